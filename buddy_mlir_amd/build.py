@@ -8,6 +8,7 @@ buddy_mlir_amd/lib/obj and rebuilt when the source or a header is newer.
 """
 from __future__ import annotations
 
+import fcntl
 import os
 import subprocess
 import sys
@@ -22,6 +23,13 @@ OBJDIR = LIBDIR / "obj"
 LIB = LIBDIR / "libbuddy_hip.so"
 RUNNER_SRC = PKG / "runner" / "buddy_hip_run.cpp"
 RUNNER = LIBDIR / "buddy_hip_run"
+TRACE_SRC = PKG / "runner" / "trace_run.cpp"
+TRACE_RUNNER = LIBDIR / "trace_run"
+# what a session built from a model folder consists of
+FOLDER_MODEL_SOURCES = [CSRC / n for n in (
+    "bf16_gemm.hip", "bf16_gemv.hip", "common.cpp", "elementwise.hip", "latent_attn.hip",
+    "linear_attn.hip", "model_folder.cpp", "model_registry.cpp", "row_ops.hip", "session.hip",
+    "session_nukopel.hip")]
 
 ARCH = "gfx950"
 # -packed-fp32-ops off: scalar float code must not be turned into v_pk_*_f32.
@@ -103,6 +111,42 @@ def _compile(src: Path, force: bool) -> Path:
     return obj
 
 
+def _run(cmd: list[str], what: str) -> None:
+    r = subprocess.run(cmd, capture_output=True, text=True)
+    if r.returncode != 0:
+        raise RuntimeError(f"{what} failed:\n{r.stdout}\n{r.stderr}")
+
+
+def _link_trace_runner(objs: list[Path]) -> None:
+    # the objects themselves: the program needs no library beside it
+    part = TRACE_RUNNER.with_name(f"trace_run.{os.getpid()}")
+    main = _compile(TRACE_SRC, False)
+    _run([_hipcc(), f"--offload-arch={ARCH}", str(main), *map(str, objs), "-o", str(part)],
+         "trace runner link")
+    os.replace(part, TRACE_RUNNER)
+
+
+def trace_runner() -> Path:
+    """The trace replay program; compiles it, and no more than it needs, when it is
+    missing or older than its sources."""
+    newest = max(f.stat().st_mtime for f in
+                 [*FOLDER_MODEL_SOURCES, TRACE_SRC, Path(__file__)])
+    newest = max(newest, _headers_mtime())
+
+    def fresh() -> bool:
+        return TRACE_RUNNER.exists() and TRACE_RUNNER.stat().st_mtime >= newest
+
+    if not fresh():
+        OBJDIR.mkdir(parents=True, exist_ok=True)
+        with open(LIBDIR / ".trace_run.lock", "w") as lock:
+            fcntl.flock(lock, fcntl.LOCK_EX)  # another call may be compiling
+            if not fresh():
+                with ThreadPoolExecutor(max_workers=8) as ex:
+                    objs = list(ex.map(lambda s: _compile(s, False), FOLDER_MODEL_SOURCES))
+                _link_trace_runner(objs)
+    return TRACE_RUNNER
+
+
 def build(force: bool = False, jobs: int = 8, verbose: bool = True) -> Path:
     OBJDIR.mkdir(parents=True, exist_ok=True)
     srcs = sources()
@@ -110,18 +154,15 @@ def build(force: bool = False, jobs: int = 8, verbose: bool = True) -> Path:
         objs = list(ex.map(lambda s: _compile(s, force), srcs))
     cmd = [_hipcc(), "-shared", "-fPIC", f"--offload-arch={ARCH}",
            "-o", str(LIB), *map(str, objs)]
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
+    _run(cmd, "link")
     # the command-line runner for the reference's w8a32 parameter files: plain
     # C++ over the C interface, found next to the library at run time
     cmd = [_hipcc(), "-O2", "-std=c++17", f"-I{ROOT / 'include'}", str(RUNNER_SRC),
            f"-L{LIBDIR}", "-lbuddy_hip", "-Wl,-rpath,$ORIGIN", "-o", str(RUNNER)]
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError(f"runner build failed:\n{r.stdout}\n{r.stderr}")
+    _run(cmd, "runner build")
+    _link_trace_runner([OBJDIR / (s.name + ".o") for s in FOLDER_MODEL_SOURCES])
     if verbose:
-        print(f"built {LIB} from {len(srcs)} sources, and {RUNNER.name}")
+        print(f"built {LIB} from {len(srcs)} sources, {RUNNER.name} and {TRACE_RUNNER.name}")
     return LIB
 
 

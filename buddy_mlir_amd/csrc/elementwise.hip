@@ -138,11 +138,13 @@ argmax_final_kernel(const float *__restrict__ pv, const int *__restrict__ pi,
 // candidates, logs it, advances position and step, then prepares the next step:
 // its embedding row and the cos/sin table of its position (shared by every
 // layer's attention kernel).  One workgroup.
+// Table: f32 rows as they are, or bfloat16 rows times a scale.
+template <typename Table>
 __global__ void __launch_bounds__(1024)
 finish_step_kernel(const float *__restrict__ pv, const int *__restrict__ pi,
                    int nparts, int *__restrict__ state, int *__restrict__ token_log,
-                   const float *__restrict__ table, int64_t hidden, int64_t vocab,
-                   float *__restrict__ x, const float *__restrict__ inv_freq,
+                   const Table *__restrict__ table, float table_scale, int64_t hidden,
+                   int64_t vocab, float *__restrict__ x, const float *__restrict__ inv_freq,
                    int half, float *__restrict__ rope, int advance, int log_cap) {
   __shared__ float sv[16];
   __shared__ int si[16];
@@ -210,9 +212,13 @@ finish_step_kernel(const float *__restrict__ pv, const int *__restrict__ pi,
   int64_t t = s_tok;
   if (t < 0 || t >= vocab)
     t = 0;
-  const float *row = table + t * hidden;
-  for (int64_t i = threadIdx.x; i < hidden; i += threads)
-    x[i] = row[i];
+  const Table *row = table + t * hidden;
+  for (int64_t i = threadIdx.x; i < hidden; i += threads) {
+    if constexpr (sizeof(Table) == 4)
+      x[i] = row[i];
+    else
+      x[i] = __uint_as_float((unsigned)row[i] << 16) * table_scale;
+  }
   if (threadIdx.x < half) {
     float sn, cs;
     sincosf(inv_freq[threadIdx.x] * (float)s_pos, &sn, &cs);
@@ -230,9 +236,23 @@ int launch_finish_step(const float *cand_v, const int *cand_i, int nparts, int *
   BH_REQUIRE(state && table && x && inv_freq && rope && head_dim > 0 &&
                  head_dim / 2 <= 256 && (nparts == 0 || (cand_v && cand_i && token_log)),
              "finish_step: bad argument");
-  hipLaunchKernelGGL(finish_step_kernel, dim3(1), dim3(nparts > 1024 ? 1024 : 256), 0, stream,
-                     cand_v, cand_i, nparts, state, token_log, table, hidden, vocab, x,
-                     inv_freq, head_dim / 2, rope, advance ? 1 : 0, token_log_cap);
+  hipLaunchKernelGGL(finish_step_kernel<float>, dim3(1), dim3(nparts > 1024 ? 1024 : 256), 0,
+                     stream, cand_v, cand_i, nparts, state, token_log, table, 1.0f, hidden, vocab,
+                     x, inv_freq, head_dim / 2, rope, advance ? 1 : 0, token_log_cap);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+int launch_finish_step_bf16(const float *cand_v, const int *cand_i, int nparts, int *state,
+                            int *token_log, const uint16_t *table, float table_scale,
+                            int64_t hidden, int64_t vocab, float *x, bool advance,
+                            int token_log_cap, hipStream_t stream) {
+  BH_REQUIRE(state && table && x && (nparts == 0 || (cand_v && cand_i && token_log)),
+             "finish_step: bad argument");
+  hipLaunchKernelGGL(finish_step_kernel<uint16_t>, dim3(1), dim3(nparts > 1024 ? 1024 : 256), 0,
+                     stream, cand_v, cand_i, nparts, state, token_log, table, table_scale, hidden,
+                     vocab, x, (const float *)nullptr, 0, (float *)nullptr, advance ? 1 : 0,
+                     token_log_cap);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }

@@ -1,0 +1,258 @@
+// linear_attn.hip -- the decaying linear-attention recurrence: one token, and a
+// prompt in chunks of 64 tokens: every chunk's own contribution to the state, a
+// scan over the chunks, then every chunk's outputs from the state it starts with
+// and its own tokens.  f32 matrix cores throughout.
+#include "linear_attn.h"
+#include "bf16_dev.h"
+
+#include <algorithm>
+
+namespace bh {
+namespace {
+
+// Grid (heads, ceil(vdim / 16)): 16 value channels x 16 slices of the key
+// dimensions, which meet in LDS in slice order.
+__global__ void __launch_bounds__(256)
+linear_step_kernel(const float *__restrict__ q, const float *__restrict__ k,
+                   const float *__restrict__ v, int dim, int vdim,
+                   const float *__restrict__ powers, float *__restrict__ state,
+                   float *__restrict__ out) {
+  __shared__ float part[16][17];
+  const int h = blockIdx.x, c = threadIdx.x & 15, slice = threadIdx.x >> 4;
+  const int vi = blockIdx.y * 16 + c;
+  const bool ok = vi < vdim;
+  const int vc = min(vi, vdim - 1);
+  const float decay = powers[h * (kLinearChunk + 1) + 1];
+  const float vv = v[(int64_t)h * vdim + vc];
+  float *S = state + (int64_t)h * dim * vdim + vc;
+  float acc = 0.f;
+  for (int d0 = slice; d0 < dim; d0 += 16 * 8) {
+    float s[8], kk[8], qq[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      const int d = min(d0 + u * 16, dim - 1);
+      s[u] = S[(int64_t)d * vdim];
+      kk[u] = k[(int64_t)h * dim + d];
+      qq[u] = q[(int64_t)h * dim + d];
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      if (d0 + u * 16 < dim) {
+        const float n = fmaf(decay, s[u], kk[u] * vv);
+        acc = fmaf(n, qq[u], acc);
+        if (ok)
+          S[(int64_t)(d0 + u * 16) * vdim] = n;
+      }
+  }
+  part[slice][c] = acc;
+  __syncthreads();
+  if (slice == 0 && ok) {
+    float t = 0.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i)
+      t += part[i][c];
+    out[(int64_t)h * vdim + vi] = t;
+  }
+}
+
+struct LinearArgs {
+  int heads, dim, vdim, ld, q_at, k_at, v_at, rows;
+  int dp; // LDS row of q / k: dim padded to 32, plus 4
+  const float *powers;
+};
+
+constexpr int kSliceV = 64, kVRow = kSliceV + 4; // value channels of a workgroup
+
+__device__ __forceinline__ void stage_rows(float *dst, int stride, const float *src, int64_t ld,
+                                           int rows, int width, int padded) {
+  for (int i = threadIdx.x; i < kLinearChunk * padded; i += 256) {
+    const int r = i / padded, c = i - r * padded;
+    dst[r * stride + c] = r < rows && c < width ? src[r * ld + c] : 0.f;
+  }
+}
+
+// Grid (chunks, heads, value slices): sum over the chunk's tokens of
+// decay^(last - i) k_i v_i^T.
+__global__ void __launch_bounds__(256)
+linear_chunk_kernel(const float *__restrict__ proj, float *__restrict__ chunk_states, LinearArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kSliceV;
+  const int rows = min(kLinearChunk, a.rows - c * kLinearChunk);
+  const int vw = min(kSliceV, a.vdim - v0);
+  float *k = lds, *v = lds + kLinearChunk * a.dp;
+  const float *src = proj + (int64_t)c * kLinearChunk * a.ld;
+  const float *pw = a.powers + h * (kLinearChunk + 1);
+  stage_rows(k, a.dp, src + a.k_at + h * a.dim, a.ld, rows, a.dim, a.dp - 4);
+  for (int i = threadIdx.x; i < kLinearChunk * kSliceV; i += 256) {
+    const int r = i / kSliceV, x = i - r * kSliceV;
+    v[r * kVRow + x] =
+        r < rows && x < vw ? src[(int64_t)r * a.ld + a.v_at + h * a.vdim + v0 + x] * pw[rows - 1 - r] : 0.f;
+  }
+  __syncthreads();
+  float *dst = chunk_states + ((int64_t)c * a.heads + h) * a.dim * a.vdim;
+  for (int dt = wave; dt * 16 < a.dim; dt += 4) {
+    f32x4 acc[kSliceV / 16];
+#pragma unroll
+    for (int t = 0; t < kSliceV / 16; ++t)
+      acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < kLinearChunk / 4; ++s) {
+      const float ka = k[(s * 4 + quad) * a.dp + dt * 16 + col];
+#pragma unroll
+      for (int t = 0; t < kSliceV / 16; ++t)
+        acc[t] = mfma_f32(ka, v[(s * 4 + quad) * kVRow + t * 16 + col], acc[t]);
+    }
+#pragma unroll
+    for (int t = 0; t < kSliceV / 16; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int d = dt * 16 + quad * 4 + r, x = t * 16 + col;
+        if (d < a.dim && x < vw)
+          dst[(int64_t)d * a.vdim + v0 + x] = acc[t][r];
+      }
+  }
+}
+
+// One thread per state element: turns the chunks' contributions into the state each
+// chunk starts with, and leaves the last one in the sequence's state.
+__global__ void __launch_bounds__(256)
+linear_scan_kernel(float *__restrict__ chunk_states, float *__restrict__ state, int per_head,
+                   int64_t total, int rows, const float *__restrict__ powers) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i >= total)
+    return;
+  const float *pw = powers + (i / per_head) * (kLinearChunk + 1);
+  float s = state[i];
+  const int chunks = (rows + kLinearChunk - 1) / kLinearChunk;
+  for (int c0 = 0; c0 < chunks; c0 += 8) {
+    float d[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      d[u] = chunk_states[(int64_t)min(c0 + u, chunks - 1) * total + i];
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      if (c0 + u < chunks) {
+        const int c = c0 + u, n = min(kLinearChunk, rows - c * kLinearChunk);
+        chunk_states[(int64_t)c * total + i] = s;
+        s = fmaf(s, pw[n], d[u]);
+      }
+  }
+  state[i] = s;
+}
+
+// Grid (chunks, heads, value slices): o_i = decay^(i+1) S^T q_i + sum over j <= i of
+// decay^(i-j) (q_i . k_j) v_j.
+__global__ void __launch_bounds__(256)
+linear_out_kernel(const float *__restrict__ proj, const float *__restrict__ chunk_states,
+                  float *__restrict__ out, LinearArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float pw[kLinearChunk + 1];
+  const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kSliceV;
+  const int rows = min(kLinearChunk, a.rows - c * kLinearChunk);
+  const int vw = min(kSliceV, a.vdim - v0);
+  float *q = lds, *k = q + kLinearChunk * a.dp, *v = k + kLinearChunk * a.dp;
+  const float *src = proj + (int64_t)c * kLinearChunk * a.ld;
+  stage_rows(q, a.dp, src + a.q_at + h * a.dim, a.ld, rows, a.dim, a.dp - 4);
+  stage_rows(k, a.dp, src + a.k_at + h * a.dim, a.ld, rows, a.dim, a.dp - 4);
+  stage_rows(v, kVRow, src + a.v_at + h * a.vdim + v0, a.ld, rows, vw, kSliceV);
+  if (threadIdx.x <= kLinearChunk)
+    pw[threadIdx.x] = a.powers[h * (kLinearChunk + 1) + threadIdx.x];
+  __syncthreads();
+  if (wave * 16 >= rows)
+    return;
+  const int qi = wave * 16 + col; // this lane's query within the chunk
+  constexpr int NV = kSliceV / 16;
+  f32x4 o[NV];
+#pragma unroll
+  for (int t = 0; t < NV; ++t)
+    o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  // state part: A = S^T (value channels x key dimensions), B = the scaled queries
+  const float *S = chunk_states + ((int64_t)c * a.heads + h) * a.dim * a.vdim + v0;
+  const float lead = pw[qi + 1];
+  for (int d0 = 0; d0 < a.dim; d0 += 4) {
+    const int d = min(d0 + quad, a.dim - 1);
+    const float qb = d0 + quad < a.dim ? q[qi * a.dp + d] * lead : 0.f;
+#pragma unroll
+    for (int t = 0; t < NV; ++t) {
+      const int x = min(t * 16 + col, vw - 1);
+      o[t] = mfma_f32(S[(int64_t)d * a.vdim + x], qb, o[t]);
+    }
+  }
+  // tokens of the chunk up to the query
+  for (int kt = 0; kt <= wave; ++kt) {
+    f32x4 s{0.f, 0.f, 0.f, 0.f};
+    const float *kr = k + (kt * 16 + col) * a.dp + quad * 8, *qr = q + qi * a.dp + quad * 8;
+    for (int t = 0; t < a.dp - 4; t += 32) {
+      Frag<float> kf, qf;
+      kf.load(kr + t);
+      qf.load(qr + t);
+      s = mfma32(kf, qf, s);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int gap = qi - (kt * 16 + quad * 4 + r);
+      s[r] = gap >= 0 ? s[r] * pw[max(gap, 0)] : 0.f;
+    }
+#pragma unroll
+    for (int t = 0; t < NV; ++t)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        o[t] = mfma_f32(v[(kt * 16 + quad * 4 + r) * kVRow + t * 16 + col], s[r], o[t]);
+  }
+  if (qi >= rows)
+    return;
+  float *dst = out + ((int64_t)c * kLinearChunk + qi) * a.heads * a.vdim + (int64_t)h * a.vdim + v0;
+#pragma unroll
+  for (int t = 0; t < NV; ++t)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int x = t * 16 + quad * 4 + r;
+      if (x < vw)
+        dst[x] = o[t][r];
+    }
+}
+
+} // namespace
+
+int launch_linear_step(const LinearStep &a, hipStream_t stream) {
+  BH_REQUIRE(a.q && a.k && a.v && a.powers && a.state && a.out && a.s.heads > 0 && a.s.dim > 0 &&
+                 a.s.vdim > 0,
+             "linear_step: bad argument");
+  hipLaunchKernelGGL(linear_step_kernel, dim3(a.s.heads, (unsigned)ceil_div(a.s.vdim, 16)),
+                     dim3(256), 0, stream, a.q, a.k, a.v, a.s.dim, a.s.vdim, a.powers, a.state,
+                     a.out);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+int launch_linear_rows(const LinearRows &a, hipStream_t stream) {
+  const LinearShape &s = a.s;
+  BH_REQUIRE(a.proj && a.powers && a.state && a.chunk_states && a.out && a.rows > 0 && s.heads > 0 &&
+                 s.dim > 0 && s.vdim > 0,
+             "linear_rows: bad argument");
+  LinearArgs p{s.heads, s.dim, s.vdim, a.ld, a.q_at, a.k_at, a.v_at, a.rows, 0, a.powers};
+  p.dp = (int)round_up(s.dim, 32) + 4;
+  const size_t out_lds = sizeof(float) * kLinearChunk * (2 * (size_t)p.dp + kVRow);
+  constexpr size_t kLimit = 156 * 1024;
+  BH_REQUIRE(out_lds <= kLimit, "linear_rows: key heads of %d values do not fit LDS", s.dim);
+  const size_t chunk_lds = sizeof(float) * kLinearChunk * ((size_t)p.dp + kVRow);
+  static DynLdsOnce once_chunk, once_out;
+  BH_CHECK_HIP(ensure_dyn_lds(once_chunk, (const void *)linear_chunk_kernel, (int)kLimit));
+  BH_CHECK_HIP(ensure_dyn_lds(once_out, (const void *)linear_out_kernel, (int)kLimit));
+  const dim3 grid((unsigned)linear_chunks(a.rows), (unsigned)s.heads,
+                  (unsigned)ceil_div(s.vdim, kSliceV));
+  hipLaunchKernelGGL(linear_chunk_kernel, grid, dim3(256), chunk_lds, stream, a.proj,
+                     a.chunk_states, p);
+  const int64_t total = (int64_t)s.heads * s.dim * s.vdim;
+  hipLaunchKernelGGL(linear_scan_kernel, dim3((unsigned)ceil_div(total, 256)), dim3(256), 0, stream,
+                     a.chunk_states, a.state, s.dim * s.vdim, total, a.rows, a.powers);
+  hipLaunchKernelGGL(linear_out_kernel, grid, dim3(256), out_lds, stream, a.proj, a.chunk_states,
+                     a.out, p);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+} // namespace bh

@@ -1,0 +1,271 @@
+// row_ops.hip -- residual, norm, convolution and routing of many rows.
+#include "row_ops.h"
+#include "bf16_dev.h"
+#include "bf16_linear.h"
+
+#include <algorithm>
+
+namespace bh {
+namespace {
+
+__global__ void __launch_bounds__(256)
+embed_rows_kernel(const uint16_t *__restrict__ table, const int *__restrict__ tokens, int width,
+                  int vocab, float scale, float *__restrict__ x) {
+  int t = tokens[blockIdx.x];
+  if (t < 0 || t >= vocab)
+    t = 0;
+  const uint16_t *row = table + (int64_t)t * width;
+  float *dst = x + (int64_t)blockIdx.x * width;
+  for (int i = threadIdx.x; i < width; i += 256)
+    dst[i] = bf_f(row[i]) * scale;
+}
+
+__device__ __forceinline__ float block_sum4(float v, float *red) {
+  v = wave_sum(v);
+  if ((threadIdx.x & 63) == 0)
+    red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) norm_rows_kernel(NormRows a) {
+  extern __shared__ float lds[]; // x' of the row, then y
+  __shared__ float red[2][4];
+  const int tid = threadIdx.x, W = a.width;
+  const int64_t r = a.pick ? a.pick[blockIdx.x] : blockIdx.x;
+  float *x = a.x + r * W;
+  float *xb = lds, *yb = lds + W;
+  float ss = 0.f;
+  for (int i = tid; i < W; i += 256) {
+    xb[i] = x[i];
+    if (a.y || a.expert_out) {
+      float y = a.y ? a.y[r * a.ldy + i] : 0.f;
+      for (int j = 0; j < a.top; ++j)
+        y = fmaf(a.expert_w[r * a.top + j], a.expert_out[(r * a.top + j) * a.lde + i], y);
+      yb[i] = y;
+      ss = fmaf(y, y, ss);
+    }
+  }
+  if (a.y || a.expert_out) {
+    const float ry = a.out_gain / sqrtf(block_sum4(ss, red[0]) / (float)W + a.eps);
+    for (int i = tid; i < W; i += 256) {
+      const float v = fmaf(yb[i], ry, xb[i]);
+      xb[i] = v;
+      if (a.write_x)
+        x[i] = v;
+    }
+  }
+  if (!a.out_f32 && !a.out_act)
+    return;
+  ss = 0.f;
+  for (int i = tid; i < W; i += 256)
+    ss = fmaf(xb[i], xb[i], ss);
+  const float g = a.gain / sqrtf(block_sum4(ss, red[1]) / (float)W + a.eps);
+  for (int i = tid; i < W; i += 256) {
+    const float v = xb[i] * g;
+    if (a.out_f32)
+      a.out_f32[(int64_t)blockIdx.x * W + i] = v;
+    if (a.out_act)
+      store_act<T>(static_cast<T *>(a.out_act) + (int64_t)blockIdx.x * a.ld_act + i, v);
+  }
+}
+
+template <typename T> __global__ void __launch_bounds__(256) conv_rows_kernel(ConvRows a) {
+  const int64_t r = blockIdx.x;
+  const int p = a.start + (int)r;
+  for (int i = threadIdx.x; i < a.width; i += 256) {
+    const float h = a.h[r * a.width + i];
+    float c = 0.f;
+    for (int b = a.taps - 1; b >= 1; --b) {
+      if (p - b < 0)
+        continue;
+      const float e = r >= b ? a.h[(r - b) * a.width + i]
+                             : a.ring[(int64_t)((p - b) % a.taps) * a.width + i];
+      c = fmaf(a.w[(int64_t)(a.taps - 1 - b) * a.width + i], e, c);
+    }
+    store_act<T>(static_cast<T *>(a.out) + r * a.ld + i,
+                 h + fmaf(a.w[(int64_t)(a.taps - 1) * a.width + i], h, c));
+  }
+}
+
+// the last min(rows, taps) rows into their slots
+__global__ void __launch_bounds__(256)
+conv_save_kernel(const float *__restrict__ h, float *__restrict__ ring, int taps, int width, int rows,
+                 int start) {
+  const int r = rows - 1 - (int)blockIdx.x;
+  const int slot = (start + r) % taps;
+  for (int i = threadIdx.x; i < width; i += 256)
+    ring[(int64_t)slot * width + i] = h[(int64_t)r * width + i];
+}
+
+template <typename T> __global__ void __launch_bounds__(256) gated_norm_rows_kernel(GatedNormRows a) {
+  extern __shared__ float lds[];
+  __shared__ float red[4];
+  const int64_t r = blockIdx.x;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < a.width; i += 256) {
+    const float v = a.x[r * a.width + i];
+    lds[i] = v;
+    ss = fmaf(v, v, ss);
+  }
+  const float g = 1.0f / sqrtf(block_sum4(ss, red) / (float)a.width + a.eps);
+  for (int i = threadIdx.x; i < a.width; i += 256)
+    store_act<T>(static_cast<T *>(a.out) + r * a.ld + i,
+                 lds[i] * g * a.w[i] * sigmoid_f(a.gate[r * a.ld_gate + i]));
+}
+
+__device__ __forceinline__ unsigned rank_key(float f) {
+  const unsigned u = __float_as_uint(f);
+  return max(u & 0x80000000u ? ~u : u | 0x80000000u, 1u);
+}
+
+// A wavefront per row, four rows per workgroup.
+template <int R>
+__global__ void __launch_bounds__(256) route_pick_kernel(RouteRows a) {
+  const int lane = threadIdx.x & 63;
+  const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row >= a.rows)
+    return;
+  float val[R];
+  unsigned key[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const int i = r * 64 + lane;
+    val[r] = a.logits[row * a.ld + min(i, a.experts - 1)];
+    key[r] = i < a.experts ? rank_key(val[r]) : 0u;
+  }
+  float mine = -INFINITY;
+  int mine_idx = 0;
+  for (int it = 0; it < a.top; ++it) {
+    unsigned best = key[0];
+#pragma unroll
+    for (int r = 1; r < R; ++r)
+      best = max(best, key[r]);
+    const unsigned m = wave_max_u32(best);
+    bool found = false;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      const unsigned long long b = __ballot(key[r] == m);
+      if (!found && b) {
+        found = true;
+        const int l = __builtin_ctzll(b);
+        const float z = lane_f(val[r], l);
+        if (lane == l)
+          key[r] = 0;
+        if (lane == it) {
+          mine = z;
+          mine_idx = r * 64 + l;
+        }
+      }
+    }
+  }
+  const float e = lane < a.top ? expf(mine - wave_max(mine)) : 0.f;
+  const float w = e / wave_sum(e);
+  if (lane < a.top) {
+    a.chosen[row * a.top + lane] = mine_idx;
+    a.weights[row * a.top + lane] = w;
+  }
+}
+
+// A workgroup per expert walks all assignments in order.
+__global__ void __launch_bounds__(1024)
+route_list_kernel(const int *__restrict__ chosen, int total, int *__restrict__ counts,
+                  int *__restrict__ lists, int list_cap) {
+  __shared__ int wave_count[16];
+  const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  int *list = lists + (int64_t)e * list_cap;
+  int have = 0;
+  for (int base = 0; base < total; base += 1024) {
+    const int i = base + tid;
+    const bool hit = i < total && chosen[i] == e;
+    const unsigned long long b = __ballot(hit);
+    if (lane == 0)
+      wave_count[wave] = __popcll(b);
+    __syncthreads();
+    int before = have;
+    for (int w = 0; w < 16; ++w) {
+      if (w < wave)
+        before += wave_count[w];
+      have += wave_count[w];
+    }
+    if (hit)
+      list[before + __popcll(b & ((1ull << lane) - 1))] = i;
+    __syncthreads();
+  }
+  if (tid == 0)
+    counts[e] = have;
+}
+
+} // namespace
+
+int launch_embed_rows(const uint16_t *table, const int *tokens, int rows, int width, int vocab,
+                      float scale, float *x, hipStream_t stream) {
+  BH_REQUIRE(table && tokens && x && rows > 0 && width > 0 && vocab > 0, "embed_rows: bad argument");
+  hipLaunchKernelGGL(embed_rows_kernel, dim3(rows), dim3(256), 0, stream, table, tokens, width,
+                     vocab, scale, x);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+int launch_norm_rows(const NormRows &a, hipStream_t stream) {
+  BH_REQUIRE(a.x && a.rows > 0 && a.width > 0 && (!a.pick || !a.write_x) &&
+                 (!a.expert_out || (a.expert_w && a.top > 0)) && (a.expert_out || a.top == 0),
+             "norm_rows: bad argument");
+  const size_t lds = 2 * sizeof(float) * (size_t)a.width;
+  constexpr size_t kLimit = 150 * 1024;
+  BH_REQUIRE(lds <= kLimit, "norm_rows: a row of %d values does not fit LDS", a.width);
+  static DynLdsOnce once_f, once_b;
+  if (a.act_f32) {
+    BH_CHECK_HIP(ensure_dyn_lds(once_f, (const void *)norm_rows_kernel<float>, (int)kLimit));
+    hipLaunchKernelGGL(norm_rows_kernel<float>, dim3(a.rows), dim3(256), lds, stream, a);
+  } else {
+    BH_CHECK_HIP(ensure_dyn_lds(once_b, (const void *)norm_rows_kernel<bf16_bits>, (int)kLimit));
+    hipLaunchKernelGGL(norm_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), lds, stream, a);
+  }
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+int launch_conv_rows(const ConvRows &a, hipStream_t stream) {
+  BH_REQUIRE(a.h && a.w && a.ring && a.out && a.taps > 0 && a.width > 0 && a.rows > 0 && a.start >= 0,
+             "conv_rows: bad argument");
+  if (a.act_f32)
+    hipLaunchKernelGGL(conv_rows_kernel<float>, dim3(a.rows), dim3(256), 0, stream, a);
+  else
+    hipLaunchKernelGGL(conv_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), 0, stream, a);
+  hipLaunchKernelGGL(conv_save_kernel, dim3(std::min(a.rows, a.taps)), dim3(256), 0, stream, a.h,
+                     a.ring, a.taps, a.width, a.rows, a.start);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+int launch_gated_norm_rows(const GatedNormRows &a, hipStream_t stream) {
+  BH_REQUIRE(a.x && a.w && a.gate && a.out && a.rows > 0 && a.width > 0 && a.width <= 16384,
+             "gated_norm_rows: bad argument");
+  const size_t lds = sizeof(float) * (size_t)a.width;
+  if (a.act_f32)
+    hipLaunchKernelGGL(gated_norm_rows_kernel<float>, dim3(a.rows), dim3(256), lds, stream, a);
+  else
+    hipLaunchKernelGGL(gated_norm_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), lds, stream, a);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+int launch_route_rows(const RouteRows &a, hipStream_t stream) {
+  BH_REQUIRE(a.logits && a.chosen && a.weights && a.counts && a.lists && a.rows > 0 &&
+                 a.experts > 0 && a.experts <= kMaxExperts && a.top > 0 && a.top <= 64 &&
+                 a.top <= a.experts && a.list_cap >= a.rows,
+             "route_rows: bad argument");
+  const dim3 grid((unsigned)ceil_div(a.rows, 4));
+  if (a.experts <= 64)
+    hipLaunchKernelGGL(route_pick_kernel<1>, grid, dim3(256), 0, stream, a);
+  else
+    hipLaunchKernelGGL(route_pick_kernel<kMaxExperts / 64>, grid, dim3(256), 0, stream, a);
+  hipLaunchKernelGGL(route_list_kernel, dim3(a.experts), dim3(1024), 0, stream, a.chosen,
+                     a.rows * a.top, a.counts, a.lists, a.list_cap);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
+} // namespace bh

@@ -471,6 +471,16 @@ int buddy_hip_session_prefill(buddy_hip_session *s, const int *tokens,
 int buddy_hip_session_prefill_all_logits(buddy_hip_session *s, const int *tokens,
                                          int n_tokens, int start_pos,
                                          float *logits_out);
+/* The same with the logits of chosen rows: `rows` (host) ascends within
+ * 0..n_tokens - 1, logits_out is [n_rows, vocab] (host or device); n_rows may be 0.
+ * A prompt may come in portions, each starting where the last one ended. */
+int buddy_hip_session_prefill_rows(buddy_hip_session *s, const int *tokens, int n_tokens,
+                                   int start_pos, const int *rows, int n_rows,
+                                   float *logits_out);
+/* Ends the sequence the session holds: what it keeps in caches and states is given
+ * back, and the next token stands at position 0.  (Beginning at position 0 does the
+ * same.) */
+int buddy_hip_session_reset(buddy_hip_session *s);
 /* Hands a device allocation to the session, which frees it when destroyed. */
 void buddy_hip_session_adopt(buddy_hip_session *s, void *device_ptr);
 /* How the prefill matmuls carry their f32 activations:
@@ -487,6 +497,34 @@ int buddy_hip_session_enqueue_steps(buddy_hip_session *s, int steps);
 const float *buddy_hip_session_logits(buddy_hip_session *s); /* device */
 buddy_hip_stream buddy_hip_session_stream(buddy_hip_session *s);
 int buddy_hip_session_vocab(buddy_hip_session *s);
+/* The name the model registry knows the session's model by. */
+const char *buddy_hip_session_architecture(buddy_hip_session *s);
+
+/* ---- models from a folder ------------------------------------------------------
+ * Builds a session from a folder with config.json and model.safetensors: the
+ * registry picks the model class by config.json's "architecture".  Every
+ * buddy_hip_session_* call above works on it except those that name the Qwen2
+ * shape's parts (set_globals, set_layer, set_kv, get_kv, get_kv_rows,
+ * decode_mirror's rows, set_prefill_precision, discard_kv), which are refused.
+ *
+ * A model with a recurrent state continues only where its state stands: a decode
+ * or prefill call must start at the position that follows the last token, or at
+ * position 0, which begins a new sequence. */
+enum {
+  BUDDY_HIP_MODEL_BF16 = 0, /* matrix products and cache in bfloat16, f32 sums */
+  BUDDY_HIP_MODEL_F32 = 1   /* every product and the cache in f32 */
+};
+typedef struct buddy_hip_model_options {
+  int dtype;         /* BUDDY_HIP_MODEL_* */
+  int max_len;       /* positions of a sequence; 0: 4096 */
+  int prefill_block; /* tokens of a prompt that go through the layers at once; 0: 2048 */
+  buddy_hip_stream stream; /* NULL: the session creates its own */
+} buddy_hip_model_options;
+/* options may be NULL.  Returns NULL on failure. */
+buddy_hip_session *buddy_hip_session_create_from_folder(const char *folder,
+                                                        const buddy_hip_model_options *options);
+/* The i-th architecture the registry knows, NULL past the last. */
+const char *buddy_hip_model_architecture(int index);
 
 /* ---- token sampler ----------------------------------------------------------
  * buddy::runtime::Sampler (runtime/include/buddy/runtime/llm/Sampler.h:38-46
