@@ -129,6 +129,11 @@ def _declare(lib):
         "buddy_hip_session_prefill": (c_int, [vp, vp, c_int, c_int, vp, vp]),
         "buddy_hip_session_set_prefill_precision": (c_int, [vp, c_int]),
         "buddy_hip_session_prefill_all_logits": (c_int, [vp, vp, c_int, c_int, vp]),
+        "buddy_hip_session_prefill_rows": (c_int, [vp, vp, c_int, c_int, vp, c_int, vp]),
+        "buddy_hip_session_reset": (c_int, [vp]),
+        "buddy_hip_session_architecture": (c_char_p, [vp]),
+        "buddy_hip_session_create_from_folder": (vp, [c_char_p, vp]),
+        "buddy_hip_model_architecture": (c_char_p, [c_int]),
         "buddy_hip_session_adopt": (None, [vp, vp]),
         "buddy_hip_w8a32_blob_sizes": (None, [vp, vp, vp]),
         "buddy_hip_w8a32_blob_layout": (i64, [vp, vp, i64]),

@@ -15,6 +15,11 @@
 //                 --kv-heads 2 --inter 8960 --vocab 151936]
 //                 [--temperature T --top-k K --top-p P --min-p P
 //                  --repeat-penalty R --repeat-last-n N --seed S]
+//   buddy_hip_run --model DIR --tokens ... [--dtype bfloat16|float32] [...]
+//
+// The second form takes a model folder (config.json and model.safetensors) of any
+// architecture the library's registry knows; everything behind the loading is the
+// same, except that no end-of-text id is assumed.
 //
 // With a temperature above 0 or a repetition penalty other than 1 the next
 // token comes from the library's sampler
@@ -42,10 +47,12 @@ void usage(FILE *f) {
         "                     --kv-heads N --inter N --vocab N]\n"
         "                     [--temperature T --top-k K --top-p P --min-p P\n"
         "                      --repeat-penalty R --repeat-last-n N --seed S]\n"
+        "       buddy_hip_run --model DIR --tokens ID,ID,... [--dtype bfloat16|float32] ...\n"
         "Runs the reference's w8a32 parameter files (arg0-w8a32-f32.data,\n"
         "arg0-w8a32-i8.data) through libbuddy_hip: prefill of the prompt tokens, then\n"
         "greedy decoding, or sampling when a temperature or a repetition penalty is\n"
-        "given.  Defaults are the DeepSeek-R1-Distill-Qwen-1.5B shape.\n",
+        "given.  Defaults are the DeepSeek-R1-Distill-Qwen-1.5B shape.  --model takes a\n"
+        "folder with config.json and model.safetensors instead.\n",
         f);
 }
 
@@ -99,9 +106,10 @@ double seconds_since(std::chrono::steady_clock::time_point t0) {
 
 int main(int argc, char **argv) {
   buddy_hip_model_shape shape = {28, 1536, 12, 2, 128, 8960, 151936, 1024, 1e-6f};
-  std::string f32_path, i8_path;
+  std::string f32_path, i8_path, folder, dtype = "bfloat16";
   std::vector<int> prompt;
   int max_new = 64, eos = 151643;
+  bool eos_given = false;
   buddy_hip_sampler_config sampling = {0.0f, 0, 1.0f, 0.0f, 1.0f, 64, 0};
   for (int i = 1; i < argc; ++i) {
     const std::string a = argv[i];
@@ -116,6 +124,8 @@ int main(int argc, char **argv) {
     const char *v = argv[++i];
     if (a == "--f32") f32_path = v;
     else if (a == "--i8") i8_path = v;
+    else if (a == "--model") folder = v;
+    else if (a == "--dtype") dtype = v;
     else if (a == "--tokens") {
       if (!parse_tokens(v, prompt)) {
         fprintf(stderr, "[Error] --tokens wants a comma separated list of ids\n");
@@ -123,7 +133,10 @@ int main(int argc, char **argv) {
       }
     } else if (a == "--max-new") max_new = atoi(v);
     else if (a == "--max-len") shape.max_len = atoi(v);
-    else if (a == "--eos") eos = atoi(v);
+    else if (a == "--eos") {
+      eos = atoi(v);
+      eos_given = true;
+    }
     else if (a == "--layers") shape.layers = atoi(v);
     else if (a == "--hidden") shape.hidden = atoi(v);
     else if (a == "--heads") shape.heads = atoi(v);
@@ -142,7 +155,9 @@ int main(int argc, char **argv) {
       return 2;
     }
   }
-  if (f32_path.empty() || i8_path.empty() || prompt.empty() || max_new < 1) {
+  const bool from_folder = !folder.empty();
+  if ((from_folder ? !f32_path.empty() || !i8_path.empty() : f32_path.empty() || i8_path.empty()) ||
+      (dtype != "bfloat16" && dtype != "float32") || prompt.empty() || max_new < 1) {
     usage(stderr);
     return 2;
   }
@@ -151,30 +166,53 @@ int main(int argc, char **argv) {
             prompt.size(), max_new, shape.max_len);
     return 2;
   }
-  for (int t : prompt)
-    if (t >= shape.vocab) {
-      fprintf(stderr, "[Error] token id %d outside the vocabulary (%d)\n", t, shape.vocab);
-      return 2;
-    }
-
-  int64_t n_f32 = 0, n_i8 = 0;
-  buddy_hip_w8a32_blob_sizes(&shape, &n_f32, &n_i8);
+  auto in_vocabulary = [&] {
+    for (int t : prompt)
+      if (t >= shape.vocab) {
+        fprintf(stderr, "[Error] token id %d outside the vocabulary (%d)\n", t, shape.vocab);
+        return false;
+      }
+    return true;
+  };
+  buddy_hip_session *s = nullptr;
   auto t0 = std::chrono::steady_clock::now();
-  std::vector<float> f32;
-  std::vector<int8_t> i8;
-  if (!read_file(f32_path, n_f32, f32) || !read_file(i8_path, n_i8, i8))
-    return 1;
-  printf("[Log] Params load time: %.3fs\n", seconds_since(t0));
+  if (from_folder) {
+    if (!eos_given)
+      eos = -1;
+    buddy_hip_model_options o = {};
+    o.dtype = dtype == "float32" ? BUDDY_HIP_MODEL_F32 : BUDDY_HIP_MODEL_BF16;
+    o.max_len = shape.max_len;
+    s = buddy_hip_session_create_from_folder(folder.c_str(), &o);
+    if (!s) {
+      fprintf(stderr, "[Error] %s\n", buddy_hip_last_error());
+      return 1;
+    }
+    shape.vocab = buddy_hip_session_vocab(s);
+    if (!in_vocabulary())
+      return 2;
+    printf("[Log] %s, load and packing: %.3fs\n", buddy_hip_session_architecture(s),
+           seconds_since(t0));
+  } else {
+    if (!in_vocabulary())
+      return 2;
+    int64_t n_f32 = 0, n_i8 = 0;
+    buddy_hip_w8a32_blob_sizes(&shape, &n_f32, &n_i8);
+    t0 = std::chrono::steady_clock::now();
+    std::vector<float> f32;
+    std::vector<int8_t> i8;
+    if (!read_file(f32_path, n_f32, f32) || !read_file(i8_path, n_i8, i8))
+      return 1;
+    printf("[Log] Params load time: %.3fs\n", seconds_since(t0));
 
-  t0 = std::chrono::steady_clock::now();
-  buddy_hip_session *s =
-      buddy_hip_session_create_from_w8a32_blobs(&shape, f32.data(), n_f32, i8.data(), n_i8);
-  if (!s) {
-    fprintf(stderr, "[Error] %s\n", buddy_hip_last_error());
-    return 1;
+    t0 = std::chrono::steady_clock::now();
+    s = buddy_hip_session_create_from_w8a32_blobs(&shape, f32.data(), n_f32, i8.data(), n_i8);
+    if (!s) {
+      fprintf(stderr, "[Error] %s\n", buddy_hip_last_error());
+      return 1;
+    }
+    std::vector<int8_t>().swap(i8); // the session holds its own packed copy
+    printf("[Log] Upload and packing: %.3fs\n", seconds_since(t0));
   }
-  std::vector<int8_t>().swap(i8); // the session holds its own packed copy
-  printf("[Log] Upload and packing: %.3fs\n", seconds_since(t0));
 
   const bool sampled = sampling.temperature > 0.0f || sampling.repeat_penalty != 1.0f;
   buddy_hip_sampler *sampler = nullptr;

@@ -144,12 +144,12 @@ def forward(cfg, tensors, tokens, layers_out=None):
 
 def to_bf16_bits(a):
     """float -> bfloat16 bit patterns, round to nearest even."""
-    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
-    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+    u = np.array(a, np.float32, order="C").view(np.uint32)
+    return np.asarray((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
 
 
 def from_bf16_bits(b):
-    return (np.asarray(b).astype(np.uint32) << 16).view(np.float32).astype(np.float64)
+    return np.asarray(np.asarray(b).astype(np.uint32) << 16).view(np.float32).astype(np.float64)
 
 
 def bf16(a):

@@ -1,0 +1,395 @@
+"""The Nukopel session on the GPU against the plain implementation of the tests:
+every mechanism, prompts and decoding, portions, sequences one after the other, far
+keys and window edges, and generation through the framework's own entry points."""
+import json
+import os
+import subprocess
+from pathlib import Path
+
+import numpy as np
+import pytest
+
+import buddy_mlir_amd as bma
+import nukopel_models as M
+import nukopel_oracle as N
+from buddy_mlir_amd import BuddyHipError
+from buddy_mlir_amd.session import FolderSession, Sampler
+
+pytestmark = pytest.mark.gpu
+
+ROOT = Path(__file__).resolve().parent.parent
+# f32: rounding of sums only.  bfloat16: 2^-9 per stored activation, a dozen of them
+# on the way through a few layers.
+BOUND = {"float32": 2e-5, "bfloat16": 4e-2}
+DTYPES = ("float32", "bfloat16")
+
+
+def tokens_for(cfg, n, seed=1):
+    return np.random.default_rng(seed).integers(0, cfg["vocab"], n).astype(np.int32)
+
+
+def check(got, want, dtype, what="", strict=False):
+    """Every row within the bound.  Of many bfloat16 rows a few may lie above it: where
+    two router logits are closer than the format's rounding, another expert is chosen."""
+    e = M.row_errors(got, want)
+    assert np.isfinite(got).all()
+    if dtype == "bfloat16" and len(e) >= 20 and not strict:
+        assert np.median(e) < BOUND[dtype] / 2 and np.mean(e > BOUND[dtype]) < 0.15, \
+            (what, float(np.median(e)), float(np.mean(e > BOUND[dtype])))
+    else:
+        assert e.max() < BOUND[dtype], (what, int(e.argmax()), float(e.max()))
+
+
+def all_rows(s, tokens, start=0):
+    return s.prefill_rows(tokens, np.arange(len(tokens)), start)
+
+
+def feed(s, tokens, cuts):
+    """The sequence in portions of the given sizes (1 = a decode step), its logits."""
+    out, at = [], 0
+    for n in cuts:
+        part = tokens[at:at + n]
+        if n == 1:
+            out.append(s.decode(int(part[0]), at)[1][None])
+        else:
+            out.append(all_rows(s, part, at))
+        at += n
+    assert at == len(tokens)
+    return np.concatenate(out)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", list(M.SIZES))
+def test_prompt_and_decoding_match_the_oracle(tmp_path, name, dtype):
+    cfg = M.SIZES[name]
+    folder, t = M.build(tmp_path, cfg, seed=len(name))
+    tokens = tokens_for(cfg, 90)
+    want = N.forward(cfg, t, tokens)
+    s = FolderSession(folder, dtype, max_len=128)
+    assert s.vocab == cfg["vocab"] and s.architecture == "Nukopel"
+    check(all_rows(s, tokens), want, dtype, "prompt")
+    check(feed(s, tokens, [1] * 90), want, dtype, "decoding")
+    check(feed(s, tokens, [70] + [1] * 20), want, dtype, "prompt, then decoding")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("what", ["latent", "linear", "experts", "shared", "convolution"])
+def test_mechanism_alone(tmp_path, what, dtype):
+    """One layer, the head an identity: the logits are the normed residual."""
+    layer = {"latent": M.latent(mlp=None), "linear": M.linear(mlp=None),
+             "experts": M.linear(mlp=M.moe(experts=9, top=4, shared_ff=0, limit=0.4)),
+             "shared": M.latent(mlp=M.moe(experts=1, top=1, shared_ff=33, shared_limit=0.3)),
+             "convolution": M.latent(window=1, mlp=None)}[what]
+    cfg = M.config([layer], width=56, vocab=64, taps=5 if what == "convolution" else 2)
+
+    def edit(t):
+        t["head"] = np.eye(64, 56)
+        if what in ("experts", "shared"):
+            t["l0.mix.o"] *= 0.0          # the feed-forward alone
+        if what == "convolution":
+            t["l0.canon1"] *= 2.0
+    folder, t = M.build(tmp_path, cfg, 3, edit)
+    tokens = tokens_for(cfg, 70)
+    want = N.forward(cfg, t, tokens)
+    s = FolderSession(folder, dtype, max_len=80)
+    check(all_rows(s, tokens), want, dtype, "prompt")
+    check(feed(s, tokens, [3] + [1] * 67), want, dtype, "decoding")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("block", [0, 16])
+def test_portions_do_not_matter(tmp_path, dtype, block):
+    """Cuts anywhere, down to two tokens and one, also where a portion is longer than
+    the block in which it goes through the layers and the ring of cache rows wraps."""
+    cfg = M.SIZES["mixed"] if dtype == "float32" else M.STEADY
+    folder, t = M.build(tmp_path, cfg)
+    tokens = tokens_for(cfg, 205, 7)
+    want = N.forward(cfg, t, tokens)
+    s = FolderSession(folder, dtype, max_len=256, prefill_block=block)
+    rng = np.random.default_rng(8)
+    for cuts in ([205], [2] * 102 + [1], [3, 64, 1, 2, 63, 65, 1, 1, 5], None, None):
+        if cuts is None:
+            cuts = []
+            while sum(cuts) < 205:
+                cuts.append(int(min(rng.choice([1, 2, 3, 17, 37, 64]), 205 - sum(cuts))))
+        check(feed(s, tokens, cuts), want, dtype, cuts, strict=True)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_sequences_one_after_the_other(tmp_path, dtype):
+    """What an earlier sequence left in caches, rings and states is not seen, whether
+    it was ended or simply overtaken by position 0."""
+    cfg = M.SIZES["mixed"] if dtype == "float32" else M.STEADY
+    folder, t = M.build(tmp_path, cfg)
+    s = FolderSession(folder, dtype, max_len=160)
+    reqs = [tokens_for(cfg, n, n) for n in (150, 1, 2, 23, 97)]
+    fresh = [feed(FolderSession(folder, dtype, max_len=160), r, [len(r)]) for r in reqs]
+    for r, f in zip(reqs, fresh):
+        check(f, N.forward(cfg, t, r), dtype)
+    for end in (True, False):
+        for i in (0, 1, 3, 0, 2, 4, 1, 0):
+            np.testing.assert_array_equal(feed(s, reqs[i], [len(reqs[i])]), fresh[i])
+            if end:
+                s.reset()
+    # decoding from position 0 over what a long prompt left
+    feed(s, reqs[0], [150])
+    check(feed(s, reqs[3], [1] * 23), N.forward(cfg, t, reqs[3]), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("decoded", [False, True])
+def test_window_edges(tmp_path, dtype, decoded):
+    """A key whose score stands out, just inside and just outside the window, from the
+    first tokens on and after the ring of cache rows has wrapped."""
+    window = 24
+    cfg, t, ask, needle, found = M.needle_model(window)
+    folder = N.write_model(tmp_path, cfg, t)
+    s = FolderSession(folder, dtype, max_len=512, prefill_block=16)   # ring of 64 rows
+    for at in (0, 1, 15, 16, 39, 40, 63, 64, 127, 200):
+        for gap in (1, window - 1, window):
+            n = at + gap + 1
+            tokens = np.random.default_rng(at + gap).integers(4, cfg["vocab"], n).astype(np.int32)
+            tokens[at], tokens[-1] = needle, ask
+            want = N.forward(cfg, t, tokens)[-1]
+            seen = want[found] > 1.0
+            assert seen == (gap < window)              # the oracle tells them apart
+            if decoded:
+                if n > 1:
+                    s.prefill(tokens[:-1], 0)
+                got = s.decode(ask, n - 1)[1]
+            else:
+                got = s.prefill(tokens, 0)[1]
+            assert (got[found] > 1.0) == seen
+            check(got[None], want[None], dtype, (at, gap))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_window_passes_over_decoded_tokens(tmp_path, dtype):
+    window = 9
+    cfg, t, ask, needle, found = M.needle_model(window)
+    folder = N.write_model(tmp_path, cfg, t)
+    s = FolderSession(folder, dtype, max_len=256)
+    tokens = np.random.default_rng(3).integers(4, cfg["vocab"], 30).astype(np.int32)
+    tokens[11] = needle
+    tokens[[12, 19, 20, 28]] = ask                     # 1, 8: visible; 9, 17: not
+    want = N.forward(cfg, t, tokens)
+    assert (want[[12, 19, 20, 28], found] > 1.0).tolist() == [True, True, False, False]
+    for cuts in ([10] + [1] * 20, [30], [11, 2, 7, 1, 9], [19, 2, 9]):
+        got = feed(s, tokens, cuts)
+        check(got, want, dtype, cuts)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("length", [1030, 4110])
+def test_far_keys_in_long_windows(tmp_path, dtype, length):
+    """One key among thousands decides; the spans that change how a step cuts its
+    window lie in between."""
+    cfg, t, ask, needle, found = M.needle_model(5000, heads=1)
+    folder = N.write_model(tmp_path, cfg, t)
+    s = FolderSession(folder, dtype, max_len=5100)
+    tokens = np.random.default_rng(5).integers(4, cfg["vocab"], length).astype(np.int32)
+    tokens[3] = needle
+    tokens[[100, 1022, 1023, length - 7, length - 3, length - 1]] = ask
+    want = N.forward(cfg, t, tokens)
+    rows = np.unique([2, 3, 4, 100, 1022, length - 8])
+    got = s.prefill_rows(tokens[:-7], rows)
+    check(got, want[rows], dtype, "prompt")
+    assert (got[np.isin(rows, [100, 1022]), found] > 1.0).all()
+    for p in range(length - 7, length):
+        got = s.decode(int(tokens[p]), p)[1]
+        check(got[None], want[p][None], dtype, p)
+        assert (got[found] > 1.0) == (tokens[p] == ask)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_slow_and_fast_decays_reach_as_far_as_they_should(tmp_path, dtype):
+    """One loud token: what later tokens still hear of it is the decay's power of the
+    gap, across the chunks of a prompt and in decoding."""
+    cfg = M.config([M.linear(decay=(0.0, 1.0, 0.99, 0.5), mlp=None)], width=40, vocab=48, taps=1)
+
+    def edit(t):
+        t["embed"][5] *= 30.0
+        t["head"] = np.eye(48, 40)
+    folder, t = M.build(tmp_path, cfg, 1, edit)
+    for at in (0, 62, 63, 64):
+        tokens = tokens_for(cfg, 260, at)
+        tokens[tokens == 5] = 6
+        tokens[at] = 5
+        want = N.forward(cfg, t, tokens)
+        s = FolderSession(folder, dtype, max_len=300, prefill_block=128)
+        check(all_rows(s, tokens), want, dtype, at)
+        check(feed(s, tokens, [66, 2, 60] + [1] * 132), want, dtype, at)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_experts_are_chosen_and_weighted(tmp_path, dtype):
+    """Every expert answers in its own coordinate, so a wrong choice or weight shows."""
+    experts = 12
+    cfg = M.config([M.linear(decay=(0.5,), mlp=M.moe(experts=experts, top=3, ff=16, shared_ff=0, limit=5.0))],
+                   width=32, vocab=64, taps=1)
+
+    def edit(t):
+        t["l0.mix.o"] *= 0.0
+        for e in range(experts):
+            d = np.zeros((32, 16))
+            d[e] = t[f"l0.mlp.e{e}.down"][e] * 3
+            t[f"l0.mlp.e{e}.down"] = d
+        t["head"] = np.eye(64, 32)
+    folder, t = M.build(tmp_path, cfg, 2, edit)
+    tokens = np.arange(64, dtype=np.int32)
+    x = t["embed"][tokens] * cfg["embedding"]["scale"]
+    h = N.scalar_norm(x, t["l0.norm2"], 1e-5)
+    assert len(np.unique(N.route(h, t["l0.mlp.router"], 3)[0])) == experts
+    z = np.sort(h @ t["l0.mlp.router"].T)
+    clear = z[:, -3] - z[:, -4] > 0.1                  # no close call
+    assert clear.sum() > 40
+    want = N.forward(cfg, t, tokens)
+    s = FolderSession(folder, dtype, max_len=64)
+    for got in (all_rows(s, tokens), feed(s, tokens, [1] * 64)):
+        for r in np.nonzero(clear)[0]:
+            check(got[r][None], want[r][None], dtype, r)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_decoding_by_the_greedy_entry_point(tmp_path, dtype):
+    """300 greedy steps on the device (captured steps, replayed) against the oracle on
+    the tokens they chose, and the same tokens from single steps, captured or not."""
+    cfg = M.SIZES["mixed"]
+    folder, t = M.build(tmp_path, cfg)
+    s = FolderSession(folder, dtype, max_len=400)
+    prompt = tokens_for(cfg, 12)
+    first, _ = s.prefill(prompt, 0)
+    out = s.decode_greedy(first, 12, 300)
+    seq = np.concatenate([prompt, [first], out]).astype(np.int32)
+    want = N.forward(cfg, t, seq)
+    # the chosen logit is the largest, up to the format's rounding
+    spread = want.std(-1)
+    for p, tok in zip(range(11, 312), seq[12:]):
+        assert want[p, tok] > want[p].max() - BOUND[dtype] * 4 * spread[p]
+    for graph in (True, False):
+        s.use_graph(graph)
+        s.prefill(prompt, 0)
+        logits = []
+        for i in range(300):
+            nxt, lg = s.decode(int(seq[12 + i]), 12 + i)
+            assert nxt == seq[13 + i]
+            logits.append(lg)
+        check(np.stack(logits), want[12:312], dtype, graph)
+
+
+def test_captured_steps_equal_launched_ones_bit_for_bit(tmp_path):
+    cfg = M.SIZES["round"]
+    folder, _ = M.build(tmp_path, cfg)
+    tokens = tokens_for(cfg, 40)
+    s = FolderSession(folder, "bfloat16", max_len=64)
+    runs = []
+    for graph in (True, False, True):
+        s.use_graph(graph)
+        runs.append(feed(s, tokens, [8] + [1] * 32))
+    np.testing.assert_array_equal(runs[0], runs[1])
+    np.testing.assert_array_equal(runs[0], runs[2])
+
+
+def test_sampling_entry_points(tmp_path):
+    """temperature 0 is the greedy choice; a seeded sampler repeats itself."""
+    cfg = M.SIZES["mixed"]
+    folder, _ = M.build(tmp_path, cfg)
+    s = FolderSession(folder, "bfloat16", max_len=128)
+    prompt = tokens_for(cfg, 9)
+    first, _ = s.prefill(prompt, 0)
+    greedy = s.decode_greedy(first, 9, 20)
+
+    def run(**kw):
+        sampler = Sampler(**kw)
+        s.prefill(prompt, 0)
+        out = [first]
+        for i in range(20):
+            out.append(s.decode_sample(sampler, out[-1], 9 + i, out))
+        return out[1:]
+    assert run(temperature=0.0) == greedy.tolist()
+    a = run(temperature=1.2, top_k=20, seed=11)
+    assert a == run(temperature=1.2, top_k=20, seed=11) and a != greedy.tolist()
+
+
+def test_positions_that_do_not_follow_are_refused(tmp_path, bh):
+    cfg = M.SIZES["mixed"]
+    folder, _ = M.build(tmp_path, cfg)
+    s = FolderSession(folder, "bfloat16", max_len=64)
+    s.prefill(tokens_for(cfg, 10), 0)
+    for bad in (lambda: s.decode(1, 9), lambda: s.decode(1, 11), lambda: s.prefill([1, 2], 12),
+                lambda: s.decode_greedy(1, 10, 60), lambda: s.prefill(tokens_for(cfg, 60), 10),
+                lambda: s.prefill_rows([1, 2], [1, 0], 10), lambda: s.decode(cfg["vocab"], 10)):
+        with pytest.raises(BuddyHipError):
+            bad()
+    s.decode(1, 10)
+    with pytest.raises(BuddyHipError):     # no token and position since the prompt
+        s.prefill([1, 2], 11)
+        s.enqueue_steps(1)
+    # what only a per-head key / value cache has
+    assert bh.buddy_hip_session_get_kv(s._h, 0, np.empty(4, np.float32).ctypes.data) != 0
+    assert bh.buddy_hip_session_discard_kv(s._h, 0, 1, 4) != 0
+
+
+@pytest.mark.parametrize("edit,text", [
+    (lambda c: c["layers"][0].update(type="other"), "other"),
+    (lambda c: c["layers"][1]["mixer"]["decay"].pop(), "decay"),
+    (lambda c: c["layers"][0]["mlp"].update(kind="dense"), "dense"),
+    (lambda c: c["layers"][0]["mlp"]["router"].update(top=99), "99"),
+    (lambda c: c.update(width=47), "expected BF16"),
+    (lambda c: c.pop("canon"), "canon"),
+    (lambda c: c["layers"].append(c["layers"][0]), "l4."),
+])
+def test_configurations_that_do_not_fit_are_refused(tmp_path, edit, text):
+    cfg = json.loads(json.dumps(M.SIZES["mixed"]))
+    folder, _ = M.build(tmp_path, cfg)
+    edit(cfg)
+    (folder / "config.json").write_text(json.dumps(cfg))
+    with pytest.raises(BuddyHipError, match=text):
+        FolderSession(folder)
+
+
+def test_command_line_runner_generates_the_same(tmp_path):
+    cfg = M.SIZES["mixed"]
+    folder, _ = M.build(tmp_path, cfg)
+    prompt = tokens_for(cfg, 11).tolist()
+    runner = bma.library_path().parent / "buddy_hip_run"
+    for dtype in DTYPES:
+        s = FolderSession(folder, dtype, max_len=128)
+        first, _ = s.prefill(prompt, 0)
+        want = [first] + s.decode_greedy(first, 11, 24).tolist()
+        s.close()
+        r = subprocess.run([str(runner), "--model", str(folder), "--dtype", dtype, "--max-new", "25",
+                            "--tokens", ",".join(map(str, prompt))],
+                           capture_output=True, text=True, timeout=100)
+        assert r.returncode == 0, r.stderr
+        ids = [line for line in r.stdout.splitlines() if line.startswith("[Output ids]")][0]
+        assert [int(x) for x in ids.split("]")[1].split()] == want
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_trace_replay(tmp_path, dtype):
+    """Two sequences one after the other, in portions, through the replay program."""
+    cfg = M.SIZES["odd"]
+    folder, t = M.build(tmp_path / "m", cfg)
+    out = tmp_path / "out"
+    out.mkdir()
+    a, b = tokens_for(cfg, 50, 1), tokens_for(cfg, 20, 2)
+    steps = [("a", a[:30], [29, 0, 7]), ("a", a[30:31], [0]), ("a", a[31:33], []), ("a", a[33:], [16, 2]),
+             ("b", b[:1], [0]), ("b", b[1:], [18])]
+    lines = [json.dumps({"step": i, "entries": [{"id": n, "tokens": x.tolist(), "want": w}],
+                         "end": ["a"] if i == 3 else ["b"] if i == 5 else []})
+             for i, (n, x, w) in enumerate(steps)]
+    r = subprocess.run([str(ROOT / "bin" / "trace_run"), "--model", str(folder), "--dtype", dtype,
+                        "--out", str(out), "--max-tokens", "50"], input="\n".join(lines) + "\n",
+                       capture_output=True, text=True, timeout=110, env=dict(os.environ))
+    assert r.returncode == 0, r.stderr
+    assert [x for x in r.stdout.splitlines() if x.startswith("done")] == [f"done {i}" for i in range(6)]
+    full = {"a": N.forward(cfg, t, a), "b": N.forward(cfg, t, b)}
+    at = {"a": 0, "b": 0}
+    for i, (n, x, w) in enumerate(steps):
+        path = out / f"{i}.f32"
+        assert path.exists() == bool(w)
+        if w:
+            got = np.fromfile(path, "<f4").reshape(len(w), cfg["vocab"])
+            check(got, full[n][at[n] + np.array(w)], dtype, i)
+        at[n] += len(x)
