@@ -3,7 +3,7 @@
 MI355X, next to the CPU oracle timed on the same host.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W]
-    python bench.py --workload gemv|mlp|prefill|llama8b|kvdiscard|w4a16|model_abi|sampler|quantize   (the other configurations)
+    python bench.py --workload gemv|mlp|prefill|llama8b|kvdiscard|w4a16|model_abi|sampler|quantize|nukopel   (the other configurations)
 
 A step is one greedy decode step (one token) at batch 1 with the KV cache
 already holding 1024 positions; weights, KV cache and activations are resident
@@ -936,6 +936,110 @@ def bench_model_abi(bh, args):
     }
 
 
+# Layers of real models, and for each a Qwen2-shaped session of the same width, number
+# of layers, heads, vocabulary, and feed-forward units per token ((top + shared) * ff).
+NUKOPEL_SIZES = {
+    "w1536": (dict(width=1536, layers="alaa", heads=12, window=1024, experts=16, top=4, ff=1792),
+              dict(hidden=1536, layers=4, heads=12, kv_heads=2, inter=8960)),
+    "w4096": (dict(width=4096, layers="ala", heads=32, window=4096, experts=16, top=4, ff=2048),
+              dict(hidden=4096, layers=3, heads=32, kv_heads=8, inter=10240)),
+}
+
+
+def _nukopel_step_bytes(cfg, context):
+    """Weights, cache rows and states one decoded token reads or writes (bfloat16
+    weights and cache, f32 state)."""
+    W = cfg["width"]
+    total = 2 * cfg["vocab"] * W
+    for layer in cfg["layers"]:
+        m, f = layer["mixer"], layer["mlp"]
+        H, D, VD = m["heads"], m["dim"], m["vdim"]
+        if layer["type"] == "latent_attention":
+            R, L = m["rot_dim"], m["kv_rank"]
+            total += 2 * (W * (H * (D + R) + L + R + H) + H * (D + VD) * L + W * H * VD)
+            total += 2 * min(context, m["mask"]["size"]) * (L + R)
+        else:
+            total += 2 * W * (2 * H * D + 3 * H * VD) + 2 * 4 * H * D * VD
+        total += 2 * W * f["router"]["experts"]
+        total += 2 * 3 * W * (f["router"]["top"] * f["expert"]["ff"] + f["shared"]["ff"])
+    return total
+
+
+def bench_nukopel(bh, args):
+    """Prefill and decode throughput of the Nukopel session at layers of real models'
+    sizes, beside the Qwen2-shaped w8a32 session of equal width, depth, heads,
+    vocabulary and feed-forward units per token."""
+    import tempfile
+
+    import torch
+
+    from buddy_mlir_amd import synthetic
+    from buddy_mlir_amd.session import FolderSession, Shape
+
+    K, W = args.steps, max(1, args.warmup)
+    prompts = (512, 2048)
+    detail = {}
+
+    def decode_s(s, first, context):
+        s.use_graph(not args.no_graph)
+        s.set_state(first, context)
+        s.enqueue_steps(W)
+        stream = torch.cuda.ExternalStream(s.stream)
+        stream.synchronize()
+        t0 = time.perf_counter()
+        s.enqueue_steps(K)
+        stream.synchronize()
+        return (time.perf_counter() - t0) / K
+
+    def prefill_s(s, toks, n=5):
+        s.prefill(toks, 0, want_logits=False)
+        t0 = time.perf_counter()
+        for _ in range(n):
+            s.prefill(toks, 0, want_logits=False)
+        return (time.perf_counter() - t0) / n
+
+    for name in args.nukopel_sizes.split(","):
+        mine, other = NUKOPEL_SIZES[name]
+        cfg = synthetic.nukopel_config(**mine)
+        shape = Shape(vocab=cfg["vocab"], max_len=4096, **other)
+        toks = synthetic.first_tokens(shape, max(prompts))
+        d = detail[name] = {"config": mine, "qwen2": other}
+        with tempfile.TemporaryDirectory() as tmp:
+            synthetic.write_nukopel_folder(tmp, cfg)
+            s = FolderSession(tmp, "bfloat16", max_len=4096)
+        for n in prompts:
+            t = prefill_s(s, toks[:n])
+            d[f"prefill_{n}"] = {"ms": t * 1e3, "tokens_per_s": n / t}
+        s.prefill(toks[:CONTEXT], 0, want_logits=False)
+        t = decode_s(s, int(toks[0]), CONTEXT)
+        b = _nukopel_step_bytes(cfg, CONTEXT)
+        d["decode"] = {"ms": t * 1e3, "tokens_per_s": 1 / t, "algorithmic_bytes": b,
+                       "hbm_frac": b / t / 1e9 / HBM_PEAK_GBPS}
+        s.close()
+        q, _ = synthetic.build_session(shape, context=CONTEXT)
+        for n in prompts:
+            t = prefill_s(q, toks[:n])
+            d[f"qwen2_prefill_{n}"] = {"ms": t * 1e3, "tokens_per_s": n / t}
+        t = decode_s(q, int(toks[0]), CONTEXT)
+        b = decode_step_bytes(shape, CONTEXT)
+        d["qwen2_decode"] = {"ms": t * 1e3, "tokens_per_s": 1 / t, "algorithmic_bytes": b,
+                             "hbm_frac": b / t / 1e9 / HBM_PEAK_GBPS}
+        q.close()
+        torch.cuda.empty_cache()
+    lead = detail[next(iter(detail))]["decode"]
+    return {
+        "metric": "nukopel_decode_tokens_per_s", "value": lead["tokens_per_s"], "unit": "tokens/s",
+        "n_gpus": 1, "steps": K, "warmup": W, "ms_per_step": lead["ms"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "Nukopel layers (latent attention, lightning attention, routed and "
+                               "shared experts), random weights: one greedy decode step at context "
+                               "1024 and prompts of 512 and 2048 tokens, beside the Qwen2-shaped "
+                               "w8a32 session of equal size",
+                   "context": CONTEXT, "hip_graph": not args.no_graph},
+        "detail": detail,
+    }
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -943,11 +1047,13 @@ def main():
     ap.add_argument("--warmup", type=int, default=8)
     ap.add_argument("--workload", default="decode",
                     choices=["decode", "gemv", "mlp", "prefill", "llama8b", "kvdiscard", "w4a16",
-                             "model_abi", "sampler", "quantize"],
+                             "model_abi", "sampler", "quantize", "nukopel"],
                     help="decode (default): the full decode step the headline metric "
                          "is quoted on; the others measure the remaining configurations")
     ap.add_argument("--mlp-rows", default="1,4,16",
                     help="--workload mlp: the row counts to time (1..16, comma separated)")
+    ap.add_argument("--nukopel-sizes", default=",".join(NUKOPEL_SIZES),
+                    help="--workload nukopel: which of the sizes to run")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-graph", action="store_true")
     ap.add_argument("--calibrate-copy", action="store_true",
@@ -972,7 +1078,7 @@ def main():
         fn = {"gemv": bench_gemv, "mlp": bench_mlp, "prefill": bench_prefill,
               "llama8b": bench_llama8b, "kvdiscard": bench_kvdiscard, "w4a16": bench_w4a16,
               "model_abi": bench_model_abi, "sampler": bench_sampler,
-              "quantize": bench_quantize}[args.workload]
+              "quantize": bench_quantize, "nukopel": bench_nukopel}[args.workload]
         print(json.dumps(fn(bh, args)))
         return
     K, W = args.steps, args.warmup

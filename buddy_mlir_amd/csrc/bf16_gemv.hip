@@ -70,7 +70,7 @@ struct RowTail { // arguments a wavefront needs only behind its first loads
   const float *y;
   float *x_out, *row_out;
   const float *conv_w;
-  float *conv_ring;
+  float *conv_ring, *conv_next;
   const int *pos;
   const float *weight, *gate;
   float *out;
@@ -80,18 +80,186 @@ struct RowTail { // arguments a wavefront needs only behind its first loads
   int taps, silu_channels, valid;
 };
 
-// Grid: workgroups of 8 wavefronts = (8 >> ks_shift) channel groups x (1 <<
-// ks_shift) slices of k that meet in LDS in slice order.
+__device__ __forceinline__ f32x4 load4(const float *p) { return *reinterpret_cast<const f32x4 *>(p); }
+__device__ __forceinline__ void save4(float *p, f32x4 v) { *reinterpret_cast<f32x4 *>(p) = v; }
+
+// What the row of this position leaves for later ones: itself in the ring, and what
+// it and the rows before it will add to the next one.
+__device__ __forceinline__ void keep_row(const RowTail &a, int K, int p, int i, float h) {
+  a.conv_ring[(int64_t)(p % a.taps) * K + i] = h;
+  float c = 0.f;
+  for (int b = a.taps - 1; b >= 1; --b) {
+    const int q = p + 1 - b;
+    if (q < 0)
+      continue;
+    const float e = b == 1 ? h : a.conv_ring[(int64_t)(q % a.taps) * K + i];
+    c = fmaf(a.conv_w[(int64_t)(a.taps - 1 - b) * K + i], e, c);
+  }
+  a.conv_next[(int64_t)((p + 1) & 1) * K + i] = c;
+}
+
+// The finished input row into act[0 .. Kp).  R > 0: K is a multiple of 4 and at most
+// 2048 * R, and every thread keeps its 4 * R values in registers from one trip to
+// memory.  R = 0: any K.  `keeper`: this workgroup stores what the row leaves behind.
+template <int INPUT, int R>
+struct RowPrologue {
+  f32x4 x[R], y[R], c[R], w[R];
+  int at[R];
+  bool in[R];
+  __device__ __forceinline__ void request(const float *src, int K, const RowTail &a) {
+    const int p = INPUT == kRowNorm && a.conv_w ? *a.pos : 0;
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+      at[r] = (r * kRowThreads + (int)threadIdx.x) * 4;
+      in[r] = at[r] < K;
+      const int i = in[r] ? at[r] : 0;
+      x[r] = load4(src + i);
+      if constexpr (INPUT == kRowNorm) {
+        if (a.y)
+          y[r] = load4(a.y + i);
+        if (a.conv_w) {
+          w[r] = load4(a.conv_w + (int64_t)(a.taps - 1) * K + i);
+          c[r] = load4(a.conv_next + (int64_t)(p & 1) * K + i);
+        }
+      } else if constexpr (INPUT == kRowGated) {
+        w[r] = load4(a.weight + i);
+        c[r] = load4(a.gate + i);
+      }
+    }
+  }
+  __device__ __forceinline__ float squares(const f32x4 (&v)[R]) const {
+    float s = 0.f;
+#pragma unroll
+    for (int r = 0; r < R; ++r)
+      if (in[r])
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          s = fmaf(v[r][j], v[r][j], s);
+    return s;
+  }
+  __device__ __forceinline__ void finish(float *act, int K, int Kp, const RowTail &a, bool keeper,
+                                         float (*red)[kRowWaves]) {
+    if constexpr (INPUT == kRowGated) {
+      const float g = 1.0f / sqrtf(block_sum(squares(x), red[0]) / (float)K + a.eps);
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          x[r][j] = x[r][j] * g * w[r][j] * sigmoid_f(c[r][j]);
+    } else if constexpr (INPUT == kRowNorm) {
+      if (a.y) {
+        const float ry = a.out_gain / sqrtf(block_sum(squares(y), red[0]) / (float)K + a.eps);
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            x[r][j] = fmaf(y[r][j], ry, x[r][j]);
+          if (keeper && a.x_out && in[r])
+            save4(a.x_out + at[r], x[r]);
+        }
+      }
+      const float g = a.gain / sqrtf(block_sum(squares(x), red[1]) / (float)K + a.eps);
+      const int p = a.conv_w ? *a.pos : 0;
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        f32x4 h;
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          h[j] = x[r][j] * g;
+        x[r] = h;
+        if (a.conv_w) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            x[r][j] += fmaf(w[r][j], h[j], p > 0 ? c[r][j] : 0.f);
+          if (keeper && in[r])
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+              keep_row(a, K, p, at[r] + j, h[j]);
+        }
+        if (keeper && a.row_out && in[r])
+          save4(a.row_out + at[r], x[r]);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < R; ++r)
+      if (at[r] < Kp)
+        save4(act + at[r], in[r] ? x[r] : f32x4{0.f, 0.f, 0.f, 0.f});
+  }
+};
 template <int INPUT>
+struct RowPrologue<INPUT, 0> {
+  const float *src;
+  __device__ __forceinline__ void request(const float *s, int, const RowTail &) { src = s; }
+  __device__ __forceinline__ void finish(float *act, int K, int Kp, const RowTail &a, bool keeper,
+                                         float (*red)[kRowWaves]) {
+    const int tid = threadIdx.x;
+    float scale = 1.f;
+    if constexpr (INPUT == kRowPlain) {
+      for (int i = tid; i < K; i += kRowThreads)
+        act[i] = src[i];
+    } else {
+      float ry = 0.f, ss = 0.f;
+      if (INPUT == kRowNorm && a.y) {
+        for (int i = tid; i < K; i += kRowThreads)
+          ss = fmaf(a.y[i], a.y[i], ss);
+        ry = a.out_gain / sqrtf(block_sum(ss, red[0]) / (float)K + a.eps);
+      }
+      ss = 0.f;
+      for (int i = tid; i < K; i += kRowThreads) {
+        float v = src[i];
+        if (INPUT == kRowNorm && a.y) {
+          v = fmaf(a.y[i], ry, v);
+          if (keeper && a.x_out)
+            a.x_out[i] = v;
+        }
+        act[i] = v;
+        ss = fmaf(v, v, ss);
+      }
+      scale = (INPUT == kRowNorm ? a.gain : 1.0f) / sqrtf(block_sum(ss, red[1]) / (float)K + a.eps);
+    }
+    const int p = INPUT == kRowNorm && a.conv_w ? *a.pos : 0;
+    for (int i = tid; i < Kp; i += kRowThreads) {
+      float h = 0.f;
+      if (i < K) {
+        h = act[i] * scale;
+        if constexpr (INPUT == kRowGated)
+          h *= a.weight[i] * sigmoid_f(a.gate[i]);
+        if constexpr (INPUT == kRowNorm) {
+          if (a.conv_w) {
+            const float raw = h;
+            h += fmaf(a.conv_w[(int64_t)(a.taps - 1) * K + i], raw,
+                      p > 0 ? a.conv_next[(int64_t)(p & 1) * K + i] : 0.f);
+            if (keeper)
+              keep_row(a, K, p, i, raw);
+          }
+          if (keeper && a.row_out)
+            a.row_out[i] = h;
+        }
+      }
+      act[i] = h;
+    }
+  }
+};
+
+// Grid: workgroups of 8 wavefronts = (8 >> ks_shift) channel groups x (1 <<
+// ks_shift) slices of k that meet in LDS in slice order.  kRowNorm: one workgroup
+// more, which multiplies nothing and stores what the row leaves behind.
+template <int INPUT, int R>
 __global__ void __launch_bounds__(kRowThreads)
 row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src, int K, int ktiles,
                 int groups, int ks_shift, int slice_tiles, RowTail a) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];
+  extern __shared__ __attribute__((aligned(16))) float act[]; // [Kp]
   __shared__ float red[2][kRowWaves];
   __shared__ float part[kRowWaves][16];
   const int Kp = ktiles * kBfTileK;
-  float *act = lds; // [Kp]
   const int tid = threadIdx.x, lane = tid & 63;
+  // the row's values first: loads return in order, and these come from the L2
+  RowPrologue<INPUT, R> row;
+  row.request(src, K, a);
+  if (INPUT == kRowNorm && blockIdx.x == gridDim.x - 1) {
+    row.finish(act, K, Kp, a, true, red);
+    return;
+  }
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int slice = wave & ((1 << ks_shift) - 1);
   const int g = blockIdx.x * (kRowWaves >> ks_shift) + (wave >> ks_shift);
@@ -102,73 +270,7 @@ row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src, int 
 #pragma unroll
   for (int u = 0; u < kAhead; ++u)
     w[u] = wp[(int64_t)min(t0 + u, ktiles - 1) * 64];
-
-  if constexpr (INPUT == kRowPlain) {
-    for (int i = tid; i < Kp; i += kRowThreads)
-      act[i] = i < K ? src[i] : 0.f;
-  } else if constexpr (INPUT == kRowGated) {
-    float *gt = lds + Kp;
-    float ss = 0.f;
-    for (int i = tid; i < K; i += kRowThreads) {
-      const float o = src[i];
-      gt[i] = a.weight[i] * sigmoid_f(a.gate[i]);
-      act[i] = o;
-      ss = fmaf(o, o, ss);
-    }
-    const float r = 1.0f / sqrtf(block_sum(ss, red[0]) / (float)K + a.eps);
-    for (int i = tid; i < Kp; i += kRowThreads)
-      act[i] = i < K ? act[i] * r * gt[i] : 0.f;
-  } else {
-    float *yb = lds + Kp, *cv = lds + 2 * Kp;
-    float ss = 0.f;
-    const int p = a.conv_w ? *a.pos : 0;
-    for (int i = tid; i < K; i += kRowThreads) {
-      act[i] = src[i];
-      if (a.y) {
-        const float y = a.y[i];
-        yb[i] = y;
-        ss = fmaf(y, y, ss);
-      }
-      if (a.conv_w) { // what earlier rows add
-        float c = 0.f;
-        for (int b = 1; b < a.taps; ++b)
-          if (p - b >= 0)
-            c = fmaf(a.conv_w[(int64_t)(a.taps - 1 - b) * K + i],
-                     a.conv_ring[(int64_t)((p - b) % a.taps) * K + i], c);
-        cv[i] = c;
-      }
-    }
-    const bool first = blockIdx.x == 0;
-    float ry = 0.f;
-    if (a.y)
-      ry = a.out_gain / sqrtf(block_sum(ss, red[0]) / (float)K + a.eps);
-    ss = 0.f;
-    for (int i = tid; i < K; i += kRowThreads) {
-      float v = act[i];
-      if (a.y)
-        v = fmaf(yb[i], ry, v);
-      act[i] = v;
-      ss = fmaf(v, v, ss);
-      if (first && a.x_out)
-        a.x_out[i] = v;
-    }
-    const float r = a.gain / sqrtf(block_sum(ss, red[1]) / (float)K + a.eps);
-    const int slot = a.conv_w ? p % a.taps : 0;
-    for (int i = tid; i < Kp; i += kRowThreads) {
-      float h = 0.f;
-      if (i < K) {
-        h = act[i] * r;
-        if (a.conv_w) {
-          if (first)
-            a.conv_ring[(int64_t)slot * K + i] = h;
-          h += fmaf(a.conv_w[(int64_t)(a.taps - 1) * K + i], h, cv[i]);
-        }
-        if (first && a.row_out)
-          a.row_out[i] = h;
-      }
-      act[i] = h;
-    }
-  }
+  row.finish(act, K, Kp, a, false, red);
   __syncthreads();
 
   const float *ap = act + (lane >> 4) * 8;
@@ -360,16 +462,22 @@ struct MoeDown {
   float *out;
 };
 
-// Grid: one channel group per workgroup; its wavefronts cut the concatenation of
-// the chosen experts' k (and the shared expert's) into slices.
-template <int WAVES>
+// Grid: one channel group (HALF: 8 of its 16 channels) per workgroup; its wavefronts
+// cut the concatenation of the chosen experts' k (and the shared expert's) into
+// slices.  With HALF a load covers the 8 channels of two consecutive tiles, so it
+// still moves whole 128-byte lines; every expert has an even number of tiles.
+template <int WAVES, bool HALF>
 __global__ void __launch_bounds__(WAVES * 64)
 moe_down_kernel(const uint4 *__restrict__ down, const float *__restrict__ act,
                 const int *__restrict__ chosen, int slice_tiles, MoeDown a) {
   __shared__ float part[WAVES][16];
+  constexpr int kStep = HALF ? 2 : 1; // tiles per load
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int g = blockIdx.x;
+  const int g = HALF ? blockIdx.x >> 1 : blockIdx.x, half = HALF ? blockIdx.x & 1 : 0;
+  // this lane's 16 bytes of a load and the k they hold
+  const int run = HALF ? (lane >> 5) * 64 + ((lane >> 3) & 3) * 16 + half * 8 + (lane & 7) : lane;
+  const int k_at = HALF ? (lane >> 5) * kBfTileK + ((lane >> 3) & 3) * 8 : (lane >> 4) * 8;
   // lane j: the j-th chosen expert and its softmax weight
   const int cj = chosen[min(lane, a.top - 1)];
   const float zj = lane < a.top ? a.chosen_logit[lane] : -INFINITY;
@@ -386,38 +494,40 @@ moe_down_kernel(const uint4 *__restrict__ down, const float *__restrict__ act,
   while (left > 0) {
     const bool sh = seg >= a.top;
     const int kt = sh ? a.shared_ktiles : a.ktiles;
-    const int run = min(left, kt - off);
+    const int n = min(left, kt - off);
     const int e = sh ? 0 : __builtin_amdgcn_readlane(cj, min(seg, 63));
     const float wt = sh ? 1.0f : lane_f(wj, min(seg, 63));
     const uint4 *wp = (sh ? a.shared_down : down + (int64_t)e * a.groups * kt * 64) +
-                      ((int64_t)g * kt + off) * 64 + lane;
-    const float *ap = act + (int64_t)seg * a.act_stride + off * kBfTileK + (lane >> 4) * 8;
+                      ((int64_t)g * kt + off) * 64 + run;
+    const float *ap = act + (int64_t)seg * a.act_stride + off * kBfTileK + k_at;
     float s = 0.f;
-    for (int t = 0; t < run; t += kAhead) {
+    for (int t = 0; t < n; t += kAhead * kStep) {
       uint4 w[kAhead];
 #pragma unroll
       for (int u = 0; u < kAhead; ++u)
-        w[u] = wp[(int64_t)min(t + u, run - 1) * 64];
+        w[u] = wp[(int64_t)min(t + u * kStep, n - kStep) * 64];
 #pragma unroll
       for (int u = 0; u < kAhead; ++u)
-        if (t + u < run)
-          s = dot_tile(w[u], ap + (t + u) * kBfTileK, s);
+        if (t + u * kStep < n)
+          s = dot_tile(w[u], ap + (t + u * kStep) * kBfTileK, s);
     }
     acc = fmaf(wt, s, acc);
-    left -= run;
+    left -= n;
     off = 0;
     ++seg;
   }
   acc = sum_rows(acc);
-  if (lane < 16)
+  if constexpr (HALF)
+    acc += __shfl_xor(acc, 8, 64);
+  if (lane < (HALF ? 8 : 16))
     part[wave][lane] = acc;
   __syncthreads();
-  if (tid < 16) {
+  if (tid < (HALF ? 8 : 16)) {
     float v = 0.f;
 #pragma unroll
     for (int s = 0; s < WAVES; ++s)
       v += part[s][tid];
-    a.out[g * 16 + tid] = v;
+    a.out[g * 16 + half * 8 + tid] = v;
   }
 }
 
@@ -446,38 +556,57 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
   BH_REQUIRE(W.tiles && W.K > 0 && W.N > 0 && W.N % 16 == 0 && W.ktiles == bf16_ktiles(W.K) &&
                  a.src && a.out,
              "row_gemv: bad argument");
-  BH_REQUIRE(!a.conv_w || (a.conv_ring && a.pos && a.taps > 0), "row_gemv: convolution operands");
+  BH_REQUIRE(!a.conv_w || (a.conv_ring && a.conv_next && a.pos && a.taps > 0),
+             "row_gemv: convolution operands");
   BH_REQUIRE(a.input != kRowGated || (a.weight && a.gate), "row_gemv: gate operands");
   BH_REQUIRE(a.x_out == nullptr || a.x_out != a.src, "row_gemv: the row is read by every workgroup");
   BH_REQUIRE(!a.max_v || a.max_i, "row_gemv: maxima without indices");
-  // slices of k: as many as keep 8 tiles per wavefront, more while the launch has
-  // fewer than 1024 wavefronts
+  // slices of k: doubled while the launch has fewer than 2048 wavefronts and each
+  // keeps four tiles
   const int groups = W.groups();
   int ks = 1;
-  while (ks < kRowWaves && (W.ktiles / (2 * ks) >= kAhead ||
-                            ((int64_t)groups * ks < 1024 && W.ktiles / (2 * ks) >= 2)))
+  while (ks < kRowWaves && (int64_t)groups * ks < 2048 && W.ktiles / (2 * ks) >= 4)
     ks *= 2;
   const int shift = shift_for(ks), per = kRowWaves >> shift;
   const int slice_tiles = (int)ceil_div(W.ktiles, ks);
-  const int arrays = a.input == kRowPlain ? 1 : a.input == kRowGated ? 2 : 3;
-  const size_t lds = sizeof(float) * (size_t)arrays * W.ktiles * kBfTileK;
+  const size_t lds = sizeof(float) * (size_t)W.ktiles * kBfTileK;
   BH_REQUIRE(lds <= 150 * 1024, "row_gemv: a row of %d values does not fit LDS", W.K);
-  RowTail t{a.y, a.x_out, a.row_out, a.conv_w, a.conv_ring, a.pos, a.weight, a.gate, a.out,
-            a.max_v, a.max_i, a.eps, a.out_gain, a.gain, a.taps, a.silu_channels, a.valid};
-  const dim3 grid((unsigned)ceil_div(groups, per)), block(kRowThreads);
-#define BH_ROW(I)                                                                              \
-  do {                                                                                         \
-    static DynLdsOnce once;                                                                    \
-    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)row_gemv_kernel<I>, 150 * 1024));          \
-    hipLaunchKernelGGL(row_gemv_kernel<I>, grid, block, lds, stream, W.tiles, a.src, W.K,      \
-                       W.ktiles, groups, shift, slice_tiles, t);                               \
+  RowTail t{a.y, a.x_out, a.row_out, a.conv_w, a.conv_ring, a.conv_next, a.pos, a.weight, a.gate,
+            a.out, a.max_v, a.max_i, a.eps, a.out_gain, a.gain, a.taps, a.silu_channels, a.valid};
+  const bool keeper = a.input == kRowNorm;
+  const dim3 grid((unsigned)(ceil_div(groups, per) + keeper)), block(kRowThreads);
+  bool quads = W.K % 4 == 0;
+  for (const void *p : {(const void *)a.src, (const void *)a.y, (const void *)a.x_out,
+                        (const void *)a.row_out, (const void *)a.conv_w, (const void *)a.conv_next,
+                        (const void *)a.weight, (const void *)a.gate})
+    quads = quads && ((uintptr_t)p & 15) == 0;
+  const int span = W.ktiles * kBfTileK; // the padding is written too
+  const int regs = !quads || span > 8192 ? 0 : span <= 2048 ? 1 : span <= 4096 ? 2 : 4;
+#define BH_ROW(I, R)                                                                             \
+  do {                                                                                           \
+    static DynLdsOnce once;                                                                      \
+    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)row_gemv_kernel<I, R>, 150 * 1024));         \
+    hipLaunchKernelGGL((row_gemv_kernel<I, R>), grid, block, lds, stream, W.tiles, a.src, W.K,   \
+                       W.ktiles, groups, shift, slice_tiles, t);                                 \
+  } while (0)
+#define BH_ROWS(I)                                                                               \
+  do {                                                                                           \
+    if (regs == 1)                                                                               \
+      BH_ROW(I, 1);                                                                              \
+    else if (regs == 2)                                                                          \
+      BH_ROW(I, 2);                                                                              \
+    else if (regs == 4)                                                                          \
+      BH_ROW(I, 4);                                                                              \
+    else                                                                                         \
+      BH_ROW(I, 0);                                                                              \
   } while (0)
   if (a.input == kRowPlain)
-    BH_ROW(kRowPlain);
+    BH_ROWS(kRowPlain);
   else if (a.input == kRowNorm)
-    BH_ROW(kRowNorm);
+    BH_ROWS(kRowNorm);
   else
-    BH_ROW(kRowGated);
+    BH_ROWS(kRowGated);
+#undef BH_ROWS
 #undef BH_ROW
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
@@ -540,13 +669,18 @@ int launch_row_moe(const RowMoe &a, hipStream_t stream) {
   d.act_stride = a.act_stride;
   d.chosen_logit = a.weights;
   d.out = a.out;
+  // slices start at even tiles
   const int total = a.top * d.ktiles + d.shared_ktiles;
-  if (total >= 64)
-    hipLaunchKernelGGL(moe_down_kernel<16>, dim3(d.groups), dim3(1024), 0, stream, a.experts.down,
-                       a.act, a.chosen, (int)ceil_div(total, 16), d);
+  auto slice = [&](int waves) { return (int)round_up(ceil_div(total, waves), 2); };
+  if (total >= 64 && d.groups < 192) // fewer workgroups than compute units: halves
+    hipLaunchKernelGGL((moe_down_kernel<16, true>), dim3(2 * d.groups), dim3(1024), 0, stream,
+                       a.experts.down, a.act, a.chosen, slice(16), d);
+  else if (total >= 64)
+    hipLaunchKernelGGL((moe_down_kernel<16, false>), dim3(d.groups), dim3(1024), 0, stream,
+                       a.experts.down, a.act, a.chosen, slice(16), d);
   else
-    hipLaunchKernelGGL(moe_down_kernel<4>, dim3(d.groups), dim3(256), 0, stream, a.experts.down,
-                       a.act, a.chosen, (int)ceil_div(total, 4), d);
+    hipLaunchKernelGGL((moe_down_kernel<4, false>), dim3(d.groups), dim3(256), 0, stream,
+                       a.experts.down, a.act, a.chosen, slice(4), d);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }

@@ -53,6 +53,7 @@ struct RowGemv {
   float *row_out = nullptr;       // the finished input row
   const float *conv_w = nullptr;  // [taps][K]
   float *conv_ring = nullptr;     // [taps][K], row of position p in slot p % taps
+  float *conv_next = nullptr;     // [2][K]: what earlier rows add at position p, in slot p % 2
   int taps = 0;
   const int *pos = nullptr;       // device: position of the row
   // kRowGated

@@ -1,5 +1,5 @@
 // latent_attn.h -- attention over a cache of latents: a row per position holds one
-// normed latent and one rotated key part that all heads share, in a ring of
+// rotated key part and one normed latent that all heads share, in a ring of
 // positions, seen through a sliding window.
 #pragma once
 
@@ -14,7 +14,12 @@ struct LatentShape {
   // cache: ring_mask + 1 (a power of two) rows of row_elems() elements
   int ring_mask = 0;
   bool f32 = false; // element type of the cache and of the activations: f32 or bfloat16
-  int row_elems() const { return (int)round_up(rank + rot_dim, 32); }
+  // a row: the rotated part from element 0, the latent from element rot8(), zeros
+  int rot8() const { return (int)round_up(rot_dim, 8); }
+  int row_elems() const { return (int)round_up(rot8() + rank16(), 32); }
+  // a query or key of a head in a prompt's attention: the unrotated part, padded, then
+  // the rotated one
+  int key_elems() const { return (int)round_up(dim16() + rot8(), 32); }
   int rank16() const { return (int)round_up(rank, 16); }
   int heads16() const { return (int)round_up(heads, 16); }
   int dim16() const { return (int)round_up(dim, 16); }
@@ -50,16 +55,19 @@ int latent_max_chunks(const LatentShape &s);
 int launch_latent_step(const LatentStep &a, int span, hipStream_t stream);
 
 // ---- many tokens ---------------------------------------------------------------
+constexpr int kLatentKeyTile = 64; // keys and values are padded to this many positions
 struct LatentRows {
   LatentShape s;
-  float *proj = nullptr; // [rows][ld]: q is rotated and scaled in place
+  const float *proj = nullptr; // [rows][ld]: q | dkv | gate at their offsets
   int ld = 0, dkv_at = 0, gate_at = 0;
   int rows = 0, start = 0; // rows hold positions start .. start + rows - 1
   const float *norm_w = nullptr;
   const double *turns = nullptr;
   void *cache = nullptr;
+  void *queries = nullptr; // [rows][heads][key_elems], rotated and scaled
   // keys and values of the visible positions first .. start + rows - 1, made from
-  // the cache: [keys][heads * dim16] and, transposed, [heads * vdim16][value_ld]
+  // the cache: [keys][heads * dim16] and, transposed, [heads * vdim16][value_ld];
+  // both with room for a multiple of kLatentKeyTile positions
   const void *keys = nullptr, *values_t = nullptr;
   int value_ld = 0;
   int first = 0;
@@ -67,7 +75,7 @@ struct LatentRows {
   int out_ld = 0;
 };
 int latent_first_visible(const LatentShape &s, int start);
-// latent norm, rotations, cache rows
+// latent norm, rotations, cache rows, queries
 int launch_latent_rows(const LatentRows &a, hipStream_t stream);
 int launch_latent_attention(const LatentRows &a, hipStream_t stream);
 

@@ -25,8 +25,21 @@ __device__ __forceinline__ void rotation(double turns, int p, float &c, float &s
 
 constexpr int kStepThreads = 512, kStepWaves = 8;
 
+// eight bfloat16 weights times eight values in LDS
+__device__ __forceinline__ float dot_run(const uint4 w, const float *x, float acc) {
+  acc = fmaf(bf_lo(w.x), x[0], acc);
+  acc = fmaf(bf_hi(w.x), x[1], acc);
+  acc = fmaf(bf_lo(w.y), x[2], acc);
+  acc = fmaf(bf_hi(w.y), x[3], acc);
+  acc = fmaf(bf_lo(w.z), x[4], acc);
+  acc = fmaf(bf_hi(w.z), x[5], acc);
+  acc = fmaf(bf_lo(w.w), x[6], acc);
+  acc = fmaf(bf_hi(w.w), x[7], acc);
+  return acc;
+}
+
 struct LatentQueryArgs {
-  int heads, dim, rot_dim, rank, row_elems, ring_mask, dkv_at, uk_groups, uk_ktiles;
+  int heads, dim, rot_dim, rot8, rank, row_elems, ring_mask, dkv_at, uk_groups, uk_ktiles;
   float scale, eps;
   const float *norm_w;
   const double *turns;
@@ -64,14 +77,14 @@ latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj
     T *row = static_cast<T *>(a.cache) + (int64_t)(p & a.ring_mask) * a.row_elems;
     for (int i = tid; i < a.row_elems; i += kStepThreads) {
       float v = 0.f;
-      if (i < a.rank) {
-        v = d[i] * r * a.norm_w[i];
-      } else if (i < a.rank + a.rot_dim) {
-        const int j = i - a.rank, f = j < half ? j : j - half;
+      if (i < a.rot_dim) {
+        const int f = i < half ? i : i - half;
         float c, s;
         rotation(a.turns[f], p, c, s);
         const float u = d[a.rank + f], w = d[a.rank + f + half];
-        v = j < half ? u * c - w * s : w * c + u * s;
+        v = i < half ? u * c - w * s : w * c + u * s;
+      } else if (i >= a.rot8 && i < a.rot8 + a.rank) {
+        v = d[i - a.rot8] * r * a.norm_w[i - a.rot8];
       }
       store_act<T>(row + i, v);
     }
@@ -80,47 +93,51 @@ latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj
   const float *q = proj + (int64_t)h * (a.dim + a.rot_dim);
   float *out = a.query + (int64_t)h * a.row_elems;
   const int Kp = a.uk_ktiles * kBfTileK;
+  // one channel group per wavefront, its first tiles asked for ahead of the query
+  const int g = blockIdx.y * kStepWaves + wave, gl = min(g, a.uk_groups - 1);
+  const uint4 *wp = uk + ((int64_t)h * a.uk_groups + gl) * a.uk_ktiles * 64 + lane;
+  constexpr int kAhead = 4;
+  uint4 w[kAhead];
+#pragma unroll
+  for (int u = 0; u < kAhead; ++u)
+    w[u] = wp[(int64_t)min(u, a.uk_ktiles - 1) * 64];
   for (int i = tid; i < Kp; i += kStepThreads)
     lds[i] = i < a.dim ? q[i] : 0.f;
   if (blockIdx.y == 0)
-    for (int i = a.rank + tid; i < a.row_elems; i += kStepThreads) {
+    for (int i = tid; i < a.row_elems; i += kStepThreads) {
+      if (i >= a.rot8 && i < a.rot8 + a.rank)
+        continue; // the latent part, below
       float v = 0.f;
-      const int j = i - a.rank;
-      if (j < a.rot_dim) {
-        const int f = j < half ? j : j - half;
+      if (i < a.rot_dim) {
+        const int f = i < half ? i : i - half;
         float c, s;
         rotation(a.turns[f], p, c, s);
-        const float u = q[a.dim + f], w = q[a.dim + f + half];
-        v = (j < half ? u * c - w * s : w * c + u * s) * a.scale;
+        const float u = q[a.dim + f], x = q[a.dim + f + half];
+        v = (i < half ? u * c - x * s : x * c + u * s) * a.scale;
       }
       out[i] = v;
     }
   __syncthreads();
-  for (int g = blockIdx.y * kStepWaves + wave; g < a.uk_groups; g += gridDim.y * kStepWaves) {
-    const uint4 *wp = uk + ((int64_t)h * a.uk_groups + g) * a.uk_ktiles * 64 + lane;
-    float acc = 0.f;
-#pragma unroll 4
-    for (int t = 0; t < a.uk_ktiles; ++t) {
-      const uint4 w = wp[(int64_t)t * 64];
-      const float *x = lds + t * kBfTileK + (lane >> 4) * 8;
-      acc = fmaf(bf_lo(w.x), x[0], acc);
-      acc = fmaf(bf_hi(w.x), x[1], acc);
-      acc = fmaf(bf_lo(w.y), x[2], acc);
-      acc = fmaf(bf_hi(w.y), x[3], acc);
-      acc = fmaf(bf_lo(w.z), x[4], acc);
-      acc = fmaf(bf_hi(w.z), x[5], acc);
-      acc = fmaf(bf_lo(w.w), x[6], acc);
-      acc = fmaf(bf_hi(w.w), x[7], acc);
+  float acc = 0.f;
+  for (int t = 0; t < a.uk_ktiles; t += kAhead) {
+    if (t > 0) {
+#pragma unroll
+      for (int u = 0; u < kAhead; ++u)
+        w[u] = wp[(int64_t)min(t + u, a.uk_ktiles - 1) * 64];
     }
-    acc = sum_rows(acc);
-    const int l = g * 16 + lane;
-    if (lane < 16 && l < a.rank)
-      out[l] = acc * a.scale;
+#pragma unroll
+    for (int u = 0; u < kAhead; ++u)
+      if (t + u < a.uk_ktiles)
+        acc = dot_run(w[u], lds + (t + u) * kBfTileK + (lane >> 4) * 8, acc);
   }
+  acc = sum_rows(acc);
+  const int l = g * 16 + lane;
+  if (lane < 16 && l < a.rank)
+    out[a.rot8 + l] = acc * a.scale;
 }
 
 struct LatentPartArgs {
-  int heads, heads16, rank16, row_elems, window, ring_mask, lds_stride;
+  int heads, heads16, rank16, rot8, row_elems, window, ring_mask, lds_stride;
   const int *pos;
   float *acc, *ml;
 };
@@ -133,13 +150,11 @@ template <typename T, int KT>
 __global__ void __launch_bounds__(KT * 256)
 latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query, LatentPartArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
-  constexpr int kThreads = KT * 256, kKeys = KT * 16;
+  constexpr int kKeys = KT * 16;
   const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int qs = a.row_elems + 4;
   T *ck = reinterpret_cast<T *>(raw);                                            // [kKeys][lds_stride]
-  float *qq = reinterpret_cast<float *>(raw + sizeof(T) * kKeys * a.lds_stride); // [16][qs]
-  float *sp = qq + 16 * qs;                                                      // [KT][4][16][16]
+  float *sp = reinterpret_cast<float *>(raw + sizeof(T) * kKeys * a.lds_stride); // [KT][4][16][16]
   const int p = *a.pos;
   const int lo = max(0, p - a.window + 1), n = p - lo + 1;
   const int k0 = blockIdx.x * kKeys, head0 = blockIdx.y * 16;
@@ -151,39 +166,55 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
     }
     return;
   }
-  constexpr int E = 16 / (int)sizeof(T);
+  // four rows of the tile per wavefront, and this lane's query values: a step of 32 k
+  // in every fourth, the first kQSteps of them in flight together
+  constexpr int E = 16 / (int)sizeof(T), kQSteps = 5;
+  const int kt = wave >> 2, quarter = wave & 3, steps = a.row_elems / 32;
   const int runs = a.row_elems / E;
-  for (int i = tid; i < kKeys * runs; i += kThreads) {
-    const int r = i / runs, c = i - r * runs;
-    uint4 v{0, 0, 0, 0};
-    if (k0 + r < n)
-      v = *reinterpret_cast<const uint4 *>(cache + (int64_t)((lo + k0 + r) & a.ring_mask) * a.row_elems + c * E);
-    *reinterpret_cast<uint4 *>(ck + r * a.lds_stride + c * E) = v;
-  }
-  const int qruns = a.row_elems / 4;
-  for (int i = tid; i < 16 * qruns; i += kThreads) {
-    const int r = i / qruns, c = i - r * qruns;
-    f32x4 v{0.f, 0.f, 0.f, 0.f};
-    if (head0 + r < a.heads)
-      v = *reinterpret_cast<const f32x4 *>(query + (int64_t)(head0 + r) * a.row_elems + c * 4);
-    *reinterpret_cast<f32x4 *>(qq + r * qs + c * 4) = v;
+  // (what columns of heads past the last compute is not used)
+  const float *qr = query + (int64_t)(head0 + col) * a.row_elems + quad * 8;
+  Frag<float> qf[kQSteps];
+#pragma unroll
+  for (int i = 0; i < kQSteps; ++i)
+    qf[i].load(qr + min(quarter + i * 4, steps - 1) * 32);
+  for (int c0 = 0; c0 < runs; c0 += 128) {
+    u32x4 v[4][2];
+    const int ca = min(c0 + lane, runs - 1), cb = min(c0 + 64 + lane, runs - 1);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) { // a row past the last key repeats it, masked below
+      const T *row = cache + (int64_t)((lo + min(k0 + wave * 4 + r, n - 1)) & a.ring_mask) * a.row_elems;
+      v[r][0] = *reinterpret_cast<const u32x4 *>(row + ca * E);
+      v[r][1] = *reinterpret_cast<const u32x4 *>(row + cb * E);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      T *row = ck + (wave * 4 + r) * a.lds_stride;
+      *reinterpret_cast<u32x4 *>(row + ca * E) = v[r][0];
+      *reinterpret_cast<u32x4 *>(row + cb * E) = v[r][1];
+    }
   }
   __syncthreads();
   {
-    const int kt = wave >> 2, quarter = wave & 3;
     f32x4 s{0.f, 0.f, 0.f, 0.f};
     const T *kr = ck + (kt * 16 + col) * a.lds_stride + quad * 8;
-    const float *qr = qq + col * qs + quad * 8;
-    for (int t = quarter; t < a.row_elems / 32; t += 4) {
+    auto score = [&](int t, const Frag<float> &q) {
       Frag<T> kf;
-      Frag<float> qf, kw;
       kf.load(kr + t * 32);
-      qf.load(qr + t * 32);
+      Frag<float> kw;
       if constexpr (sizeof(T) == 2)
         kw = widen(kf.v);
       else
         kw = kf;
-      s = mfma32(kw, qf, s);
+      s = mfma32(kw, q, s);
+    };
+#pragma unroll
+    for (int i = 0; i < kQSteps; ++i)
+      if (quarter + i * 4 < steps)
+        score(quarter + i * 4, qf[i]);
+    for (int t = quarter + kQSteps * 4; t < steps; t += 4) {
+      Frag<float> q;
+      q.load(qr + t * 32);
+      score(t, q);
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r)
@@ -233,7 +264,7 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
     for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        o = mfma_f32(load_act<T>(ck + (kt * 16 + quad * 4 + r) * a.lds_stride + lt * 16 + col),
+        o = mfma_f32(load_act<T>(ck + (kt * 16 + quad * 4 + r) * a.lds_stride + a.rot8 + lt * 16 + col),
                      pr[kt][r], o);
     *reinterpret_cast<f32x4 *>(acc + lt * 16 + quad * 4) = o;
   }
@@ -293,27 +324,34 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
   for (int i = 0; i < kStepWaves; ++i)
     l += red[1][i];
   const float inv = 1.0f / l;
+  // the partials in four parts: 128 threads take four latent dimensions each of every
+  // fourth chunk, eight in flight
   const int64_t step = (int64_t)a.heads16 * a.rank16;
-  for (int i = tid; i < Kp; i += kStepThreads) {
-    float o = 0.f;
-    if (i < a.rank) {
+  const int part4 = tid >> 7;
+  float *fold = wt + ((a.chunks + 3) & ~3); // [4][Kp]
+  for (int i = (tid & 127) * 4; i < Kp; i += 512) {
+    f32x4 o{0.f, 0.f, 0.f, 0.f};
+    if (i < a.rank16) {
       const float *q = a.acc + (int64_t)h * a.rank16 + i;
-      int c = 0;
-      for (; c + 8 <= a.chunks; c += 8) {
-        float v[8];
+      for (int c = part4; c < a.chunks; c += 32) {
+        f32x4 v[8];
 #pragma unroll
         for (int u = 0; u < 8; ++u)
-          v[u] = q[(c + u) * step];
+          v[u] = *reinterpret_cast<const f32x4 *>(q + min(c + u * 4, a.chunks - 1) * step);
 #pragma unroll
-        for (int u = 0; u < 8; ++u) // an empty partial's accumulators were never written
-          o = wt[c + u] != 0.f ? fmaf(wt[c + u], v[u], o) : o;
+        for (int u = 0; u < 8; ++u) {
+          const float e = c + u * 4 < a.chunks ? wt[min(c + u * 4, a.chunks - 1)] : 0.f;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) // an empty partial's accumulators were never written
+            o[j] = e != 0.f ? fmaf(e, v[u][j], o[j]) : o[j];
+        }
       }
-      for (; c < a.chunks; ++c)
-        o = wt[c] != 0.f ? fmaf(wt[c], q[c * step], o) : o;
-      o *= inv;
     }
-    x[i] = o;
+    *reinterpret_cast<f32x4 *>(fold + part4 * Kp + i) = o;
   }
+  __syncthreads();
+  for (int i = tid; i < Kp; i += kStepThreads)
+    x[i] = i < a.rank ? ((fold[i] + fold[Kp + i]) + (fold[2 * Kp + i] + fold[3 * Kp + i])) * inv : 0.f;
   __syncthreads();
   float acc = 0.f;
   const float *xp = x + (lane >> 4) * 8;
@@ -325,17 +363,8 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
     }
 #pragma unroll
     for (int u = 0; u < kAhead; ++u)
-      if (t + u < t1) {
-        const float *v = xp + (t + u) * kBfTileK;
-        acc = fmaf(bf_lo(w[u].x), v[0], acc);
-        acc = fmaf(bf_hi(w[u].x), v[1], acc);
-        acc = fmaf(bf_lo(w[u].y), v[2], acc);
-        acc = fmaf(bf_hi(w[u].y), v[3], acc);
-        acc = fmaf(bf_lo(w[u].z), v[4], acc);
-        acc = fmaf(bf_hi(w[u].z), v[5], acc);
-        acc = fmaf(bf_lo(w[u].w), v[6], acc);
-        acc = fmaf(bf_hi(w[u].w), v[7], acc);
-      }
+      if (t + u < t1)
+        acc = dot_run(w[u], xp + (t + u) * kBfTileK, acc);
   }
   acc = sum_rows(acc);
   if (lane < 16)
@@ -353,21 +382,22 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
 // ---- many tokens -----------------------------------------------------------------
 
 struct LatentRowsArgs {
-  int heads, dim, rot_dim, rank, row_elems, ring_mask, dkv_at, ld, start;
+  int heads, dim, dim16, rot_dim, rot8, rank, row_elems, key_elems, ring_mask, dkv_at, ld, start;
   float scale, eps;
   const float *norm_w;
   const double *turns;
 };
 
-// One workgroup per token: the cache row, and the queries rotated and scaled in place.
+// One workgroup per token: its cache row and its queries.
 template <typename T>
 __global__ void __launch_bounds__(256)
-latent_rows_kernel(float *__restrict__ proj, T *__restrict__ cache, LatentRowsArgs a) {
+latent_rows_kernel(const float *__restrict__ proj, T *__restrict__ cache, T *__restrict__ queries,
+                   LatentRowsArgs a) {
   extern __shared__ float lds[]; // cos, sin of this position
   __shared__ float red[4];
   const int tid = threadIdx.x, half = a.rot_dim / 2;
   const int p = a.start + blockIdx.x;
-  float *row = proj + (int64_t)blockIdx.x * a.ld;
+  const float *row = proj + (int64_t)blockIdx.x * a.ld;
   const float *d = row + a.dkv_at;
   for (int f = tid; f < half; f += 256)
     rotation(a.turns[f], p, lds[f], lds[half + f]);
@@ -379,212 +409,305 @@ latent_rows_kernel(float *__restrict__ proj, T *__restrict__ cache, LatentRowsAr
     red[tid >> 6] = ss;
   __syncthreads();
   const float r = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.rank + a.eps);
+  // value j of the rotated vector that starts at v
+  auto turned = [&](const float *v, int j) {
+    const int f = j < half ? j : j - half;
+    const float u = v[f], w = v[f + half], c = lds[f], s = lds[half + f];
+    return j < half ? u * c - w * s : w * c + u * s;
+  };
   T *out = cache + (int64_t)(p & a.ring_mask) * a.row_elems;
   for (int i = tid; i < a.row_elems; i += 256) {
     float v = 0.f;
-    if (i < a.rank) {
-      v = d[i] * r * a.norm_w[i];
-    } else if (i < a.rank + a.rot_dim) {
-      const int j = i - a.rank, f = j < half ? j : j - half;
-      const float u = d[a.rank + f], w = d[a.rank + f + half];
-      v = j < half ? u * lds[f] - w * lds[half + f] : w * lds[f] + u * lds[half + f];
-    }
+    if (i < a.rot_dim)
+      v = turned(d + a.rank, i);
+    else if (i >= a.rot8 && i < a.rot8 + a.rank)
+      v = d[i - a.rot8] * r * a.norm_w[i - a.rot8];
     store_act<T>(out + i, v);
   }
-  const int per = a.dim + half; // work items per head: unrotated values, then pairs
-  for (int i = tid; i < a.heads * per; i += 256) {
-    const int h = i / per, j = i - h * per;
-    float *q = row + (int64_t)h * (a.dim + a.rot_dim);
-    if (j < a.dim) {
-      q[j] *= a.scale;
-    } else {
-      const int f = j - a.dim;
-      const float u = q[a.dim + f], w = q[a.dim + f + half];
-      q[a.dim + f] = (u * lds[f] - w * lds[half + f]) * a.scale;
-      q[a.dim + f + half] = (w * lds[f] + u * lds[half + f]) * a.scale;
+  T *qo = queries + (int64_t)blockIdx.x * a.heads * a.key_elems;
+  for (int h = tid >> 6; h < a.heads; h += 4) {
+    const float *q = row + (int64_t)h * (a.dim + a.rot_dim);
+    for (int k = tid & 63; k < a.key_elems; k += 64) {
+      float v = 0.f;
+      if (k < a.dim)
+        v = q[k] * a.scale;
+      else if (k >= a.dim16 && k < a.dim16 + a.rot_dim)
+        v = turned(q + a.dim, k - a.dim16) * a.scale;
+      store_act<T>(qo + (int64_t)h * a.key_elems + k, v);
     }
   }
 }
 
 struct LatentAttnArgs {
-  int heads, dim, dim16, rot_dim, vdim, vdim16, rank, row_elems, window, ring_mask;
+  int heads, dim16, rot8, vdim, nv, row_elems, window, ring_mask;
   int ld, gate_at, rows, start, first, value_ld, out_ld;
-  int kd, k_stride, v_stride; // LDS: padded key size, row strides of the K / Q and V^T tiles
+  int kd, k_stride, v_stride; // elements of a key; LDS row strides of the K and V^T tiles
 };
 
-constexpr int kTileKeys = 32;
+// Keys of a tile: 128 bytes of a V^T row.
+template <typename T> struct KeyTile {
+  static constexpr int kKeys = 128 / (int)sizeof(T);
+};
 
-// Grid (query blocks, heads).  A wavefront owns 16 queries; the workgroup's share
-// tiles of 32 keys through LDS.  S^T = K . Q^T leaves a lane with keys of one
-// query, which is the B operand of O^T += V^T . P^T as it lies.
-template <typename T, int NV>
+// Grid (heads, query blocks).  A wavefront owns 16 * QT queries, the workgroup's four
+// share tiles of kKeys keys through LDS; the next tile is on its way in registers
+// meanwhile.  S^T = K . Q^T leaves a lane with keys of one query, which is the B
+// operand of O^T += V^T . P^T as it lies (of 32 keys in bfloat16: a lane's eight are
+// keys 4q .. 4q + 3 of both halves, and V^T rows are stored in that order).
+// NK: 32-element steps of a key, NV: 16-channel groups of a value, at most.
+template <typename T, int NK, int NV, int QT>
 __global__ void __launch_bounds__(256)
-latent_attention_kernel(const float *__restrict__ proj, const T *__restrict__ keys,
+latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ keys,
                         const T *__restrict__ values_t, const T *__restrict__ cache,
-                        T *__restrict__ out, LatentAttnArgs a) {
+                        const float *__restrict__ proj, T *__restrict__ out, LatentAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
-  constexpr int E = 16 / (int)sizeof(T);
-  const int threads = blockDim.x, waves = threads >> 6, block = waves * 16;
+  constexpr int E = 16 / (int)sizeof(T), KEYS = KeyTile<T>::kKeys, SUB = KEYS / 16;
+  constexpr int KL = NK, VL = (NV + 1) / 2; // 16-byte loads per thread and tile
   const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int h = blockIdx.y;
-  // long blocks first
-  const int qb = gridDim.x - 1 - blockIdx.x, q0 = qb * block;
-  T *qt = reinterpret_cast<T *>(raw);                // [block][k_stride]
-  T *kt = qt + block * a.k_stride;                   // [32][k_stride]
-  T *vt = kt + kTileKeys * a.k_stride;               // [vdim16][v_stride]
-  for (int i = tid; i < block * a.kd; i += threads) {
-    const int r = i / a.kd, k = i - r * a.kd;
-    float v = 0.f;
-    if (q0 + r < a.rows) {
-      const float *q = proj + (int64_t)(q0 + r) * a.ld + (int64_t)h * (a.dim + a.rot_dim);
-      if (k < a.dim)
-        v = q[k];
-      else if (k >= a.dim16 && k < a.dim16 + a.rot_dim)
-        v = q[a.dim + k - a.dim16];
-    }
-    store_act<T>(qt + r * a.k_stride + k, v);
-  }
-  const int last_q = min(q0 + block, a.rows) - 1;
-  const int key_hi = a.start + last_q - a.first;                                      // last visible
-  const int key_lo = max(0, a.start + q0 - a.window + 1 - a.first) & ~(kTileKeys - 1); // tile of the first
-  const int nkeys = a.start + a.rows - a.first;
-  const int my_q = a.start + q0 + wave * 16 + col - a.first; // this lane's query as a key index
+  const int h = blockIdx.x;
+  constexpr int kBlock = 64 * QT;
+  const int q0 = (gridDim.y - 1 - blockIdx.y) * kBlock; // long blocks first
+  T *kt = reinterpret_cast<T *>(raw); // [KEYS][k_stride]
+  T *vt = kt + KEYS * a.k_stride;     // [16 * nv][v_stride]
+  const int nk = a.kd / 32;
 
-  f32x4 o[NV];
+  // this lane's queries as key indexes, and their fragments
+  int my_q[QT];
+  Frag<T> qf[QT][NK];
 #pragma unroll
-  for (int v = 0; v < NV; ++v)
-    o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
-  const int nv = a.vdim16 / 16;
-  const int64_t kld = (int64_t)a.heads * a.dim16;
-  for (int k0 = key_lo; k0 <= key_hi; k0 += kTileKeys) {
-    __syncthreads(); // the previous tile has been read (and the queries are staged)
-    const int kruns = a.dim16 / E;
-    for (int i = tid; i < kTileKeys * kruns; i += threads) {
-      const int r = i / kruns, c = i - r * kruns;
-      uint4 v{0, 0, 0, 0};
-      if (k0 + r < nkeys)
-        v = *reinterpret_cast<const uint4 *>(keys + (k0 + r) * kld + h * a.dim16 + c * E);
-      *reinterpret_cast<uint4 *>(kt + r * a.k_stride + c * E) = v;
-    }
-    const int tail = a.kd - a.dim16; // the shared rotated part and the padding
-    for (int i = tid; i < kTileKeys * tail; i += threads) {
-      const int r = i / tail, c = i - r * tail;
-      T v = 0;
-      if (k0 + r < nkeys && c < a.rot_dim)
-        v = cache[(int64_t)((a.first + k0 + r) & a.ring_mask) * a.row_elems + a.rank + c];
-      kt[r * a.k_stride + a.dim16 + c] = v;
-    }
-    constexpr int vruns = kTileKeys / E;
-    for (int i = tid; i < a.vdim16 * vruns; i += threads) {
-      const int r = i / vruns, c = i - r * vruns;
-      uint4 v = *reinterpret_cast<const uint4 *>(values_t + (int64_t)(h * a.vdim16 + r) * a.value_ld + k0 + c * E);
-      if (k0 + c * E + E > nkeys) { // columns past the last key hold anything
-        T e[E];
-        __builtin_memcpy(e, &v, 16);
+  for (int u = 0; u < QT; ++u) {
+    const int r = q0 + (wave * QT + u) * 16 + col;
+    my_q[u] = a.start + r - a.first;
+    const T *q = queries + ((int64_t)min(r, a.rows - 1) * a.heads + h) * a.kd + quad * 8;
 #pragma unroll
-        for (int j = 0; j < E; ++j)
-          if (k0 + c * E + j >= nkeys)
-            e[j] = 0;
-        __builtin_memcpy(&v, e, 16);
+    for (int t = 0; t < NK; ++t)
+      qf[u][t].load(q + min(t, nk - 1) * 32);
+  }
+  const int nkeys = a.start + a.rows - a.first;
+  const int last_q = min(q0 + kBlock, a.rows) - 1;
+  const int key_hi = a.start + last_q - a.first;                               // last visible
+  const int key_lo = max(0, a.start + q0 - a.window + 1 - a.first) & ~(KEYS - 1); // tile of the first
+  const int wave_q0 = a.start + q0 + wave * 16 * QT - a.first, wave_q1 = wave_q0 + 16 * QT - 1;
+
+  // the 16-byte runs this thread moves.  A key's runs: its head's part, the shared
+  // rotated part; the rest of the row in LDS stays zero.
+  const int runs_head = a.dim16 / E, runs = runs_head + a.rot8 / E;
+  const T *ksrc[KL];
+  int kkey[KL], kdst[KL], kstep[KL];
+  bool kring[KL];
+#pragma unroll
+  for (int i = 0; i < KL; ++i) {
+    const int id = min(i * 256 + tid, KEYS * runs - 1); // past the end: the last one again
+    const int r = id / runs, c = id - r * runs;
+    kkey[i] = r;
+    kdst[i] = r * a.k_stride + (c < runs_head ? c * E : a.dim16 + (c - runs_head) * E);
+    kring[i] = c >= runs_head;
+    kstep[i] = c < runs_head ? a.heads * a.dim16 : a.row_elems;
+    ksrc[i] = c < runs_head ? keys + h * a.dim16 + c * E : cache + (c - runs_head) * E;
+  }
+  const T *vsrc[VL];
+  int vdst[VL], vcol[VL];
+  const int vruns = 16 * a.nv * 8;
+#pragma unroll
+  for (int i = 0; i < VL; ++i) {
+    const int id = min(i * 256 + tid, vruns - 1), r = id >> 3, c = id & 7;
+    vsrc[i] = values_t + (int64_t)(h * 16 * a.nv + r) * a.value_ld + c * E;
+    vcol[i] = c * E;
+    // bfloat16: the run's two halves of four keys go to their places in the lane order
+    vdst[i] = r * a.v_stride + (sizeof(T) == 2 ? (c >> 2) * 32 + (c & 1) * 16 + ((c >> 1) & 1) * 4 : c * E);
+  }
+  u32x4 kr[KL], vr[VL];
+  auto fetch = [&](int k0, u32x4 (&kr)[KL], u32x4 (&vr)[VL]) {
+#pragma unroll
+    for (int i = 0; i < KL; ++i) {
+      const int k = min(k0 + kkey[i], nkeys - 1); // masked past the end
+      const int row = kring[i] ? (a.first + k) & a.ring_mask : k;
+      kr[i] = *reinterpret_cast<const u32x4 *>(ksrc[i] + (int64_t)row * kstep[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < VL; ++i)
+      vr[i] = *reinterpret_cast<const u32x4 *>(vsrc[i] + k0);
+  };
+  fetch(key_lo, kr, vr);
+  if (runs * E < a.kd) { // the padding of the keys
+    const int pad = a.kd - runs * E, at = a.dim16 + a.rot8;
+    for (int i = tid; i < KEYS * pad; i += 256)
+      kt[(i / pad) * a.k_stride + at + i % pad] = 0;
+  }
+
+  f32x4 o[QT][NV];
+  float m[QT], l[QT];
+#pragma unroll
+  for (int u = 0; u < QT; ++u) {
+    m[u] = -INFINITY;
+    l[u] = 0.f;
+#pragma unroll
+    for (int v = 0; v < NV; ++v)
+      o[u][v] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  for (int k0 = key_lo; k0 <= key_hi; k0 += KEYS) {
+    __syncthreads(); // the previous tile has been read
+#pragma unroll
+    for (int i = 0; i < KL; ++i)
+      *reinterpret_cast<u32x4 *>(kt + kdst[i]) = kr[i];
+    if (k0 + KEYS > nkeys) { // value columns past the last key hold anything
+#pragma unroll
+      for (int i = 0; i < VL; ++i) {
+        const int keep = nkeys - k0 - vcol[i];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          if constexpr (sizeof(T) == 4)
+            vr[i][j] = j < keep ? vr[i][j] : 0u;
+          else
+            vr[i][j] = 2 * j + 1 < keep ? vr[i][j] : 2 * j < keep ? vr[i][j] & 0xffffu : 0u;
+        }
       }
-      *reinterpret_cast<uint4 *>(vt + r * a.v_stride + c * E) = v;
+    }
+#pragma unroll
+    for (int i = 0; i < VL; ++i) {
+      if constexpr (sizeof(T) == 2) {
+        *reinterpret_cast<uint2 *>(vt + vdst[i]) = uint2{vr[i][0], vr[i][1]};
+        *reinterpret_cast<uint2 *>(vt + vdst[i] + 8) = uint2{vr[i][2], vr[i][3]};
+      } else {
+        *reinterpret_cast<u32x4 *>(vt + vdst[i]) = vr[i];
+      }
     }
     __syncthreads();
-    f32x4 s0{0.f, 0.f, 0.f, 0.f}, s1 = s0;
-    const T *qr = qt + (wave * 16 + col) * a.k_stride + quad * 8;
-    const T *kr = kt + col * a.k_stride + quad * 8;
-    for (int t = 0; t < a.kd; t += 32) {
-      Frag<T> q, ka, kb;
-      q.load(qr + t);
-      ka.load(kr + t);
-      kb.load(kr + 16 * a.k_stride + t);
-      s0 = mfma32(ka, q, s0);
-      s1 = mfma32(kb, q, s1);
-    }
-    float mt = m;
+    fetch(min(k0 + KEYS, (nkeys - 1) & ~(KEYS - 1)), kr, vr);
+    if (k0 > wave_q1 || k0 + KEYS - 1 <= wave_q0 - a.window)
+      continue; // nothing of this tile is visible to this wavefront
+    f32x4 s[QT][SUB];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int ka = k0 + quad * 4 + r, kb = ka + 16;
-      s0[r] = ka <= my_q && my_q - ka < a.window ? s0[r] : -INFINITY;
-      s1[r] = kb <= my_q && my_q - kb < a.window ? s1[r] : -INFINITY;
-      mt = fmaxf(mt, fmaxf(s0[r], s1[r]));
-    }
-    {
+    for (int u = 0; u < QT; ++u)
+#pragma unroll
+      for (int b = 0; b < SUB; ++b)
+        s[u][b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const T *kp = kt + col * a.k_stride + quad * 8;
+#pragma unroll
+    for (int t = 0; t < NK; ++t)
+      if (t < nk) {
+#pragma unroll
+        for (int b = 0; b < SUB; ++b) {
+          Frag<T> kf;
+          kf.load(kp + b * 16 * a.k_stride + t * 32);
+#pragma unroll
+          for (int u = 0; u < QT; ++u)
+            s[u][b] = mfma32(kf, qf[u][t], s[u][b]);
+        }
+      }
+    const bool whole = k0 + KEYS - 1 <= wave_q0 && wave_q1 - k0 < a.window;
+    float alpha[QT];
+#pragma unroll
+    for (int u = 0; u < QT; ++u) {
+      float mt = m[u];
+      if (!whole) {
+#pragma unroll
+        for (int b = 0; b < SUB; ++b)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const int gap = my_q[u] - (k0 + b * 16 + quad * 4 + r);
+            s[u][b][r] = gap >= 0 && gap < a.window ? s[u][b][r] : -INFINITY;
+          }
+      }
+#pragma unroll
+      for (int b = 0; b < SUB; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          mt = fmaxf(mt, s[u][b][r]);
       float x, y;
       lane_pair<16>(mt, x, y);
       mt = fmaxf(x, y);
       lane_pair<32>(mt, x, y);
       mt = fmaxf(x, y);
-    }
-    const float base = mt == -INFINITY ? 0.f : mt; // nothing visible so far
-    const float alpha = fast_exp(m - base);
-    m = mt;
-    float sum = 0.f;
+      const float base = mt == -INFINITY ? 0.f : mt; // nothing visible so far
+      alpha[u] = fast_exp(m[u] - base);
+      m[u] = mt;
+      float sum = 0.f;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      s0[r] = fast_exp(s0[r] - base);
-      s1[r] = fast_exp(s1[r] - base);
-      sum += s0[r] + s1[r];
-    }
-    l = fmaf(l, alpha, sum);
-    if constexpr (sizeof(T) == 2) {
-      uint4 hi, lo;
-      unsigned *ph = reinterpret_cast<unsigned *>(&hi), *pl = reinterpret_cast<unsigned *>(&lo);
+      for (int b = 0; b < SUB; ++b)
 #pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        ph[j] = pack_bf(s0[2 * j], s0[2 * j + 1]);
-        pl[j] = pack_bf(s0[2 * j] - bf_lo(ph[j]), s0[2 * j + 1] - bf_hi(ph[j]));
-        ph[2 + j] = pack_bf(s1[2 * j], s1[2 * j + 1]);
-        pl[2 + j] = pack_bf(s1[2 * j] - bf_lo(ph[2 + j]), s1[2 * j + 1] - bf_hi(ph[2 + j]));
-      }
+        for (int r = 0; r < 4; ++r) {
+          s[u][b][r] = fast_exp(s[u][b][r] - base);
+          sum += s[u][b][r];
+        }
+      l[u] = fmaf(l[u], alpha[u], sum);
+    }
+#pragma unroll
+    for (int u = 0; u < QT; ++u)
 #pragma unroll
       for (int v = 0; v < NV; ++v)
-        if (v < nv) {
-          const T *vr = vt + (v * 16 + col) * a.v_stride + quad * 4;
-          const uint2 va = *reinterpret_cast<const uint2 *>(vr), vb = *reinterpret_cast<const uint2 *>(vr + 16);
-          const uint4 vv{va.x, va.y, vb.x, vb.y};
+        if (v < a.nv) {
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            o[v][r] *= alpha;
-          o[v] = mfma_bf16(vv, hi, o[v]);
-          o[v] = mfma_bf16(vv, lo, o[v]);
+            o[u][v][r] *= alpha[u];
+        }
+    if constexpr (sizeof(T) == 2) {
+      // the weights as two bfloat16 terms
+      uint4 hi[QT][SUB / 2], lo[QT][SUB / 2];
+#pragma unroll
+      for (int u = 0; u < QT; ++u)
+#pragma unroll
+        for (int b = 0; b < SUB / 2; ++b) {
+          unsigned ph[4], pl[4];
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const f32x4 &x = s[u][2 * b + (j >> 1)];
+            const float x0 = x[2 * (j & 1)], x1 = x[2 * (j & 1) + 1];
+            ph[j] = pack_bf(x0, x1);
+            pl[j] = pack_bf(x0 - bf_lo(ph[j]), x1 - bf_hi(ph[j]));
+          }
+          hi[u][b] = uint4{ph[0], ph[1], ph[2], ph[3]};
+          lo[u][b] = uint4{pl[0], pl[1], pl[2], pl[3]};
+        }
+#pragma unroll
+      for (int v = 0; v < NV; ++v)
+        if (v < a.nv) {
+#pragma unroll
+          for (int b = 0; b < SUB / 2; ++b) {
+            const uint4 vv = *reinterpret_cast<const uint4 *>(vt + (v * 16 + col) * a.v_stride + b * 32 + quad * 8);
+#pragma unroll
+            for (int u = 0; u < QT; ++u) {
+              o[u][v] = mfma_bf16(vv, hi[u][b], o[u][v]);
+              o[u][v] = mfma_bf16(vv, lo[u][b], o[u][v]);
+            }
+          }
         }
     } else {
 #pragma unroll
       for (int v = 0; v < NV; ++v)
-        if (v < nv) {
-          const float *vr = reinterpret_cast<const float *>(vt) + (v * 16 + col) * a.v_stride + quad * 4;
-          const f32x4 va = *reinterpret_cast<const f32x4 *>(vr), vb = *reinterpret_cast<const f32x4 *>(vr + 16);
+        if (v < a.nv) {
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
-            o[v][r] *= alpha;
+          for (int b = 0; b < SUB; ++b) {
+            const f32x4 vv = *reinterpret_cast<const f32x4 *>(vt + (v * 16 + col) * a.v_stride + b * 16 + quad * 4);
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
-            o[v] = mfma_f32(va[r], s0[r], o[v]);
+            for (int u = 0; u < QT; ++u)
 #pragma unroll
-          for (int r = 0; r < 4; ++r)
-            o[v] = mfma_f32(vb[r], s1[r], o[v]);
+              for (int r = 0; r < 4; ++r)
+                o[u][v] = mfma_f32(vv[r], s[u][b][r], o[u][v]);
+          }
         }
     }
   }
-  l = sum_rows(l);
-  const int qi = q0 + wave * 16 + col;
-  if (qi >= a.rows)
-    return;
-  const float f = sigmoid_f(proj[(int64_t)qi * a.ld + a.gate_at + h]) / l;
-  T *dst = out + (int64_t)qi * a.out_ld + (int64_t)h * a.vdim;
 #pragma unroll
-  for (int v = 0; v < NV; ++v)
-    if (v < nv) {
+  for (int u = 0; u < QT; ++u) {
+    const float sum = sum_rows(l[u]);
+    const int qi = q0 + (wave * QT + u) * 16 + col;
+    if (qi >= a.rows)
+      continue;
+    const float f = sigmoid_f(proj[(int64_t)qi * a.ld + a.gate_at + h]) / sum;
+    T *dst = out + (int64_t)qi * a.out_ld + (int64_t)h * a.vdim;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int c = v * 16 + quad * 4 + r;
-        if (c < a.vdim)
-          store_act<T>(dst + c, o[v][r] * f);
+    for (int v = 0; v < NV; ++v)
+      if (v < a.nv) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int c = v * 16 + quad * 4 + r;
+          if (c < a.vdim)
+            store_act<T>(dst + c, o[u][v][r] * f);
+        }
       }
-    }
+  }
 }
 
 bool shape_ok(const LatentShape &s) {
@@ -595,8 +718,7 @@ bool shape_ok(const LatentShape &s) {
 size_t part_lds(const LatentShape &s, int kt, int *stride) {
   // rows of the tile start 4 banks apart
   *stride = s.row_elems() + (s.f32 ? 4 : 8);
-  return (size_t)(s.f32 ? 4 : 2) * 16 * kt * *stride + 4 * (size_t)16 * (s.row_elems() + 4) +
-         4 * (size_t)kt * 4 * 256;
+  return (size_t)(s.f32 ? 4 : 2) * 16 * kt * *stride + 4 * (size_t)kt * 4 * 256;
 }
 constexpr size_t kLdsLimit = 156 * 1024;
 
@@ -627,7 +749,7 @@ int launch_latent_step(const LatentStep &a, int span, hipStream_t stream) {
              "latent_step: matrix shapes");
   const int re = s.row_elems();
   {
-    LatentQueryArgs q{s.heads, s.dim, s.rot_dim, s.rank, re, s.ring_mask, a.dkv_at,
+    LatentQueryArgs q{s.heads, s.dim, s.rot_dim, s.rot8(), s.rank, re, s.ring_mask, a.dkv_at,
                       s.rank16() / 16, a.uk_t.ktiles, s.scale, s.eps, a.norm_w, a.turns, a.pos,
                       a.cache, a.query};
     const dim3 grid((unsigned)(s.heads + 1), (unsigned)ceil_div(q.uk_groups, kStepWaves));
@@ -643,7 +765,7 @@ int launch_latent_step(const LatentStep &a, int span, hipStream_t stream) {
   }
   const LatentCut cut = latent_step_cut(s, span);
   {
-    LatentPartArgs p{s.heads, s.heads16(), s.rank16(), re, s.window, s.ring_mask, 0, a.pos,
+    LatentPartArgs p{s.heads, s.heads16(), s.rank16(), s.rot8(), re, s.window, s.ring_mask, 0, a.pos,
                      a.part_acc, a.part_ml};
     const size_t lds = part_lds(s, cut.key_tiles, &p.lds_stride);
     BH_REQUIRE(lds <= kLdsLimit, "latent_step: a cache row of %d values does not fit LDS", re);
@@ -670,7 +792,7 @@ int launch_latent_step(const LatentStep &a, int span, hipStream_t stream) {
   {
     LatentFoldArgs f{s.heads16(), s.rank, s.rank16(), s.vdim, s.vdim16() / 16, a.uv.ktiles,
                      cut.chunks, a.part_acc, a.part_ml, a.proj + a.gate_at, a.out};
-    const size_t lds = sizeof(float) * ((size_t)a.uv.ktiles * kBfTileK + (size_t)cut.chunks);
+    const size_t lds = sizeof(float) * ((size_t)5 * a.uv.ktiles * kBfTileK + (size_t)round_up(cut.chunks, 4));
     BH_REQUIRE(lds <= kLdsLimit, "latent_step: %d partials do not fit LDS", cut.chunks);
     static DynLdsOnce once;
     BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_value_kernel, (int)kLdsLimit));
@@ -685,75 +807,69 @@ int latent_first_visible(const LatentShape &s, int start) { return std::max(0, s
 
 int launch_latent_rows(const LatentRows &a, hipStream_t stream) {
   const LatentShape &s = a.s;
-  BH_REQUIRE(shape_ok(s) && a.proj && a.norm_w && a.turns && a.cache && a.rows > 0 && a.start >= 0 &&
-                 a.rows + std::min(a.start, s.window - 1) <= s.ring_mask + 1,
+  BH_REQUIRE(shape_ok(s) && a.proj && a.norm_w && a.turns && a.cache && a.queries && a.rows > 0 &&
+                 a.start >= 0 && a.rows + std::min(a.start, s.window - 1) <= s.ring_mask + 1,
              "latent_rows: bad argument (%d rows from %d)", a.rows, a.start);
-  LatentRowsArgs r{s.heads, s.dim, s.rot_dim, s.rank, s.row_elems(), s.ring_mask, a.dkv_at, a.ld,
-                   a.start, s.scale, s.eps, a.norm_w, a.turns};
+  LatentRowsArgs r{s.heads, s.dim, s.dim16(), s.rot_dim, s.rot8(), s.rank, s.row_elems(),
+                   s.key_elems(), s.ring_mask, a.dkv_at, a.ld, a.start, s.scale, s.eps, a.norm_w,
+                   a.turns};
   const size_t lds = sizeof(float) * (size_t)std::max(2, s.rot_dim);
   if (s.f32)
     hipLaunchKernelGGL(latent_rows_kernel<float>, dim3(a.rows), dim3(256), lds, stream, a.proj,
-                       static_cast<float *>(a.cache), r);
+                       static_cast<float *>(a.cache), static_cast<float *>(a.queries), r);
   else
     hipLaunchKernelGGL(latent_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), lds, stream, a.proj,
-                       static_cast<bf16_bits *>(a.cache), r);
+                       static_cast<bf16_bits *>(a.cache), static_cast<bf16_bits *>(a.queries), r);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }
 
 namespace {
-template <typename T, int NV>
-int launch_attention(const LatentRows &a, const LatentAttnArgs &p, int waves, size_t lds,
-                     hipStream_t stream) {
+template <typename T, int NK, int NV, int QT>
+int launch_attention(const LatentRows &a, const LatentAttnArgs &p, size_t lds, hipStream_t stream) {
   static DynLdsOnce once;
-  BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_attention_kernel<T, NV>, (int)kLdsLimit));
-  hipLaunchKernelGGL((latent_attention_kernel<T, NV>),
-                     dim3((unsigned)ceil_div(a.rows, 16 * waves), (unsigned)a.s.heads),
-                     dim3(waves * 64), lds, stream, a.proj, static_cast<const T *>(a.keys),
-                     static_cast<const T *>(a.values_t), static_cast<const T *>(a.cache),
+  BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_attention_kernel<T, NK, NV, QT>, (int)kLdsLimit));
+  hipLaunchKernelGGL((latent_attention_kernel<T, NK, NV, QT>),
+                     dim3((unsigned)a.s.heads, (unsigned)ceil_div(a.rows, 64 * QT)), dim3(256), lds,
+                     stream, static_cast<const T *>(a.queries), static_cast<const T *>(a.keys),
+                     static_cast<const T *>(a.values_t), static_cast<const T *>(a.cache), a.proj,
                      static_cast<T *>(a.out), p);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }
 template <typename T>
-int launch_attention_any(const LatentRows &a, const LatentAttnArgs &p, int waves, size_t lds,
-                         hipStream_t stream) {
-  const int nv = p.vdim16 / 16;
-  if (nv <= 4)
-    return launch_attention<T, 4>(a, p, waves, lds, stream);
-  if (nv <= 8)
-    return launch_attention<T, 8>(a, p, waves, lds, stream);
-  if (nv <= 16)
-    return launch_attention<T, 16>(a, p, waves, lds, stream);
-  BH_REQUIRE(nv <= 32, "latent_attention: value heads of %d", a.s.vdim);
-  return launch_attention<T, 32>(a, p, waves, lds, stream);
+int launch_attention_any(const LatentRows &a, LatentAttnArgs &p, hipStream_t stream) {
+  p.k_stride = p.kd + 16 / (int)sizeof(T); // rows start 4 banks apart
+  p.v_stride = KeyTile<T>::kKeys + 16 / (int)sizeof(T);
+  const size_t lds = sizeof(T) * ((size_t)KeyTile<T>::kKeys * p.k_stride + (size_t)16 * p.nv * p.v_stride);
+  const int nk = p.kd / 32;
+  BH_REQUIRE(lds <= kLdsLimit && nk <= 18 && p.nv <= 32,
+             "latent_attention: heads of %d and %d values", p.kd, a.s.vdim);
+  // two query tiles per wavefront halve the LDS reads, where they leave enough workgroups
+  const bool two = ceil_div(a.rows, 128) * a.s.heads >= 192;
+  if (nk <= 4 && p.nv <= 4)
+    return two ? launch_attention<T, 4, 4, 2>(a, p, lds, stream)
+               : launch_attention<T, 4, 4, 1>(a, p, lds, stream);
+  if (nk <= 6 && p.nv <= 8)
+    return two && sizeof(T) == 2 ? launch_attention<T, 6, 8, sizeof(T) == 2 ? 2 : 1>(a, p, lds, stream)
+                                 : launch_attention<T, 6, 8, 1>(a, p, lds, stream);
+  if (nk <= 10 && p.nv <= 16)
+    return launch_attention<T, 10, 16, 1>(a, p, lds, stream);
+  return launch_attention<T, 18, 32, 1>(a, p, lds, stream);
 }
 } // namespace
 
 int launch_latent_attention(const LatentRows &a, hipStream_t stream) {
   const LatentShape &s = a.s;
-  BH_REQUIRE(shape_ok(s) && a.proj && a.cache && a.keys && a.values_t && a.out && a.rows > 0 &&
-                 a.start >= 0 && a.first == latent_first_visible(s, a.start) &&
-                 a.value_ld % kTileKeys == 0 && a.value_ld >= a.start + a.rows - a.first,
+  BH_REQUIRE(shape_ok(s) && a.proj && a.cache && a.queries && a.keys && a.values_t && a.out &&
+                 a.rows > 0 && a.start >= 0 && a.first == latent_first_visible(s, a.start) &&
+                 a.value_ld % kLatentKeyTile == 0 && a.value_ld >= a.start + a.rows - a.first,
              "latent_attention: bad argument");
-  const int esz = s.f32 ? 4 : 2, pad = 16 / esz;
-  LatentAttnArgs p{s.heads, s.dim, s.dim16(), s.rot_dim, s.vdim, s.vdim16(), s.rank, s.row_elems(),
-                   s.window, s.ring_mask, a.ld, a.gate_at, a.rows, a.start, a.first, a.value_ld,
-                   a.out_ld, 0, 0, 0};
-  p.kd = (int)round_up(s.dim16() + s.rot_dim, 32);
-  p.k_stride = p.kd + pad;
-  p.v_stride = kTileKeys + pad;
-  int waves = 4;
-  auto lds_bytes = [&](int w) {
-    return (size_t)esz * ((size_t)(16 * w + kTileKeys) * p.k_stride + (size_t)s.vdim16() * p.v_stride);
-  };
-  while (waves > 1 && (lds_bytes(waves) > kLdsLimit || a.rows <= 16 * (waves / 2)))
-    waves /= 2;
-  const size_t lds = lds_bytes(waves);
-  BH_REQUIRE(lds <= kLdsLimit, "latent_attention: heads of %d + %d values do not fit LDS", p.kd,
-             s.vdim);
-  return s.f32 ? launch_attention_any<float>(a, p, waves, lds, stream)
-               : launch_attention_any<bf16_bits>(a, p, waves, lds, stream);
+  LatentAttnArgs p{s.heads, s.dim16(), s.rot8(), s.vdim, s.vdim16() / 16, s.row_elems(), s.window,
+                   s.ring_mask, a.ld, a.gate_at, a.rows, a.start, a.first, a.value_ld, a.out_ld,
+                   s.key_elems(), 0, 0};
+  return s.f32 ? launch_attention_any<float>(a, p, stream)
+               : launch_attention_any<bf16_bits>(a, p, stream);
 }
 
 } // namespace bh

@@ -57,54 +57,75 @@ linear_step_kernel(const float *__restrict__ q, const float *__restrict__ k,
 
 struct LinearArgs {
   int heads, dim, vdim, ld, q_at, k_at, v_at, rows;
-  int dp; // LDS row of q / k: dim padded to 32, plus 4
+  int dp;     // LDS row of q / k: dim padded to 32, plus 4
+  bool quads; // rows can be moved four floats at a time
   const float *powers;
 };
 
-constexpr int kSliceV = 64, kVRow = kSliceV + 4; // value channels of a workgroup
-
+// Rows 0..kLinearChunk - 1 of src into LDS as [.][stride]; rows past `rows` and columns
+// past `width` (of `padded`, a multiple of 4) as zeros.  With `quads` (width, ld and
+// the address are multiples of four floats) 16 bytes a load, eight in flight.
+template <int THREADS>
 __device__ __forceinline__ void stage_rows(float *dst, int stride, const float *src, int64_t ld,
-                                           int rows, int width, int padded) {
-  for (int i = threadIdx.x; i < kLinearChunk * padded; i += 256) {
-    const int r = i / padded, c = i - r * padded;
-    dst[r * stride + c] = r < rows && c < width ? src[r * ld + c] : 0.f;
+                                           int rows, int total_rows, int width, int padded, bool quads) {
+  const int cols = padded / 4, c = threadIdx.x % cols * 4, per = THREADS / cols;
+  int r = threadIdx.x / cols;
+  if (r >= per)
+    return;
+  if (quads) {
+#pragma unroll 8
+    for (; r < total_rows; r += per) {
+      f32x4 v{0.f, 0.f, 0.f, 0.f};
+      if (r < rows && c < width)
+        v = *reinterpret_cast<const f32x4 *>(src + r * ld + c);
+      *reinterpret_cast<f32x4 *>(dst + r * stride + c) = v;
+    }
+  } else {
+    for (; r < total_rows; r += per) {
+      f32x4 v;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        v[j] = r < rows && c + j < width ? src[r * ld + c + j] : 0.f;
+      *reinterpret_cast<f32x4 *>(dst + r * stride + c) = v;
+    }
   }
 }
 
-// Grid (chunks, heads, value slices): sum over the chunk's tokens of
+// Grid (chunks, heads, value slices of SV channels): sum over the chunk's tokens of
 // decay^(last - i) k_i v_i^T.
-__global__ void __launch_bounds__(256)
+template <int SV>
+__global__ void __launch_bounds__(SV * 4)
 linear_chunk_kernel(const float *__restrict__ proj, float *__restrict__ chunk_states, LinearArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
+  __shared__ float pw[kLinearChunk];
+  constexpr int kThreads = SV * 4, kWaves = kThreads / 64, kVRow = SV + 4;
   const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kSliceV;
+  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * SV;
   const int rows = min(kLinearChunk, a.rows - c * kLinearChunk);
-  const int vw = min(kSliceV, a.vdim - v0);
+  const int vw = min(SV, a.vdim - v0);
   float *k = lds, *v = lds + kLinearChunk * a.dp;
   const float *src = proj + (int64_t)c * kLinearChunk * a.ld;
-  const float *pw = a.powers + h * (kLinearChunk + 1);
-  stage_rows(k, a.dp, src + a.k_at + h * a.dim, a.ld, rows, a.dim, a.dp - 4);
-  for (int i = threadIdx.x; i < kLinearChunk * kSliceV; i += 256) {
-    const int r = i / kSliceV, x = i - r * kSliceV;
-    v[r * kVRow + x] =
-        r < rows && x < vw ? src[(int64_t)r * a.ld + a.v_at + h * a.vdim + v0 + x] * pw[rows - 1 - r] : 0.f;
-  }
+  stage_rows<kThreads>(k, a.dp, src + a.k_at + h * a.dim, a.ld, rows, kLinearChunk, a.dim, a.dp - 4, a.quads);
+  stage_rows<kThreads>(v, kVRow, src + a.v_at + h * a.vdim + v0, a.ld, rows, kLinearChunk, vw, SV, a.quads);
+  if (threadIdx.x < kLinearChunk) // of a token: what is left of it at the chunk's end
+    pw[threadIdx.x] = threadIdx.x < rows ? a.powers[h * (kLinearChunk + 1) + rows - 1 - threadIdx.x] : 0.f;
   __syncthreads();
   float *dst = chunk_states + ((int64_t)c * a.heads + h) * a.dim * a.vdim;
-  for (int dt = wave; dt * 16 < a.dim; dt += 4) {
-    f32x4 acc[kSliceV / 16];
+  for (int dt = wave; dt * 16 < a.dim; dt += kWaves) {
+    f32x4 acc[SV / 16];
 #pragma unroll
-    for (int t = 0; t < kSliceV / 16; ++t)
+    for (int t = 0; t < SV / 16; ++t)
       acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
     for (int s = 0; s < kLinearChunk / 4; ++s) {
-      const float ka = k[(s * 4 + quad) * a.dp + dt * 16 + col];
+      const float ka = k[(s * 4 + quad) * a.dp + dt * 16 + col] * pw[s * 4 + quad];
 #pragma unroll
-      for (int t = 0; t < kSliceV / 16; ++t)
+      for (int t = 0; t < SV / 16; ++t)
         acc[t] = mfma_f32(ka, v[(s * 4 + quad) * kVRow + t * 16 + col], acc[t]);
     }
 #pragma unroll
-    for (int t = 0; t < kSliceV / 16; ++t)
+    for (int t = 0; t < SV / 16; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int d = dt * 16 + quad * 4 + r, x = t * 16 + col;
@@ -141,48 +162,49 @@ linear_scan_kernel(float *__restrict__ chunk_states, float *__restrict__ state, 
   state[i] = s;
 }
 
-// Grid (chunks, heads, value slices): o_i = decay^(i+1) S^T q_i + sum over j <= i of
-// decay^(i-j) (q_i . k_j) v_j.
-__global__ void __launch_bounds__(256)
+// Grid (chunks, heads, value slices of SV channels): o_i = decay^(i+1) S^T q_i + sum
+// over j <= i of decay^(i-j) (q_i . k_j) v_j.  A wavefront owns 16 queries and 64 value
+// channels.  The state takes the place of the chunk's keys and values in LDS once
+// those have been used; its loads are in flight meanwhile.
+template <int SV>
+__global__ void __launch_bounds__(SV * 4)
 linear_out_kernel(const float *__restrict__ proj, const float *__restrict__ chunk_states,
                   float *__restrict__ out, LinearArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float pw[kLinearChunk + 1];
-  const int lane = threadIdx.x & 63, col = lane & 15, quad = lane >> 4;
-  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * kSliceV;
+  constexpr int kThreads = SV * 4, kVRow = SV + 4, NV = 4, kStateLoads = 8;
+  const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int qt = wave & 3, vt0 = wave >> 2 << 6; // query tile, first value channel
+  const int c = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * SV;
   const int rows = min(kLinearChunk, a.rows - c * kLinearChunk);
-  const int vw = min(kSliceV, a.vdim - v0);
-  float *q = lds, *k = q + kLinearChunk * a.dp, *v = k + kLinearChunk * a.dp;
+  const int vw = min(SV, a.vdim - v0);
+  float *q = lds, *k = q + kLinearChunk * a.dp, *v = k + kLinearChunk * a.dp, *st = k;
   const float *src = proj + (int64_t)c * kLinearChunk * a.ld;
-  stage_rows(q, a.dp, src + a.q_at + h * a.dim, a.ld, rows, a.dim, a.dp - 4);
-  stage_rows(k, a.dp, src + a.k_at + h * a.dim, a.ld, rows, a.dim, a.dp - 4);
-  stage_rows(v, kVRow, src + a.v_at + h * a.vdim + v0, a.ld, rows, vw, kSliceV);
-  if (threadIdx.x <= kLinearChunk)
-    pw[threadIdx.x] = a.powers[h * (kLinearChunk + 1) + threadIdx.x];
+  const float *S = chunk_states + ((int64_t)c * a.heads + h) * a.dim * a.vdim + v0;
+  stage_rows<kThreads>(q, a.dp, src + a.q_at + h * a.dim, a.ld, rows, kLinearChunk, a.dim, a.dp - 4, a.quads);
+  stage_rows<kThreads>(k, a.dp, src + a.k_at + h * a.dim, a.ld, rows, kLinearChunk, a.dim, a.dp - 4, a.quads);
+  stage_rows<kThreads>(v, kVRow, src + a.v_at + h * a.vdim + v0, a.ld, rows, kLinearChunk, vw, SV, a.quads);
+  if (tid <= kLinearChunk)
+    pw[tid] = a.powers[h * (kLinearChunk + 1) + tid];
+  // the first rows of the state: SV / 4 threads a row, 16 rows a pass
+  const int sc = tid % (SV / 4) * 4, sr = tid / (SV / 4);
+  f32x4 ahead[kStateLoads];
+  if (a.quads) {
+#pragma unroll
+    for (int i = 0; i < kStateLoads; ++i)
+      ahead[i] = *reinterpret_cast<const f32x4 *>(S + (int64_t)min(sr + i * 16, a.dim - 1) * a.vdim +
+                                                  (sc < vw ? sc : 0));
+  }
   __syncthreads();
-  if (wave * 16 >= rows)
-    return;
-  const int qi = wave * 16 + col; // this lane's query within the chunk
-  constexpr int NV = kSliceV / 16;
+  const int qi = qt * 16 + col; // this lane's query within the chunk
   f32x4 o[NV];
 #pragma unroll
   for (int t = 0; t < NV; ++t)
     o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-  // state part: A = S^T (value channels x key dimensions), B = the scaled queries
-  const float *S = chunk_states + ((int64_t)c * a.heads + h) * a.dim * a.vdim + v0;
-  const float lead = pw[qi + 1];
-  for (int d0 = 0; d0 < a.dim; d0 += 4) {
-    const int d = min(d0 + quad, a.dim - 1);
-    const float qb = d0 + quad < a.dim ? q[qi * a.dp + d] * lead : 0.f;
-#pragma unroll
-    for (int t = 0; t < NV; ++t) {
-      const int x = min(t * 16 + col, vw - 1);
-      o[t] = mfma_f32(S[(int64_t)d * a.vdim + x], qb, o[t]);
-    }
-  }
+  const bool busy = qt * 16 < rows;
   // tokens of the chunk up to the query
-  for (int kt = 0; kt <= wave; ++kt) {
+  for (int kt = 0; busy && kt <= qt; ++kt) {
     f32x4 s{0.f, 0.f, 0.f, 0.f};
     const float *kr = k + (kt * 16 + col) * a.dp + quad * 8, *qr = q + qi * a.dp + quad * 8;
     for (int t = 0; t < a.dp - 4; t += 32) {
@@ -200,19 +222,77 @@ linear_out_kernel(const float *__restrict__ proj, const float *__restrict__ chun
     for (int t = 0; t < NV; ++t)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        o[t] = mfma_f32(v[(kt * 16 + quad * 4 + r) * kVRow + t * 16 + col], s[r], o[t]);
+        o[t] = mfma_f32(v[(kt * 16 + quad * 4 + r) * kVRow + vt0 + t * 16 + col], s[r], o[t]);
+  }
+  __syncthreads();
+  if (a.quads) {
+#pragma unroll
+    for (int i = 0; i < kStateLoads; ++i)
+      if (sr + i * 16 < a.dim)
+        *reinterpret_cast<f32x4 *>(st + (sr + i * 16) * kVRow + sc) = ahead[i];
+    for (int r = sr + kStateLoads * 16; r < a.dim; r += 16)
+      *reinterpret_cast<f32x4 *>(st + r * kVRow + sc) =
+          *reinterpret_cast<const f32x4 *>(S + (int64_t)r * a.vdim + (sc < vw ? sc : 0));
+  } else {
+    for (int r = sr; r < a.dim; r += 16)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        st[r * kVRow + sc + j] = sc + j < vw ? S[(int64_t)r * a.vdim + sc + j] : 0.f;
+  }
+  __syncthreads();
+  if (!busy)
+    return;
+  // state part: A = S^T (value channels x key dimensions), B = the scaled queries
+  const float lead = pw[qi + 1];
+#pragma unroll 4
+  for (int d0 = 0; d0 < a.dim; d0 += 4) {
+    const int d = min(d0 + quad, a.dim - 1);
+    const float qb = d0 + quad < a.dim ? q[qi * a.dp + d] * lead : 0.f;
+#pragma unroll
+    for (int t = 0; t < NV; ++t)
+      o[t] = mfma_f32(st[d * kVRow + vt0 + t * 16 + col], qb, o[t]);
   }
   if (qi >= rows)
     return;
   float *dst = out + ((int64_t)c * kLinearChunk + qi) * a.heads * a.vdim + (int64_t)h * a.vdim + v0;
 #pragma unroll
-  for (int t = 0; t < NV; ++t)
+  for (int t = 0; t < NV; ++t) {
+    const int x = vt0 + t * 16 + quad * 4;
+    if (a.quads && x < vw) {
+      *reinterpret_cast<f32x4 *>(dst + x) = o[t];
+    } else {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int x = t * 16 + quad * 4 + r;
-      if (x < vw)
-        dst[x] = o[t][r];
+      for (int r = 0; r < 4; ++r)
+        if (x + r < vw)
+          dst[x + r] = o[t][r];
     }
+  }
+}
+
+template <int SV>
+size_t out_lds_bytes(const LinearArgs &p) {
+  // q, then keys and values or the state
+  const size_t own = (size_t)kLinearChunk * (p.dp + SV + 4), state = (size_t)p.dim * (SV + 4);
+  return sizeof(float) * ((size_t)kLinearChunk * p.dp + std::max(own, state));
+}
+constexpr size_t kLinearLds = 156 * 1024;
+
+template <int SV> int launch_rows(const LinearRows &a, const LinearArgs &p, hipStream_t stream) {
+  const LinearShape &s = a.s;
+  const size_t chunk_lds = sizeof(float) * kLinearChunk * ((size_t)p.dp + SV + 4);
+  static DynLdsOnce once_chunk, once_out;
+  BH_CHECK_HIP(ensure_dyn_lds(once_chunk, (const void *)linear_chunk_kernel<SV>, (int)kLinearLds));
+  BH_CHECK_HIP(ensure_dyn_lds(once_out, (const void *)linear_out_kernel<SV>, (int)kLinearLds));
+  const dim3 grid((unsigned)linear_chunks(a.rows), (unsigned)s.heads, (unsigned)ceil_div(s.vdim, SV));
+  hipLaunchKernelGGL(linear_chunk_kernel<SV>, grid, dim3(SV * 4), chunk_lds, stream, a.proj,
+                     a.chunk_states, p);
+  const int64_t total = (int64_t)s.heads * s.dim * s.vdim;
+  hipLaunchKernelGGL(linear_scan_kernel, dim3((unsigned)ceil_div(total, 256)), dim3(256), 0, stream,
+                     a.chunk_states, a.state, s.dim * s.vdim, total, a.rows, a.powers);
+  hipLaunchKernelGGL(linear_out_kernel<SV>, grid, dim3(SV * 4), out_lds_bytes<SV>(p), stream, a.proj,
+                     a.chunk_states, a.out, p);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
 }
 
 } // namespace
@@ -233,26 +313,16 @@ int launch_linear_rows(const LinearRows &a, hipStream_t stream) {
   BH_REQUIRE(a.proj && a.powers && a.state && a.chunk_states && a.out && a.rows > 0 && s.heads > 0 &&
                  s.dim > 0 && s.vdim > 0,
              "linear_rows: bad argument");
-  LinearArgs p{s.heads, s.dim, s.vdim, a.ld, a.q_at, a.k_at, a.v_at, a.rows, 0, a.powers};
+  LinearArgs p{s.heads, s.dim, s.vdim, a.ld, a.q_at, a.k_at, a.v_at, a.rows, 0, false, a.powers};
   p.dp = (int)round_up(s.dim, 32) + 4;
-  const size_t out_lds = sizeof(float) * kLinearChunk * (2 * (size_t)p.dp + kVRow);
-  constexpr size_t kLimit = 156 * 1024;
-  BH_REQUIRE(out_lds <= kLimit, "linear_rows: key heads of %d values do not fit LDS", s.dim);
-  const size_t chunk_lds = sizeof(float) * kLinearChunk * ((size_t)p.dp + kVRow);
-  static DynLdsOnce once_chunk, once_out;
-  BH_CHECK_HIP(ensure_dyn_lds(once_chunk, (const void *)linear_chunk_kernel, (int)kLimit));
-  BH_CHECK_HIP(ensure_dyn_lds(once_out, (const void *)linear_out_kernel, (int)kLimit));
-  const dim3 grid((unsigned)linear_chunks(a.rows), (unsigned)s.heads,
-                  (unsigned)ceil_div(s.vdim, kSliceV));
-  hipLaunchKernelGGL(linear_chunk_kernel, grid, dim3(256), chunk_lds, stream, a.proj,
-                     a.chunk_states, p);
-  const int64_t total = (int64_t)s.heads * s.dim * s.vdim;
-  hipLaunchKernelGGL(linear_scan_kernel, dim3((unsigned)ceil_div(total, 256)), dim3(256), 0, stream,
-                     a.chunk_states, a.state, s.dim * s.vdim, total, a.rows, a.powers);
-  hipLaunchKernelGGL(linear_out_kernel, grid, dim3(256), out_lds, stream, a.proj, a.chunk_states,
-                     a.out, p);
-  BH_CHECK_HIP(hipGetLastError());
-  return BUDDY_HIP_OK;
+  p.quads = s.dim % 4 == 0 && s.vdim % 4 == 0 && a.ld % 4 == 0 && a.q_at % 4 == 0 &&
+            a.k_at % 4 == 0 && a.v_at % 4 == 0 && ((uintptr_t)a.proj & 15) == 0 &&
+            ((uintptr_t)a.chunk_states & 15) == 0 && ((uintptr_t)a.out & 15) == 0;
+  if (s.vdim > 64 && out_lds_bytes<128>(p) <= kLinearLds)
+    return launch_rows<128>(a, p, stream);
+  BH_REQUIRE(out_lds_bytes<64>(p) <= kLinearLds, "linear_rows: key heads of %d values do not fit LDS",
+             s.dim);
+  return launch_rows<64>(a, p, stream);
 }
 
 } // namespace bh

@@ -31,17 +31,19 @@ struct NormRows {
 int launch_norm_rows(const NormRows &a, hipStream_t stream);
 
 // out[r] = h[r] + causal convolution over time per channel; rows before the first
-// come from the ring ([taps][width], position p in slot p % taps).
+// come from the ring ([taps][width], position p in slot p % taps).  Afterwards the
+// ring holds the last rows, and conv_next ([2][width], position p in slot p % 2) what
+// they add at the position that follows.
 struct ConvRows {
   const float *h = nullptr; // [rows][width]
   const float *w = nullptr; // [taps][width]
-  float *ring = nullptr;
+  float *ring = nullptr, *next = nullptr;
   int taps = 0, width = 0, rows = 0, start = 0;
   void *out = nullptr;
   int ld = 0;
   bool act_f32 = false;
 };
-int launch_conv_rows(const ConvRows &a, hipStream_t stream); // and saves the last rows in the ring
+int launch_conv_rows(const ConvRows &a, hipStream_t stream); 
 
 // out[r] = (x[r] / rms(x[r])) * w * sigmoid(gate[r])
 struct GatedNormRows {

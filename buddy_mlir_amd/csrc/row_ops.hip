@@ -89,14 +89,25 @@ template <typename T> __global__ void __launch_bounds__(256) conv_rows_kernel(Co
   }
 }
 
-// the last min(rows, taps) rows into their slots
-__global__ void __launch_bounds__(256)
-conv_save_kernel(const float *__restrict__ h, float *__restrict__ ring, int taps, int width, int rows,
-                 int start) {
-  const int r = rows - 1 - (int)blockIdx.x;
-  const int slot = (start + r) % taps;
-  for (int i = threadIdx.x; i < width; i += 256)
-    ring[(int64_t)slot * width + i] = h[(int64_t)r * width + i];
+// one thread per channel: the last rows into their slots, and what the ring adds next
+__global__ void __launch_bounds__(64)
+conv_save_kernel(const float *__restrict__ h, const float *__restrict__ w, float *__restrict__ ring,
+                 float *__restrict__ next, int taps, int width, int rows, int start) {
+  const int i = blockIdx.x * 64 + threadIdx.x;
+  if (i >= width)
+    return;
+  const int end = start + rows;
+  float c = 0.f;
+  for (int b = taps - 1; b >= 1; --b) {
+    if (end - b < 0)
+      continue;
+    const float e = rows >= b ? h[(int64_t)(rows - b) * width + i]
+                              : ring[(int64_t)((end - b) % taps) * width + i];
+    c = fmaf(w[(int64_t)(taps - 1 - b) * width + i], e, c);
+    if (rows >= b)
+      ring[(int64_t)((end - b) % taps) * width + i] = e;
+  }
+  next[(int64_t)(end & 1) * width + i] = c;
 }
 
 template <typename T> __global__ void __launch_bounds__(256) gated_norm_rows_kernel(GatedNormRows a) {
@@ -228,14 +239,14 @@ int launch_norm_rows(const NormRows &a, hipStream_t stream) {
 }
 
 int launch_conv_rows(const ConvRows &a, hipStream_t stream) {
-  BH_REQUIRE(a.h && a.w && a.ring && a.out && a.taps > 0 && a.width > 0 && a.rows > 0 && a.start >= 0,
+  BH_REQUIRE(a.h && a.w && a.ring && a.next && a.out && a.taps > 0 && a.width > 0 && a.rows > 0 && a.start >= 0,
              "conv_rows: bad argument");
   if (a.act_f32)
     hipLaunchKernelGGL(conv_rows_kernel<float>, dim3(a.rows), dim3(256), 0, stream, a);
   else
     hipLaunchKernelGGL(conv_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), 0, stream, a);
-  hipLaunchKernelGGL(conv_save_kernel, dim3(std::min(a.rows, a.taps)), dim3(256), 0, stream, a.h,
-                     a.ring, a.taps, a.width, a.rows, a.start);
+  hipLaunchKernelGGL(conv_save_kernel, dim3((unsigned)ceil_div(a.width, 64)), dim3(64), 0, stream,
+                     a.h, a.w, a.ring, a.next, a.taps, a.width, a.rows, a.start);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }

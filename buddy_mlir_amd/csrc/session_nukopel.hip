@@ -132,6 +132,7 @@ struct Part {
 struct NukopelLayer {
   float norm1 = 0.f, norm1b = 0.f, norm2 = 0.f, norm2b = 0.f;
   float *conv_w = nullptr, *conv_ring = nullptr; // [taps][width] each
+  float *conv_next = nullptr;                    // [2][width]
   Bf16Matrix in;                                 // q | dkv | g, or q | k | v | g
   Part q, k, v, dkv, g;
   int silu_channels = 0;
@@ -183,7 +184,7 @@ struct NukopelSession : Session {
   float *pf_x = nullptr, *pf_y = nullptr, *pf_h = nullptr, *pf_proj = nullptr, *pf_lin = nullptr,
         *pf_states = nullptr, *pf_router = nullptr, *pf_weights = nullptr, *pf_experts = nullptr,
         *pf_logits = nullptr;
-  void *pf_act = nullptr, *pf_mix = nullptr, *pf_keys = nullptr, *pf_values = nullptr,
+  void *pf_act = nullptr, *pf_mix = nullptr, *pf_keys = nullptr, *pf_values = nullptr, *pf_queries = nullptr,
        *pf_moe = nullptr, *pf_shared = nullptr;
   int ld_act = 0, ld_mix = 0, max_proj = 0;
   static constexpr int kLogitRows = 256; // rows of the head multiplied at once
@@ -384,6 +385,7 @@ struct NukopelSession : Session {
             t[(size_t)j * W + ch] = w[(size_t)ch * cfg.taps + j];
         L.conv_w = device_copy(t);
         L.conv_ring = device_zeros<float>((size_t)cfg.taps * W);
+        L.conv_next = device_zeros<float>((size_t)2 * W);
       }
       load_mixer(f, p, c, L);
       mix_max = std::max(mix_max, c.heads * c.vdim);
@@ -494,6 +496,7 @@ struct NukopelSession : Session {
         RowGemv g = norm_gemv(L.in, L.norm1, proj);
         g.conv_w = L.conv_w;
         g.conv_ring = L.conv_ring;
+        g.conv_next = L.conv_next;
         g.taps = cfg.taps;
         g.pos = state + 1;
         g.silu_channels = L.silu_channels;
@@ -594,7 +597,7 @@ struct NukopelSession : Session {
     return BUDDY_HIP_OK;
   }
   static int key_cap(const LatentShape &s, int rows) {
-    return (int)round_up((int64_t)std::min(s.window - 1, s.ring_mask + 1) + rows, 32);
+    return (int)round_up((int64_t)std::min(s.window - 1, s.ring_mask + 1) + rows, kLatentKeyTile);
   }
   int ensure_block(int rows) {
     if (rows <= pf_rows)
@@ -602,7 +605,7 @@ struct NukopelSession : Session {
     BH_CHECK_HIP(hipStreamSynchronize(stream));
     free_block();
     const size_t n = (size_t)rows, T = opt.f32 ? 4 : 2;
-    size_t keys = 0, values = 0, lin = 0, states = 0, e16 = 0, top = 0, experts = 0, moe = 0, shared = 0;
+    size_t keys = 0, values = 0, queries = 0, lin = 0, states = 0, e16 = 0, top = 0, experts = 0, moe = 0, shared = 0;
     for (size_t i = 0; i < layers.size(); ++i) {
       const NukopelLayer &L = layers[i];
       const LayerConfig &c = cfg.layers[i];
@@ -610,6 +613,7 @@ struct NukopelSession : Session {
         const size_t cap = (size_t)key_cap(L.lat, rows);
         keys = std::max(keys, cap * L.uk.N);
         values = std::max(values, cap * L.uv.N);
+        queries = std::max(queries, n * c.heads * L.lat.key_elems());
       } else {
         lin = std::max(lin, n * c.heads * c.vdim);
         states = std::max(states, (size_t)linear_chunks(rows) * c.heads * c.dim * c.vdim);
@@ -631,6 +635,7 @@ struct NukopelSession : Session {
     rc |= block_alloc(&pf_mix, T * n * ld_mix);
     rc |= block_alloc(&pf_keys, T * keys);
     rc |= block_alloc(&pf_values, T * values);
+    rc |= block_alloc(&pf_queries, T * queries);
     rc |= block_alloc(&pf_lin, 4 * lin);
     rc |= block_alloc(&pf_states, 4 * states);
     rc |= block_alloc(&pf_router, 4 * n * e16);
@@ -678,14 +683,16 @@ struct NukopelSession : Session {
     r.cache = L.cache;
     r.first = latent_first_visible(L.lat, start);
     const int keys = start + n - r.first;
+    r.queries = pf_queries;
     r.keys = pf_keys;
     r.values_t = pf_values;
-    r.value_ld = (int)round_up(keys, 32);
+    r.value_ld = (int)round_up(keys, kLatentKeyTile);
     r.out = pf_mix;
     r.out_ld = ld_mix;
     if ((rc = launch_latent_rows(r, stream)))
       return rc;
-    RowsGemm k = gemm(L.uk, L.cache, L.lat.row_elems(), keys, kOutAct, pf_keys, L.uk.N);
+    const char *latents = static_cast<const char *>(L.cache) + L.lat.rot8() * (opt.f32 ? 4 : 2);
+    RowsGemm k = gemm(L.uk, latents, L.lat.row_elems(), keys, kOutAct, pf_keys, L.uk.N);
     k.ring_base = r.first & L.lat.ring_mask;
     k.ring_mask = L.lat.ring_mask;
     if ((rc = launch_rows_gemm(k, stream)))
@@ -808,6 +815,7 @@ struct NukopelSession : Session {
       cv.h = pf_h;
       cv.w = L.conv_w;
       cv.ring = L.conv_ring;
+      cv.next = L.conv_next;
       cv.taps = cfg.taps;
       cv.width = cfg.width;
       cv.rows = n;

@@ -103,3 +103,83 @@ def build_session(shape: Shape, context: int, keep_host: bool = False,
 def first_tokens(shape: Shape, n: int, seed: int = SEED + 9999) -> np.ndarray:
     rng = np.random.default_rng(seed)
     return rng.integers(0, shape.vocab, n).astype(np.int64)
+
+
+# ---- Nukopel ---------------------------------------------------------------------
+
+def nukopel_config(width: int, layers: str, heads: int, *, dim: int = 128, rot_dim: int = 64,
+                   kv_rank: int = 512, window: int = 1024, experts: int = 16, top: int = 4,
+                   ff: int = 1792, vocab: int = 32768, taps: int = 4) -> dict:
+    """A configuration of the layers of a real model; `layers`: a letter per layer, a =
+    latent attention, l = lightning."""
+    mlp = {"kind": "moe", "router": {"experts": experts, "top": top},
+           "expert": {"ff": ff, "limit": 7.0}, "shared": {"ff": ff, "limit": 7.0}}
+    latent = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": dim, "kv_rank": kv_rank,
+              "mask": {"size": window}, "rot": {"base": 1e6, "dims": rot_dim},
+              "scale": (dim + rot_dim) ** -0.5}
+    linear = {"heads": heads, "dim": dim, "vdim": dim,
+              "decay": [1.0 - 2.0 ** -(3 + 5.0 * h / heads) for h in range(heads)]}
+    return {"architecture": "Nukopel", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": width ** 0.5}, "canon": {"taps": taps},
+            "layers": [{"type": "latent_attention" if c == "a" else "lightning",
+                        "mixer": latent if c == "a" else linear, "mlp": mlp} for c in layers]}
+
+
+def nukopel_shapes(cfg: dict):
+    """(name, shape, standard deviation) of every tensor; None: a gain of one."""
+    W, V = cfg["width"], cfg["vocab"]
+    yield "embed", (V, W), W ** -0.5
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        H, D, VD = m["heads"], m["dim"], m["vdim"]
+        for n in ("norm1", "norm1b", "norm2", "norm2b"):
+            yield p + n, (), None
+        yield p + "canon1", (W, cfg["canon"]["taps"]), 0.3
+        if layer["type"] == "latent_attention":
+            R, L = m["rot_dim"], m["kv_rank"]
+            mats = {"q": (H * (D + R), W), "dkv": (L + R, W), "uk": (H * D, L), "uv": (H * VD, L),
+                    "g": (H, W), "o": (W, H * VD)}
+            yield p + "mix.dkv.norm", (L,), None
+        else:
+            mats = {"q": (H * D, W), "k": (H * D, W), "v": (H * VD, W), "g": (H * VD, W),
+                    "o": (W, H * VD)}
+            yield p + "mix.norm", (H * VD,), None
+        for n, s in mats.items():
+            yield p + "mix." + n, s, s[1] ** -0.5
+        yield p + "mlp.router", (f["router"]["experts"], W), W ** -0.5
+        names = [(f"e{e}", f["expert"]["ff"]) for e in range(f["router"]["experts"])]
+        for n, ff in names + [("shared", f["shared"]["ff"])]:
+            yield f"{p}mlp.{n}.gate", (ff, W), W ** -0.5
+            yield f"{p}mlp.{n}.up", (ff, W), W ** -0.5
+            yield f"{p}mlp.{n}.down", (W, ff), ff ** -0.5
+    yield "final.norm", (), None
+    yield "head", (V, W), W ** -0.5
+
+
+def write_nukopel_folder(folder, cfg: dict, seed: int = SEED):
+    """config.json and model.safetensors with random weights in bfloat16."""
+    import json
+    import struct
+    from math import prod
+    from pathlib import Path
+
+    folder = Path(folder)
+    folder.mkdir(parents=True, exist_ok=True)
+    (folder / "config.json").write_text(json.dumps(cfg))
+    tensors, head, at = list(nukopel_shapes(cfg)), {}, 0
+    for name, shape, _ in tensors:
+        size = 2 * prod(shape)
+        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + size]}
+        at += size
+    text = json.dumps(head).encode()
+    text += b" " * (-len(text) % 8)
+    g = _gen(seed)
+    with open(folder / "model.safetensors", "wb") as f:
+        f.write(struct.pack("<Q", len(text)) + text)
+        for _, shape, std in tensors:
+            if std is None:
+                t = torch.ones(shape, dtype=torch.bfloat16)
+            else:
+                t = (torch.randn(shape, generator=g, device="cuda") * std).bfloat16().cpu()
+            f.write(t.reshape(-1).view(torch.int16).numpy().tobytes())
+    return folder
