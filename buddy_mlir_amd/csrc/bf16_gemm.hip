@@ -289,19 +289,24 @@ int launch_shape(const RowsGemm &a, hipStream_t stream) {
   const int64_t rows = GROUPED ? ceil_div(a.list_total, a.experts) : a.rows;
   const int64_t all_blocks = GROUPED ? std::min<int64_t>(a.experts, a.list_total) : 1;
   constexpr int P = OUT == kOutExpertAct ? 2 : 1; // groups come in pairs
-  const int rt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;
-  auto workgroups = [&](int gt) {
-    return ceil_div(a.W.groups(), 4 * gt) * ceil_div(rows, 16 * rt) * all_blocks;
+  auto workgroups = [&](int rt, int gt) {
+    return ceil_div(a.W.groups(), 4 * gt / P) * ceil_div(rows, 16 * rt) * all_blocks;
   };
-  const bool wide = workgroups(2) >= 256;
-  if (rt == 1)
-    return wide ? launch_variant<T, 1, 2 * P, OUT, GROUPED>(a, stream)
-                : launch_variant<T, 1, P, OUT, GROUPED>(a, stream);
-  if (rt == 2)
-    return wide ? launch_variant<T, 2, 2 * P, OUT, GROUPED>(a, stream)
-                : launch_variant<T, 2, P, OUT, GROUPED>(a, stream);
-  return wide ? launch_variant<T, 4, 2 * P, OUT, GROUPED>(a, stream)
-              : launch_variant<T, 4, P, OUT, GROUPED>(a, stream);
+  if (rows <= 16)
+    return workgroups(1, 2 * P) >= 256 ? launch_variant<T, 1, 2 * P, OUT, GROUPED>(a, stream)
+                                       : launch_variant<T, 1, P, OUT, GROUPED>(a, stream);
+  if (rows <= 32)
+    return workgroups(2, 2 * P) >= 256 ? launch_variant<T, 2, 2 * P, OUT, GROUPED>(a, stream)
+                                       : launch_variant<T, 2, P, OUT, GROUPED>(a, stream);
+  // what a workgroup fetches per product shrinks with both sides of its tile
+  if constexpr (sizeof(T) == 2) {
+    // -- but one such workgroup fills a compute unit: whole rounds of 256 pay
+    const int64_t w = workgroups(8, 4);
+    if (rows > 64 && w >= 240 && w * 5 >= round_up(w, 256) * 4)
+      return launch_variant<T, 8, 4, OUT, GROUPED>(a, stream);
+  }
+  return workgroups(4, 2 * P) >= 256 ? launch_variant<T, 4, 2 * P, OUT, GROUPED>(a, stream)
+                                     : launch_variant<T, 4, P, OUT, GROUPED>(a, stream);
 }
 
 template <typename T> int launch_typed(const RowsGemm &a, hipStream_t stream) {

@@ -441,7 +441,7 @@ latent_rows_kernel(const float *__restrict__ proj, T *__restrict__ cache, T *__r
 struct LatentAttnArgs {
   int heads, dim16, rot8, vdim, nv, row_elems, window, ring_mask;
   int ld, gate_at, rows, start, first, value_ld, out_ld;
-  int kd, k_stride, v_stride; // elements of a key; LDS row strides of the K and V^T tiles
+  int kd; // elements of a query
 };
 
 // Keys of a tile: 128 bytes of a V^T row.
@@ -454,9 +454,15 @@ template <typename T> struct KeyTile {
 // meanwhile.  S^T = K . Q^T leaves a lane with keys of one query, which is the B
 // operand of O^T += V^T . P^T as it lies (of 32 keys in bfloat16: a lane's eight are
 // keys 4q .. 4q + 3 of both halves, and V^T rows are stored in that order).
-// NK: 32-element steps of a key, NV: 16-channel groups of a value, at most.
+// NK: 32-element steps of a key, NV: 16-channel groups of a value, at most; smaller
+// heads are padded with zeros (keys) or with rows whose results are not stored
+// (values), so that the loop has no branches.
+//
+// The running maximum a lane subtracts follows the scores only when one exceeds it by
+// more than kSlack: the weights stay below e^kSlack, and the sums are rescaled a few
+// times per query instead of once per tile.
 template <typename T, int NK, int NV, int QT>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, QT == 1 && NV <= 8 ? 2 : 1)
 latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ keys,
                         const T *__restrict__ values_t, const T *__restrict__ cache,
                         const float *__restrict__ proj, T *__restrict__ out, LatentAttnArgs a) {
@@ -468,9 +474,10 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
   const int h = blockIdx.x;
   constexpr int kBlock = 64 * QT;
   const int q0 = (gridDim.y - 1 - blockIdx.y) * kBlock; // long blocks first
-  T *kt = reinterpret_cast<T *>(raw); // [KEYS][k_stride]
-  T *vt = kt + KEYS * a.k_stride;     // [16 * nv][v_stride]
-  const int nk = a.kd / 32;
+  constexpr int kKeyRow = NK * 32 + E, kValueRow = KEYS + E; // rows start 4 banks apart
+  constexpr float kSlack = 8.0f;
+  T *kt = reinterpret_cast<T *>(raw); // [KEYS][kKeyRow]
+  T *vt = kt + KEYS * kKeyRow;        // [16 * NV][kValueRow]
 
   // this lane's queries as key indexes, and their fragments
   int my_q[QT];
@@ -481,8 +488,12 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
     my_q[u] = a.start + r - a.first;
     const T *q = queries + ((int64_t)min(r, a.rows - 1) * a.heads + h) * a.kd + quad * 8;
 #pragma unroll
-    for (int t = 0; t < NK; ++t)
-      qf[u][t].load(q + min(t, nk - 1) * 32);
+    for (int t = 0; t < NK; ++t) {
+      if (t * 32 < a.kd)
+        qf[u][t].load(q + t * 32);
+      else
+        qf[u][t] = Frag<T>{};
+    }
   }
   const int nkeys = a.start + a.rows - a.first;
   const int last_q = min(q0 + kBlock, a.rows) - 1;
@@ -501,7 +512,7 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
     const int id = min(i * 256 + tid, KEYS * runs - 1); // past the end: the last one again
     const int r = id / runs, c = id - r * runs;
     kkey[i] = r;
-    kdst[i] = r * a.k_stride + (c < runs_head ? c * E : a.dim16 + (c - runs_head) * E);
+    kdst[i] = r * kKeyRow + (c < runs_head ? c * E : a.dim16 + (c - runs_head) * E);
     kring[i] = c >= runs_head;
     kstep[i] = c < runs_head ? a.heads * a.dim16 : a.row_elems;
     ksrc[i] = c < runs_head ? keys + h * a.dim16 + c * E : cache + (c - runs_head) * E;
@@ -515,7 +526,7 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
     vsrc[i] = values_t + (int64_t)(h * 16 * a.nv + r) * a.value_ld + c * E;
     vcol[i] = c * E;
     // bfloat16: the run's two halves of four keys go to their places in the lane order
-    vdst[i] = r * a.v_stride + (sizeof(T) == 2 ? (c >> 2) * 32 + (c & 1) * 16 + ((c >> 1) & 1) * 4 : c * E);
+    vdst[i] = r * kValueRow + (sizeof(T) == 2 ? (c >> 2) * 32 + (c & 1) * 16 + ((c >> 1) & 1) * 4 : c * E);
   }
   u32x4 kr[KL], vr[VL];
   auto fetch = [&](int k0, u32x4 (&kr)[KL], u32x4 (&vr)[VL]) {
@@ -530,10 +541,10 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       vr[i] = *reinterpret_cast<const u32x4 *>(vsrc[i] + k0);
   };
   fetch(key_lo, kr, vr);
-  if (runs * E < a.kd) { // the padding of the keys
-    const int pad = a.kd - runs * E, at = a.dim16 + a.rot8;
+  if (runs * E < NK * 32) { // the padding of the keys
+    const int pad = NK * 32 - runs * E, at = a.dim16 + a.rot8;
     for (int i = tid; i < KEYS * pad; i += 256)
-      kt[(i / pad) * a.k_stride + at + i % pad] = 0;
+      kt[(i / pad) * kKeyRow + at + i % pad] = 0;
   }
 
   f32x4 o[QT][NV];
@@ -583,24 +594,30 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
 #pragma unroll
       for (int b = 0; b < SUB; ++b)
         s[u][b] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const T *kp = kt + col * a.k_stride + quad * 8;
+    // the fragments of the next step are read while this one is multiplied
+    const T *kp = kt + col * kKeyRow + quad * 8;
+    Frag<T> kf[2][SUB];
 #pragma unroll
-    for (int t = 0; t < NK; ++t)
-      if (t < nk) {
+    for (int b = 0; b < SUB; ++b)
+      kf[0][b].load(kp + b * 16 * kKeyRow);
 #pragma unroll
-        for (int b = 0; b < SUB; ++b) {
-          Frag<T> kf;
-          kf.load(kp + b * 16 * a.k_stride + t * 32);
+    for (int t = 0; t < NK; ++t) {
+      if (t + 1 < NK) {
 #pragma unroll
-          for (int u = 0; u < QT; ++u)
-            s[u][b] = mfma32(kf, qf[u][t], s[u][b]);
-        }
+        for (int b = 0; b < SUB; ++b)
+          kf[(t + 1) & 1][b].load(kp + b * 16 * kKeyRow + (t + 1) * 32);
       }
+      __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+      for (int b = 0; b < SUB; ++b)
+#pragma unroll
+        for (int u = 0; u < QT; ++u)
+          s[u][b] = mfma32(kf[t & 1][b], qf[u][t], s[u][b]);
+      __builtin_amdgcn_sched_barrier(0);
+    }
     const bool whole = k0 + KEYS - 1 <= wave_q0 && wave_q1 - k0 < a.window;
-    float alpha[QT];
 #pragma unroll
     for (int u = 0; u < QT; ++u) {
-      float mt = m[u];
       if (!whole) {
 #pragma unroll
         for (int b = 0; b < SUB; ++b)
@@ -610,6 +627,7 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
             s[u][b][r] = gap >= 0 && gap < a.window ? s[u][b][r] : -INFINITY;
           }
       }
+      float mt = s[u][0][0];
 #pragma unroll
       for (int b = 0; b < SUB; ++b)
 #pragma unroll
@@ -620,28 +638,26 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       mt = fmaxf(x, y);
       lane_pair<32>(mt, x, y);
       mt = fmaxf(x, y);
-      const float base = mt == -INFINITY ? 0.f : mt; // nothing visible so far
-      alpha[u] = fast_exp(m[u] - base);
-      m[u] = mt;
-      float sum = 0.f;
+      if (__any(mt > m[u] + kSlack)) { // -inf + kSlack stays below every score
+        mt = fmaxf(mt, m[u]);
+        const float alpha = mt == -INFINITY ? 1.f : fast_exp(m[u] - mt);
+        m[u] = mt;
+        l[u] *= alpha;
+#pragma unroll
+        for (int v = 0; v < NV; ++v)
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            o[u][v][r] *= alpha;
+      }
+      const float base = m[u] == -INFINITY ? 0.f : m[u]; // nothing visible so far
 #pragma unroll
       for (int b = 0; b < SUB; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           s[u][b][r] = fast_exp(s[u][b][r] - base);
-          sum += s[u][b][r];
+          l[u] += s[u][b][r];
         }
-      l[u] = fmaf(l[u], alpha[u], sum);
     }
-#pragma unroll
-    for (int u = 0; u < QT; ++u)
-#pragma unroll
-      for (int v = 0; v < NV; ++v)
-        if (v < a.nv) {
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            o[u][v][r] *= alpha[u];
-        }
     if constexpr (sizeof(T) == 2) {
       // the weights as two bfloat16 terms
       uint4 hi[QT][SUB / 2], lo[QT][SUB / 2];
@@ -660,32 +676,48 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
           hi[u][b] = uint4{ph[0], ph[1], ph[2], ph[3]};
           lo[u][b] = uint4{pl[0], pl[1], pl[2], pl[3]};
         }
+      constexpr int G = NV < 4 ? NV : 4; // value tiles read ahead
+      const T *vp = vt + col * kValueRow + quad * 8;
+      Frag<T> vf[2][G][SUB / 2];
 #pragma unroll
-      for (int v = 0; v < NV; ++v)
-        if (v < a.nv) {
+      for (int v = 0; v < G; ++v)
 #pragma unroll
-          for (int b = 0; b < SUB / 2; ++b) {
-            const uint4 vv = *reinterpret_cast<const uint4 *>(vt + (v * 16 + col) * a.v_stride + b * 32 + quad * 8);
+        for (int b = 0; b < SUB / 2; ++b)
+          vf[0][v][b].load(vp + v * 16 * kValueRow + b * 32);
 #pragma unroll
-            for (int u = 0; u < QT; ++u) {
-              o[u][v] = mfma_bf16(vv, hi[u][b], o[u][v]);
-              o[u][v] = mfma_bf16(vv, lo[u][b], o[u][v]);
-            }
-          }
+      for (int v0 = 0; v0 < NV; v0 += G) {
+        if (v0 + G < NV) {
+#pragma unroll
+          for (int v = 0; v < G; ++v)
+#pragma unroll
+            for (int b = 0; b < SUB / 2; ++b)
+              vf[(v0 / G + 1) & 1][v][b].load(vp + (v0 + G + v) * 16 * kValueRow + b * 32);
         }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int b = 0; b < SUB / 2; ++b)
+#pragma unroll
+          for (int u = 0; u < QT; ++u) {
+#pragma unroll
+            for (int v = 0; v < G; ++v)
+              o[u][v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, hi[u][b], o[u][v0 + v]);
+#pragma unroll
+            for (int v = 0; v < G; ++v)
+              o[u][v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, lo[u][b], o[u][v0 + v]);
+          }
+        __builtin_amdgcn_sched_barrier(0);
+      }
     } else {
 #pragma unroll
       for (int v = 0; v < NV; ++v)
-        if (v < a.nv) {
 #pragma unroll
-          for (int b = 0; b < SUB; ++b) {
-            const f32x4 vv = *reinterpret_cast<const f32x4 *>(vt + (v * 16 + col) * a.v_stride + b * 16 + quad * 4);
+        for (int b = 0; b < SUB; ++b) {
+          const f32x4 vv = *reinterpret_cast<const f32x4 *>(vt + (v * 16 + col) * kValueRow + b * 16 + quad * 4);
 #pragma unroll
-            for (int u = 0; u < QT; ++u)
+          for (int u = 0; u < QT; ++u)
 #pragma unroll
-              for (int r = 0; r < 4; ++r)
-                o[u][v] = mfma_f32(vv[r], s[u][b][r], o[u][v]);
-          }
+            for (int r = 0; r < 4; ++r)
+              o[u][v] = mfma_f32(vv[r], s[u][b][r], o[u][v]);
         }
     }
   }
@@ -826,7 +858,10 @@ int launch_latent_rows(const LatentRows &a, hipStream_t stream) {
 
 namespace {
 template <typename T, int NK, int NV, int QT>
-int launch_attention(const LatentRows &a, const LatentAttnArgs &p, size_t lds, hipStream_t stream) {
+int launch_attention(const LatentRows &a, const LatentAttnArgs &p, hipStream_t stream) {
+  constexpr int E = 16 / (int)sizeof(T), KEYS = KeyTile<T>::kKeys;
+  constexpr size_t lds = sizeof(T) * ((size_t)KEYS * (NK * 32 + E) + (size_t)16 * NV * (KEYS + E));
+  static_assert(lds <= kLdsLimit, "the tiles must fit LDS");
   static DynLdsOnce once;
   BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_attention_kernel<T, NK, NV, QT>, (int)kLdsLimit));
   hipLaunchKernelGGL((latent_attention_kernel<T, NK, NV, QT>),
@@ -838,24 +873,24 @@ int launch_attention(const LatentRows &a, const LatentAttnArgs &p, size_t lds, h
   return BUDDY_HIP_OK;
 }
 template <typename T>
-int launch_attention_any(const LatentRows &a, LatentAttnArgs &p, hipStream_t stream) {
-  p.k_stride = p.kd + 16 / (int)sizeof(T); // rows start 4 banks apart
-  p.v_stride = KeyTile<T>::kKeys + 16 / (int)sizeof(T);
-  const size_t lds = sizeof(T) * ((size_t)KeyTile<T>::kKeys * p.k_stride + (size_t)16 * p.nv * p.v_stride);
+int launch_attention_any(const LatentRows &a, const LatentAttnArgs &p, hipStream_t stream) {
   const int nk = p.kd / 32;
-  BH_REQUIRE(lds <= kLdsLimit && nk <= 18 && p.nv <= 32,
-             "latent_attention: heads of %d and %d values", p.kd, a.s.vdim);
+  BH_REQUIRE(nk <= 18 && p.nv <= 32, "latent_attention: heads of %d and %d values", p.kd, a.s.vdim);
   // two query tiles per wavefront halve the LDS reads, where they leave enough workgroups
-  const bool two = ceil_div(a.rows, 128) * a.s.heads >= 192;
+  const bool two = getenv("QT2") && sizeof(T) == 2 && ceil_div(a.rows, 128) * a.s.heads >= 192;
+  if (nk <= 2 && p.nv <= 2)
+    return launch_attention<T, 2, 2, 1>(a, p, stream);
   if (nk <= 4 && p.nv <= 4)
-    return two ? launch_attention<T, 4, 4, 2>(a, p, lds, stream)
-               : launch_attention<T, 4, 4, 1>(a, p, lds, stream);
-  if (nk <= 6 && p.nv <= 8)
-    return two && sizeof(T) == 2 ? launch_attention<T, 6, 8, sizeof(T) == 2 ? 2 : 1>(a, p, lds, stream)
-                                 : launch_attention<T, 6, 8, 1>(a, p, lds, stream);
+    return launch_attention<T, 4, 4, 1>(a, p, stream);
+  if (nk <= 6 && p.nv <= 8) {
+    if constexpr (sizeof(T) == 2)
+      if (two)
+        return launch_attention<T, 6, 8, 2>(a, p, stream);
+    return launch_attention<T, 6, 8, 1>(a, p, stream);
+  }
   if (nk <= 10 && p.nv <= 16)
-    return launch_attention<T, 10, 16, 1>(a, p, lds, stream);
-  return launch_attention<T, 18, 32, 1>(a, p, lds, stream);
+    return launch_attention<T, 10, 16, 1>(a, p, stream);
+  return launch_attention<T, 18, 32, 1>(a, p, stream);
 }
 } // namespace
 
@@ -867,7 +902,7 @@ int launch_latent_attention(const LatentRows &a, hipStream_t stream) {
              "latent_attention: bad argument");
   LatentAttnArgs p{s.heads, s.dim16(), s.rot8(), s.vdim, s.vdim16() / 16, s.row_elems(), s.window,
                    s.ring_mask, a.ld, a.gate_at, a.rows, a.start, a.first, a.value_ld, a.out_ld,
-                   s.key_elems(), 0, 0};
+                   s.key_elems()};
   return s.f32 ? launch_attention_any<float>(a, p, stream)
                : launch_attention_any<bf16_bits>(a, p, stream);
 }

@@ -28,64 +28,120 @@ __device__ __forceinline__ float block_sum4(float v, float *red) {
   return (red[0] + red[1]) + (red[2] + red[3]);
 }
 
-template <typename T>
+// V consecutive values of a row at a time: 4 where every row is 16-byte aligned, else 1
+template <int V> struct Run {
+  float v[V];
+};
+template <int V> __device__ __forceinline__ Run<V> load_run(const float *p) {
+  Run<V> r;
+  if constexpr (V == 4) {
+    const f32x4 x = *reinterpret_cast<const f32x4 *>(p);
+#pragma unroll
+    for (int j = 0; j < V; ++j)
+      r.v[j] = x[j];
+  } else {
+    r.v[0] = *p;
+  }
+  return r;
+}
+template <int V> __device__ __forceinline__ void store_run(float *p, const Run<V> &r) {
+  if constexpr (V == 4)
+    *reinterpret_cast<f32x4 *>(p) = f32x4{r.v[0], r.v[1], r.v[2], r.v[3]};
+  else
+    *p = r.v[0];
+}
+template <int V> __device__ __forceinline__ void store_run(bf16_bits *p, const Run<V> &r) {
+  if constexpr (V == 4)
+    *reinterpret_cast<uint2 *>(p) = uint2{pack_bf(r.v[0], r.v[1]), pack_bf(r.v[2], r.v[3])};
+  else
+    *p = f_bf(r.v[0]);
+}
+
+template <typename T, int V>
 __global__ void __launch_bounds__(256) norm_rows_kernel(NormRows a) {
-  extern __shared__ float lds[]; // x' of the row, then y
+  extern __shared__ __attribute__((aligned(16))) float lds[]; // x' of the row, then y
   __shared__ float red[2][4];
-  const int tid = threadIdx.x, W = a.width;
+  const int tid = threadIdx.x * V, W = a.width;
   const int64_t r = a.pick ? a.pick[blockIdx.x] : blockIdx.x;
   float *x = a.x + r * W;
   float *xb = lds, *yb = lds + W;
+  const bool pending = a.y || a.expert_out;
   float ss = 0.f;
-  for (int i = tid; i < W; i += 256) {
-    xb[i] = x[i];
-    if (a.y || a.expert_out) {
-      float y = a.y ? a.y[r * a.ldy + i] : 0.f;
-      for (int j = 0; j < a.top; ++j)
-        y = fmaf(a.expert_w[r * a.top + j], a.expert_out[(r * a.top + j) * a.lde + i], y);
-      yb[i] = y;
-      ss = fmaf(y, y, ss);
+  for (int i = tid; i < W; i += 256 * V) {
+    store_run<V>(xb + i, load_run<V>(x + i));
+    if (pending) {
+      Run<V> y{};
+      if (a.y)
+        y = load_run<V>(a.y + r * a.ldy + i);
+      for (int j = 0; j < a.top; ++j) {
+        const float w = a.expert_w[r * a.top + j];
+        const Run<V> e = load_run<V>(a.expert_out + (r * a.top + j) * a.lde + i);
+#pragma unroll
+        for (int k = 0; k < V; ++k)
+          y.v[k] = fmaf(w, e.v[k], y.v[k]);
+      }
+      store_run<V>(yb + i, y);
+#pragma unroll
+      for (int k = 0; k < V; ++k)
+        ss = fmaf(y.v[k], y.v[k], ss);
     }
   }
-  if (a.y || a.expert_out) {
+  float sx = 0.f;
+  if (pending) {
     const float ry = a.out_gain / sqrtf(block_sum4(ss, red[0]) / (float)W + a.eps);
-    for (int i = tid; i < W; i += 256) {
-      const float v = fmaf(yb[i], ry, xb[i]);
-      xb[i] = v;
+    for (int i = tid; i < W; i += 256 * V) {
+      Run<V> v = load_run<V>(xb + i);
+      const Run<V> y = load_run<V>(yb + i);
+#pragma unroll
+      for (int k = 0; k < V; ++k)
+        v.v[k] = fmaf(y.v[k], ry, v.v[k]);
+      store_run<V>(xb + i, v);
       if (a.write_x)
-        x[i] = v;
+        store_run<V>(x + i, v);
     }
   }
   if (!a.out_f32 && !a.out_act)
     return;
-  ss = 0.f;
-  for (int i = tid; i < W; i += 256)
-    ss = fmaf(xb[i], xb[i], ss);
-  const float g = a.gain / sqrtf(block_sum4(ss, red[1]) / (float)W + a.eps);
-  for (int i = tid; i < W; i += 256) {
-    const float v = xb[i] * g;
+  for (int i = tid; i < W; i += 256 * V) {
+    const Run<V> v = load_run<V>(xb + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k)
+      sx = fmaf(v.v[k], v.v[k], sx);
+  }
+  const float g = a.gain / sqrtf(block_sum4(sx, red[1]) / (float)W + a.eps);
+  for (int i = tid; i < W; i += 256 * V) {
+    Run<V> v = load_run<V>(xb + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k)
+      v.v[k] *= g;
     if (a.out_f32)
-      a.out_f32[(int64_t)blockIdx.x * W + i] = v;
+      store_run<V>(a.out_f32 + (int64_t)blockIdx.x * W + i, v);
     if (a.out_act)
-      store_act<T>(static_cast<T *>(a.out_act) + (int64_t)blockIdx.x * a.ld_act + i, v);
+      store_run<V>(static_cast<T *>(a.out_act) + (int64_t)blockIdx.x * a.ld_act + i, v);
   }
 }
 
-template <typename T> __global__ void __launch_bounds__(256) conv_rows_kernel(ConvRows a) {
+template <typename T, int V> __global__ void __launch_bounds__(256) conv_rows_kernel(ConvRows a) {
   const int64_t r = blockIdx.x;
   const int p = a.start + (int)r;
-  for (int i = threadIdx.x; i < a.width; i += 256) {
-    const float h = a.h[r * a.width + i];
-    float c = 0.f;
+  for (int i = (blockIdx.y * 256 + threadIdx.x) * V; i < a.width; i += gridDim.y * 256 * V) {
+    const Run<V> h = load_run<V>(a.h + r * a.width + i);
+    Run<V> c{};
     for (int b = a.taps - 1; b >= 1; --b) {
       if (p - b < 0)
         continue;
-      const float e = r >= b ? a.h[(r - b) * a.width + i]
-                             : a.ring[(int64_t)((p - b) % a.taps) * a.width + i];
-      c = fmaf(a.w[(int64_t)(a.taps - 1 - b) * a.width + i], e, c);
+      const Run<V> e = load_run<V>(r >= b ? a.h + (r - b) * a.width + i
+                                          : a.ring + (int64_t)((p - b) % a.taps) * a.width + i);
+      const Run<V> w = load_run<V>(a.w + (int64_t)(a.taps - 1 - b) * a.width + i);
+#pragma unroll
+      for (int k = 0; k < V; ++k)
+        c.v[k] = fmaf(w.v[k], e.v[k], c.v[k]);
     }
-    store_act<T>(static_cast<T *>(a.out) + r * a.ld + i,
-                 h + fmaf(a.w[(int64_t)(a.taps - 1) * a.width + i], h, c));
+    const Run<V> w = load_run<V>(a.w + (int64_t)(a.taps - 1) * a.width + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k)
+      c.v[k] = h.v[k] + fmaf(w.v[k], h.v[k], c.v[k]);
+    store_run<V>(static_cast<T *>(a.out) + r * a.ld + i, c);
   }
 }
 
@@ -226,14 +282,28 @@ int launch_norm_rows(const NormRows &a, hipStream_t stream) {
   const size_t lds = 2 * sizeof(float) * (size_t)a.width;
   constexpr size_t kLimit = 150 * 1024;
   BH_REQUIRE(lds <= kLimit, "norm_rows: a row of %d values does not fit LDS", a.width);
-  static DynLdsOnce once_f, once_b;
+  bool quads = a.width % 4 == 0 && a.ldy % 4 == 0 && a.lde % 4 == 0 && a.ld_act % 4 == 0;
+  for (const void *p : {(const void *)a.x, (const void *)a.y, (const void *)a.expert_out,
+                        (const void *)a.out_f32, (const void *)a.out_act})
+    quads = quads && ((uintptr_t)p & 15) == 0;
+#define BH_NORM(T, V)                                                                          \
+  do {                                                                                         \
+    static DynLdsOnce once;                                                                    \
+    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)norm_rows_kernel<T, V>, (int)kLimit));     \
+    hipLaunchKernelGGL((norm_rows_kernel<T, V>), dim3(a.rows), dim3(256), lds, stream, a);     \
+  } while (0)
   if (a.act_f32) {
-    BH_CHECK_HIP(ensure_dyn_lds(once_f, (const void *)norm_rows_kernel<float>, (int)kLimit));
-    hipLaunchKernelGGL(norm_rows_kernel<float>, dim3(a.rows), dim3(256), lds, stream, a);
+    if (quads)
+      BH_NORM(float, 4);
+    else
+      BH_NORM(float, 1);
   } else {
-    BH_CHECK_HIP(ensure_dyn_lds(once_b, (const void *)norm_rows_kernel<bf16_bits>, (int)kLimit));
-    hipLaunchKernelGGL(norm_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), lds, stream, a);
+    if (quads)
+      BH_NORM(bf16_bits, 4);
+    else
+      BH_NORM(bf16_bits, 1);
   }
+#undef BH_NORM
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }
@@ -241,10 +311,17 @@ int launch_norm_rows(const NormRows &a, hipStream_t stream) {
 int launch_conv_rows(const ConvRows &a, hipStream_t stream) {
   BH_REQUIRE(a.h && a.w && a.ring && a.next && a.out && a.taps > 0 && a.width > 0 && a.rows > 0 && a.start >= 0,
              "conv_rows: bad argument");
-  if (a.act_f32)
-    hipLaunchKernelGGL(conv_rows_kernel<float>, dim3(a.rows), dim3(256), 0, stream, a);
+  const bool quads = a.width % 4 == 0 && a.ld % 4 == 0 &&
+                     (((uintptr_t)a.h | (uintptr_t)a.w | (uintptr_t)a.ring | (uintptr_t)a.out) & 15) == 0;
+  const dim3 grid((unsigned)a.rows, (unsigned)std::min<int64_t>(4, ceil_div(a.width, quads ? 1024 : 256)));
+  if (a.act_f32 && quads)
+    hipLaunchKernelGGL((conv_rows_kernel<float, 4>), grid, dim3(256), 0, stream, a);
+  else if (a.act_f32)
+    hipLaunchKernelGGL((conv_rows_kernel<float, 1>), grid, dim3(256), 0, stream, a);
+  else if (quads)
+    hipLaunchKernelGGL((conv_rows_kernel<bf16_bits, 4>), grid, dim3(256), 0, stream, a);
   else
-    hipLaunchKernelGGL(conv_rows_kernel<bf16_bits>, dim3(a.rows), dim3(256), 0, stream, a);
+    hipLaunchKernelGGL((conv_rows_kernel<bf16_bits, 1>), grid, dim3(256), 0, stream, a);
   hipLaunchKernelGGL(conv_save_kernel, dim3((unsigned)ceil_div(a.width, 64)), dim3(64), 0, stream,
                      a.h, a.w, a.ring, a.next, a.taps, a.width, a.rows, a.start);
   BH_CHECK_HIP(hipGetLastError());
