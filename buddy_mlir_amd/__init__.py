@@ -133,6 +133,10 @@ def _declare(lib):
         "buddy_hip_session_reset": (c_int, [vp]),
         "buddy_hip_session_architecture": (c_char_p, [vp]),
         "buddy_hip_session_create_from_folder": (vp, [c_char_p, vp]),
+        "buddy_hip_bf16_tiles_bytes": (sz, [i64, i64]),
+        "buddy_hip_pack_bf16_tiles": (c_int, [vp, i64, i64, vp, vp]),
+        "buddy_hip_gemm_bf16": (c_int, [vp, i64, c_int, vp, vp, i64, i64, i64, i64, vp]),
+        "buddy_hip_gemv_bf16": (c_int, [vp, vp, vp, i64, i64, vp]),
         "buddy_hip_model_architecture": (c_char_p, [c_int]),
         "buddy_hip_session_adopt": (None, [vp, vp]),
         "buddy_hip_w8a32_blob_sizes": (None, [vp, vp, vp]),

@@ -277,7 +277,7 @@ int launch_variant(const RowsGemm &a, hipStream_t stream) {
   BH_REQUIRE(blocks <= 65535, "rows_gemm: %lld row blocks", (long long)blocks);
   hipLaunchKernelGGL((rows_gemm_kernel<T, RT, GT, OUT, GROUPED>),
                      dim3((unsigned)ceil_div(d.groups, per), (unsigned)blocks), dim3(kGemmThreads),
-                     0, stream, a.W.tiles, a.W.ktiles, a.W.ktiles / ActTraits<T>::kTiles, d);
+                     0, stream, a.W.tiles, a.W.ktiles, (int)ceil_div(a.W.K, ActTraits<T>::kElems), d);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }
@@ -349,3 +349,26 @@ int launch_rows_gemm(const RowsGemm &a, hipStream_t stream) {
 }
 
 } // namespace bh
+
+extern "C" {
+
+int buddy_hip_gemm_bf16(const void *A, int64_t lda, int dtype, const void *tiles, float *C,
+                        int64_t ldc, int64_t M, int64_t K, int64_t N, buddy_hip_stream stream) try {
+  BH_REQUIRE(A && tiles && C && M > 0 && K > 0 && N > 0 && M < (1 << 30) && K < (1 << 30) &&
+                 N < (1 << 30) && lda < (1 << 30) && ldc < (1 << 30) &&
+                 (dtype == BUDDY_HIP_MODEL_BF16 || dtype == BUDDY_HIP_MODEL_F32),
+             "gemm_bf16: bad argument");
+  bh::RowsGemm g;
+  g.W.tiles = static_cast<const uint4 *>(tiles);
+  g.W.K = (int)K;
+  g.W.N = (int)bh::round_up(N, 16);
+  g.W.ktiles = bh::bf16_ktiles(K);
+  g.A = A;
+  g.lda = (int)lda;
+  g.f32 = dtype == BUDDY_HIP_MODEL_F32;
+  g.rows = (int)M;
+  g.C = C;
+  g.ldc = (int)ldc;
+  return bh::launch_rows_gemm(g, bh::as_stream(stream));
+} BH_CATCH_INT("buddy_hip_gemm_bf16")
+}

@@ -67,7 +67,6 @@ __device__ __forceinline__ float block_sum(float v, float *red) {
 }
 
 struct RowTail { // arguments a wavefront needs only behind its first loads
-  const float *y;
   float *x_out, *row_out;
   const float *conv_w;
   float *conv_ring, *conv_next;
@@ -103,11 +102,13 @@ __device__ __forceinline__ void keep_row(const RowTail &a, int K, int p, int i, 
 // memory.  R = 0: any K.  `keeper`: this workgroup stores what the row leaves behind.
 template <int INPUT, int R>
 struct RowPrologue {
-  f32x4 x[R], y[R], c[R], w[R];
+  f32x4 x[R], y[R], c[2][R], w[R];
+  const float *yp;
   int at[R];
   bool in[R];
-  __device__ __forceinline__ void request(const float *src, int K, const RowTail &a) {
-    const int p = INPUT == kRowNorm && a.conv_w ? *a.pos : 0;
+  __device__ __forceinline__ void request(const float *src, const float *ysrc, const float *conv_next,
+                                          int K, const RowTail &a) {
+    yp = ysrc;
 #pragma unroll
     for (int r = 0; r < R; ++r) {
       at[r] = (r * kRowThreads + (int)threadIdx.x) * 4;
@@ -115,15 +116,16 @@ struct RowPrologue {
       const int i = in[r] ? at[r] : 0;
       x[r] = load4(src + i);
       if constexpr (INPUT == kRowNorm) {
-        if (a.y)
-          y[r] = load4(a.y + i);
-        if (a.conv_w) {
+        if (yp)
+          y[r] = load4(yp + i);
+        if (conv_next) { // both slots: which one counts depends on the position
+          c[0][r] = load4(conv_next + i);
+          c[1][r] = load4(conv_next + K + i);
           w[r] = load4(a.conv_w + (int64_t)(a.taps - 1) * K + i);
-          c[r] = load4(a.conv_next + (int64_t)(p & 1) * K + i);
         }
       } else if constexpr (INPUT == kRowGated) {
         w[r] = load4(a.weight + i);
-        c[r] = load4(a.gate + i);
+        c[0][r] = load4(a.gate + i);
       }
     }
   }
@@ -145,9 +147,9 @@ struct RowPrologue {
       for (int r = 0; r < R; ++r)
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-          x[r][j] = x[r][j] * g * w[r][j] * sigmoid_f(c[r][j]);
+          x[r][j] = x[r][j] * g * w[r][j] * sigmoid_f(c[0][r][j]);
     } else if constexpr (INPUT == kRowNorm) {
-      if (a.y) {
+      if (yp) {
         const float ry = a.out_gain / sqrtf(block_sum(squares(y), red[0]) / (float)K + a.eps);
 #pragma unroll
         for (int r = 0; r < R; ++r) {
@@ -170,7 +172,7 @@ struct RowPrologue {
         if (a.conv_w) {
 #pragma unroll
           for (int j = 0; j < 4; ++j)
-            x[r][j] += fmaf(w[r][j], h[j], p > 0 ? c[r][j] : 0.f);
+            x[r][j] += fmaf(w[r][j], h[j], p == 0 ? 0.f : p & 1 ? c[1][r][j] : c[0][r][j]);
           if (keeper && in[r])
 #pragma unroll
             for (int j = 0; j < 4; ++j)
@@ -188,8 +190,12 @@ struct RowPrologue {
 };
 template <int INPUT>
 struct RowPrologue<INPUT, 0> {
-  const float *src;
-  __device__ __forceinline__ void request(const float *s, int, const RowTail &) { src = s; }
+  const float *src, *yp;
+  __device__ __forceinline__ void request(const float *s, const float *ysrc, const float *, int,
+                                          const RowTail &) {
+    src = s;
+    yp = ysrc;
+  }
   __device__ __forceinline__ void finish(float *act, int K, int Kp, const RowTail &a, bool keeper,
                                          float (*red)[kRowWaves]) {
     const int tid = threadIdx.x;
@@ -199,16 +205,16 @@ struct RowPrologue<INPUT, 0> {
         act[i] = src[i];
     } else {
       float ry = 0.f, ss = 0.f;
-      if (INPUT == kRowNorm && a.y) {
+      if (INPUT == kRowNorm && yp) {
         for (int i = tid; i < K; i += kRowThreads)
-          ss = fmaf(a.y[i], a.y[i], ss);
+          ss = fmaf(yp[i], yp[i], ss);
         ry = a.out_gain / sqrtf(block_sum(ss, red[0]) / (float)K + a.eps);
       }
       ss = 0.f;
       for (int i = tid; i < K; i += kRowThreads) {
         float v = src[i];
-        if (INPUT == kRowNorm && a.y) {
-          v = fmaf(a.y[i], ry, v);
+        if (INPUT == kRowNorm && yp) {
+          v = fmaf(yp[i], ry, v);
           if (keeper && a.x_out)
             a.x_out[i] = v;
         }
@@ -246,8 +252,9 @@ struct RowPrologue<INPUT, 0> {
 // more, which multiplies nothing and stores what the row leaves behind.
 template <int INPUT, int R>
 __global__ void __launch_bounds__(kRowThreads)
-row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src, int K, int ktiles,
-                int groups, int ks_shift, int slice_tiles, RowTail a) {
+row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src,
+                const float *__restrict__ y, const float *conv_next, int K, int ktiles, int groups,
+                int ks_shift, int slice_tiles, RowTail a) {
   extern __shared__ __attribute__((aligned(16))) float act[]; // [Kp]
   __shared__ float red[2][kRowWaves];
   __shared__ float part[kRowWaves][16];
@@ -255,7 +262,7 @@ row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src, int 
   const int tid = threadIdx.x, lane = tid & 63;
   // the row's values first: loads return in order, and these come from the L2
   RowPrologue<INPUT, R> row;
-  row.request(src, K, a);
+  row.request(src, y, conv_next, K, a);
   if (INPUT == kRowNorm && blockIdx.x == gridDim.x - 1) {
     row.finish(act, K, Kp, a, true, red);
     return;
@@ -571,7 +578,7 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
   const int slice_tiles = (int)ceil_div(W.ktiles, ks);
   const size_t lds = sizeof(float) * (size_t)W.ktiles * kBfTileK;
   BH_REQUIRE(lds <= 150 * 1024, "row_gemv: a row of %d values does not fit LDS", W.K);
-  RowTail t{a.y, a.x_out, a.row_out, a.conv_w, a.conv_ring, a.conv_next, a.pos, a.weight, a.gate,
+  RowTail t{a.x_out, a.row_out, a.conv_w, a.conv_ring, a.conv_next, a.pos, a.weight, a.gate,
             a.out, a.max_v, a.max_i, a.eps, a.out_gain, a.gain, a.taps, a.silu_channels, a.valid};
   const bool keeper = a.input == kRowNorm;
   const dim3 grid((unsigned)(ceil_div(groups, per) + keeper)), block(kRowThreads);
@@ -586,8 +593,9 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
   do {                                                                                           \
     static DynLdsOnce once;                                                                      \
     BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)row_gemv_kernel<I, R>, 150 * 1024));         \
-    hipLaunchKernelGGL((row_gemv_kernel<I, R>), grid, block, lds, stream, W.tiles, a.src, W.K,   \
-                       W.ktiles, groups, shift, slice_tiles, t);                                 \
+    hipLaunchKernelGGL((row_gemv_kernel<I, R>), grid, block, lds, stream, W.tiles, a.src, a.y,   \
+                       a.conv_w ? a.conv_next : nullptr, W.K, W.ktiles, groups, shift,           \
+                       slice_tiles, t);                                                          \
   } while (0)
 #define BH_ROWS(I)                                                                               \
   do {                                                                                           \
@@ -686,3 +694,29 @@ int launch_row_moe(const RowMoe &a, hipStream_t stream) {
 }
 
 } // namespace bh
+
+extern "C" {
+
+size_t buddy_hip_bf16_tiles_bytes(int64_t K, int64_t N) {
+  return K > 0 && N > 0 ? bh::bf16_tiles_bytes(K, N) : 0;
+}
+
+int buddy_hip_pack_bf16_tiles(const uint16_t *W, int64_t K, int64_t N, void *tiles,
+                              buddy_hip_stream stream) try {
+  BH_REQUIRE(K < (1 << 30) && N < (1 << 30), "pack_bf16_tiles: bad size");
+  return bh::launch_pack_bf16(W, K, 1, N, K, tiles, bh::as_stream(stream));
+} BH_CATCH_INT("buddy_hip_pack_bf16_tiles")
+
+int buddy_hip_gemv_bf16(const float *x, const void *tiles, float *y, int64_t K, int64_t N,
+                        buddy_hip_stream stream) try {
+  BH_REQUIRE(K > 0 && N > 0 && K < (1 << 30) && N < (1 << 30), "gemv_bf16: bad size");
+  bh::RowGemv g;
+  g.W.tiles = static_cast<const uint4 *>(tiles);
+  g.W.K = (int)K;
+  g.W.N = (int)bh::round_up(N, 16);
+  g.W.ktiles = bh::bf16_ktiles(K);
+  g.src = x;
+  g.out = y;
+  return bh::launch_row_gemv(g, bh::as_stream(stream));
+} BH_CATCH_INT("buddy_hip_gemv_bf16")
+}

@@ -39,11 +39,10 @@ __device__ __forceinline__ float dot_run(const uint4 w, const float *x, float ac
 }
 
 struct LatentQueryArgs {
-  int heads, dim, rot_dim, rot8, rank, row_elems, ring_mask, dkv_at, uk_groups, uk_ktiles;
+  int heads, rot8, rank, row_elems, ring_mask, dkv_at;
   float scale, eps;
   const float *norm_w;
   const double *turns;
-  const int *pos;
   void *cache;
   float *query;
 };
@@ -52,12 +51,14 @@ struct LatentQueryArgs {
 // row, the others a head's query in the space of a cache row.
 template <typename T>
 __global__ void __launch_bounds__(kStepThreads)
-latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj, LatentQueryArgs a) {
+latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj,
+                    const int *__restrict__ pos, int uk_groups, int uk_ktiles, int dim, int rot_dim,
+                    LatentQueryArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int h = blockIdx.x, half = a.rot_dim / 2;
-  const int p = *a.pos;
+  const int h = blockIdx.x, half = rot_dim / 2;
+  const int p = *pos;
   if (h == a.heads) {
     if (blockIdx.y)
       return;
@@ -77,7 +78,7 @@ latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj
     T *row = static_cast<T *>(a.cache) + (int64_t)(p & a.ring_mask) * a.row_elems;
     for (int i = tid; i < a.row_elems; i += kStepThreads) {
       float v = 0.f;
-      if (i < a.rot_dim) {
+      if (i < rot_dim) {
         const int f = i < half ? i : i - half;
         float c, s;
         rotation(a.turns[f], p, c, s);
@@ -90,44 +91,44 @@ latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj
     }
     return;
   }
-  const float *q = proj + (int64_t)h * (a.dim + a.rot_dim);
+  const float *q = proj + (int64_t)h * (dim + rot_dim);
   float *out = a.query + (int64_t)h * a.row_elems;
-  const int Kp = a.uk_ktiles * kBfTileK;
+  const int Kp = uk_ktiles * kBfTileK;
   // one channel group per wavefront, its first tiles asked for ahead of the query
-  const int g = blockIdx.y * kStepWaves + wave, gl = min(g, a.uk_groups - 1);
-  const uint4 *wp = uk + ((int64_t)h * a.uk_groups + gl) * a.uk_ktiles * 64 + lane;
+  const int g = blockIdx.y * kStepWaves + wave, gl = min(g, uk_groups - 1);
+  const uint4 *wp = uk + ((int64_t)h * uk_groups + gl) * uk_ktiles * 64 + lane;
   constexpr int kAhead = 4;
   uint4 w[kAhead];
 #pragma unroll
   for (int u = 0; u < kAhead; ++u)
-    w[u] = wp[(int64_t)min(u, a.uk_ktiles - 1) * 64];
+    w[u] = wp[(int64_t)min(u, uk_ktiles - 1) * 64];
   for (int i = tid; i < Kp; i += kStepThreads)
-    lds[i] = i < a.dim ? q[i] : 0.f;
+    lds[i] = i < dim ? q[i] : 0.f;
   if (blockIdx.y == 0)
     for (int i = tid; i < a.row_elems; i += kStepThreads) {
       if (i >= a.rot8 && i < a.rot8 + a.rank)
         continue; // the latent part, below
       float v = 0.f;
-      if (i < a.rot_dim) {
+      if (i < rot_dim) {
         const int f = i < half ? i : i - half;
         float c, s;
         rotation(a.turns[f], p, c, s);
-        const float u = q[a.dim + f], x = q[a.dim + f + half];
+        const float u = q[dim + f], x = q[dim + f + half];
         v = (i < half ? u * c - x * s : x * c + u * s) * a.scale;
       }
       out[i] = v;
     }
   __syncthreads();
   float acc = 0.f;
-  for (int t = 0; t < a.uk_ktiles; t += kAhead) {
+  for (int t = 0; t < uk_ktiles; t += kAhead) {
     if (t > 0) {
 #pragma unroll
       for (int u = 0; u < kAhead; ++u)
-        w[u] = wp[(int64_t)min(t + u, a.uk_ktiles - 1) * 64];
+        w[u] = wp[(int64_t)min(t + u, uk_ktiles - 1) * 64];
     }
 #pragma unroll
     for (int u = 0; u < kAhead; ++u)
-      if (t + u < a.uk_ktiles)
+      if (t + u < uk_ktiles)
         acc = dot_run(w[u], lds + (t + u) * kBfTileK + (lane >> 4) * 8, acc);
   }
   acc = sum_rows(acc);
@@ -137,27 +138,40 @@ latent_query_kernel(const uint4 *__restrict__ uk, const float *__restrict__ proj
 }
 
 struct LatentPartArgs {
-  int heads, heads16, rank16, rot8, row_elems, window, ring_mask, lds_stride;
-  const int *pos;
+  int heads16, rank16, rot8;
   float *acc, *ml;
 };
 
-// Grid (chunks, heads16 / 16).  Four wavefronts per key tile of 16 positions: each
-// takes a quarter of the score's k, then all share out the latent dimensions.
+// Grid (chunks, heads16 / 16).  WK wavefronts per key tile of 16 positions: each
+// takes its share of the score's k, then all share out the latent dimensions.
 // S^T = C . Q^T leaves a lane with 4 keys of one head, which is the B operand of
 // O^T += C^T . P^T as it lies.
-template <typename T, int KT>
-__global__ void __launch_bounds__(KT * 256)
-latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query, LatentPartArgs a) {
+template <typename T, int KT, int WK>
+__global__ void __launch_bounds__(KT * WK * 64)
+latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
+                   const int *__restrict__ pos, int row_elems, int window, int ring_mask,
+                   int lds_stride, LatentPartArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
   constexpr int kKeys = KT * 16;
   const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   T *ck = reinterpret_cast<T *>(raw);                                            // [kKeys][lds_stride]
-  float *sp = reinterpret_cast<float *>(raw + sizeof(T) * kKeys * a.lds_stride); // [KT][4][16][16]
-  const int p = *a.pos;
-  const int lo = max(0, p - a.window + 1), n = p - lo + 1;
-  const int k0 = blockIdx.x * kKeys, head0 = blockIdx.y * 16;
+  float *sp = reinterpret_cast<float *>(raw + sizeof(T) * kKeys * lds_stride); // [KT][WK][16][16]
+  const int head0 = blockIdx.y * 16;
+  // this lane's query values: a step of 32 k in every WK-th, the first kQSteps of them
+  // in flight together, asked for before the position is known
+  constexpr int E = 16 / (int)sizeof(T), kQSteps = 20 / WK + (20 % WK != 0), kRows = 16 / WK;
+  const int kt = wave / WK, share = wave % WK, steps = row_elems / 32;
+  const int runs = row_elems / E;
+  // (what columns of heads past the last compute is not used)
+  const float *qr = query + (int64_t)(head0 + col) * row_elems + quad * 8;
+  Frag<float> qf[kQSteps];
+#pragma unroll
+  for (int i = 0; i < kQSteps; ++i)
+    qf[i].load(qr + min(share + i * WK, steps - 1) * 32);
+  const int p = *pos;
+  const int lo = max(0, p - window + 1), n = p - lo + 1;
+  const int k0 = blockIdx.x * kKeys;
   float *ml = a.ml + ((int64_t)blockIdx.x * a.heads16 + head0) * 2;
   if (k0 >= n) { // nothing visible: an empty partial
     if (tid < 16) {
@@ -166,29 +180,18 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
     }
     return;
   }
-  // four rows of the tile per wavefront, and this lane's query values: a step of 32 k
-  // in every fourth, the first kQSteps of them in flight together
-  constexpr int E = 16 / (int)sizeof(T), kQSteps = 5;
-  const int kt = wave >> 2, quarter = wave & 3, steps = a.row_elems / 32;
-  const int runs = a.row_elems / E;
-  // (what columns of heads past the last compute is not used)
-  const float *qr = query + (int64_t)(head0 + col) * a.row_elems + quad * 8;
-  Frag<float> qf[kQSteps];
-#pragma unroll
-  for (int i = 0; i < kQSteps; ++i)
-    qf[i].load(qr + min(quarter + i * 4, steps - 1) * 32);
   for (int c0 = 0; c0 < runs; c0 += 128) {
-    u32x4 v[4][2];
+    u32x4 v[kRows][2];
     const int ca = min(c0 + lane, runs - 1), cb = min(c0 + 64 + lane, runs - 1);
 #pragma unroll
-    for (int r = 0; r < 4; ++r) { // a row past the last key repeats it, masked below
-      const T *row = cache + (int64_t)((lo + min(k0 + wave * 4 + r, n - 1)) & a.ring_mask) * a.row_elems;
+    for (int r = 0; r < kRows; ++r) { // a row past the last key repeats it, masked below
+      const T *row = cache + (int64_t)((lo + min(k0 + wave * kRows + r, n - 1)) & ring_mask) * row_elems;
       v[r][0] = *reinterpret_cast<const u32x4 *>(row + ca * E);
       v[r][1] = *reinterpret_cast<const u32x4 *>(row + cb * E);
     }
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      T *row = ck + (wave * 4 + r) * a.lds_stride;
+    for (int r = 0; r < kRows; ++r) {
+      T *row = ck + (wave * kRows + r) * lds_stride;
       *reinterpret_cast<u32x4 *>(row + ca * E) = v[r][0];
       *reinterpret_cast<u32x4 *>(row + cb * E) = v[r][1];
     }
@@ -196,7 +199,7 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
   __syncthreads();
   {
     f32x4 s{0.f, 0.f, 0.f, 0.f};
-    const T *kr = ck + (kt * 16 + col) * a.lds_stride + quad * 8;
+    const T *kr = ck + (kt * 16 + col) * lds_stride + quad * 8;
     auto score = [&](int t, const Frag<float> &q) {
       Frag<T> kf;
       kf.load(kr + t * 32);
@@ -209,9 +212,9 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
     };
 #pragma unroll
     for (int i = 0; i < kQSteps; ++i)
-      if (quarter + i * 4 < steps)
-        score(quarter + i * 4, qf[i]);
-    for (int t = quarter + kQSteps * 4; t < steps; t += 4) {
+      if (share + i * WK < steps)
+        score(share + i * WK, qf[i]);
+    for (int t = share + kQSteps * WK; t < steps; t += WK) {
       Frag<float> q;
       q.load(qr + t * 32);
       score(t, q);
@@ -230,8 +233,8 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
       const int key = quad * 4 + r;
       float s = 0.f;
 #pragma unroll
-      for (int w = 0; w < 4; ++w)
-        s += sp[(((kt * 4 + w) * 16) + key) * 16 + col];
+      for (int w = 0; w < WK; ++w)
+        s += sp[(((kt * WK + w) * 16) + key) * 16 + col];
       s = k0 + kt * 16 + key < n ? s : -INFINITY;
       pr[kt][r] = s;
       m = fmaxf(m, s);
@@ -258,49 +261,67 @@ latent_part_kernel(const T *__restrict__ cache, const float *__restrict__ query,
     ml[lane * 2 + 1] = l;
   }
   float *acc = a.acc + ((int64_t)blockIdx.x * a.heads16 + head0 + col) * a.rank16;
-  for (int lt = wave; lt < a.rank16 / 16; lt += KT * 4) {
+  for (int lt = wave; lt < a.rank16 / 16; lt += KT * WK) {
     f32x4 o{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int kt = 0; kt < KT; ++kt)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        o = mfma_f32(load_act<T>(ck + (kt * 16 + quad * 4 + r) * a.lds_stride + a.rot8 + lt * 16 + col),
+        o = mfma_f32(load_act<T>(ck + (kt * 16 + quad * 4 + r) * lds_stride + a.rot8 + lt * 16 + col),
                      pr[kt][r], o);
     *reinterpret_cast<f32x4 *>(acc + lt * 16 + quad * 4) = o;
   }
 }
 
 struct LatentFoldArgs {
-  int heads16, rank, rank16, vdim, groups, ktiles, chunks;
-  const float *acc, *ml, *gate;
+  int rank, vdim;
+  const float *gate;
   float *out;
 };
 
 // Grid (heads, parts of the value channels): folds the partials of a head, then
 // four channel groups of its value matrix, k in two slices.
 __global__ void __launch_bounds__(kStepThreads)
-latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
+latent_value_kernel(const uint4 *__restrict__ uv, const float *__restrict__ part_acc,
+                    const float *__restrict__ part_ml, int groups, int ktiles, int chunks, int heads16,
+                    int rank16, LatentFoldArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   __shared__ float part[kStepWaves][16];
   __shared__ float red[2][kStepWaves];
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = blockIdx.x;
-  const int Kp = a.ktiles * kBfTileK;
+  const int Kp = ktiles * kBfTileK;
   float *x = lds, *wt = lds + Kp; // [Kp], [chunks]
   const int gi = wave >> 1, slice = wave & 1;
-  const int g = blockIdx.y * 4 + gi, gl = min(g, a.groups - 1);
-  const int half = (a.ktiles + 1) / 2;
-  const int t0 = slice * half, t1 = min(t0 + half, a.ktiles);
-  const uint4 *wp = uv + ((int64_t)h * a.groups + gl) * a.ktiles * 64 + lane;
+  const int g = blockIdx.y * 4 + gi, gl = min(g, groups - 1);
+  const int half = (ktiles + 1) / 2;
+  const int t0 = slice * half, t1 = min(t0 + half, ktiles);
+  const uint4 *wp = uv + ((int64_t)h * groups + gl) * ktiles * 64 + lane;
+  // loads return in order: what is needed first is asked for first
+  float2 ml{-INFINITY, 0.f}; // (maximum, sum) of this thread's first chunk
+  if (tid < chunks)
+    ml = *reinterpret_cast<const float2 *>(part_ml + ((int64_t)tid * heads16 + h) * 2);
+  // the partials in four parts: 128 threads take four latent dimensions each of every
+  // fourth chunk, eight in flight, the first eight before their weights are known
+  const int64_t step = (int64_t)heads16 * rank16;
+  const int part4 = tid >> 7, i0 = (tid & 127) * 4;
+  auto partials = [&](int i, int c, f32x4 (&v)[8]) {
+    const float *q = part_acc + (int64_t)h * rank16 + i;
+#pragma unroll
+    for (int u = 0; u < 8; ++u)
+      v[u] = *reinterpret_cast<const f32x4 *>(q + min(c + u * 4, chunks - 1) * step);
+  };
+  f32x4 v[8];
+  partials(min(i0, rank16 - 4), part4, v);
   constexpr int kAhead = 8;
   uint4 w[kAhead];
 #pragma unroll
   for (int u = 0; u < kAhead; ++u)
-    w[u] = wp[(int64_t)min(t0 + u, a.ktiles - 1) * 64];
-  float m = -INFINITY;
-  for (int c = tid; c < a.chunks; c += kStepThreads)
-    m = fmaxf(m, a.ml[((int64_t)c * a.heads16 + h) * 2]);
+    w[u] = wp[(int64_t)min(t0 + u, ktiles - 1) * 64];
+  float m = ml.x;
+  for (int c = tid + kStepThreads; c < chunks; c += kStepThreads)
+    m = fmaxf(m, part_ml[((int64_t)c * heads16 + h) * 2]);
   m = wave_max(m);
   if (lane == 0)
     red[0][wave] = m;
@@ -309,11 +330,12 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
   for (int i = 0; i < kStepWaves; ++i)
     m = fmaxf(m, red[0][i]);
   float l = 0.f;
-  for (int c = tid; c < a.chunks; c += kStepThreads) {
-    const float *q = a.ml + ((int64_t)c * a.heads16 + h) * 2;
-    const float e = q[1] > 0.f ? fast_exp(q[0] - m) : 0.f;
+  for (int c = tid; c < chunks; c += kStepThreads) {
+    if (c != tid)
+      ml = *reinterpret_cast<const float2 *>(part_ml + ((int64_t)c * heads16 + h) * 2);
+    const float e = ml.y > 0.f ? fast_exp(ml.x - m) : 0.f;
     wt[c] = e;
-    l = fmaf(e, q[1], l);
+    l = fmaf(e, ml.y, l);
   }
   l = wave_sum(l);
   if (lane == 0)
@@ -324,23 +346,16 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
   for (int i = 0; i < kStepWaves; ++i)
     l += red[1][i];
   const float inv = 1.0f / l;
-  // the partials in four parts: 128 threads take four latent dimensions each of every
-  // fourth chunk, eight in flight
-  const int64_t step = (int64_t)a.heads16 * a.rank16;
-  const int part4 = tid >> 7;
-  float *fold = wt + ((a.chunks + 3) & ~3); // [4][Kp]
-  for (int i = (tid & 127) * 4; i < Kp; i += 512) {
+  float *fold = wt + ((chunks + 3) & ~3); // [4][Kp]
+  for (int i = i0; i < Kp; i += 512) {
     f32x4 o{0.f, 0.f, 0.f, 0.f};
-    if (i < a.rank16) {
-      const float *q = a.acc + (int64_t)h * a.rank16 + i;
-      for (int c = part4; c < a.chunks; c += 32) {
-        f32x4 v[8];
-#pragma unroll
-        for (int u = 0; u < 8; ++u)
-          v[u] = *reinterpret_cast<const f32x4 *>(q + min(c + u * 4, a.chunks - 1) * step);
+    if (i < rank16) {
+      for (int c = part4; c < chunks; c += 32) {
+        if (i != i0 || c != part4)
+          partials(i, c, v);
 #pragma unroll
         for (int u = 0; u < 8; ++u) {
-          const float e = c + u * 4 < a.chunks ? wt[min(c + u * 4, a.chunks - 1)] : 0.f;
+          const float e = c + u * 4 < chunks ? wt[min(c + u * 4, chunks - 1)] : 0.f;
 #pragma unroll
           for (int j = 0; j < 4; ++j) // an empty partial's accumulators were never written
             o[j] = e != 0.f ? fmaf(e, v[u][j], o[j]) : o[j];
@@ -359,7 +374,7 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
     if (t > t0) {
 #pragma unroll
       for (int u = 0; u < kAhead; ++u)
-        w[u] = wp[(int64_t)min(t + u, a.ktiles - 1) * 64];
+        w[u] = wp[(int64_t)min(t + u, ktiles - 1) * 64];
     }
 #pragma unroll
     for (int u = 0; u < kAhead; ++u)
@@ -372,7 +387,7 @@ latent_value_kernel(const uint4 *__restrict__ uv, LatentFoldArgs a) {
   __syncthreads();
   if (tid < 64) {
     const int gg = blockIdx.y * 4 + (tid >> 4), v = gg * 16 + (tid & 15);
-    if (gg < a.groups && v < a.vdim)
+    if (gg < groups && v < a.vdim)
       a.out[(int64_t)h * a.vdim + v] =
           (part[(tid >> 4) * 2][tid & 15] + part[(tid >> 4) * 2 + 1][tid & 15]) *
           sigmoid_f(a.gate[h]);
@@ -449,7 +464,7 @@ template <typename T> struct KeyTile {
   static constexpr int kKeys = 128 / (int)sizeof(T);
 };
 
-// Grid (heads, query blocks).  A wavefront owns 16 * QT queries, the workgroup's four
+// Grid (heads, query blocks).  A wavefront owns 16 queries, the workgroup's four
 // share tiles of kKeys keys through LDS; the next tile is on its way in registers
 // meanwhile.  S^T = K . Q^T leaves a lane with keys of one query, which is the B
 // operand of O^T += V^T . P^T as it lies (of 32 keys in bfloat16: a lane's eight are
@@ -461,8 +476,8 @@ template <typename T> struct KeyTile {
 // The running maximum a lane subtracts follows the scores only when one exceeds it by
 // more than kSlack: the weights stay below e^kSlack, and the sums are rescaled a few
 // times per query instead of once per tile.
-template <typename T, int NK, int NV, int QT>
-__global__ void __launch_bounds__(256, QT == 1 && NV <= 8 ? 2 : 1)
+template <typename T, int NK, int NV>
+__global__ void __launch_bounds__(256, NV <= 8 ? 2 : 1)
 latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ keys,
                         const T *__restrict__ values_t, const T *__restrict__ cache,
                         const float *__restrict__ proj, T *__restrict__ out, LatentAttnArgs a) {
@@ -472,34 +487,29 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
   const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = blockIdx.x;
-  constexpr int kBlock = 64 * QT;
+  constexpr int kBlock = 64;
   const int q0 = (gridDim.y - 1 - blockIdx.y) * kBlock; // long blocks first
   constexpr int kKeyRow = NK * 32 + E, kValueRow = KEYS + E; // rows start 4 banks apart
   constexpr float kSlack = 8.0f;
   T *kt = reinterpret_cast<T *>(raw); // [KEYS][kKeyRow]
   T *vt = kt + KEYS * kKeyRow;        // [16 * NV][kValueRow]
 
-  // this lane's queries as key indexes, and their fragments
-  int my_q[QT];
-  Frag<T> qf[QT][NK];
+  // this lane's query, also as a key index, and its fragments
+  const int qi = q0 + wave * 16 + col, my_q = a.start + qi - a.first;
+  Frag<T> qf[NK];
+  const T *q = queries + ((int64_t)min(qi, a.rows - 1) * a.heads + h) * a.kd + quad * 8;
 #pragma unroll
-  for (int u = 0; u < QT; ++u) {
-    const int r = q0 + (wave * QT + u) * 16 + col;
-    my_q[u] = a.start + r - a.first;
-    const T *q = queries + ((int64_t)min(r, a.rows - 1) * a.heads + h) * a.kd + quad * 8;
-#pragma unroll
-    for (int t = 0; t < NK; ++t) {
-      if (t * 32 < a.kd)
-        qf[u][t].load(q + t * 32);
-      else
-        qf[u][t] = Frag<T>{};
-    }
+  for (int t = 0; t < NK; ++t) {
+    if (t * 32 < a.kd)
+      qf[t].load(q + t * 32);
+    else
+      qf[t] = Frag<T>{};
   }
   const int nkeys = a.start + a.rows - a.first;
   const int last_q = min(q0 + kBlock, a.rows) - 1;
   const int key_hi = a.start + last_q - a.first;                               // last visible
   const int key_lo = max(0, a.start + q0 - a.window + 1 - a.first) & ~(KEYS - 1); // tile of the first
-  const int wave_q0 = a.start + q0 + wave * 16 * QT - a.first, wave_q1 = wave_q0 + 16 * QT - 1;
+  const int wave_q0 = a.start + q0 + wave * 16 - a.first, wave_q1 = wave_q0 + 15;
 
   // the 16-byte runs this thread moves.  A key's runs: its head's part, the shared
   // rotated part; the rest of the row in LDS stays zero.
@@ -547,16 +557,11 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       kt[(i / pad) * kKeyRow + at + i % pad] = 0;
   }
 
-  f32x4 o[QT][NV];
-  float m[QT], l[QT];
+  f32x4 o[NV];
+  float m = -INFINITY, l = 0.f;
 #pragma unroll
-  for (int u = 0; u < QT; ++u) {
-    m[u] = -INFINITY;
-    l[u] = 0.f;
-#pragma unroll
-    for (int v = 0; v < NV; ++v)
-      o[u][v] = f32x4{0.f, 0.f, 0.f, 0.f};
-  }
+  for (int v = 0; v < NV; ++v)
+    o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
   for (int k0 = key_lo; k0 <= key_hi; k0 += KEYS) {
     __syncthreads(); // the previous tile has been read
 #pragma unroll
@@ -588,12 +593,10 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
     fetch(min(k0 + KEYS, (nkeys - 1) & ~(KEYS - 1)), kr, vr);
     if (k0 > wave_q1 || k0 + KEYS - 1 <= wave_q0 - a.window)
       continue; // nothing of this tile is visible to this wavefront
-    f32x4 s[QT][SUB];
-#pragma unroll
-    for (int u = 0; u < QT; ++u)
+    f32x4 s[SUB];
 #pragma unroll
       for (int b = 0; b < SUB; ++b)
-        s[u][b] = f32x4{0.f, 0.f, 0.f, 0.f};
+        s[b] = f32x4{0.f, 0.f, 0.f, 0.f};
     // the fragments of the next step are read while this one is multiplied
     const T *kp = kt + col * kKeyRow + quad * 8;
     Frag<T> kf[2][SUB];
@@ -610,71 +613,64 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
       for (int b = 0; b < SUB; ++b)
-#pragma unroll
-        for (int u = 0; u < QT; ++u)
-          s[u][b] = mfma32(kf[t & 1][b], qf[u][t], s[u][b]);
+        s[b] = mfma32(kf[t & 1][b], qf[t], s[b]);
       __builtin_amdgcn_sched_barrier(0);
     }
     const bool whole = k0 + KEYS - 1 <= wave_q0 && wave_q1 - k0 < a.window;
-#pragma unroll
-    for (int u = 0; u < QT; ++u) {
-      if (!whole) {
-#pragma unroll
-        for (int b = 0; b < SUB; ++b)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            const int gap = my_q[u] - (k0 + b * 16 + quad * 4 + r);
-            s[u][b][r] = gap >= 0 && gap < a.window ? s[u][b][r] : -INFINITY;
-          }
-      }
-      float mt = s[u][0][0];
-#pragma unroll
-      for (int b = 0; b < SUB; ++b)
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          mt = fmaxf(mt, s[u][b][r]);
-      float x, y;
-      lane_pair<16>(mt, x, y);
-      mt = fmaxf(x, y);
-      lane_pair<32>(mt, x, y);
-      mt = fmaxf(x, y);
-      if (__any(mt > m[u] + kSlack)) { // -inf + kSlack stays below every score
-        mt = fmaxf(mt, m[u]);
-        const float alpha = mt == -INFINITY ? 1.f : fast_exp(m[u] - mt);
-        m[u] = mt;
-        l[u] *= alpha;
-#pragma unroll
-        for (int v = 0; v < NV; ++v)
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            o[u][v][r] *= alpha;
-      }
-      const float base = m[u] == -INFINITY ? 0.f : m[u]; // nothing visible so far
+    if (!whole) {
 #pragma unroll
       for (int b = 0; b < SUB; ++b)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          s[u][b][r] = fast_exp(s[u][b][r] - base);
-          l[u] += s[u][b][r];
+          const int gap = my_q - (k0 + b * 16 + quad * 4 + r);
+          s[b][r] = gap >= 0 && gap < a.window ? s[b][r] : -INFINITY;
         }
     }
+    float mt = s[0][0];
+#pragma unroll
+    for (int b = 0; b < SUB; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        mt = fmaxf(mt, s[b][r]);
+    float x, y;
+    lane_pair<16>(mt, x, y);
+    mt = fmaxf(x, y);
+    lane_pair<32>(mt, x, y);
+    mt = fmaxf(x, y);
+    if (__any(mt > m + kSlack)) { // -inf + kSlack stays below every score
+      mt = fmaxf(mt, m);
+      const float alpha = mt == -INFINITY ? 1.f : fast_exp(m - mt);
+      m = mt;
+      l *= alpha;
+#pragma unroll
+      for (int v = 0; v < NV; ++v)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          o[v][r] *= alpha;
+    }
+    const float base = m == -INFINITY ? 0.f : m; // nothing visible so far
+#pragma unroll
+    for (int b = 0; b < SUB; ++b)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        s[b][r] = fast_exp(s[b][r] - base);
+        l += s[b][r];
+      }
     if constexpr (sizeof(T) == 2) {
       // the weights as two bfloat16 terms
-      uint4 hi[QT][SUB / 2], lo[QT][SUB / 2];
-#pragma unroll
-      for (int u = 0; u < QT; ++u)
+      uint4 hi[SUB / 2], lo[SUB / 2];
 #pragma unroll
         for (int b = 0; b < SUB / 2; ++b) {
           unsigned ph[4], pl[4];
 #pragma unroll
           for (int j = 0; j < 4; ++j) {
-            const f32x4 &x = s[u][2 * b + (j >> 1)];
+            const f32x4 &x = s[2 * b + (j >> 1)];
             const float x0 = x[2 * (j & 1)], x1 = x[2 * (j & 1) + 1];
             ph[j] = pack_bf(x0, x1);
             pl[j] = pack_bf(x0 - bf_lo(ph[j]), x1 - bf_hi(ph[j]));
           }
-          hi[u][b] = uint4{ph[0], ph[1], ph[2], ph[3]};
-          lo[u][b] = uint4{pl[0], pl[1], pl[2], pl[3]};
+          hi[b] = uint4{ph[0], ph[1], ph[2], ph[3]};
+          lo[b] = uint4{pl[0], pl[1], pl[2], pl[3]};
         }
       constexpr int G = NV < 4 ? NV : 4; // value tiles read ahead
       const T *vp = vt + col * kValueRow + quad * 8;
@@ -695,16 +691,14 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
         }
         __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-        for (int b = 0; b < SUB / 2; ++b)
+        for (int b = 0; b < SUB / 2; ++b) {
 #pragma unroll
-          for (int u = 0; u < QT; ++u) {
+          for (int v = 0; v < G; ++v)
+            o[v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, hi[b], o[v0 + v]);
 #pragma unroll
-            for (int v = 0; v < G; ++v)
-              o[u][v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, hi[u][b], o[u][v0 + v]);
-#pragma unroll
-            for (int v = 0; v < G; ++v)
-              o[u][v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, lo[u][b], o[u][v0 + v]);
-          }
+          for (int v = 0; v < G; ++v)
+            o[v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, lo[b], o[v0 + v]);
+        }
         __builtin_amdgcn_sched_barrier(0);
       }
     } else {
@@ -714,32 +708,26 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
         for (int b = 0; b < SUB; ++b) {
           const f32x4 vv = *reinterpret_cast<const f32x4 *>(vt + (v * 16 + col) * kValueRow + b * 16 + quad * 4);
 #pragma unroll
-          for (int u = 0; u < QT; ++u)
-#pragma unroll
-            for (int r = 0; r < 4; ++r)
-              o[u][v] = mfma_f32(vv[r], s[u][b][r], o[u][v]);
+          for (int r = 0; r < 4; ++r)
+            o[v] = mfma_f32(vv[r], s[b][r], o[v]);
         }
     }
   }
+  const float sum = sum_rows(l);
+  if (qi >= a.rows)
+    return;
+  const float f = sigmoid_f(proj[(int64_t)qi * a.ld + a.gate_at + h]) / sum;
+  T *dst = out + (int64_t)qi * a.out_ld + (int64_t)h * a.vdim;
 #pragma unroll
-  for (int u = 0; u < QT; ++u) {
-    const float sum = sum_rows(l[u]);
-    const int qi = q0 + (wave * QT + u) * 16 + col;
-    if (qi >= a.rows)
-      continue;
-    const float f = sigmoid_f(proj[(int64_t)qi * a.ld + a.gate_at + h]) / sum;
-    T *dst = out + (int64_t)qi * a.out_ld + (int64_t)h * a.vdim;
+  for (int v = 0; v < NV; ++v)
+    if (v < a.nv) {
 #pragma unroll
-    for (int v = 0; v < NV; ++v)
-      if (v < a.nv) {
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int c = v * 16 + quad * 4 + r;
-          if (c < a.vdim)
-            store_act<T>(dst + c, o[u][v][r] * f);
-        }
+      for (int r = 0; r < 4; ++r) {
+        const int c = v * 16 + quad * 4 + r;
+        if (c < a.vdim)
+          store_act<T>(dst + c, o[v][r] * f);
       }
-  }
+    }
 }
 
 bool shape_ok(const LatentShape &s) {
@@ -747,10 +735,11 @@ bool shape_ok(const LatentShape &s) {
          s.rank > 0 && s.window > 0 && s.ring_mask > 0 && ((s.ring_mask + 1) & s.ring_mask) == 0;
 }
 
+constexpr int part_waves(int key_tiles) { return key_tiles <= 2 ? 8 : 4; } // per key tile
 size_t part_lds(const LatentShape &s, int kt, int *stride) {
   // rows of the tile start 4 banks apart
   *stride = s.row_elems() + (s.f32 ? 4 : 8);
-  return (size_t)(s.f32 ? 4 : 2) * 16 * kt * *stride + 4 * (size_t)kt * 4 * 256;
+  return (size_t)(s.f32 ? 4 : 2) * 16 * kt * *stride + 4 * (size_t)kt * part_waves(kt) * 256;
 }
 constexpr size_t kLdsLimit = 156 * 1024;
 
@@ -758,7 +747,7 @@ constexpr size_t kLdsLimit = 156 * 1024;
 
 LatentCut latent_step_cut(const LatentShape &s, int span) {
   span = std::min(span, s.window);
-  int kt = span <= 1024 ? 1 : span <= 4096 ? 2 : 4, stride;
+  int kt = span <= 2048 ? 1 : span <= 8192 ? 2 : 4, stride;
   while (kt > 1 && part_lds(s, kt, &stride) > kLdsLimit)
     kt /= 2;
   return {kt, (int)ceil_div(span, 16 * kt)};
@@ -766,7 +755,7 @@ LatentCut latent_step_cut(const LatentShape &s, int span) {
 
 int latent_max_chunks(const LatentShape &s) {
   int most = 1; // the cuts change at these spans
-  for (int span : {1024, 4096, s.window})
+  for (int span : {2048, 8192, s.window})
     most = std::max(most, latent_step_cut(s, span).chunks);
   return most;
 }
@@ -781,33 +770,36 @@ int launch_latent_step(const LatentStep &a, int span, hipStream_t stream) {
              "latent_step: matrix shapes");
   const int re = s.row_elems();
   {
-    LatentQueryArgs q{s.heads, s.dim, s.rot_dim, s.rot8(), s.rank, re, s.ring_mask, a.dkv_at,
-                      s.rank16() / 16, a.uk_t.ktiles, s.scale, s.eps, a.norm_w, a.turns, a.pos,
-                      a.cache, a.query};
-    const dim3 grid((unsigned)(s.heads + 1), (unsigned)ceil_div(q.uk_groups, kStepWaves));
-    const size_t lds = sizeof(float) * (size_t)q.uk_ktiles * kBfTileK;
+    LatentQueryArgs q{s.heads, s.rot8(), s.rank, re, s.ring_mask, a.dkv_at, s.scale, s.eps, a.norm_w,
+                      a.turns, a.cache, a.query};
+    const int groups = s.rank16() / 16;
+    const dim3 grid((unsigned)(s.heads + 1), (unsigned)ceil_div(groups, kStepWaves));
+    const size_t lds = sizeof(float) * (size_t)a.uk_t.ktiles * kBfTileK;
     BH_REQUIRE(lds <= 60 * 1024, "latent_step: head of %d values", s.dim);
     if (s.f32)
       hipLaunchKernelGGL(latent_query_kernel<float>, grid, dim3(kStepThreads), lds, stream,
-                         a.uk_t.tiles, a.proj, q);
+                         a.uk_t.tiles, a.proj, a.pos, groups, a.uk_t.ktiles, s.dim, s.rot_dim, q);
     else
       hipLaunchKernelGGL(latent_query_kernel<bf16_bits>, grid, dim3(kStepThreads), lds, stream,
-                         a.uk_t.tiles, a.proj, q);
+                         a.uk_t.tiles, a.proj, a.pos, groups, a.uk_t.ktiles, s.dim, s.rot_dim, q);
     BH_CHECK_HIP(hipGetLastError());
   }
   const LatentCut cut = latent_step_cut(s, span);
   {
-    LatentPartArgs p{s.heads, s.heads16(), s.rank16(), s.rot8(), re, s.window, s.ring_mask, 0, a.pos,
-                     a.part_acc, a.part_ml};
-    const size_t lds = part_lds(s, cut.key_tiles, &p.lds_stride);
+    LatentPartArgs p{s.heads16(), s.rank16(), s.rot8(), a.part_acc, a.part_ml};
+    int stride = 0;
+    const size_t lds = part_lds(s, cut.key_tiles, &stride);
     BH_REQUIRE(lds <= kLdsLimit, "latent_step: a cache row of %d values does not fit LDS", re);
     const dim3 grid((unsigned)cut.chunks, (unsigned)(s.heads16() / 16));
 #define BH_PART(T, KT)                                                                           \
   do {                                                                                           \
     static DynLdsOnce once;                                                                      \
-    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_part_kernel<T, KT>, (int)kLdsLimit)); \
-    hipLaunchKernelGGL((latent_part_kernel<T, KT>), grid, dim3(KT * 256), lds, stream,           \
-                       static_cast<const T *>(a.cache), a.query, p);                             \
+    constexpr int WK = part_waves(KT);                                                           \
+    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_part_kernel<T, KT, WK>,               \
+                                (int)kLdsLimit));                                                \
+    hipLaunchKernelGGL((latent_part_kernel<T, KT, WK>), grid, dim3(KT * WK * 64), lds, stream,   \
+                       static_cast<const T *>(a.cache), a.query, a.pos, re, s.window,            \
+                       s.ring_mask, stride, p);                                                  \
   } while (0)
     if (s.f32) {
       if (cut.key_tiles == 1) BH_PART(float, 1);
@@ -822,14 +814,15 @@ int launch_latent_step(const LatentStep &a, int span, hipStream_t stream) {
     BH_CHECK_HIP(hipGetLastError());
   }
   {
-    LatentFoldArgs f{s.heads16(), s.rank, s.rank16(), s.vdim, s.vdim16() / 16, a.uv.ktiles,
-                     cut.chunks, a.part_acc, a.part_ml, a.proj + a.gate_at, a.out};
+    LatentFoldArgs f{s.rank, s.vdim, a.proj + a.gate_at, a.out};
+    const int groups = s.vdim16() / 16;
     const size_t lds = sizeof(float) * ((size_t)5 * a.uv.ktiles * kBfTileK + (size_t)round_up(cut.chunks, 4));
     BH_REQUIRE(lds <= kLdsLimit, "latent_step: %d partials do not fit LDS", cut.chunks);
     static DynLdsOnce once;
     BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_value_kernel, (int)kLdsLimit));
-    hipLaunchKernelGGL(latent_value_kernel, dim3((unsigned)s.heads, (unsigned)ceil_div(f.groups, 4)),
-                       dim3(kStepThreads), lds, stream, a.uv.tiles, f);
+    hipLaunchKernelGGL(latent_value_kernel, dim3((unsigned)s.heads, (unsigned)ceil_div(groups, 4)),
+                       dim3(kStepThreads), lds, stream, a.uv.tiles, a.part_acc, a.part_ml, groups,
+                       a.uv.ktiles, cut.chunks, s.heads16(), s.rank16(), f);
     BH_CHECK_HIP(hipGetLastError());
   }
   return BUDDY_HIP_OK;
@@ -857,15 +850,15 @@ int launch_latent_rows(const LatentRows &a, hipStream_t stream) {
 }
 
 namespace {
-template <typename T, int NK, int NV, int QT>
+template <typename T, int NK, int NV>
 int launch_attention(const LatentRows &a, const LatentAttnArgs &p, hipStream_t stream) {
   constexpr int E = 16 / (int)sizeof(T), KEYS = KeyTile<T>::kKeys;
   constexpr size_t lds = sizeof(T) * ((size_t)KEYS * (NK * 32 + E) + (size_t)16 * NV * (KEYS + E));
   static_assert(lds <= kLdsLimit, "the tiles must fit LDS");
   static DynLdsOnce once;
-  BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_attention_kernel<T, NK, NV, QT>, (int)kLdsLimit));
-  hipLaunchKernelGGL((latent_attention_kernel<T, NK, NV, QT>),
-                     dim3((unsigned)a.s.heads, (unsigned)ceil_div(a.rows, 64 * QT)), dim3(256), lds,
+  BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)latent_attention_kernel<T, NK, NV>, (int)kLdsLimit));
+  hipLaunchKernelGGL((latent_attention_kernel<T, NK, NV>),
+                     dim3((unsigned)a.s.heads, (unsigned)ceil_div(a.rows, 64)), dim3(256), lds,
                      stream, static_cast<const T *>(a.queries), static_cast<const T *>(a.keys),
                      static_cast<const T *>(a.values_t), static_cast<const T *>(a.cache), a.proj,
                      static_cast<T *>(a.out), p);
@@ -876,21 +869,15 @@ template <typename T>
 int launch_attention_any(const LatentRows &a, const LatentAttnArgs &p, hipStream_t stream) {
   const int nk = p.kd / 32;
   BH_REQUIRE(nk <= 18 && p.nv <= 32, "latent_attention: heads of %d and %d values", p.kd, a.s.vdim);
-  // two query tiles per wavefront halve the LDS reads, where they leave enough workgroups
-  const bool two = getenv("QT2") && sizeof(T) == 2 && ceil_div(a.rows, 128) * a.s.heads >= 192;
   if (nk <= 2 && p.nv <= 2)
-    return launch_attention<T, 2, 2, 1>(a, p, stream);
+    return launch_attention<T, 2, 2>(a, p, stream);
   if (nk <= 4 && p.nv <= 4)
-    return launch_attention<T, 4, 4, 1>(a, p, stream);
-  if (nk <= 6 && p.nv <= 8) {
-    if constexpr (sizeof(T) == 2)
-      if (two)
-        return launch_attention<T, 6, 8, 2>(a, p, stream);
-    return launch_attention<T, 6, 8, 1>(a, p, stream);
-  }
+    return launch_attention<T, 4, 4>(a, p, stream);
+  if (nk <= 6 && p.nv <= 8)
+    return launch_attention<T, 6, 8>(a, p, stream);
   if (nk <= 10 && p.nv <= 16)
-    return launch_attention<T, 10, 16, 1>(a, p, stream);
-  return launch_attention<T, 18, 32, 1>(a, p, stream);
+    return launch_attention<T, 10, 16>(a, p, stream);
+  return launch_attention<T, 18, 32>(a, p, stream);
 }
 } // namespace
 

@@ -500,6 +500,25 @@ int buddy_hip_session_vocab(buddy_hip_session *s);
 /* The name the model registry knows the session's model by. */
 const char *buddy_hip_session_architecture(buddy_hip_session *s);
 
+/* ---- matrices kept in bfloat16 ---------------------------------------------------
+ * W[N,K] bfloat16 bit patterns, row-major (out, in), packed once into 1 KiB tiles of
+ * 16 channels x 32 k in the matrix cores' operand order, K padded to 64 and N to 16
+ * with zeros: tile (g = n/16, c = k/32) at byte (g * ceil64(K)/32 + c) * 1024, lane
+ * L's 16 bytes hold k = c*32 + (L/16)*8 + 0..7 of channel g*16 + L%16.
+ * gemm: C[M, N] f32 = A[M, K] . W^T with f32 sums; A is bfloat16 (dtype
+ * BUDDY_HIP_MODEL_BF16) or f32 (BUDDY_HIP_MODEL_F32: f32 products), 16-byte aligned
+ * rows with lda a multiple of 8; ldc a multiple of 4, at least ceil16(N): the padding
+ * channels are written.  gemv: y[ceil16(N)] = x[K] . W^T, f32 multiply-adds.
+ * What the matrix products of folder models are made of; no counterpart in the
+ * reference. */
+size_t buddy_hip_bf16_tiles_bytes(int64_t K, int64_t N);
+int buddy_hip_pack_bf16_tiles(const uint16_t *W, int64_t K, int64_t N, void *tiles,
+                              buddy_hip_stream stream);
+int buddy_hip_gemm_bf16(const void *A, int64_t lda, int dtype, const void *tiles, float *C,
+                        int64_t ldc, int64_t M, int64_t K, int64_t N, buddy_hip_stream stream);
+int buddy_hip_gemv_bf16(const float *x, const void *tiles, float *y, int64_t K, int64_t N,
+                        buddy_hip_stream stream);
+
 /* ---- models from a folder ------------------------------------------------------
  * Builds a session from a folder with config.json and model.safetensors: the
  * registry picks the model class by config.json's "architecture".  Every

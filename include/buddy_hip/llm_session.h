@@ -17,6 +17,10 @@
  *   buddy::runtime::runGeneration(prompt, session, vocab, maxNewTokens, stops,
  *                                 sampler, codec, quiet);
  *
+ * loadWeights({"folder"}) takes a model folder (config.json, model.safetensors) of
+ * any architecture the library's registry knows instead; of the shape only max_len
+ * counts then.
+ *
  * Behaviour follows the generated class: prefill() leaves the logits of every
  * prompt row for logitsData(row) and sets the position to the token count
  * (gen_session.py:1345-1369); decode() runs one step at the current position
@@ -52,10 +56,23 @@ public:
   }
 
   /// {f32 file, int8 file}: the two parameter files of the w8a32 package
-  /// (tools/buddy-codegen/gen_config.py:55-58).
+  /// (tools/buddy-codegen/gen_config.py:55-58); or {folder}.
   void loadWeights(const std::vector<std::string> &weightPaths) override {
+    if (weightPaths.size() == 1) {
+      if (session_)
+        buddy_hip_session_destroy(session_);
+      buddy_hip_model_options options = {};
+      options.max_len = shape_.max_len;
+      session_ = buddy_hip_session_create_from_folder(weightPaths[0].c_str(), &options);
+      if (!session_)
+        fail("loadWeights");
+      shape_.vocab = buddy_hip_session_vocab(session_);
+      folder_ = true;
+      position_ = 0;
+      return;
+    }
     if (weightPaths.size() != 2)
-      throw std::runtime_error("HipLLMSession: expected {f32 file, int8 file}");
+      throw std::runtime_error("HipLLMSession: expected {f32 file, int8 file} or {folder}");
     int64_t nF32 = 0, nI8 = 0;
     buddy_hip_w8a32_blob_sizes(&shape_, &nF32, &nI8);
     std::vector<float> f32((size_t)nF32);
@@ -68,6 +85,7 @@ public:
         buddy_hip_session_create_from_w8a32_blobs(&shape_, f32.data(), nF32, i8.data(), nI8);
     if (!session_)
       fail("loadWeights");
+    folder_ = false;
     position_ = 0;
   }
 
@@ -111,7 +129,9 @@ public:
 
   bool handleKVCacheOverflow(int keepTokenNum, float ropeTheta = 10000.0f) override {
     requireLoaded();
-    if (position_ < shape_.max_len)
+    // a folder model keeps windows and states, no cache that tokens could be dropped
+    // from: its sequence ends at max_len
+    if (folder_ || position_ < shape_.max_len)
       return false;
     const int currentTokens = std::min(position_, shape_.max_len);
     keepTokenNum = std::clamp(keepTokenNum, 0, currentTokens - 1);
@@ -149,7 +169,8 @@ private:
   buddy_hip_model_shape shape_;
   buddy_hip_session *session_ = nullptr;
   int position_ = 0;
-  int rows_ = 0; // rows of logits_ that are valid
+  int rows_ = 0;        // rows of logits_ that are valid
+  bool folder_ = false; // loaded from a model folder
   std::vector<float> logits_;
 };
 

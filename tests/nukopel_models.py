@@ -47,7 +47,7 @@ SIZES = {
                    linear(decay=(0.0, 0.3, 1.0, 0.999, 0.7), dim=9, vdim=5,
                           mlp=moe(experts=3, top=3, ff=17, shared_ff=0))],
                   width=44, vocab=37, taps=6, embed=1.0),
-    "round": config([latent(heads=4, dim=64, rot=32, vdim=64, rank=128, window=64,
+    "even": config([latent(heads=4, dim=64, rot=32, vdim=64, rank=128, window=64,
                             mlp=moe(experts=8, top=2, ff=64, shared_ff=128)),
                      linear(decay=(0.9, 0.99), dim=64, vdim=64,
                             mlp=moe(experts=8, top=1, ff=128, shared_ff=64))],
@@ -57,9 +57,19 @@ SIZES = {
     "wide_heads": config([latent(heads=2, dim=96, rot=64, vdim=136, rank=150, window=40),
                           latent(heads=1, dim=40, rot=16, vdim=270, rank=64, window=25),
                           linear(decay=(0.97, 0.4), dim=130, vdim=140)], width=96),
+    # rows of other lengths than multiples of four, and of thousands of values
+    "width_46": config([latent(mlp=moe(experts=3, top=2, ff=11, shared_ff=6)), linear()], width=46),
+    "width_2600": config([latent(heads=1), linear(decay=(0.9,))], width=2600),
+    "width_4400": config([latent(heads=1, mlp=moe(experts=2, top=1, ff=2100, shared_ff=70))], width=4400),
+    "width_8300": config([linear(decay=(0.9,), mlp=None)], width=8300, vocab=33),
     "many_experts": config([linear(mlp=moe(experts=70, top=6, ff=8, shared_ff=8)),
                             latent(mlp=moe(experts=130, top=9, ff=4, shared_ff=20))], width=64),
 }
+# sizes at which the prompt kernels take their large tiles; for a long prompt
+LARGE = config([latent(heads=24, dim=128, rot=64, vdim=128, rank=160, window=300,
+                       mlp=moe(experts=4, top=2, ff=2100, shared_ff=2100)),
+                linear(decay=(0.9, 0.99, 0.999), dim=128, vdim=128, mlp=None)], width=256, vocab=300)
+
 # every expert is chosen, so no rounding can choose another one
 _all = moe(experts=3, top=3)
 STEADY = config([latent(mlp=_all), linear(mlp=_all), latent(window=7, heads=2, mlp=_all),

@@ -73,6 +73,18 @@ def test_prompt_and_decoding_match_the_oracle(tmp_path, name, dtype):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
+def test_long_prompt_at_real_head_sizes(tmp_path, dtype):
+    cfg = M.LARGE
+    folder, t = M.build(tmp_path, cfg)
+    tokens = tokens_for(cfg, 1100)
+    want = N.forward(cfg, t, tokens)
+    s = FolderSession(folder, dtype, max_len=1200)
+    check(all_rows(s, tokens), want, dtype, "prompt")
+    got = feed(s, tokens, [700, 384] + [1] * 16)
+    check(got, want, dtype, "portions, then decoding")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("what", ["latent", "linear", "experts", "shared", "convolution"])
 def test_mechanism_alone(tmp_path, what, dtype):
     """One layer, the head an identity: the logits are the normed residual."""
@@ -278,7 +290,7 @@ def test_long_decoding_by_the_greedy_entry_point(tmp_path, dtype):
 
 
 def test_captured_steps_equal_launched_ones_bit_for_bit(tmp_path):
-    cfg = M.SIZES["round"]
+    cfg = M.SIZES["even"]
     folder, _ = M.build(tmp_path, cfg)
     tokens = tokens_for(cfg, 40)
     s = FolderSession(folder, "bfloat16", max_len=64)
