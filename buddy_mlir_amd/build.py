@@ -27,9 +27,9 @@ TRACE_SRC = PKG / "runner" / "trace_run.cpp"
 TRACE_RUNNER = LIBDIR / "trace_run"
 # what a session built from a model folder consists of
 FOLDER_MODEL_SOURCES = [CSRC / n for n in (
-    "bf16_gemm.hip", "bf16_gemv.hip", "common.cpp", "elementwise.hip", "latent_attn.hip",
-    "linear_attn.hip", "model_folder.cpp", "model_registry.cpp", "row_ops.hip", "session.hip",
-    "session_nukopel.hip")]
+    "bf16_gemm.hip", "bf16_gemv.hip", "common.cpp", "delta_rule.hip", "elementwise.hip",
+    "head_attn.hip", "latent_attn.hip", "linear_attn.hip", "model_folder.cpp", "model_registry.cpp",
+    "row_ops.hip", "session.hip", "session_lirulix.hip", "session_nukopel.hip")]
 
 ARCH = "gfx950"
 # -packed-fp32-ops off: scalar float code must not be turned into v_pk_*_f32.

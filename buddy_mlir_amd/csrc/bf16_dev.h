@@ -5,6 +5,12 @@
 
 namespace bh {
 
+// How a gate and an up value become one.
+enum GatedAct {
+  kActClamped = 0, // g = min(g, limit), u = clamp(u, +-limit): g * sigmoid(1.702 g) * (u + 1)
+  kActGeluTanh = 1 // gelu(g) * u, the tanh form of gelu
+};
+
 typedef float f32x4 __attribute__((ext_vector_type(4)));
 typedef unsigned u32x4 __attribute__((ext_vector_type(4)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
@@ -24,10 +30,17 @@ __device__ __forceinline__ unsigned pack_bf(float a, float b) {
 }
 __device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f(float z) { return z * sigmoid_f(z); }
+// z * (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))) / 2, by (1 + tanh(y)) / 2 = sigmoid(2 y)
+__device__ __forceinline__ float gelu_tanh_f(float z) {
+  return z * sigmoid_f(1.59576912160573071f * fmaf(0.044715f * z * z, z, z));
+}
 __device__ __forceinline__ float expert_act(float g, float u, float limit) {
   g = fminf(g, limit);
   u = fminf(fmaxf(u, -limit), limit);
   return g * sigmoid_f(1.702f * g) * (u + 1.0f);
+}
+__device__ __forceinline__ float gated_act(GatedAct act, float g, float u, float limit) {
+  return act == kActGeluTanh ? gelu_tanh_f(g) * u : expert_act(g, u, limit);
 }
 
 // an element of an activation buffer

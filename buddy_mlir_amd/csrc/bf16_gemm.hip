@@ -27,6 +27,7 @@ struct GemmDev {
   int rows, K, groups; // groups of one matrix
   int ring_base, ring_mask;
   int silu_channels;
+  GatedAct act;
   float limit;
   const int *counts, *lists;
   int experts, list_cap, list_div;
@@ -231,7 +232,7 @@ rows_gemm_kernel(const uint4 *__restrict__ W, int ktiles, int steps, GemmDev a) 
         const f32x4 up = acc[g + kGroups][r];
 #pragma unroll
         for (int j = 0; j < 4; ++j)
-          v[j] = expert_act(v[j], up[j], a.limit);
+          v[j] = gated_act(a.act, v[j], up[j], a.limit);
         store4<T>(static_cast<T *>(a.C) + (int64_t)orow * a.ldc + ch, v);
       } else if constexpr (OUT == kOutF32) {
 #pragma unroll
@@ -263,6 +264,7 @@ int launch_variant(const RowsGemm &a, hipStream_t stream) {
   d.ring_base = a.ring_base;
   d.ring_mask = a.ring_mask;
   d.silu_channels = a.silu_channels;
+  d.act = a.act;
   d.limit = a.limit;
   d.counts = a.counts;
   d.lists = a.lists;

@@ -77,6 +77,8 @@ struct RowTail { // arguments a wavefront needs only behind its first loads
   int *max_i;
   float eps, out_gain, gain;
   int taps, silu_channels, valid;
+  const float *add, *norm_w;
+  GatedAct act;
 };
 
 __device__ __forceinline__ f32x4 load4(const float *p) { return *reinterpret_cast<const f32x4 *>(p); }
@@ -126,6 +128,12 @@ struct RowPrologue {
       } else if constexpr (INPUT == kRowGated) {
         w[r] = load4(a.weight + i);
         c[0][r] = load4(a.gate + i);
+      } else if constexpr (INPUT == kRowResidual) {
+        if (yp)
+          y[r] = load4(yp + i);
+        if (a.add)
+          c[0][r] = load4(a.add + i);
+        w[r] = load4(a.norm_w + i);
       }
     }
   }
@@ -148,6 +156,28 @@ struct RowPrologue {
 #pragma unroll
         for (int j = 0; j < 4; ++j)
           x[r][j] = x[r][j] * g * w[r][j] * sigmoid_f(c[0][r][j]);
+    } else if constexpr (INPUT == kRowResidual) {
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          if (yp)
+            x[r][j] += y[r][j];
+          if (a.add)
+            x[r][j] += c[0][r][j];
+        }
+        if (keeper && a.x_out && in[r])
+          save4(a.x_out + at[r], x[r]);
+      }
+      const float g = 1.0f / sqrtf(block_sum(squares(x), red[1]) / (float)K + a.eps);
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          x[r][j] = x[r][j] * g * w[r][j];
+        if (keeper && a.row_out && in[r])
+          save4(a.row_out + at[r], x[r]);
+      }
     } else if constexpr (INPUT == kRowNorm) {
       if (yp) {
         const float ry = a.out_gain / sqrtf(block_sum(squares(y), red[0]) / (float)K + a.eps);
@@ -218,6 +248,14 @@ struct RowPrologue<INPUT, 0> {
           if (keeper && a.x_out)
             a.x_out[i] = v;
         }
+        if constexpr (INPUT == kRowResidual) {
+          if (yp)
+            v += yp[i];
+          if (a.add)
+            v += a.add[i];
+          if (keeper && a.x_out)
+            a.x_out[i] = v;
+        }
         act[i] = v;
         ss = fmaf(v, v, ss);
       }
@@ -230,6 +268,11 @@ struct RowPrologue<INPUT, 0> {
         h = act[i] * scale;
         if constexpr (INPUT == kRowGated)
           h *= a.weight[i] * sigmoid_f(a.gate[i]);
+        if constexpr (INPUT == kRowResidual) {
+          h *= a.norm_w[i];
+          if (keeper && a.row_out)
+            a.row_out[i] = h;
+        }
         if constexpr (INPUT == kRowNorm) {
           if (a.conv_w) {
             const float raw = h;
@@ -248,9 +291,10 @@ struct RowPrologue<INPUT, 0> {
 };
 
 // Grid: workgroups of 8 wavefronts = (8 >> ks_shift) channel groups x (1 <<
-// ks_shift) slices of k that meet in LDS in slice order.  kRowNorm: one workgroup
-// more, which multiplies nothing and stores what the row leaves behind.
-template <int INPUT, int R>
+// ks_shift) slices of k that meet in LDS in slice order.  kRowNorm, kRowResidual: one
+// workgroup more, which multiplies nothing and stores what the row leaves behind.
+// GATED: neighbouring channel groups are group i of one matrix and of the other.
+template <int INPUT, int R, bool GATED>
 __global__ void __launch_bounds__(kRowThreads)
 row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src,
                 const float *__restrict__ y, const float *conv_next, int K, int ktiles, int groups,
@@ -263,7 +307,7 @@ row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src,
   // the row's values first: loads return in order, and these come from the L2
   RowPrologue<INPUT, R> row;
   row.request(src, y, conv_next, K, a);
-  if (INPUT == kRowNorm && blockIdx.x == gridDim.x - 1) {
+  if ((INPUT == kRowNorm || INPUT == kRowResidual) && blockIdx.x == gridDim.x - 1) {
     row.finish(act, K, Kp, a, true, red);
     return;
   }
@@ -272,7 +316,7 @@ row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src,
   const int g = blockIdx.x * (kRowWaves >> ks_shift) + (wave >> ks_shift);
   const int gl = min(g, groups - 1); // a wavefront past the last group repeats it and stores nothing
   const int t0 = slice * slice_tiles, t1 = min(t0 + slice_tiles, ktiles);
-  const uint4 *wp = W + (int64_t)gl * ktiles * 64 + lane;
+  const uint4 *wp = W + (int64_t)(GATED ? (gl & 1) * (groups >> 1) + (gl >> 1) : gl) * ktiles * 64 + lane;
   uint4 w[kAhead];
 #pragma unroll
   for (int u = 0; u < kAhead; ++u)
@@ -305,6 +349,19 @@ row_gemv_kernel(const uint4 *__restrict__ W, const float *__restrict__ src,
     part[wave][lane] = acc;
   __syncthreads();
   const int gi = tid >> 4;
+  if constexpr (GATED) {
+    if (gi < (kRowWaves >> ks_shift) / 2) {
+      const int go = blockIdx.x * ((kRowWaves >> ks_shift) / 2) + gi;
+      float vg = 0.f, vu = 0.f;
+      for (int s = 0; s < (1 << ks_shift); ++s) {
+        vg += part[((2 * gi) << ks_shift) + s][tid & 15];
+        vu += part[((2 * gi + 1) << ks_shift) + s][tid & 15];
+      }
+      if (go < groups / 2)
+        a.out[go * 16 + (tid & 15)] = gated_act(a.act, vg, vu, 0.f);
+    }
+    return;
+  }
   if (gi < (kRowWaves >> ks_shift)) {
     const int go = blockIdx.x * (kRowWaves >> ks_shift) + gi;
     float v = 0.f;
@@ -568,52 +625,61 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
   BH_REQUIRE(a.input != kRowGated || (a.weight && a.gate), "row_gemv: gate operands");
   BH_REQUIRE(a.x_out == nullptr || a.x_out != a.src, "row_gemv: the row is read by every workgroup");
   BH_REQUIRE(!a.max_v || a.max_i, "row_gemv: maxima without indices");
+  BH_REQUIRE(a.input != kRowResidual || a.norm_w, "row_gemv: no norm weight");
+  BH_REQUIRE(!a.gated || (a.input == kRowResidual && W.N % 32 == 0 && !a.max_v && a.act == kActGeluTanh),
+             "row_gemv: gated form");
   // slices of k: doubled while the launch has fewer than 2048 wavefronts and each
   // keeps four tiles
   const int groups = W.groups();
   int ks = 1;
-  while (ks < kRowWaves && (int64_t)groups * ks < 2048 && W.ktiles / (2 * ks) >= 4)
+  while (ks < (a.gated ? kRowWaves / 2 : kRowWaves) && (int64_t)groups * ks < 2048 && W.ktiles / (2 * ks) >= 4)
     ks *= 2;
   const int shift = shift_for(ks), per = kRowWaves >> shift;
   const int slice_tiles = (int)ceil_div(W.ktiles, ks);
   const size_t lds = sizeof(float) * (size_t)W.ktiles * kBfTileK;
   BH_REQUIRE(lds <= 150 * 1024, "row_gemv: a row of %d values does not fit LDS", W.K);
   RowTail t{a.x_out, a.row_out, a.conv_w, a.conv_ring, a.conv_next, a.pos, a.weight, a.gate,
-            a.out, a.max_v, a.max_i, a.eps, a.out_gain, a.gain, a.taps, a.silu_channels, a.valid};
-  const bool keeper = a.input == kRowNorm;
+            a.out, a.max_v, a.max_i, a.eps, a.out_gain, a.gain, a.taps, a.silu_channels, a.valid,
+            a.add, a.norm_w, a.act};
+  const bool keeper = a.input == kRowNorm || a.input == kRowResidual;
   const dim3 grid((unsigned)(ceil_div(groups, per) + keeper)), block(kRowThreads);
   bool quads = W.K % 4 == 0;
   for (const void *p : {(const void *)a.src, (const void *)a.y, (const void *)a.x_out,
                         (const void *)a.row_out, (const void *)a.conv_w, (const void *)a.conv_next,
-                        (const void *)a.weight, (const void *)a.gate})
+                        (const void *)a.weight, (const void *)a.gate, (const void *)a.add,
+                        (const void *)a.norm_w})
     quads = quads && ((uintptr_t)p & 15) == 0;
   const int span = W.ktiles * kBfTileK; // the padding is written too
   const int regs = !quads || span > 8192 ? 0 : span <= 2048 ? 1 : span <= 4096 ? 2 : 4;
-#define BH_ROW(I, R)                                                                             \
+#define BH_ROW(I, R, G)                                                                          \
   do {                                                                                           \
     static DynLdsOnce once;                                                                      \
-    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)row_gemv_kernel<I, R>, 150 * 1024));         \
-    hipLaunchKernelGGL((row_gemv_kernel<I, R>), grid, block, lds, stream, W.tiles, a.src, a.y,   \
+    BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)row_gemv_kernel<I, R, G>, 150 * 1024));       \
+    hipLaunchKernelGGL((row_gemv_kernel<I, R, G>), grid, block, lds, stream, W.tiles, a.src, a.y,\
                        a.conv_w ? a.conv_next : nullptr, W.K, W.ktiles, groups, shift,           \
                        slice_tiles, t);                                                          \
   } while (0)
-#define BH_ROWS(I)                                                                               \
+#define BH_ROWS(I, G)                                                                            \
   do {                                                                                           \
     if (regs == 1)                                                                               \
-      BH_ROW(I, 1);                                                                              \
+      BH_ROW(I, 1, G);                                                                           \
     else if (regs == 2)                                                                          \
-      BH_ROW(I, 2);                                                                              \
+      BH_ROW(I, 2, G);                                                                           \
     else if (regs == 4)                                                                          \
-      BH_ROW(I, 4);                                                                              \
+      BH_ROW(I, 4, G);                                                                           \
     else                                                                                         \
-      BH_ROW(I, 0);                                                                              \
+      BH_ROW(I, 0, G);                                                                           \
   } while (0)
   if (a.input == kRowPlain)
-    BH_ROWS(kRowPlain);
+    BH_ROWS(kRowPlain, false);
   else if (a.input == kRowNorm)
-    BH_ROWS(kRowNorm);
+    BH_ROWS(kRowNorm, false);
+  else if (a.input == kRowGated)
+    BH_ROWS(kRowGated, false);
+  else if (a.gated)
+    BH_ROWS(kRowResidual, true);
   else
-    BH_ROWS(kRowGated);
+    BH_ROWS(kRowResidual, false);
 #undef BH_ROWS
 #undef BH_ROW
   BH_CHECK_HIP(hipGetLastError());

@@ -9,7 +9,7 @@
 // the order (j, L/16) the A operands of eight v_mfma_f32_16x16x4_f32.
 #pragma once
 
-#include "common.h"
+#include "bf16_dev.h"
 
 namespace bh {
 
@@ -39,7 +39,8 @@ enum RowInput {
   kRowNorm = 1,    // x' = src + y * (out_gain / rms(y)) (src alone without y), then
                    // x' * (gain / rms(x')), then, with conv_w, itself plus its
                    // causal convolution over the ring of earlier rows
-  kRowGated = 2    // (src / rms(src)) * weight * sigmoid(gate)
+  kRowGated = 2,   // (src / rms(src)) * weight * sigmoid(gate)
+  kRowResidual = 3 // x' = src + y + add (each may be missing), then x' / rms(x') * norm_w
 };
 struct RowGemv {
   Bf16Matrix W;
@@ -58,6 +59,12 @@ struct RowGemv {
   const int *pos = nullptr;       // device: position of the row
   // kRowGated
   const float *weight = nullptr, *gate = nullptr;
+  // kRowResidual (also eps, y, x_out, row_out)
+  const float *add = nullptr, *norm_w = nullptr;
+  // kRowResidual: W holds two matrices of N / 2 channels, the second one behind the
+  // first; out [N / 2] = gated activation of the two
+  bool gated = false;
+  GatedAct act = kActGeluTanh;
   // output: channels below silu_channels go through silu
   float *out = nullptr;
   int silu_channels = 0;
@@ -98,7 +105,7 @@ enum GemmOut {
   kOutF32 = 0,       // C f32 [rows][ldc]
   kOutAct = 1,       // C in A's type [rows][ldc]
   kOutActTrans = 2,  // C in A's type [N][ldc], a row per channel
-  kOutExpertAct = 3  // two matrices: the clamped gated activation, A's type [rows][ldc]
+  kOutExpertAct = 3  // two matrices: the gated activation of both, A's type [rows][ldc]
 };
 struct RowsGemm {
   Bf16Matrix W;               // kOutExpertAct: N channels each, second one behind the first
@@ -112,7 +119,8 @@ struct RowsGemm {
   void *C = nullptr;
   int ldc = 0;
   int silu_channels = 0;      // kOutF32: these first channels go through silu
-  float limit = 0.f;          // kOutExpertAct
+  GatedAct act = kActClamped; // kOutExpertAct
+  float limit = 0.f;
   // Grouped form: matrix e applies to the rows listed for it.  lists[e][i] is an
   // assignment id; it reads A row id / list_div and writes C row id.
   int experts = 0;

@@ -33,10 +33,11 @@ int launch_finish_step(const float *cand_v, const int *cand_i, int nparts, int *
                        int *token_log, const float *table, int64_t hidden, int64_t vocab,
                        float *x, const float *inv_freq, int head_dim, float *rope,
                        bool advance, int token_log_cap, hipStream_t stream);
-// The same over a bfloat16 table whose rows are scaled, without an angle table.
+// The same over a bfloat16 table whose rows are scaled or, with norm_w ([hidden]),
+// normed: row / rms(row) * norm_w; without an angle table.
 int launch_finish_step_bf16(const float *cand_v, const int *cand_i, int nparts, int *state,
                             int *token_log, const uint16_t *table, float table_scale,
-                            int64_t hidden, int64_t vocab, float *x, bool advance,
-                            int token_log_cap, hipStream_t stream);
+                            const float *norm_w, float eps, int64_t hidden, int64_t vocab, float *x,
+                            bool advance, int token_log_cap, hipStream_t stream);
 
 } // namespace bh

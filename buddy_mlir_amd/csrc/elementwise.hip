@@ -138,14 +138,15 @@ argmax_final_kernel(const float *__restrict__ pv, const int *__restrict__ pi,
 // candidates, logs it, advances position and step, then prepares the next step:
 // its embedding row and the cos/sin table of its position (shared by every
 // layer's attention kernel).  One workgroup.
-// Table: f32 rows as they are, or bfloat16 rows times a scale.
+// Table: f32 rows as they are, or bfloat16 rows times a scale or normed.
 template <typename Table>
 __global__ void __launch_bounds__(1024)
 finish_step_kernel(const float *__restrict__ pv, const int *__restrict__ pi,
                    int nparts, int *__restrict__ state, int *__restrict__ token_log,
                    const Table *__restrict__ table, float table_scale, int64_t hidden,
                    int64_t vocab, float *__restrict__ x, const float *__restrict__ inv_freq,
-                   int half, float *__restrict__ rope, int advance, int log_cap) {
+                   int half, float *__restrict__ rope, int advance, int log_cap,
+                   const float *__restrict__ norm_w, float eps) {
   __shared__ float sv[16];
   __shared__ int si[16];
   __shared__ int s_tok, s_pos;
@@ -213,9 +214,30 @@ finish_step_kernel(const float *__restrict__ pv, const int *__restrict__ pi,
   if (t < 0 || t >= vocab)
     t = 0;
   const Table *row = table + t * hidden;
+  float gain = table_scale;
+  if constexpr (sizeof(Table) == 2) {
+    if (norm_w) {
+      float ss = 0.f;
+      for (int64_t i = threadIdx.x; i < hidden; i += threads) {
+        const float v = __uint_as_float((unsigned)row[i] << 16);
+        ss = fmaf(v, v, ss);
+      }
+      ss = wave_sum(ss);
+      __syncthreads(); // the candidates have been read
+      if ((threadIdx.x & 63) == 0)
+        sv[threadIdx.x >> 6] = ss;
+      __syncthreads();
+      ss = 0.f;
+      for (int w = 0; w < threads / 64; ++w)
+        ss += sv[w];
+      gain = 1.0f / sqrtf(ss / (float)hidden + eps);
+    }
+  }
   for (int64_t i = threadIdx.x; i < hidden; i += threads) {
     if constexpr (sizeof(Table) == 4)
       x[i] = row[i];
+    else if (norm_w)
+      x[i] = __uint_as_float((unsigned)row[i] << 16) * gain * norm_w[i];
     else
       x[i] = __uint_as_float((unsigned)row[i] << 16) * table_scale;
   }
@@ -238,21 +260,22 @@ int launch_finish_step(const float *cand_v, const int *cand_i, int nparts, int *
              "finish_step: bad argument");
   hipLaunchKernelGGL(finish_step_kernel<float>, dim3(1), dim3(nparts > 1024 ? 1024 : 256), 0,
                      stream, cand_v, cand_i, nparts, state, token_log, table, 1.0f, hidden, vocab,
-                     x, inv_freq, head_dim / 2, rope, advance ? 1 : 0, token_log_cap);
+                     x, inv_freq, head_dim / 2, rope, advance ? 1 : 0, token_log_cap,
+                     (const float *)nullptr, 0.f);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }
 
 int launch_finish_step_bf16(const float *cand_v, const int *cand_i, int nparts, int *state,
                             int *token_log, const uint16_t *table, float table_scale,
-                            int64_t hidden, int64_t vocab, float *x, bool advance,
-                            int token_log_cap, hipStream_t stream) {
+                            const float *norm_w, float eps, int64_t hidden, int64_t vocab, float *x,
+                            bool advance, int token_log_cap, hipStream_t stream) {
   BH_REQUIRE(state && table && x && (nparts == 0 || (cand_v && cand_i && token_log)),
              "finish_step: bad argument");
   hipLaunchKernelGGL(finish_step_kernel<uint16_t>, dim3(1), dim3(nparts > 1024 ? 1024 : 256), 0,
                      stream, cand_v, cand_i, nparts, state, token_log, table, table_scale, hidden,
                      vocab, x, (const float *)nullptr, 0, (float *)nullptr, advance ? 1 : 0,
-                     token_log_cap);
+                     token_log_cap, norm_w, eps);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }

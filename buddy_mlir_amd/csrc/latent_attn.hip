@@ -8,20 +8,13 @@
 // two bfloat16 terms each (17 bits), all summed in f32.
 #include "latent_attn.h"
 #include "bf16_dev.h"
+#include "flash_tile.h"
+#include "rotary.h"
 
 #include <algorithm>
 
 namespace bh {
 namespace {
-
-// cos and sin of position * turns (turns of the full circle per position); the
-// product is reduced to a fraction of a turn in double, so a far position keeps
-// its 32-bit angle
-__device__ __forceinline__ void rotation(double turns, int p, float &c, float &s) {
-  double t = turns * (double)p;
-  t -= rint(t);
-  sincospif(2.0f * (float)t, &s, &c);
-}
 
 constexpr int kStepThreads = 512, kStepWaves = 8;
 
@@ -459,38 +452,26 @@ struct LatentAttnArgs {
   int kd; // elements of a query
 };
 
-// Keys of a tile: 128 bytes of a V^T row.
-template <typename T> struct KeyTile {
-  static constexpr int kKeys = 128 / (int)sizeof(T);
-};
-
 // Grid (heads, query blocks).  A wavefront owns 16 queries, the workgroup's four
 // share tiles of kKeys keys through LDS; the next tile is on its way in registers
-// meanwhile.  S^T = K . Q^T leaves a lane with keys of one query, which is the B
-// operand of O^T += V^T . P^T as it lies (of 32 keys in bfloat16: a lane's eight are
-// keys 4q .. 4q + 3 of both halves, and V^T rows are stored in that order).
+// meanwhile.
 // NK: 32-element steps of a key, NV: 16-channel groups of a value, at most; smaller
 // heads are padded with zeros (keys) or with rows whose results are not stored
 // (values), so that the loop has no branches.
-//
-// The running maximum a lane subtracts follows the scores only when one exceeds it by
-// more than kSlack: the weights stay below e^kSlack, and the sums are rescaled a few
-// times per query instead of once per tile.
 template <typename T, int NK, int NV>
 __global__ void __launch_bounds__(256, NV <= 8 ? 2 : 1)
 latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ keys,
                         const T *__restrict__ values_t, const T *__restrict__ cache,
                         const float *__restrict__ proj, T *__restrict__ out, LatentAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) unsigned char raw[];
-  constexpr int E = 16 / (int)sizeof(T), KEYS = KeyTile<T>::kKeys, SUB = KEYS / 16;
+  constexpr int E = 16 / (int)sizeof(T), KEYS = KeyTile<T>::kKeys;
   constexpr int KL = NK, VL = (NV + 1) / 2; // 16-byte loads per thread and tile
   const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = blockIdx.x;
   constexpr int kBlock = 64;
   const int q0 = (gridDim.y - 1 - blockIdx.y) * kBlock; // long blocks first
-  constexpr int kKeyRow = NK * 32 + E, kValueRow = KEYS + E; // rows start 4 banks apart
-  constexpr float kSlack = 8.0f;
+  constexpr int kKeyRow = Flash<T, NK, NV>::kKeyRow, kValueRow = Flash<T, NK, NV>::kValueRow;
   T *kt = reinterpret_cast<T *>(raw); // [KEYS][kKeyRow]
   T *vt = kt + KEYS * kKeyRow;        // [16 * NV][kValueRow]
 
@@ -535,8 +516,7 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
     const int id = min(i * 256 + tid, vruns - 1), r = id >> 3, c = id & 7;
     vsrc[i] = values_t + (int64_t)(h * 16 * a.nv + r) * a.value_ld + c * E;
     vcol[i] = c * E;
-    // bfloat16: the run's two halves of four keys go to their places in the lane order
-    vdst[i] = r * kValueRow + (sizeof(T) == 2 ? (c >> 2) * 32 + (c & 1) * 16 + ((c >> 1) & 1) * 4 : c * E);
+    vdst[i] = Flash<T, NK, NV>::value_at(r, c);
   }
   u32x4 kr[KL], vr[VL];
   auto fetch = [&](int k0, u32x4 (&kr)[KL], u32x4 (&vr)[VL]) {
@@ -557,11 +537,7 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       kt[(i / pad) * kKeyRow + at + i % pad] = 0;
   }
 
-  f32x4 o[NV];
-  float m = -INFINITY, l = 0.f;
-#pragma unroll
-  for (int v = 0; v < NV; ++v)
-    o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+  Flash<T, NK, NV> flash;
   for (int k0 = key_lo; k0 <= key_hi; k0 += KEYS) {
     __syncthreads(); // the previous tile has been read
 #pragma unroll
@@ -581,139 +557,16 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       }
     }
 #pragma unroll
-    for (int i = 0; i < VL; ++i) {
-      if constexpr (sizeof(T) == 2) {
-        *reinterpret_cast<uint2 *>(vt + vdst[i]) = uint2{vr[i][0], vr[i][1]};
-        *reinterpret_cast<uint2 *>(vt + vdst[i] + 8) = uint2{vr[i][2], vr[i][3]};
-      } else {
-        *reinterpret_cast<u32x4 *>(vt + vdst[i]) = vr[i];
-      }
-    }
+    for (int i = 0; i < VL; ++i)
+      Flash<T, NK, NV>::store_value(vt, vdst[i], vr[i]);
     __syncthreads();
     fetch(min(k0 + KEYS, (nkeys - 1) & ~(KEYS - 1)), kr, vr);
     if (k0 > wave_q1 || k0 + KEYS - 1 <= wave_q0 - a.window)
       continue; // nothing of this tile is visible to this wavefront
-    f32x4 s[SUB];
-#pragma unroll
-      for (int b = 0; b < SUB; ++b)
-        s[b] = f32x4{0.f, 0.f, 0.f, 0.f};
-    // the fragments of the next step are read while this one is multiplied
-    const T *kp = kt + col * kKeyRow + quad * 8;
-    Frag<T> kf[2][SUB];
-#pragma unroll
-    for (int b = 0; b < SUB; ++b)
-      kf[0][b].load(kp + b * 16 * kKeyRow);
-#pragma unroll
-    for (int t = 0; t < NK; ++t) {
-      if (t + 1 < NK) {
-#pragma unroll
-        for (int b = 0; b < SUB; ++b)
-          kf[(t + 1) & 1][b].load(kp + b * 16 * kKeyRow + (t + 1) * 32);
-      }
-      __builtin_amdgcn_sched_barrier(0);
-#pragma unroll
-      for (int b = 0; b < SUB; ++b)
-        s[b] = mfma32(kf[t & 1][b], qf[t], s[b]);
-      __builtin_amdgcn_sched_barrier(0);
-    }
     const bool whole = k0 + KEYS - 1 <= wave_q0 && wave_q1 - k0 < a.window;
-    if (!whole) {
-#pragma unroll
-      for (int b = 0; b < SUB; ++b)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int gap = my_q - (k0 + b * 16 + quad * 4 + r);
-          s[b][r] = gap >= 0 && gap < a.window ? s[b][r] : -INFINITY;
-        }
-    }
-    float mt = s[0][0];
-#pragma unroll
-    for (int b = 0; b < SUB; ++b)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        mt = fmaxf(mt, s[b][r]);
-    float x, y;
-    lane_pair<16>(mt, x, y);
-    mt = fmaxf(x, y);
-    lane_pair<32>(mt, x, y);
-    mt = fmaxf(x, y);
-    if (__any(mt > m + kSlack)) { // -inf + kSlack stays below every score
-      mt = fmaxf(mt, m);
-      const float alpha = mt == -INFINITY ? 1.f : fast_exp(m - mt);
-      m = mt;
-      l *= alpha;
-#pragma unroll
-      for (int v = 0; v < NV; ++v)
-#pragma unroll
-        for (int r = 0; r < 4; ++r)
-          o[v][r] *= alpha;
-    }
-    const float base = m == -INFINITY ? 0.f : m; // nothing visible so far
-#pragma unroll
-    for (int b = 0; b < SUB; ++b)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        s[b][r] = fast_exp(s[b][r] - base);
-        l += s[b][r];
-      }
-    if constexpr (sizeof(T) == 2) {
-      // the weights as two bfloat16 terms
-      uint4 hi[SUB / 2], lo[SUB / 2];
-#pragma unroll
-        for (int b = 0; b < SUB / 2; ++b) {
-          unsigned ph[4], pl[4];
-#pragma unroll
-          for (int j = 0; j < 4; ++j) {
-            const f32x4 &x = s[2 * b + (j >> 1)];
-            const float x0 = x[2 * (j & 1)], x1 = x[2 * (j & 1) + 1];
-            ph[j] = pack_bf(x0, x1);
-            pl[j] = pack_bf(x0 - bf_lo(ph[j]), x1 - bf_hi(ph[j]));
-          }
-          hi[b] = uint4{ph[0], ph[1], ph[2], ph[3]};
-          lo[b] = uint4{pl[0], pl[1], pl[2], pl[3]};
-        }
-      constexpr int G = NV < 4 ? NV : 4; // value tiles read ahead
-      const T *vp = vt + col * kValueRow + quad * 8;
-      Frag<T> vf[2][G][SUB / 2];
-#pragma unroll
-      for (int v = 0; v < G; ++v)
-#pragma unroll
-        for (int b = 0; b < SUB / 2; ++b)
-          vf[0][v][b].load(vp + v * 16 * kValueRow + b * 32);
-#pragma unroll
-      for (int v0 = 0; v0 < NV; v0 += G) {
-        if (v0 + G < NV) {
-#pragma unroll
-          for (int v = 0; v < G; ++v)
-#pragma unroll
-            for (int b = 0; b < SUB / 2; ++b)
-              vf[(v0 / G + 1) & 1][v][b].load(vp + (v0 + G + v) * 16 * kValueRow + b * 32);
-        }
-        __builtin_amdgcn_sched_barrier(0);
-#pragma unroll
-        for (int b = 0; b < SUB / 2; ++b) {
-#pragma unroll
-          for (int v = 0; v < G; ++v)
-            o[v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, hi[b], o[v0 + v]);
-#pragma unroll
-          for (int v = 0; v < G; ++v)
-            o[v0 + v] = mfma_bf16(vf[(v0 / G) & 1][v][b].v, lo[b], o[v0 + v]);
-        }
-        __builtin_amdgcn_sched_barrier(0);
-      }
-    } else {
-#pragma unroll
-      for (int v = 0; v < NV; ++v)
-#pragma unroll
-        for (int b = 0; b < SUB; ++b) {
-          const f32x4 vv = *reinterpret_cast<const f32x4 *>(vt + (v * 16 + col) * kValueRow + b * 16 + quad * 4);
-#pragma unroll
-          for (int r = 0; r < 4; ++r)
-            o[v] = mfma_f32(vv[r], s[b][r], o[v]);
-        }
-    }
+    flash.tile(kt, vt, qf, whole, my_q - k0, a.window);
   }
-  const float sum = sum_rows(l);
+  const float sum = sum_rows(flash.l);
   if (qi >= a.rows)
     return;
   const float f = sigmoid_f(proj[(int64_t)qi * a.ld + a.gate_at + h]) / sum;
@@ -725,7 +578,7 @@ latent_attention_kernel(const T *__restrict__ queries, const T *__restrict__ key
       for (int r = 0; r < 4; ++r) {
         const int c = v * 16 + quad * 4 + r;
         if (c < a.vdim)
-          store_act<T>(dst + c, o[v][r] * f);
+          store_act<T>(dst + c, flash.o[v][r] * f);
       }
     }
 }

@@ -88,6 +88,15 @@ ModelFolder::~ModelFolder() {
     munmap(map_, map_bytes_);
 }
 
+int ModelFolder::size(const std::string &name, size_t axis) const {
+  const auto it = tensors_.find(name);
+  if (it == tensors_.end())
+    throw std::runtime_error("no tensor " + name);
+  if (axis >= it->second.shape.size() || it->second.shape[axis] <= 0 || it->second.shape[axis] > (1 << 24))
+    throw std::runtime_error("tensor " + name + " has shape " + shape_text(it->second.shape));
+  return (int)it->second.shape[axis];
+}
+
 const TensorView &ModelFolder::bf16(const std::string &name, const std::vector<int64_t> &shape) const {
   const auto it = tensors_.find(name);
   if (it == tensors_.end())

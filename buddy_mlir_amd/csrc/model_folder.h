@@ -36,6 +36,8 @@ public:
   const Json &config() const { return config_; }
   std::string architecture() const { return config_.at("architecture").string(); }
   bool has(const std::string &name) const { return tensors_.count(name) != 0; }
+  // a size that only the tensor's shape gives
+  int size(const std::string &name, size_t axis) const;
   // the tensor, which must be bfloat16 of exactly this shape
   const TensorView &bf16(const std::string &name, const std::vector<int64_t> &shape) const;
   // a bfloat16 tensor of one element

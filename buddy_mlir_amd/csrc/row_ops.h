@@ -6,12 +6,15 @@
 
 namespace bh {
 
-// x[r] = scale * table[token[r]] (bfloat16 table)
+// x[r] = scale * table[token[r]] (bfloat16 table); with norm_w ([width]) then
+// x[r] / rms(x[r]) * norm_w
 int launch_embed_rows(const uint16_t *table, const int *tokens, int rows, int width, int vocab,
-                      float scale, float *x, hipStream_t stream);
+                      float scale, const float *norm_w, float eps, float *x, hipStream_t stream);
 
 // Per row: x' = x + y * (out_gain / rms(y)), then x' * (gain / rms(x')).  y may be
-// missing, a row, or a row plus the weighted outputs of the row's experts.
+// missing, a row, or a row plus the weighted outputs of the row's experts.  `plain_y`:
+// x' = x + y.  `add`: one row that is added to every x' as well.  `norm_w`: a weight
+// per channel on the normed row.
 struct NormRows {
   float *x = nullptr;            // [rows][width]
   bool write_x = false;          // x' goes back into x
@@ -21,6 +24,8 @@ struct NormRows {
   const float *expert_w = nullptr;   // [rows][top]
   int lde = 0, top = 0;
   float out_gain = 1.f, gain = 1.f, eps = 0.f;
+  bool plain_y = false;
+  const float *add = nullptr, *norm_w = nullptr; // [width]
   int rows = 0, width = 0;
   const int *pick = nullptr;     // output row r is made from row pick[r]; `rows` counts outputs
   float *out_f32 = nullptr;      // [rows][width]

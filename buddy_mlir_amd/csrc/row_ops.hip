@@ -8,24 +8,37 @@
 namespace bh {
 namespace {
 
-__global__ void __launch_bounds__(256)
-embed_rows_kernel(const uint16_t *__restrict__ table, const int *__restrict__ tokens, int width,
-                  int vocab, float scale, float *__restrict__ x) {
-  int t = tokens[blockIdx.x];
-  if (t < 0 || t >= vocab)
-    t = 0;
-  const uint16_t *row = table + (int64_t)t * width;
-  float *dst = x + (int64_t)blockIdx.x * width;
-  for (int i = threadIdx.x; i < width; i += 256)
-    dst[i] = bf_f(row[i]) * scale;
-}
-
 __device__ __forceinline__ float block_sum4(float v, float *red) {
   v = wave_sum(v);
   if ((threadIdx.x & 63) == 0)
     red[threadIdx.x >> 6] = v;
   __syncthreads();
   return (red[0] + red[1]) + (red[2] + red[3]);
+}
+
+__global__ void __launch_bounds__(256)
+embed_rows_kernel(const uint16_t *__restrict__ table, const int *__restrict__ tokens, int width,
+                  int vocab, float scale, const float *__restrict__ norm_w, float eps,
+                  float *__restrict__ x) {
+  __shared__ float red[4];
+  int t = tokens[blockIdx.x];
+  if (t < 0 || t >= vocab)
+    t = 0;
+  const uint16_t *row = table + (int64_t)t * width;
+  float *dst = x + (int64_t)blockIdx.x * width;
+  if (norm_w) {
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < width; i += 256) {
+      const float v = bf_f(row[i]) * scale;
+      ss = fmaf(v, v, ss);
+    }
+    const float g = scale / sqrtf(block_sum4(ss, red) / (float)width + eps);
+    for (int i = threadIdx.x; i < width; i += 256)
+      dst[i] = bf_f(row[i]) * g * norm_w[i];
+    return;
+  }
+  for (int i = threadIdx.x; i < width; i += 256)
+    dst[i] = bf_f(row[i]) * scale;
 }
 
 // V consecutive values of a row at a time: 4 where every row is 16-byte aligned, else 1
@@ -65,7 +78,7 @@ __global__ void __launch_bounds__(256) norm_rows_kernel(NormRows a) {
   const int64_t r = a.pick ? a.pick[blockIdx.x] : blockIdx.x;
   float *x = a.x + r * W;
   float *xb = lds, *yb = lds + W;
-  const bool pending = a.y || a.expert_out;
+  const bool pending = a.y || a.expert_out || a.add;
   float ss = 0.f;
   for (int i = tid; i < W; i += 256 * V) {
     store_run<V>(xb + i, load_run<V>(x + i));
@@ -80,6 +93,12 @@ __global__ void __launch_bounds__(256) norm_rows_kernel(NormRows a) {
         for (int k = 0; k < V; ++k)
           y.v[k] = fmaf(w, e.v[k], y.v[k]);
       }
+      if (a.add) { // (only with plain_y)
+        const Run<V> e = load_run<V>(a.add + i);
+#pragma unroll
+        for (int k = 0; k < V; ++k)
+          y.v[k] += e.v[k];
+      }
       store_run<V>(yb + i, y);
 #pragma unroll
       for (int k = 0; k < V; ++k)
@@ -88,7 +107,7 @@ __global__ void __launch_bounds__(256) norm_rows_kernel(NormRows a) {
   }
   float sx = 0.f;
   if (pending) {
-    const float ry = a.out_gain / sqrtf(block_sum4(ss, red[0]) / (float)W + a.eps);
+    const float ry = a.plain_y ? 1.0f : a.out_gain / sqrtf(block_sum4(ss, red[0]) / (float)W + a.eps);
     for (int i = tid; i < W; i += 256 * V) {
       Run<V> v = load_run<V>(xb + i);
       const Run<V> y = load_run<V>(yb + i);
@@ -114,6 +133,12 @@ __global__ void __launch_bounds__(256) norm_rows_kernel(NormRows a) {
 #pragma unroll
     for (int k = 0; k < V; ++k)
       v.v[k] *= g;
+    if (a.norm_w) {
+      const Run<V> w = load_run<V>(a.norm_w + i);
+#pragma unroll
+      for (int k = 0; k < V; ++k)
+        v.v[k] *= w.v[k];
+    }
     if (a.out_f32)
       store_run<V>(a.out_f32 + (int64_t)blockIdx.x * W + i, v);
     if (a.out_act)
@@ -267,24 +292,25 @@ route_list_kernel(const int *__restrict__ chosen, int total, int *__restrict__ c
 } // namespace
 
 int launch_embed_rows(const uint16_t *table, const int *tokens, int rows, int width, int vocab,
-                      float scale, float *x, hipStream_t stream) {
+                      float scale, const float *norm_w, float eps, float *x, hipStream_t stream) {
   BH_REQUIRE(table && tokens && x && rows > 0 && width > 0 && vocab > 0, "embed_rows: bad argument");
   hipLaunchKernelGGL(embed_rows_kernel, dim3(rows), dim3(256), 0, stream, table, tokens, width,
-                     vocab, scale, x);
+                     vocab, scale, norm_w, eps, x);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }
 
 int launch_norm_rows(const NormRows &a, hipStream_t stream) {
   BH_REQUIRE(a.x && a.rows > 0 && a.width > 0 && (!a.pick || !a.write_x) &&
-                 (!a.expert_out || (a.expert_w && a.top > 0)) && (a.expert_out || a.top == 0),
+                 (!a.expert_out || (a.expert_w && a.top > 0)) && (a.expert_out || a.top == 0) &&
+                 (!a.add || a.plain_y),
              "norm_rows: bad argument");
   const size_t lds = 2 * sizeof(float) * (size_t)a.width;
   constexpr size_t kLimit = 150 * 1024;
   BH_REQUIRE(lds <= kLimit, "norm_rows: a row of %d values does not fit LDS", a.width);
   bool quads = a.width % 4 == 0 && a.ldy % 4 == 0 && a.lde % 4 == 0 && a.ld_act % 4 == 0;
   for (const void *p : {(const void *)a.x, (const void *)a.y, (const void *)a.expert_out,
-                        (const void *)a.out_f32, (const void *)a.out_act})
+                        (const void *)a.add, (const void *)a.norm_w, (const void *)a.out_f32, (const void *)a.out_act})
     quads = quads && ((uintptr_t)p & 15) == 0;
 #define BH_NORM(T, V)                                                                          \
   do {                                                                                         \

@@ -16,12 +16,10 @@
 //   [choice of experts -> gate | up -> activation] -> [down of all of them, summed]
 // The residual sum and norms that stand between two matrix products are computed by
 // every workgroup of the second one.
-#include "bf16_linear.h"
 #include "elementwise.h"
+#include "folder_session.h"
 #include "latent_attn.h"
 #include "linear_attn.h"
-#include "model_registry.h"
-#include "row_ops.h"
 
 #include <algorithm>
 #include <cmath>
@@ -34,13 +32,6 @@
 
 namespace bh {
 namespace {
-
-int positive(const Json &j, const char *key) {
-  const int64_t v = j.at(key).integer();
-  if (v <= 0 || v > (1 << 24))
-    throw std::runtime_error(std::string("config: \"") + key + "\" out of range");
-  return (int)v;
-}
 
 struct ExpertConfig {
   int ff = 0;
@@ -124,11 +115,6 @@ struct NukopelConfig {
   }
 };
 
-// One input of a fused projection: where its channels lie in the result.
-struct Part {
-  int at = 0, n = 0;
-};
-
 struct NukopelLayer {
   float norm1 = 0.f, norm1b = 0.f, norm2 = 0.f, norm2b = 0.f;
   float *conv_w = nullptr, *conv_ring = nullptr; // [taps][width] each
@@ -152,21 +138,12 @@ struct NukopelLayer {
   Bf16Matrix gate_up, down, shared_gate_up, shared_down; // of the first expert
 };
 
-int pow2_at_least(int64_t v) {
-  int p = 2;
-  while (p < v)
-    p *= 2;
-  return p;
-}
-
-struct NukopelSession : Session {
+struct NukopelSession : FolderSession {
   NukopelConfig cfg;
-  ModelOptions opt;
   std::vector<NukopelLayer> layers;
   uint16_t *embed = nullptr; // [vocab][width] bfloat16
   Bf16Matrix head;
   float final_norm = 1.f;
-  int seq_len = 0; // tokens the state holds
   int longest_window = 1;
 
   // one token
@@ -176,93 +153,21 @@ struct NukopelSession : Session {
   int *chosen = nullptr;
   int act_stride = 64;
 
-  // a block of a prompt, grown on demand to `pf_rows` rows
-  int pf_rows = 0;
-  std::vector<void *> pf_owned;
-  int *pf_tokens = nullptr, *pf_chosen = nullptr, *pf_counts = nullptr, *pf_lists = nullptr,
-      *pf_pick = nullptr;
+  // a block of a prompt
+  int *pf_chosen = nullptr, *pf_counts = nullptr, *pf_lists = nullptr;
   float *pf_x = nullptr, *pf_y = nullptr, *pf_h = nullptr, *pf_proj = nullptr, *pf_lin = nullptr,
         *pf_states = nullptr, *pf_router = nullptr, *pf_weights = nullptr, *pf_experts = nullptr,
         *pf_logits = nullptr;
   void *pf_act = nullptr, *pf_mix = nullptr, *pf_keys = nullptr, *pf_values = nullptr, *pf_queries = nullptr,
        *pf_moe = nullptr, *pf_shared = nullptr;
   int ld_act = 0, ld_mix = 0, max_proj = 0;
-  static constexpr int kLogitRows = 256; // rows of the head multiplied at once
 
-  NukopelSession(const Json &config, const ModelOptions &o) : cfg(config), opt(o) {}
-  ~NukopelSession() override {
-    if (stream)
-      (void)hipStreamSynchronize(stream);
-    free_block();
-  }
-  void free_block() {
-    for (void *p : pf_owned)
-      (void)hipFree(p);
-    pf_owned.clear();
-    pf_rows = 0;
-  }
+  NukopelSession(const Json &config, const ModelOptions &o) : FolderSession(o), cfg(config) {}
 
   const char *architecture() const override { return "Nukopel"; }
-  int ready() const override { return BUDDY_HIP_OK; }
   int width16() const { return (int)round_up(cfg.width, 16); }
 
   // ---- loading -------------------------------------------------------------------
-  // a bfloat16 tensor on the device, freed when it goes out of scope
-  struct Upload {
-    uint16_t *p = nullptr;
-    Upload(const TensorView &t, hipStream_t stream) {
-      if (hipMalloc((void **)&p, t.bytes) != hipSuccess)
-        throw std::bad_alloc();
-      if (hipMemcpyAsync(p, t.data, t.bytes, hipMemcpyHostToDevice, stream) != hipSuccess) {
-        (void)hipFree(p);
-        throw std::runtime_error("upload failed");
-      }
-    }
-    ~Upload() { (void)hipFree(p); } // waits for the work that reads it
-    Upload(const Upload &) = delete;
-    Upload &operator=(const Upload &) = delete;
-  };
-  void must(int rc) {
-    if (rc)
-      throw std::runtime_error(buddy_hip_last_error());
-  }
-  template <typename T> T *device(size_t n) {
-    T *p = nullptr;
-    must(alloc(&p, n));
-    return p;
-  }
-  template <typename T> T *device_copy(const std::vector<T> &v) {
-    T *p = device<T>(v.size());
-    if (hipMemcpy(p, v.data(), v.size() * sizeof(T), hipMemcpyHostToDevice) != hipSuccess)
-      throw std::runtime_error("upload failed");
-    return p;
-  }
-  template <typename T> T *device_zeros(size_t n) {
-    T *p = device<T>(n);
-    if (hipMemsetAsync(p, 0, n * sizeof(T), stream) != hipSuccess)
-      throw std::runtime_error("clear failed");
-    return p;
-  }
-  Bf16Matrix matrix(int64_t N, int64_t K) {
-    Bf16Matrix m;
-    m.N = (int)round_up(N, 16);
-    m.K = (int)K;
-    m.ktiles = bf16_ktiles(K);
-    m.tiles = reinterpret_cast<const uint4 *>(device<char>(bf16_tiles_bytes(K, N)));
-    return m;
-  }
-  // packs `src` (element (n, k) at n * sn + k * sk) as channels from `at` on
-  void pack(const Bf16Matrix &m, int at, const uint16_t *src, int64_t sn, int64_t sk, int64_t N) {
-    must(launch_pack_bf16(src, sn, sk, N, m.K, const_cast<uint4 *>(m.tiles) + (int64_t)(at / 16) * m.ktiles * 64,
-                          stream));
-  }
-  Bf16Matrix load_matrix(const ModelFolder &f, const std::string &name, int64_t N, int64_t K) {
-    Upload u(f.bf16(name, {N, K}), stream);
-    Bf16Matrix m = matrix(N, K);
-    pack(m, 0, u.p, K, 1, N);
-    return m;
-  }
-
   void load_mixer(const ModelFolder &f, const std::string &p, const LayerConfig &c, NukopelLayer &L) {
     const int W = cfg.width;
     std::vector<std::pair<std::string, Part *>> parts;
@@ -277,17 +182,8 @@ struct NukopelSession : Session {
       L.v.n = L.g.n = heads_v;
       parts = {{"q", &L.q}, {"k", &L.k}, {"v", &L.v}, {"g", &L.g}};
     }
-    int at = 0;
-    for (auto &part : parts) {
-      part.second->at = at;
-      at += (int)round_up(part.second->n, 16);
-    }
-    L.in = matrix(at, W);
-    for (auto &part : parts) {
-      Upload u(f.bf16(p + "mix." + part.first, {part.second->n, W}), stream);
-      pack(L.in, part.second->at, u.p, W, 1, part.second->n);
-    }
-    max_proj = std::max(max_proj, at);
+    L.in = load_parts(f, p + "mix.", parts, W);
+    max_proj = std::max(max_proj, L.in.N);
     L.o = load_matrix(f, p + "mix.o", W, heads_v);
     if (!c.latent) {
       L.silu_channels = L.g.at; // q, k and v, not the gate
@@ -361,12 +257,7 @@ struct NukopelSession : Session {
 
   void load(const ModelFolder &f) {
     const int W = cfg.width;
-    {
-      const TensorView &t = f.bf16("embed", {cfg.vocab, W});
-      embed = device<uint16_t>((size_t)cfg.vocab * W);
-      if (hipMemcpy(embed, t.data, t.bytes, hipMemcpyHostToDevice) != hipSuccess)
-        throw std::runtime_error("upload failed");
-    }
+    embed = device_bf16(f.bf16("embed", {cfg.vocab, W}));
     head = load_matrix(f, "head", cfg.vocab, W);
     final_norm = f.scalar("final.norm");
     int mix_max = 1, e16 = 16, query = 0, parts = 0, parts_ml = 0, top = 1;
@@ -443,27 +334,8 @@ struct NukopelSession : Session {
     seq_len = 0;
     return BUDDY_HIP_OK;
   }
-  int seek(int pos) override {
-    if (pos == 0)
-      return seq_len == 0 ? BUDDY_HIP_OK : reset();
-    BH_REQUIRE(pos == seq_len,
-               "Nukopel: position %d asked for, but the state holds %d tokens (continue there, or "
-               "begin at 0)",
-               pos, seq_len);
-    return BUDDY_HIP_OK;
-  }
-  void stepped() override { ++seq_len; }
-
   // ---- one token -------------------------------------------------------------------
-  // Keys the attention launches cover: the number of visible ones rounded up to a
-  // quarter of a power of two, so that a few captured steps serve all positions.
-  int step_span(int pos) const {
-    const int need = std::min(pos + 1, longest_window);
-    int unit = 64;
-    while (unit * 8 <= need)
-      unit *= 2;
-    return (int)round_up(need, unit);
-  }
+  int step_span(int pos) const { return key_span(std::min(pos + 1, longest_window)); }
   std::pair<int, int> step_key(int pos) const override { return {step_span(pos), 0}; }
 
   int enqueue_step(int pos) override {
@@ -580,30 +452,19 @@ struct NukopelSession : Session {
     if ((rc = launch_row_gemv(g, stream)))
       return rc;
     return launch_finish_step_bf16(group_max_v, group_max_i, head.groups(), state, token_log, embed,
-                                   cfg.embed_scale, W, cfg.vocab, x[0], true, token_log_cap, stream);
+                                   cfg.embed_scale, nullptr, 0.f, W, cfg.vocab, x[0], true, token_log_cap, stream);
   }
 
   int prepare_step() override {
     return launch_finish_step_bf16(nullptr, nullptr, 0, state, token_log, embed, cfg.embed_scale,
-                                   cfg.width, cfg.vocab, x[0], false, token_log_cap, stream);
+                                   nullptr, 0.f, cfg.width, cfg.vocab, x[0], false, token_log_cap, stream);
   }
 
   // ---- many tokens -----------------------------------------------------------------
-  template <typename T> int block_alloc(T **p, size_t bytes) {
-    void *q = nullptr;
-    BH_CHECK_HIP(hipMalloc(&q, std::max<size_t>(bytes, 16)));
-    pf_owned.push_back(q);
-    *p = static_cast<T *>(q);
-    return BUDDY_HIP_OK;
-  }
   static int key_cap(const LatentShape &s, int rows) {
     return (int)round_up((int64_t)std::min(s.window - 1, s.ring_mask + 1) + rows, kLatentKeyTile);
   }
-  int ensure_block(int rows) {
-    if (rows <= pf_rows)
-      return BUDDY_HIP_OK;
-    BH_CHECK_HIP(hipStreamSynchronize(stream));
-    free_block();
+  int alloc_block(int rows) override {
     const size_t n = (size_t)rows, T = opt.f32 ? 4 : 2;
     size_t keys = 0, values = 0, queries = 0, lin = 0, states = 0, e16 = 0, top = 0, experts = 0, moe = 0, shared = 0;
     for (size_t i = 0; i < layers.size(); ++i) {
@@ -626,8 +487,7 @@ struct NukopelSession : Session {
         shared = std::max(shared, n * round_up(c.shared_expert.ff, 16));
       }
     }
-    int rc = block_alloc(&pf_tokens, 4 * n);
-    rc |= block_alloc(&pf_x, 4 * n * cfg.width);
+    int rc = block_alloc(&pf_x, 4 * n * cfg.width);
     rc |= block_alloc(&pf_h, 4 * n * cfg.width);
     rc |= block_alloc(&pf_y, 4 * n * width16());
     rc |= block_alloc(&pf_act, T * n * ld_act);
@@ -646,26 +506,8 @@ struct NukopelSession : Session {
     rc |= block_alloc(&pf_moe, T * moe);
     rc |= block_alloc(&pf_shared, T * shared);
     rc |= block_alloc(&pf_experts, 4 * n * top * width16());
-    rc |= block_alloc(&pf_pick, 4 * n);
     rc |= block_alloc(&pf_logits, 4 * (size_t)std::min(rows, kLogitRows) * head.N);
-    if (rc)
-      return rc;
-    pf_rows = rows;
-    return BUDDY_HIP_OK;
-  }
-
-  RowsGemm gemm(const Bf16Matrix &W, const void *A, int lda, int rows, GemmOut out, void *C,
-                int ldc) const {
-    RowsGemm g;
-    g.W = W;
-    g.A = A;
-    g.lda = lda;
-    g.f32 = opt.f32;
-    g.rows = rows;
-    g.out = out;
-    g.C = C;
-    g.ldc = ldc;
-    return g;
+    return rc;
   }
 
   int latent_rows(NukopelLayer &L, int n, int start) {
@@ -787,11 +629,9 @@ struct NukopelSession : Session {
     return BUDDY_HIP_OK;
   }
 
-  // One block of tokens (in pf_tokens) through all layers; the rows listed go on to
-  // the head.
-  int run_block(int n, int start, const int *rows, int n_rows, float *dst) {
+  int run_block(int n, int start, const int *rows, int n_rows, float *dst) override {
     int rc;
-    if ((rc = launch_embed_rows(embed, pf_tokens, n, cfg.width, cfg.vocab, cfg.embed_scale, pf_x, stream)))
+    if ((rc = launch_embed_rows(embed, pf_tokens, n, cfg.width, cfg.vocab, cfg.embed_scale, nullptr, 0.f, pf_x, stream)))
       return rc;
     NormRows pend; // residual and norm, with the output x does not hold yet
     pend.x = pf_x;
@@ -856,65 +696,8 @@ struct NukopelSession : Session {
     }
     if (n_rows == 0)
       return BUDDY_HIP_OK;
-    BH_CHECK_HIP(hipMemcpyAsync(pf_pick, rows, sizeof(int) * n_rows, hipMemcpyHostToDevice, stream));
     pend.gain = final_norm;
-    if (n_rows == 1) {
-      pend.rows = 1;
-      pend.pick = pf_pick;
-      pend.out_f32 = hrow;
-      if ((rc = launch_norm_rows(pend, stream)))
-        return rc;
-      RowGemv g;
-      g.W = head;
-      g.src = hrow;
-      g.out = logits;
-      if ((rc = launch_row_gemv(g, stream)))
-        return rc;
-      if (dst != logits)
-        BH_CHECK_HIP(hipMemcpyAsync(dst, logits, sizeof(float) * vocab, hipMemcpyDeviceToDevice, stream));
-      return BUDDY_HIP_OK;
-    }
-    for (int r0 = 0; r0 < n_rows; r0 += kLogitRows) {
-      const int m = std::min(kLogitRows, n_rows - r0);
-      NormRows p = pend;
-      p.rows = m;
-      p.pick = pf_pick + r0;
-      p.out_act = pf_act;
-      if ((rc = launch_norm_rows(p, stream)))
-        return rc;
-      if ((rc = launch_rows_gemm(gemm(head, pf_act, ld_act, m, kOutF32, pf_logits, head.N), stream)))
-        return rc;
-      BH_CHECK_HIP(hipMemcpy2DAsync(dst + (size_t)r0 * vocab, sizeof(float) * vocab, pf_logits,
-                                    sizeof(float) * head.N, sizeof(float) * vocab, m,
-                                    hipMemcpyDeviceToDevice, stream));
-    }
-    return BUDDY_HIP_OK;
-  }
-
-  int prefill_rows(const int *tokens, int n, int start, const int *rows, int n_rows,
-                   float *dst) override {
-    int rc;
-    if ((rc = seek(start)))
-      return rc;
-    if ((rc = ensure_block(std::min(n, opt.prefill_block))))
-      return rc;
-    next_pos = -1; // the device's position is the one of the last decode step
-    int done_rows = 0;
-    std::vector<int> local;
-    for (int at = 0; at < n; at += opt.prefill_block) {
-      const int m = std::min(opt.prefill_block, n - at);
-      local.clear();
-      while (done_rows + (int)local.size() < n_rows && rows[done_rows + local.size()] < at + m)
-        local.push_back(rows[done_rows + local.size()] - at);
-      BH_CHECK_HIP(hipMemcpyAsync(pf_tokens, tokens + at, sizeof(int) * m, hipMemcpyDefault, stream));
-      if ((rc = run_block(m, start + at, local.data(), (int)local.size(),
-                          dst ? dst + (size_t)done_rows * vocab : nullptr)))
-        return rc;
-      BH_CHECK_HIP(hipStreamSynchronize(stream)); // `local` is reused
-      done_rows += (int)local.size();
-      seq_len = start + at + m;
-    }
-    return BUDDY_HIP_OK;
+    return logit_rows(pend, head, rows, n_rows, hrow, pf_act, pf_logits, dst);
   }
 };
 
