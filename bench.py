@@ -3,7 +3,7 @@
 MI355X, next to the CPU oracle timed on the same host.
 
     python bench.py [--gpus 1] [--steps K] [--warmup W]
-    python bench.py --workload gemv|mlp|prefill|llama8b|kvdiscard|w4a16|model_abi|sampler|quantize|nukopel   (the other configurations)
+    python bench.py --workload gemv|mlp|prefill|llama8b|kvdiscard|w4a16|model_abi|sampler|quantize|nukopel|lirulix   (the other configurations)
 
 A step is one greedy decode step (one token) at batch 1 with the KV cache
 already holding 1024 positions; weights, KV cache and activations are resident
@@ -965,38 +965,64 @@ def _nukopel_step_bytes(cfg, context):
     return total
 
 
+def _decode_seconds(s, first, context, args):
+    """One greedy step of a session that holds `context` tokens."""
+    import torch
+
+    K, W = args.steps, max(1, args.warmup)
+    s.use_graph(not args.no_graph)
+    s.set_state(first, context)
+    s.enqueue_steps(W)
+    stream = torch.cuda.ExternalStream(s.stream)
+    stream.synchronize()
+    t0 = time.perf_counter()
+    s.enqueue_steps(K)
+    stream.synchronize()
+    return (time.perf_counter() - t0) / K
+
+
+def _prefill_seconds(s, toks, n=5):
+    s.prefill(toks, 0, want_logits=False)
+    t0 = time.perf_counter()
+    for _ in range(n):
+        s.prefill(toks, 0, want_logits=False)
+    return (time.perf_counter() - t0) / n
+
+
+def _folder_model_times(write, cfg, toks, prompts, step_bytes, args):
+    """Prompts and one decode step of a model folder with random weights."""
+    import tempfile
+
+    from buddy_mlir_amd.session import FolderSession
+
+    d = {}
+    with tempfile.TemporaryDirectory() as tmp:
+        write(tmp, cfg)
+        s = FolderSession(tmp, "bfloat16", max_len=4096)
+    for n in prompts:
+        t = _prefill_seconds(s, toks[:n])
+        d[f"prefill_{n}"] = {"ms": t * 1e3, "tokens_per_s": n / t}
+    s.prefill(toks[:CONTEXT], 0, want_logits=False)
+    t = _decode_seconds(s, int(toks[0]), CONTEXT, args)
+    b = step_bytes(cfg, CONTEXT)
+    d["decode"] = {"ms": t * 1e3, "tokens_per_s": 1 / t, "algorithmic_bytes": b,
+                   "hbm_frac": b / t / 1e9 / HBM_PEAK_GBPS}
+    s.close()
+    return d
+
+
 def bench_nukopel(bh, args):
     """Prefill and decode throughput of the Nukopel session at layers of real models'
     sizes, beside the Qwen2-shaped w8a32 session of equal width, depth, heads,
     vocabulary and feed-forward units per token."""
-    import tempfile
-
     import torch
 
     from buddy_mlir_amd import synthetic
-    from buddy_mlir_amd.session import FolderSession, Shape
+    from buddy_mlir_amd.session import Shape
 
     K, W = args.steps, max(1, args.warmup)
     prompts = (512, 2048)
     detail = {}
-
-    def decode_s(s, first, context):
-        s.use_graph(not args.no_graph)
-        s.set_state(first, context)
-        s.enqueue_steps(W)
-        stream = torch.cuda.ExternalStream(s.stream)
-        stream.synchronize()
-        t0 = time.perf_counter()
-        s.enqueue_steps(K)
-        stream.synchronize()
-        return (time.perf_counter() - t0) / K
-
-    def prefill_s(s, toks, n=5):
-        s.prefill(toks, 0, want_logits=False)
-        t0 = time.perf_counter()
-        for _ in range(n):
-            s.prefill(toks, 0, want_logits=False)
-        return (time.perf_counter() - t0) / n
 
     for name in args.nukopel_sizes.split(","):
         mine, other = NUKOPEL_SIZES[name]
@@ -1004,23 +1030,13 @@ def bench_nukopel(bh, args):
         shape = Shape(vocab=cfg["vocab"], max_len=4096, **other)
         toks = synthetic.first_tokens(shape, max(prompts))
         d = detail[name] = {"config": mine, "qwen2": other}
-        with tempfile.TemporaryDirectory() as tmp:
-            synthetic.write_nukopel_folder(tmp, cfg)
-            s = FolderSession(tmp, "bfloat16", max_len=4096)
-        for n in prompts:
-            t = prefill_s(s, toks[:n])
-            d[f"prefill_{n}"] = {"ms": t * 1e3, "tokens_per_s": n / t}
-        s.prefill(toks[:CONTEXT], 0, want_logits=False)
-        t = decode_s(s, int(toks[0]), CONTEXT)
-        b = _nukopel_step_bytes(cfg, CONTEXT)
-        d["decode"] = {"ms": t * 1e3, "tokens_per_s": 1 / t, "algorithmic_bytes": b,
-                       "hbm_frac": b / t / 1e9 / HBM_PEAK_GBPS}
-        s.close()
+        d.update(_folder_model_times(synthetic.write_nukopel_folder, cfg, toks, prompts,
+                                     _nukopel_step_bytes, args))
         q, _ = synthetic.build_session(shape, context=CONTEXT)
         for n in prompts:
-            t = prefill_s(q, toks[:n])
+            t = _prefill_seconds(q, toks[:n])
             d[f"qwen2_prefill_{n}"] = {"ms": t * 1e3, "tokens_per_s": n / t}
-        t = decode_s(q, int(toks[0]), CONTEXT)
+        t = _decode_seconds(q, int(toks[0]), CONTEXT, args)
         b = decode_step_bytes(shape, CONTEXT)
         d["qwen2_decode"] = {"ms": t * 1e3, "tokens_per_s": 1 / t, "algorithmic_bytes": b,
                              "hbm_frac": b / t / 1e9 / HBM_PEAK_GBPS}
@@ -1040,6 +1056,69 @@ def bench_nukopel(bh, args):
     }
 
 
+# Layers of real models, and for each a Nukopel model of the same width, number of layers
+# (attention and linear ones alike), heads, vocabulary and feed-forward units per token.
+LIRULIX_SIZES = {
+    "w1536": (dict(width=1536, layers="fdsf", heads=12, kv_heads=2, window=1024, ff=8960), "w1536"),
+    "w4096": (dict(width=4096, layers="fds", heads=32, kv_heads=8, window=4096, ff=10240), "w4096"),
+}
+
+
+def _lirulix_step_bytes(cfg, context):
+    """Weights, cache rows and states one decoded token reads or writes (bfloat16
+    weights and cache, f32 state)."""
+    from math import prod
+
+    from buddy_mlir_amd import synthetic
+
+    total = 2 * sum(prod(s) for n, s, _ in synthetic.lirulix_shapes(cfg) if n != "embed")
+    for layer in cfg["layers"]:
+        m = layer["mixer"]
+        if layer["type"] == "channel_delta":
+            total += 2 * 4 * m["heads"] * m["dim"] * m["vdim"]
+        else:
+            maps = 2 if layer["type"] == "attention_2" else 1
+            keys = min(context, m["mask"]["size"]) if "mask" in m else context
+            total += 2 * keys * m["kv_heads"] * (maps * m["dim"] + m["vdim"])
+    return total
+
+
+def bench_lirulix(bh, args):
+    """Prefill and decode throughput of the Lirulix session at layers of real models'
+    sizes, beside a Nukopel session of equal size."""
+    import numpy as np
+
+    from buddy_mlir_amd import synthetic
+
+    K, W = args.steps, max(1, args.warmup)
+    prompts = (512, 2048)
+    detail = {}
+    for name in args.lirulix_sizes.split(","):
+        mine, other = LIRULIX_SIZES[name]
+        other = NUKOPEL_SIZES[other][0]
+        cfg, ncfg = synthetic.lirulix_config(**mine), synthetic.nukopel_config(**other)
+        toks = np.random.default_rng(1).integers(0, cfg["vocab"], max(prompts))
+        detail[name] = {
+            "config": mine,
+            **_folder_model_times(synthetic.write_lirulix_folder, cfg, toks, prompts,
+                                  _lirulix_step_bytes, args),
+            "nukopel": {"config": other,
+                        **_folder_model_times(synthetic.write_nukopel_folder, ncfg, toks, prompts,
+                                              _nukopel_step_bytes, args)}}
+    lead = detail[next(iter(detail))]["decode"]
+    return {
+        "metric": "lirulix_decode_tokens_per_s", "value": lead["tokens_per_s"], "unit": "tokens/s",
+        "n_gpus": 1, "steps": K, "warmup": W, "ms_per_step": lead["ms"], "higher_is_better": True,
+        "scaling": "weak", "vs_baseline": None, "dtype": "bf16", "data": "synthetic",
+        "config": {"workload": "Lirulix layers (attention with a sink, differential attention, gated "
+                               "delta rule, dense feed-forward), random weights: one greedy decode "
+                               "step at context 1024 and prompts of 512 and 2048 tokens, beside a "
+                               "Nukopel model of equal size",
+                   "context": CONTEXT, "hip_graph": not args.no_graph},
+        "detail": detail,
+    }
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1047,13 +1126,15 @@ def main():
     ap.add_argument("--warmup", type=int, default=8)
     ap.add_argument("--workload", default="decode",
                     choices=["decode", "gemv", "mlp", "prefill", "llama8b", "kvdiscard", "w4a16",
-                             "model_abi", "sampler", "quantize", "nukopel"],
+                             "model_abi", "sampler", "quantize", "nukopel", "lirulix"],
                     help="decode (default): the full decode step the headline metric "
                          "is quoted on; the others measure the remaining configurations")
     ap.add_argument("--mlp-rows", default="1,4,16",
                     help="--workload mlp: the row counts to time (1..16, comma separated)")
     ap.add_argument("--nukopel-sizes", default=",".join(NUKOPEL_SIZES),
                     help="--workload nukopel: which of the sizes to run")
+    ap.add_argument("--lirulix-sizes", default=",".join(LIRULIX_SIZES),
+                    help="--workload lirulix: which of the sizes to run")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--no-graph", action="store_true")
     ap.add_argument("--calibrate-copy", action="store_true",
@@ -1078,7 +1159,8 @@ def main():
         fn = {"gemv": bench_gemv, "mlp": bench_mlp, "prefill": bench_prefill,
               "llama8b": bench_llama8b, "kvdiscard": bench_kvdiscard, "w4a16": bench_w4a16,
               "model_abi": bench_model_abi, "sampler": bench_sampler,
-              "quantize": bench_quantize, "nukopel": bench_nukopel}[args.workload]
+              "quantize": bench_quantize, "nukopel": bench_nukopel,
+              "lirulix": bench_lirulix}[args.workload]
         print(json.dumps(fn(bh, args)))
         return
     K, W = args.steps, args.warmup

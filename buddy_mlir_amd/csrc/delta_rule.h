@@ -5,7 +5,7 @@
 // Everything behind the projections is f32.
 #pragma once
 
-#include "common.h"
+#include "bf16_linear.h"
 
 namespace bh {
 
@@ -23,6 +23,9 @@ struct DeltaShape {
   const float *decay_bias = nullptr; // [heads * dim]
   const float *decay_speed = nullptr; // [heads]: log g = decay_speed * softplus(. + bias)
   const float *norm_w = nullptr;      // [vdim]
+  Bf16Matrix decay, gate;             // the same two matrices for many rows
+  int dim32() const { return (int)round_up(dim, 32); }
+  int vdim16() const { return (int)round_up(vdim, 16); }
 };
 
 struct DeltaRows {
@@ -38,5 +41,12 @@ struct DeltaRows {
 };
 // Token by token: a step of decoding, short portions.
 int launch_delta_scan(const DeltaRows &a, hipStream_t stream);
+
+// A prompt in chunks of kDeltaChunk tokens.  Within a chunk the writes are solved for as
+// one triangular system; the state goes from chunk to chunk.
+constexpr int kDeltaChunk = 64;
+// floats of scratch for `rows` tokens; 0: the state's size is not one the chunks take
+size_t delta_workspace(const DeltaShape &s, int rows);
+int launch_delta_chunks(const DeltaRows &a, float *workspace, hipStream_t stream);
 
 } // namespace bh

@@ -1,4 +1,16 @@
-// delta_rule.hip -- the gated delta rule, token by token.
+// delta_rule.hip -- the gated delta rule: token by token, and a prompt in chunks.
+//
+// Chunks of 64 tokens, four blocks of 16.  With G_t the product of the decays from the
+// chunk's first token to t (per key channel) and S0 the state ahead of the chunk, the
+// writes u solve
+//   u_t + beta_t sum_{s<t} a_ts u_s = beta_t (v_t - S0^T (G_t k_t)),
+//   a_ts = sum_d k_t k_s G_t / G_s,
+// so u = U - W S0 with W and U free of the state, and
+//   o_t = S0^T (G_t q_t) + sum_{s<=t} b_ts u_s,   b_ts = sum_d q_t k_s G_t / G_s,
+//   S = diag(G_last) S0 + sum_s (G_last / G_s k_s) u_s^T.
+// Quotients of G are taken of logarithms that are summed within a block, and between
+// blocks through the border of the later one, so that every factor is at most 1 however
+// strong a decay is.  f32 throughout.
 #include "delta_rule.h"
 #include "bf16_dev.h"
 
@@ -187,12 +199,469 @@ delta_keep_kernel(const float *__restrict__ proj, int ld, int rows, int start, i
     ring[(int64_t)((start + rows - b) % taps) * channels + c] = proj[(int64_t)(rows - b) * ld + c];
 }
 
+int keep_rows(const DeltaRows &a, hipStream_t stream) {
+  const DeltaShape &s = a.s;
+  if (s.taps > 1)
+    hipLaunchKernelGGL(delta_keep_kernel, dim3((unsigned)ceil_div(s.channels, 64)), dim3(64), 0, stream,
+                       a.proj, a.ld, a.rows, a.start, s.taps, s.channels, a.ring);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
+}
+
 bool delta_ok(const DeltaRows &a) {
   const DeltaShape &s = a.s;
   return a.proj && a.ring && a.state && a.out && a.rows > 0 && (!a.pos || a.rows == 1) && s.heads > 0 &&
          s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim > 0 && s.vdim > 0 && s.taps > 0 &&
          s.decay_rank > 0 && s.gate_rank > 0 && s.channels > 0 && s.conv_w && s.decay_w && s.gate_w &&
          s.decay_bias && s.decay_speed && s.norm_w;
+}
+
+
+// ---- chunks ------------------------------------------------------------------------
+
+constexpr int kC = kDeltaChunk, kBlock = 16, kBlocks = kC / kBlock;
+constexpr int kChunkThreads = 512;
+constexpr float kLog2e = 1.44269504088896341f;
+__device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
+
+// Where the parts of a chunk and head lie in the workspace, in floats.
+struct ChunkParts {
+  int dp, v16;                     // dim32, vdim16
+  int w, q, kt, b, ut, last, size; // W, G q: [64][dim32]; (G_last / G k)^T: [dim32][64]; b: [64][64];
+                                   // U^T, later u^T: [vdim16][64]; G_last: [dim32]
+};
+ChunkParts chunk_parts(const DeltaShape &s) {
+  const int d = kC * s.dim32();
+  ChunkParts p;
+  p.dp = s.dim32();
+  p.v16 = s.vdim16();
+  p.w = 0;
+  p.q = d;
+  p.kt = 2 * d;
+  p.b = 3 * d;
+  p.ut = p.b + kC * kC;
+  p.last = p.ut + kC * s.vdim16();
+  p.size = p.last + s.dim32();
+  return p;
+}
+
+struct DeltaPrepArgs {
+  DeltaShape s;
+  const float *proj, *ring;
+  int ld, rows, start;
+  float *conv; // [rows][channels]
+  float *dots; // [rows][kv_heads]: q . k
+};
+
+// A wavefront per row and head: convolution and silu of a query and key head, made unit
+// vectors, or of a value head.
+__global__ void __launch_bounds__(256) delta_prep_kernel(DeltaPrepArgs a) {
+  const DeltaShape &s = a.s;
+  const int lane = threadIdx.x & 63;
+  const int64_t id = (int64_t)blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int units = s.kv_heads + s.heads;
+  if (id >= (int64_t)a.rows * units)
+    return;
+  const int r = (int)(id / units), u = (int)(id - (int64_t)r * units), p = a.start + r;
+  const float *row = a.proj + (int64_t)r * a.ld;
+  float *out = a.conv + (int64_t)r * s.channels;
+  if (u >= s.kv_heads) {
+    const int at = s.v_at + (u - s.kv_heads) * s.vdim;
+    for (int i = lane; i < s.vdim; i += 64)
+      out[at + i] = short_conv(s, row, a.ld, r, a.ring, p, at + i);
+    return;
+  }
+  const int qa = s.q_at + u * s.dim, ka = s.k_at + u * s.dim;
+  float qq = 0.f, kk = 0.f, qk = 0.f;
+  constexpr int kKeep = 4; // values a lane keeps in registers
+  float qv[kKeep], kv[kKeep];
+#pragma unroll
+  for (int j = 0; j < kKeep; ++j) {
+    const int i = lane + j * 64;
+    qv[j] = kv[j] = 0.f;
+    if (i < s.dim) {
+      qv[j] = short_conv(s, row, a.ld, r, a.ring, p, qa + i);
+      kv[j] = short_conv(s, row, a.ld, r, a.ring, p, ka + i);
+    }
+    qq = fmaf(qv[j], qv[j], qq);
+    kk = fmaf(kv[j], kv[j], kk);
+    qk = fmaf(qv[j], kv[j], qk);
+  }
+  const float rq = 1.0f / sqrtf(wave_sum(qq) + kUnitEps) / sqrtf((float)s.dim);
+  const float rk = 1.0f / sqrtf(wave_sum(kk) + kUnitEps);
+  qk = wave_sum(qk);
+#pragma unroll
+  for (int j = 0; j < kKeep; ++j) {
+    const int i = lane + j * 64;
+    if (i < s.dim) {
+      out[qa + i] = qv[j] * rq;
+      out[ka + i] = kv[j] * rk;
+    }
+  }
+  if (lane == 0)
+    a.dots[(int64_t)r * s.kv_heads + u] = qk * rq * rk;
+}
+
+struct DeltaChunkArgs {
+  DeltaShape s;
+  const float *conv, *dots, *decay; // decay: [rows][ld_decay], before bias and softplus
+  const float *proj;
+  int ld, ld_decay, rows;
+  float *parts;
+  ChunkParts at;
+};
+
+// Grid (chunks, heads): everything about a chunk that does not need the state.
+__global__ void __launch_bounds__(kChunkThreads) delta_chunk_kernel(DeltaChunkArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const DeltaShape &s = a.s;
+  const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int c = blockIdx.x, h = blockIdx.y, g = h / (s.heads / s.kv_heads);
+  const int dim = s.dim, dp = a.at.dp, row_at = dp + 4;
+  constexpr int kARow = kC + 4;
+  float *ks = lds;                  // [64][row_at]
+  float *qs = ks + kC * row_at;     // [64][row_at]
+  float *gs = qs + kC * row_at;     // [64][row_at]: log2 decay, summed from the block's first token
+  float *as = gs + kC * row_at;     // [64][kARow]: beta_t a_ts
+  float *tot = as + kC * kARow;     // [kBlocks][dp]: a block's sum
+  float *beta = tot + kBlocks * dp; // [64]
+  const int r0 = c * kC, rows = min(kC, a.rows - r0);
+  float *out = a.parts + ((int64_t)c * s.heads + h) * a.at.size;
+  {
+    const float speed = s.decay_speed[h] * kLog2e;
+    const float *conv = a.conv + (int64_t)r0 * s.channels;
+    for (int i = tid; i < kC * dp; i += kChunkThreads) {
+      const int r = i / dp, d = i - r * dp;
+      float k = 0.f, q = 0.f, l = 0.f; // a row past the last: no write, no decay
+      if (r < rows && d < dim) {
+        k = conv[(int64_t)r * s.channels + s.k_at + g * dim + d];
+        q = conv[(int64_t)r * s.channels + s.q_at + g * dim + d];
+        l = speed * softplus_f(a.decay[(int64_t)(r0 + r) * a.ld_decay + h * dim + d] + s.decay_bias[h * dim + d]);
+        l = fmaxf(l, -200.f); // 2^-200 is no f32 number: the same as none left
+      }
+      ks[r * row_at + d] = k;
+      qs[r * row_at + d] = q;
+      gs[r * row_at + d] = l;
+    }
+    if (tid < kC)
+      beta[tid] = tid < rows ? sigmoid_f(a.proj[(int64_t)(r0 + tid) * a.ld + s.beta_at + h]) : 0.f;
+  }
+  for (int i = tid; i < kC * kARow; i += kChunkThreads)
+    as[i] = 0.f;
+  __syncthreads();
+  for (int i = tid; i < kBlocks * dp; i += kChunkThreads) {
+    const int b = i / dp, d = i - b * dp;
+    float *p = gs + b * kBlock * row_at + d, v[kBlock];
+#pragma unroll
+    for (int t = 0; t < kBlock; ++t)
+      v[t] = p[t * row_at];
+#pragma unroll
+    for (int t = 1; t < kBlock; ++t)
+      v[t] += v[t - 1];
+#pragma unroll
+    for (int t = 0; t < kBlock; ++t)
+      p[t * row_at] = v[t];
+    tot[i] = v[kBlock - 1];
+  }
+  __syncthreads();
+  // pairs of different blocks: a product of 16 x 16 over the key channels each
+  if (wave < 6) {
+    const int bi = wave < 1 ? 1 : wave < 3 ? 2 : 3, bj = wave < 1 ? 0 : wave < 3 ? wave - 1 : wave - 3;
+    const float *kt = ks + (bi * kBlock + col) * row_at, *qt = qs + (bi * kBlock + col) * row_at;
+    const float *gt = gs + (bi * kBlock + col) * row_at;
+    const float *kr = ks + (bj * kBlock + col) * row_at, *gr = gs + (bj * kBlock + col) * row_at;
+    f32x4 sa{0.f, 0.f, 0.f, 0.f}, sb = sa;
+    for (int d0 = quad * 8; d0 < dp; d0 += 32)
+#pragma unroll
+      for (int j0 = 0; j0 < 8; j0 += 4) {
+        const int d = d0 + j0;
+        f32x4 left = *reinterpret_cast<const f32x4 *>(gt + d);
+        f32x4 right = *reinterpret_cast<const f32x4 *>(tot + bj * dp + d) - *reinterpret_cast<const f32x4 *>(gr + d);
+        for (int b = bj + 1; b < bi; ++b)
+          right += *reinterpret_cast<const f32x4 *>(tot + b * dp + d);
+        const f32x4 k = *reinterpret_cast<const f32x4 *>(kt + d), q = *reinterpret_cast<const f32x4 *>(qt + d);
+        const f32x4 w = *reinterpret_cast<const f32x4 *>(kr + d);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float l = exp2_f(left[j]), x = w[j] * exp2_f(right[j]);
+          sa = mfma_f32(k[j] * l, x, sa);
+          sb = mfma_f32(q[j] * l, x, sb);
+        }
+      }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = bi * kBlock + quad * 4 + r, x = bj * kBlock + col;
+      as[t * kARow + x] = sa[r] * beta[t];
+      out[a.at.b + t * kC + x] = sb[r];
+      out[a.at.b + x * kC + t] = 0.f;
+    }
+  }
+  // pairs within a block: a lane each, 120 of them on two wavefronts
+  {
+    const int b = wave >> 1, id = (wave & 1) * 60 + lane;
+    if (lane < 60) {
+      int t = (int)((1.0f + sqrtf((float)(8 * id + 1))) * 0.5f);
+      t -= t * (t - 1) / 2 > id;
+      t += (t + 1) * t / 2 <= id;
+      const int x = id - t * (t - 1) / 2; // x < t
+      const int tr = (b * kBlock + t) * row_at, xr = (b * kBlock + x) * row_at;
+      float sa = 0.f, sb = 0.f;
+      for (int d = 0; d < dp; d += 4) {
+        const f32x4 gap = *reinterpret_cast<const f32x4 *>(gs + tr + d) - *reinterpret_cast<const f32x4 *>(gs + xr + d);
+        const f32x4 k = *reinterpret_cast<const f32x4 *>(ks + tr + d), q = *reinterpret_cast<const f32x4 *>(qs + tr + d);
+        const f32x4 w = *reinterpret_cast<const f32x4 *>(ks + xr + d);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float e = w[j] * exp2_f(gap[j]);
+          sa = fmaf(k[j], e, sa);
+          sb = fmaf(q[j], e, sb);
+        }
+      }
+      const int ta = b * kBlock + t, xa = b * kBlock + x;
+      as[ta * kARow + xa] = sa * beta[ta];
+      out[a.at.b + ta * kC + xa] = sb;
+      out[a.at.b + xa * kC + ta] = 0.f;
+    } else {
+      // the block's own tokens, four per wavefront at a time
+      for (int t = (wave & 1) * 8 + lane - 60; t < (wave & 1) * 8 + 8; t += 4) {
+        const int r = b * kBlock + t;
+        out[a.at.b + r * kC + r] = r < rows ? a.dots[(int64_t)(r0 + r) * s.kv_heads + g] : 0.f;
+      }
+    }
+  }
+  __syncthreads();
+  auto before = [&](int b, int d) { // decay of the blocks ahead of block b
+    float v = 0.f;
+    for (int i = 0; i < b; ++i)
+      v += tot[i * dp + d];
+    return v;
+  };
+  if (wave >= 4) {
+    for (int i = tid - 256; i < kC * dp; i += 256) {
+      const int t = i / dp, d = i - t * dp;
+      out[a.at.q + i] = qs[t * row_at + d] * exp2_f(before(t / kBlock, d) + gs[t * row_at + d]);
+    }
+    for (int i = tid - 256; i < kC * dp; i += 256) {
+      const int d = i / kC, t = i - d * kC, b = t / kBlock;
+      float left = tot[b * dp + d] - gs[t * row_at + d];
+      for (int j = b + 1; j < kBlocks; ++j)
+        left += tot[j * dp + d];
+      out[a.at.kt + i] = ks[t * row_at + d] * exp2_f(left);
+    }
+    for (int d = tid - 256; d < dp; d += 256)
+      out[a.at.last + d] = exp2_f(before(kBlocks, d));
+    return;
+  }
+  // the triangular system, a thread per right-hand side
+  const int v16 = a.at.v16;
+  for (int i = tid; i < dp + v16; i += 256) {
+    float x[kC];
+    if (i < dp) {
+#pragma unroll
+      for (int b = 0; b < kBlocks; ++b) {
+        const float ahead = before(b, i);
+#pragma unroll
+        for (int t = b * kBlock; t < (b + 1) * kBlock; ++t)
+          x[t] = beta[t] * ks[t * row_at + i] * exp2_f(ahead + gs[t * row_at + i]);
+      }
+    } else {
+      const int v = i - dp;
+      const float *src = a.conv + (int64_t)r0 * s.channels + s.v_at + h * s.vdim + min(v, s.vdim - 1);
+#pragma unroll
+      for (int t = 0; t < kC; ++t)
+        x[t] = src[(int64_t)min(t, rows - 1) * s.channels];
+#pragma unroll
+      for (int t = 0; t < kC; ++t)
+        x[t] = v < s.vdim ? x[t] * beta[t] : 0.f;
+    }
+#pragma unroll
+    for (int t = 1; t < kC; ++t) {
+      float sum = x[t];
+#pragma unroll
+      for (int y = 0; y < t; y += 4) {
+        const f32x4 m = *reinterpret_cast<const f32x4 *>(as + t * kARow + y);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (y + j < t)
+            sum = fmaf(-m[j], x[y + j], sum);
+      }
+      x[t] = sum;
+    }
+    if (i < dp) {
+#pragma unroll
+      for (int t = 0; t < kC; ++t)
+        out[a.at.w + t * dp + i] = x[t];
+    } else {
+      float *u = out + a.at.ut + (i - dp) * kC;
+#pragma unroll
+      for (int t = 0; t < kC; t += 4)
+        *reinterpret_cast<f32x4 *>(u + t) = f32x4{x[t], x[t + 1], x[t + 2], x[t + 3]};
+    }
+  }
+}
+
+struct DeltaCarryArgs {
+  int heads, dim, vdim, rows, chunks;
+  const float *parts;
+  ChunkParts at;
+  float *state, *out; // out: [rows][heads * vdim]
+};
+
+// Grid (heads, value slices of 16): the state from chunk to chunk, and the outputs.  A
+// wavefront takes 16 tokens of a chunk (products with the state) and every fourth tile
+// of 16 key channels (the state itself, in registers).  ND: 32-channel steps, at most.
+// What the chunk after this one needs is on its way meanwhile.
+template <int ND>
+__global__ void __launch_bounds__(256, 1) delta_carry_kernel(DeltaCarryArgs a) {
+  constexpr int dp_max = ND * 32, kTiles = (2 * ND + 3) / 4; // state tiles per wavefront
+  constexpr int kSRow = dp_max + 4, kURow = kC + 4;
+  __shared__ __attribute__((aligned(16))) float st[16 * kSRow], ut[16 * kURow];
+  const int tid = threadIdx.x, lane = tid & 63, col = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int h = blockIdx.x, v0 = blockIdx.y * 16, v = v0 + col;
+  const int dp = (a.dim + 31) & ~31, nd = dp / 32;
+  float *S = a.state + (int64_t)h * a.dim * a.vdim;
+  f32x4 own[kTiles];
+#pragma unroll
+  for (int i = 0; i < kTiles; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = (wave + i * 4) * 16 + quad * 4 + r;
+      own[i][r] = d < a.dim && v < a.vdim ? S[(int64_t)d * a.vdim + v] : 0.f;
+    }
+  struct Chunk {
+    Frag<float> w[ND], q[ND], b[2], k[kTiles][2];
+    f32x4 u, last[kTiles];
+  };
+  auto fetch = [&](int c, Chunk &x) {
+    const float *p = a.parts + ((int64_t)min(c, a.chunks - 1) * a.heads + h) * a.at.size;
+    const float *row = p + (int64_t)(wave * 16 + col) * dp + quad * 8;
+#pragma unroll
+    for (int t = 0; t < ND; ++t) {
+      const int d = min(t, nd - 1) * 32;
+      x.w[t].load(row + a.at.w + d);
+      x.q[t].load(row + a.at.q + d);
+    }
+    x.u = *reinterpret_cast<const f32x4 *>(p + a.at.ut + (int64_t)(v0 + col) * kC + wave * 16 + quad * 4);
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+      x.b[t].load(p + a.at.b + (wave * 16 + col) * kC + t * 32 + quad * 8);
+#pragma unroll
+    for (int i = 0; i < kTiles; ++i) {
+      const int d0 = min((wave + i * 4) * 16, dp - 16);
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+        x.k[i][t].load(p + a.at.kt + (int64_t)(d0 + col) * kC + t * 32 + quad * 8);
+      x.last[i] = *reinterpret_cast<const f32x4 *>(p + a.at.last + d0 + quad * 4);
+    }
+  };
+  Chunk cur;
+  fetch(0, cur);
+  for (int c = 0; c < a.chunks; ++c) {
+    Chunk next;
+    fetch(c + 1, next);
+#pragma unroll
+    for (int i = 0; i < kTiles; ++i)
+      if ((wave + i * 4) * 16 < dp)
+        *reinterpret_cast<f32x4 *>(st + col * kSRow + (wave + i * 4) * 16 + quad * 4) = own[i];
+    __syncthreads();
+    f32x4 ws{0.f, 0.f, 0.f, 0.f}, o = ws;
+#pragma unroll
+    for (int t = 0; t < ND; ++t)
+      if (t < nd) {
+        Frag<float> sf;
+        sf.load(st + col * kSRow + t * 32 + quad * 8);
+        ws = mfma32(cur.w[t], sf, ws);
+        o = mfma32(cur.q[t], sf, o);
+      }
+    const f32x4 u = cur.u - ws;
+    *reinterpret_cast<f32x4 *>(ut + col * kURow + wave * 16 + quad * 4) = u;
+    __syncthreads();
+    Frag<float> uf[2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+      uf[t].load(ut + col * kURow + t * 32 + quad * 8);
+#pragma unroll
+    for (int i = 0; i < kTiles; ++i) {
+      f32x4 n = own[i] * cur.last[i];
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+        n = mfma32(cur.k[i][t], uf[t], n);
+      own[i] = n;
+    }
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+      if (t * 32 <= wave * 16 + 15)
+        o = mfma32(cur.b[t], uf[t], o);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = c * kC + wave * 16 + quad * 4 + r;
+      if (row < a.rows && v < a.vdim)
+        a.out[((int64_t)row * a.heads + h) * a.vdim + v] = o[r];
+    }
+    cur = next;
+  }
+#pragma unroll
+  for (int i = 0; i < kTiles; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = (wave + i * 4) * 16 + quad * 4 + r;
+      if (d < a.dim && v < a.vdim)
+        S[(int64_t)d * a.vdim + v] = own[i][r];
+    }
+}
+
+struct DeltaGateArgs {
+  int heads, vdim, rows, ld_gate, out_ld;
+  float eps;
+};
+
+// A wavefront per row and head: the output's norm and gate.
+template <typename T>
+__global__ void __launch_bounds__(256)
+delta_gate_kernel(const float *__restrict__ o, const float *__restrict__ gate, const float *__restrict__ norm_w,
+                  T *__restrict__ out, DeltaGateArgs a) {
+  const int lane = threadIdx.x & 63;
+  const int64_t id = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (id >= (int64_t)a.rows * a.heads)
+    return;
+  const int64_t row = id / a.heads;
+  const int at = (int)(id - row * a.heads) * a.vdim;
+  const float *x = o + id * a.vdim;
+  float ss = 0.f;
+  for (int i = lane; i < a.vdim; i += 64)
+    ss = fmaf(x[i], x[i], ss);
+  const float f = 1.0f / sqrtf(wave_sum(ss) / (float)a.vdim + a.eps);
+  for (int i = lane; i < a.vdim; i += 64)
+    store_act<T>(out + row * a.out_ld + at + i,
+                 x[i] * f * norm_w[i] * sigmoid_f(gate[row * a.ld_gate + at + i]));
+}
+
+constexpr size_t kChunkLdsLimit = 156 * 1024;
+size_t chunk_lds(const DeltaShape &s) {
+  return sizeof(float) * ((size_t)3 * kC * (s.dim32() + 4) + (size_t)kC * (kC + 4) + kBlocks * s.dim32() + kC);
+}
+struct Workspace {
+  size_t conv, dots, decay, gate, out, parts, size; // offsets in floats
+};
+Workspace workspace(const DeltaShape &s, int rows) {
+  Workspace w;
+  size_t at = 0;
+  auto take = [&](size_t n) {
+    const size_t here = at;
+    at += (size_t)round_up((int64_t)n, 64);
+    return here;
+  };
+  const size_t n = (size_t)rows;
+  w.conv = take(n * s.channels);
+  w.dots = take(n * s.kv_heads);
+  w.decay = take(n * s.decay.N);
+  w.gate = take(n * s.gate.N);
+  w.out = take(n * s.heads * s.vdim);
+  w.parts = take((size_t)ceil_div(rows, kC) * s.heads * chunk_parts(s).size);
+  w.size = at;
+  return w;
 }
 
 } // namespace
@@ -229,9 +698,70 @@ int launch_delta_scan(const DeltaRows &a, hipStream_t stream) {
 #undef BH_SCANS
 #undef BH_SCAN
   BH_CHECK_HIP(hipGetLastError());
-  if (a.rows > 1 && s.taps > 1)
-    hipLaunchKernelGGL(delta_keep_kernel, dim3((unsigned)ceil_div(s.channels, 64)), dim3(64), 0, stream,
-                       a.proj, a.ld, a.rows, a.start, s.taps, s.channels, a.ring);
+  return a.rows > 1 ? keep_rows(a, stream) : BUDDY_HIP_OK;
+}
+
+size_t delta_workspace(const DeltaShape &s, int rows) {
+  if (s.dim > 256 || chunk_lds(s) > kChunkLdsLimit)
+    return 0;
+  return workspace(s, rows).size;
+}
+
+int launch_delta_chunks(const DeltaRows &a, float *ws, hipStream_t stream) {
+  const DeltaShape &s = a.s;
+  BH_REQUIRE(delta_ok(a) && !a.pos && ws && ((uintptr_t)ws & 15) == 0 && delta_workspace(s, a.rows) > 0 &&
+                 s.decay.tiles && s.gate.tiles && s.decay.K == s.decay_rank && s.gate.K == s.gate_rank &&
+                 s.decay.N >= s.heads * s.dim && s.gate.N >= s.heads * s.vdim,
+             "delta_chunks: bad argument");
+  const Workspace w = workspace(s, a.rows);
+  int rc;
+  // the outer halves of the low-rank projections, on f32 activations
+  for (const bool gate : {false, true}) {
+    RowsGemm g;
+    g.W = gate ? s.gate : s.decay;
+    g.A = a.proj + (gate ? s.gate_at : s.decay_at);
+    g.lda = a.ld;
+    g.f32 = true;
+    g.rows = a.rows;
+    g.C = ws + (gate ? w.gate : w.decay);
+    g.ldc = g.W.N;
+    if ((rc = launch_rows_gemm(g, stream)))
+      return rc;
+  }
+  DeltaPrepArgs p{s, a.proj, a.ring, a.ld, a.rows, a.start, ws + w.conv, ws + w.dots};
+  hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)ceil_div((int64_t)a.rows * (s.kv_heads + s.heads), 4)),
+                     dim3(256), 0, stream, p);
+  BH_CHECK_HIP(hipGetLastError());
+  if ((rc = keep_rows(a, stream)))
+    return rc;
+  const int chunks = (int)ceil_div(a.rows, kC);
+  DeltaChunkArgs c{s, ws + w.conv, ws + w.dots, ws + w.decay, a.proj, a.ld, s.decay.N, a.rows, ws + w.parts,
+                   chunk_parts(s)};
+  static DynLdsOnce once;
+  BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)delta_chunk_kernel, (int)kChunkLdsLimit));
+  hipLaunchKernelGGL(delta_chunk_kernel, dim3((unsigned)chunks, (unsigned)s.heads), dim3(kChunkThreads),
+                     chunk_lds(s), stream, c);
+  BH_CHECK_HIP(hipGetLastError());
+  DeltaCarryArgs k{s.heads, s.dim, s.vdim, a.rows, chunks, ws + w.parts, chunk_parts(s), a.state, ws + w.out};
+  const dim3 grid((unsigned)s.heads, (unsigned)(s.vdim16() / 16));
+  const int nd = s.dim32() / 32;
+  if (nd <= 1)
+    hipLaunchKernelGGL(delta_carry_kernel<1>, grid, dim3(256), 0, stream, k);
+  else if (nd <= 2)
+    hipLaunchKernelGGL(delta_carry_kernel<2>, grid, dim3(256), 0, stream, k);
+  else if (nd <= 4)
+    hipLaunchKernelGGL(delta_carry_kernel<4>, grid, dim3(256), 0, stream, k);
+  else
+    hipLaunchKernelGGL(delta_carry_kernel<8>, grid, dim3(256), 0, stream, k);
+  BH_CHECK_HIP(hipGetLastError());
+  DeltaGateArgs e{s.heads, s.vdim, a.rows, s.gate.N, a.out_ld, s.eps};
+  const dim3 rows_grid((unsigned)ceil_div((int64_t)a.rows * s.heads, 4));
+  if (a.act_f32)
+    hipLaunchKernelGGL(delta_gate_kernel<float>, rows_grid, dim3(256), 0, stream, ws + w.out, ws + w.gate, s.norm_w,
+                       static_cast<float *>(a.out), e);
+  else
+    hipLaunchKernelGGL(delta_gate_kernel<bf16_bits>, rows_grid, dim3(256), 0, stream, ws + w.out, ws + w.gate,
+                       s.norm_w, static_cast<bf16_bits *>(a.out), e);
   BH_CHECK_HIP(hipGetLastError());
   return BUDDY_HIP_OK;
 }

@@ -145,9 +145,11 @@ struct LirulixSession : FolderSession {
         *hrow = nullptr, *part_acc = nullptr, *part_ml = nullptr;
 
   // a block of a prompt
-  float *pf_x = nullptr, *pf_y = nullptr, *pf_proj = nullptr, *pf_maps = nullptr, *pf_logits = nullptr;
+  float *pf_x = nullptr, *pf_y = nullptr, *pf_proj = nullptr, *pf_maps = nullptr, *pf_delta = nullptr,
+        *pf_logits = nullptr;
   void *pf_act = nullptr, *pf_mix = nullptr, *pf_queries = nullptr, *pf_ff = nullptr;
   int ld_act = 0, ld_mix = 0, max_proj = 0;
+  static constexpr int kScanRows = 12; // the delta rule takes fewer rows token by token
 
   LirulixSession(const Json &config, const ModelOptions &o) : FolderSession(o), cfg(config) {}
 
@@ -237,6 +239,8 @@ struct LirulixSession : FolderSession {
     s.conv_w = device_copy(conv);
     s.decay_w = device_bf16(f.bf16(p + "a2", {c.heads * c.dim, s.decay_rank}));
     s.gate_w = device_bf16(f.bf16(p + "g2", {c.heads * c.vdim, s.gate_rank}));
+    s.decay = load_matrix(f, p + "a2", c.heads * c.dim, s.decay_rank);
+    s.gate = load_matrix(f, p + "g2", c.heads * c.vdim, s.gate_rank);
     s.decay_bias = device_copy(f.values(p + "dt_bias", {c.heads * c.dim}));
     std::vector<float> speed = f.values(p + "A_log", {c.heads});
     for (float &v : speed)
@@ -437,13 +441,15 @@ struct LirulixSession : FolderSession {
   // ---- many tokens -----------------------------------------------------------------
   int alloc_block(int rows) override {
     const size_t n = (size_t)rows, T = opt.f32 ? 4 : 2;
-    size_t queries = 0, maps = 0, ff = 0;
+    size_t queries = 0, maps = 0, ff = 0, delta = 0;
     for (size_t i = 0; i < layers.size(); ++i) {
       const LirulixLayer &L = layers[i];
       if (cfg.layers[i].kind != kDelta) {
         queries = std::max(queries, (size_t)L.head.map_heads() * L.head.dim32());
         if (L.head.maps > 1 || L.head.gated)
           maps = std::max(maps, (size_t)L.head.map_heads() * L.head.vdim);
+      } else {
+        delta = std::max(delta, delta_workspace(L.delta, rows));
       }
       ff = std::max(ff, (size_t)round_up(cfg.layers[i].ff, 16));
     }
@@ -454,6 +460,7 @@ struct LirulixSession : FolderSession {
     rc |= block_alloc(&pf_mix, T * n * ld_mix);
     rc |= block_alloc(&pf_queries, T * n * queries);
     rc |= block_alloc(&pf_maps, 4 * n * maps);
+    rc |= block_alloc(&pf_delta, 4 * delta);
     rc |= block_alloc(&pf_ff, T * n * ff);
     rc |= block_alloc(&pf_logits, 4 * (size_t)std::min(rows, kLogitRows) * head.N);
     return rc;
@@ -473,7 +480,8 @@ struct LirulixSession : FolderSession {
       d.out = pf_mix;
       d.out_ld = ld_mix;
       d.act_f32 = opt.f32;
-      return launch_delta_scan(d, stream);
+      return n < kScanRows || !delta_workspace(L.delta, n) ? launch_delta_scan(d, stream)
+                                                           : launch_delta_chunks(d, pf_delta, stream);
     }
     HeadRows a;
     a.s = L.head;

@@ -157,7 +157,82 @@ def nukopel_shapes(cfg: dict):
 
 
 def write_nukopel_folder(folder, cfg: dict, seed: int = SEED):
-    """config.json and model.safetensors with random weights in bfloat16."""
+    return write_folder(folder, cfg, nukopel_shapes(cfg), seed)
+
+
+# ---- Lirulix ---------------------------------------------------------------------
+
+def lirulix_config(width: int, layers: str, heads: int, *, kv_heads: int = 2, dim: int = 128,
+                   window: int = 1024, ff: int = 8960, vocab: int = 32768, taps: int = 4,
+                   loop: tuple = (0, 1, 1)) -> dict:
+    """A configuration of the layers of a real model; `layers`: a letter per layer, f =
+    attention over everything, s = differential attention through a window, d = gated
+    delta rule."""
+    kinds = {
+        "f": ("attention",
+              {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": dim ** -0.5,
+               "rot": {"base": 1e6, "dims": dim,
+                       "scaling": {"factor": 4.0, "original": 8192, "fast": 32.0, "slow": 1.0}}}),
+        "s": ("attention_2",
+              {"heads": heads, "kv_heads": kv_heads, "dim": dim // 2, "vdim": dim, "diff": 0.5,
+               "scale": (dim // 2) ** -0.5, "mask": {"size": window},
+               "rot": {"base": 1e5, "dims": dim // 2,
+                       "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}),
+        "d": ("channel_delta",
+              {"heads": heads, "kv_heads": heads, "dim": dim, "vdim": dim, "conv": taps}),
+    }
+    return {"architecture": "Lirulix", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "loop": {"start": loop[0], "stop": loop[1], "times": loop[2]},
+            "layers": [{"type": kinds[c][0], "mixer": kinds[c][1], "mlp": {"kind": "dense", "ff": ff}}
+                       for c in layers]}
+
+
+def lirulix_shapes(cfg: dict, rank: int = 128):
+    """(name, shape, standard deviation) of every tensor; `rank`: of the decay's and the
+    gate's inner projections."""
+    W, V = cfg["width"], cfg["vocab"]
+    yield "embed", (V, W), 1.0
+    yield "embed.norm", (W,), 0.1
+    yield "loop.step", (cfg["loop"]["times"], W), 0.1
+    for i, layer in enumerate(cfg["layers"]):
+        p, m, ff = f"l{i}.", layer["mixer"], layer["mlp"]["ff"]
+        H, G, D, VD = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        yield p + "norm1", (W,), 0.1
+        yield p + "norm2", (W,), 0.1
+        if layer["type"] == "attention":
+            mats = {"q": (H * D, W), "k": (G * D, W), "v": (G * VD, W)}
+            yield p + "mix.sink", (H,), 1.0
+        elif layer["type"] == "attention_2":
+            mats = {"q": (H * 2 * D, W), "k": (G * 2 * D, W), "v": (G * VD, W), "g": (H * VD, W)}
+            for n in ("lq1", "lk1", "lq2", "lk2"):
+                yield p + "mix." + n, (D,), 0.1
+        else:
+            mats = {"q": (G * D, W), "k": (G * D, W), "v": (H * VD, W), "b": (H, W),
+                    "a1": (rank, W), "a2": (H * D, rank), "g1": (rank, W), "g2": (H * VD, rank)}
+            for n, c in (("q", G * D), ("k", G * D), ("v", H * VD)):
+                yield f"{p}mix.{n}.conv", (c, m["conv"]), 0.5
+            yield p + "mix.A_log", (H,), 1.0
+            yield p + "mix.dt_bias", (H * D,), 1.0
+            yield p + "mix.norm", (VD,), 1.0
+        for n, s in mats.items():
+            yield p + "mix." + n, s, s[1] ** -0.5
+        yield p + "mix.o", (W, H * VD), (H * VD) ** -0.5
+        yield p + "mlp.gate", (ff, W), W ** -0.5
+        yield p + "mlp.up", (ff, W), W ** -0.5
+        yield p + "mlp.down", (W, ff), ff ** -0.5
+    yield "final.norm", (W,), 0.1
+    yield "head", (V, W), W ** -0.5
+
+
+def write_lirulix_folder(folder, cfg: dict, seed: int = SEED):
+    return write_folder(folder, cfg, lirulix_shapes(cfg), seed)
+
+
+# ---- model folders ---------------------------------------------------------------
+
+def write_folder(folder, cfg: dict, shapes, seed: int = SEED):
+    """config.json and model.safetensors with random weights in bfloat16; shapes: (name,
+    shape, standard deviation or None for ones) of every tensor."""
     import json
     import struct
     from math import prod
@@ -166,7 +241,7 @@ def write_nukopel_folder(folder, cfg: dict, seed: int = SEED):
     folder = Path(folder)
     folder.mkdir(parents=True, exist_ok=True)
     (folder / "config.json").write_text(json.dumps(cfg))
-    tensors, head, at = list(nukopel_shapes(cfg)), {}, 0
+    tensors, head, at = list(shapes), {}, 0
     for name, shape, _ in tensors:
         size = 2 * prod(shape)
         head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + size]}
