@@ -79,6 +79,7 @@ struct RowTail { // arguments a wavefront needs only behind its first loads
   int taps, silu_channels, valid;
   const float *add, *norm_w;
   GatedAct act;
+  int head_dim;
 };
 
 __device__ __forceinline__ f32x4 load4(const float *p) { return *reinterpret_cast<const f32x4 *>(p); }
@@ -128,6 +129,9 @@ struct RowPrologue {
       } else if constexpr (INPUT == kRowGated) {
         w[r] = load4(a.weight + i);
         c[0][r] = load4(a.gate + i);
+      } else if constexpr (INPUT == kRowHeadGated) {
+        w[r] = load4(a.weight + i % a.head_dim);
+        c[0][r] = load4(a.gate + i);
       } else if constexpr (INPUT == kRowResidual) {
         if (yp)
           y[r] = load4(yp + i);
@@ -156,6 +160,26 @@ struct RowPrologue {
 #pragma unroll
         for (int j = 0; j < 4; ++j)
           x[r][j] = x[r][j] * g * w[r][j] * sigmoid_f(c[0][r][j]);
+    } else if constexpr (INPUT == kRowHeadGated) {
+      // the squares of four values each meet in LDS, where the row goes afterwards
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+        if (in[r])
+          act[at[r] >> 2] = fmaf(x[r][0], x[r][0], x[r][1] * x[r][1]) + fmaf(x[r][2], x[r][2], x[r][3] * x[r][3]);
+      __syncthreads();
+      const int per = a.head_dim >> 2;
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        const float *sq = act + (in[r] ? at[r] / a.head_dim * per : 0);
+        float ss = 0.f;
+        for (int i = 0; i < per; ++i)
+          ss += sq[i];
+        const float g = 1.0f / sqrtf(ss / (float)a.head_dim + a.eps);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          x[r][j] = x[r][j] * g * w[r][j] * sigmoid_f(c[0][r][j]);
+      }
+      __syncthreads();
     } else if constexpr (INPUT == kRowResidual) {
 #pragma unroll
       for (int r = 0; r < R; ++r) {
@@ -233,6 +257,19 @@ struct RowPrologue<INPUT, 0> {
     if constexpr (INPUT == kRowPlain) {
       for (int i = tid; i < K; i += kRowThreads)
         act[i] = src[i];
+    } else if constexpr (INPUT == kRowHeadGated) {
+      float *scales = act + Kp; // [heads]
+      for (int h = tid >> 6; h * a.head_dim < K; h += kRowWaves) {
+        float ss = 0.f;
+        for (int i = tid & 63; i < a.head_dim; i += 64)
+          ss = fmaf(src[h * a.head_dim + i], src[h * a.head_dim + i], ss);
+        ss = wave_sum(ss);
+        if ((tid & 63) == 0)
+          scales[h] = 1.0f / sqrtf(ss / (float)a.head_dim + a.eps);
+      }
+      __syncthreads();
+      for (int i = tid; i < K; i += kRowThreads)
+        act[i] = src[i] * scales[i / a.head_dim] * a.weight[i % a.head_dim];
     } else {
       float ry = 0.f, ss = 0.f;
       if (INPUT == kRowNorm && yp) {
@@ -268,6 +305,8 @@ struct RowPrologue<INPUT, 0> {
         h = act[i] * scale;
         if constexpr (INPUT == kRowGated)
           h *= a.weight[i] * sigmoid_f(a.gate[i]);
+        if constexpr (INPUT == kRowHeadGated)
+          h *= sigmoid_f(a.gate[i]);
         if constexpr (INPUT == kRowResidual) {
           h *= a.norm_w[i];
           if (keeper && a.row_out)
@@ -543,7 +582,7 @@ moe_down_kernel(const uint4 *__restrict__ down, const float *__restrict__ act,
   const int run = HALF ? (lane >> 5) * 64 + ((lane >> 3) & 3) * 16 + half * 8 + (lane & 7) : lane;
   const int k_at = HALF ? (lane >> 5) * kBfTileK + ((lane >> 3) & 3) * 8 : (lane >> 4) * 8;
   // lane j: the j-th chosen expert and its softmax weight
-  const int cj = chosen[min(lane, a.top - 1)];
+  const int cj = a.top > 0 ? chosen[min(lane, a.top - 1)] : 0;
   const float zj = lane < a.top ? a.chosen_logit[lane] : -INFINITY;
   const float ej = lane < a.top ? expf(zj - wave_max(zj)) : 0.f;
   const float wj = ej / wave_sum(ej);
@@ -595,6 +634,9 @@ moe_down_kernel(const uint4 *__restrict__ down, const float *__restrict__ act,
   }
 }
 
+// slices start at even tiles
+int down_slice(int total, int waves) { return (int)round_up(ceil_div(total, waves), 2); }
+
 int shift_for(int v) {
   int s = 0;
   while ((1 << (s + 1)) <= v)
@@ -622,12 +664,27 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
              "row_gemv: bad argument");
   BH_REQUIRE(!a.conv_w || (a.conv_ring && a.conv_next && a.pos && a.taps > 0),
              "row_gemv: convolution operands");
-  BH_REQUIRE(a.input != kRowGated || (a.weight && a.gate), "row_gemv: gate operands");
+  BH_REQUIRE((a.input != kRowGated && a.input != kRowHeadGated) || (a.weight && a.gate), "row_gemv: gate operands");
+  BH_REQUIRE(a.input != kRowHeadGated || (a.head_dim > 0 && W.K % a.head_dim == 0), "row_gemv: heads of %d values",
+             a.head_dim);
   BH_REQUIRE(a.x_out == nullptr || a.x_out != a.src, "row_gemv: the row is read by every workgroup");
   BH_REQUIRE(!a.max_v || a.max_i, "row_gemv: maxima without indices");
   BH_REQUIRE(a.input != kRowResidual || a.norm_w, "row_gemv: no norm weight");
   BH_REQUIRE(!a.gated || (a.input == kRowResidual && W.N % 32 == 0 && !a.max_v && a.act == kActGeluTanh),
              "row_gemv: gated form");
+  if (a.input == kRowPlain && a.src_padded && !a.silu_channels && !a.max_v && ((uintptr_t)a.src & 15) == 0 &&
+      W.ktiles >= 64 && (W.groups() < 192 || W.ktiles > 256)) {
+    // a long row and few channels: as many slices of k as the experts' down product takes
+    MoeDown d{W.tiles, W.groups(), 0, 1, W.ktiles, 0, nullptr, a.out};
+    if (W.groups() < 192)
+      hipLaunchKernelGGL((moe_down_kernel<16, true>), dim3(2 * W.groups()), dim3(1024), 0, stream,
+                         (const uint4 *)nullptr, a.src, (const int *)nullptr, down_slice(W.ktiles, 16), d);
+    else
+      hipLaunchKernelGGL((moe_down_kernel<16, false>), dim3(W.groups()), dim3(1024), 0, stream,
+                         (const uint4 *)nullptr, a.src, (const int *)nullptr, down_slice(W.ktiles, 16), d);
+    BH_CHECK_HIP(hipGetLastError());
+    return BUDDY_HIP_OK;
+  }
   // slices of k: doubled while the launch has fewer than 2048 wavefronts and each
   // keeps four tiles
   const int groups = W.groups();
@@ -636,14 +693,14 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
     ks *= 2;
   const int shift = shift_for(ks), per = kRowWaves >> shift;
   const int slice_tiles = (int)ceil_div(W.ktiles, ks);
-  const size_t lds = sizeof(float) * (size_t)W.ktiles * kBfTileK;
+  const size_t lds = sizeof(float) * ((size_t)W.ktiles * kBfTileK + (a.head_dim ? W.K / a.head_dim : 0));
   BH_REQUIRE(lds <= 150 * 1024, "row_gemv: a row of %d values does not fit LDS", W.K);
   RowTail t{a.x_out, a.row_out, a.conv_w, a.conv_ring, a.conv_next, a.pos, a.weight, a.gate,
             a.out, a.max_v, a.max_i, a.eps, a.out_gain, a.gain, a.taps, a.silu_channels, a.valid,
-            a.add, a.norm_w, a.act};
+            a.add, a.norm_w, a.act, a.head_dim};
   const bool keeper = a.input == kRowNorm || a.input == kRowResidual;
   const dim3 grid((unsigned)(ceil_div(groups, per) + keeper)), block(kRowThreads);
-  bool quads = W.K % 4 == 0;
+  bool quads = W.K % 4 == 0 && a.head_dim % 4 == 0;
   for (const void *p : {(const void *)a.src, (const void *)a.y, (const void *)a.x_out,
                         (const void *)a.row_out, (const void *)a.conv_w, (const void *)a.conv_next,
                         (const void *)a.weight, (const void *)a.gate, (const void *)a.add,
@@ -676,6 +733,8 @@ int launch_row_gemv(const RowGemv &a, hipStream_t stream) {
     BH_ROWS(kRowNorm, false);
   else if (a.input == kRowGated)
     BH_ROWS(kRowGated, false);
+  else if (a.input == kRowHeadGated)
+    BH_ROWS(kRowHeadGated, false);
   else if (a.gated)
     BH_ROWS(kRowResidual, true);
   else
@@ -743,9 +802,8 @@ int launch_row_moe(const RowMoe &a, hipStream_t stream) {
   d.act_stride = a.act_stride;
   d.chosen_logit = a.weights;
   d.out = a.out;
-  // slices start at even tiles
   const int total = a.top * d.ktiles + d.shared_ktiles;
-  auto slice = [&](int waves) { return (int)round_up(ceil_div(total, waves), 2); };
+  auto slice = [&](int waves) { return down_slice(total, waves); };
   if (total >= 64 && d.groups < 192) // fewer workgroups than compute units: halves
     hipLaunchKernelGGL((moe_down_kernel<16, true>), dim3(2 * d.groups), dim3(1024), 0, stream,
                        a.experts.down, a.act, a.chosen, slice(16), d);

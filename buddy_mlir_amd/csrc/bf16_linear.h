@@ -40,12 +40,15 @@ enum RowInput {
                    // x' * (gain / rms(x')), then, with conv_w, itself plus its
                    // causal convolution over the ring of earlier rows
   kRowGated = 2,   // (src / rms(src)) * weight * sigmoid(gate)
-  kRowResidual = 3 // x' = src + y + add (each may be missing), then x' / rms(x') * norm_w
+  kRowResidual = 3, // x' = src + y + add (each may be missing), then x' / rms(x') * norm_w
+  kRowHeadGated = 4 // like kRowGated with the mean over heads of head_dim values each,
+                    // which share the weight [head_dim]
 };
 struct RowGemv {
   Bf16Matrix W;
   RowInput input = kRowPlain;
   const float *src = nullptr;
+  bool src_padded = false; // src has (finite) values up to a multiple of 64
   float eps = 0.f;
   // kRowNorm
   const float *y = nullptr;
@@ -57,8 +60,9 @@ struct RowGemv {
   float *conv_next = nullptr;     // [2][K]: what earlier rows add at position p, in slot p % 2
   int taps = 0;
   const int *pos = nullptr;       // device: position of the row
-  // kRowGated
+  // kRowGated, kRowHeadGated
   const float *weight = nullptr, *gate = nullptr;
+  int head_dim = 0;
   // kRowResidual (also eps, y, x_out, row_out)
   const float *add = nullptr, *norm_w = nullptr;
   // kRowResidual: W holds two matrices of N / 2 channels, the second one behind the

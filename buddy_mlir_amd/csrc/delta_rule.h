@@ -35,12 +35,17 @@ struct DeltaRows {
   const int *pos = nullptr;        // device: in place of `start`, for one row
   float *ring = nullptr;           // [taps][channels], position p in slot p % taps
   float *state = nullptr;          // [heads][dim][vdim]
-  void *out = nullptr;             // [rows][out_ld], normed and gated
+  float *o = nullptr, *gate = nullptr; // launch_delta_scan: [rows][heads * vdim], outputs ahead of norm and gate
+  void *out = nullptr;             // launch_delta_chunks: [rows][out_ld], normed and gated
   int out_ld = 0;
   bool act_f32 = true;             // type of out: f32 or bfloat16
 };
 // Token by token: a step of decoding, short portions.
 int launch_delta_scan(const DeltaRows &a, hipStream_t stream);
+
+// out = per head o / rms(o) * norm_w * sigmoid(gate)
+int launch_delta_gate(const DeltaShape &s, const float *o, const float *gate, int ld_gate, int rows, void *out,
+                      int out_ld, bool act_f32, hipStream_t stream);
 
 // A prompt in chunks of kDeltaChunk tokens.  Within a chunk the writes are solved for as
 // one triangular system; the state goes from chunk to chunk.

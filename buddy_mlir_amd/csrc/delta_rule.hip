@@ -19,34 +19,42 @@
 namespace bh {
 namespace {
 
-constexpr int kScanThreads = 1024, kScanWaves = kScanThreads / 64;
 constexpr float kUnitEps = 1e-6f; // of the unit vectors
 
-__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+// log(1 + e^z); what rounding 1 + e loses of a small e is made up for by e / ((1 + e) - 1)
+__device__ __forceinline__ float softplus_f(float z) {
+  const float e = fast_exp(-fabsf(z)), u = 1.0f + e, d = u - 1.0f;
+  const float l = __builtin_amdgcn_logf(u) * 0.693147180559945309f;
+  return fmaxf(z, 0.f) + (d == 0.f ? e : l * (e / d));
+}
 
+__device__ __forceinline__ float dot_run8(uint4 v, const float *x, float acc) {
+  acc = fmaf(bf_lo(v.x), x[0], acc);
+  acc = fmaf(bf_hi(v.x), x[1], acc);
+  acc = fmaf(bf_lo(v.y), x[2], acc);
+  acc = fmaf(bf_hi(v.y), x[3], acc);
+  acc = fmaf(bf_lo(v.z), x[4], acc);
+  acc = fmaf(bf_hi(v.z), x[5], acc);
+  acc = fmaf(bf_lo(v.w), x[6], acc);
+  return fmaf(bf_hi(v.w), x[7], acc);
+}
+__device__ __forceinline__ float sum8(float v) { // over eight neighbouring lanes
+  v = quad_sum(v);
+  return v + __shfl_xor(v, 4, 64);
+}
 // Row `w` of a bfloat16 matrix times x (LDS), by eight neighbouring lanes; all of them
 // get the sum.
 __device__ __forceinline__ float row_dot8(const uint16_t *__restrict__ w, const float *x, int n) {
   const int l = threadIdx.x & 7;
   float acc = 0.f;
   if (n % 8 == 0) {
-    for (int i = l * 8; i < n; i += 64) {
-      const uint4 v = *reinterpret_cast<const uint4 *>(w + i);
-      acc = fmaf(bf_lo(v.x), x[i], acc);
-      acc = fmaf(bf_hi(v.x), x[i + 1], acc);
-      acc = fmaf(bf_lo(v.y), x[i + 2], acc);
-      acc = fmaf(bf_hi(v.y), x[i + 3], acc);
-      acc = fmaf(bf_lo(v.z), x[i + 4], acc);
-      acc = fmaf(bf_hi(v.z), x[i + 5], acc);
-      acc = fmaf(bf_lo(v.w), x[i + 6], acc);
-      acc = fmaf(bf_hi(v.w), x[i + 7], acc);
-    }
+    for (int i = l * 8; i < n; i += 64)
+      acc = dot_run8(*reinterpret_cast<const uint4 *>(w + i), x + i, acc);
   } else {
     for (int i = l; i < n; i += 8)
       acc = fmaf(bf_f(w[i]), x[i], acc);
   }
-  acc = quad_sum(acc);
-  return acc + __shfl_xor(acc, 4, 64);
+  return sum8(acc);
 }
 
 // The convolution of column c at position p; `row`: the projections of that position,
@@ -54,74 +62,128 @@ __device__ __forceinline__ float row_dot8(const uint16_t *__restrict__ w, const 
 __device__ __forceinline__ float short_conv(const DeltaShape &s, const float *row, int ld, int have,
                                             const float *__restrict__ ring, int p, int c) {
   float v = 0.f;
-  for (int b = s.taps - 1; b >= 0; --b) {
-    if (p - b < 0)
-      continue;
-    const float e = b <= have ? row[c - (int64_t)b * ld] : ring[(int64_t)((p - b) % s.taps) * s.channels + c];
-    v = fmaf(s.conv_w[(int64_t)(s.taps - 1 - b) * s.channels + c], e, v);
+  for (int b0 = 0; b0 < s.taps; b0 += 4) {
+    float e[4], w[4]; // asked for together
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int b = b0 + i;
+      const bool some = b < s.taps && b <= p;
+      const float *from = !some || b <= have ? row + c - (int64_t)(some ? b : 0) * ld
+                                             : ring + (int64_t)((p - b) % s.taps) * s.channels + c;
+      e[i] = *from;
+      w[i] = s.conv_w[(int64_t)(some ? s.taps - 1 - b : 0) * s.channels + c];
+      w[i] = some ? w[i] : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      v = fmaf(w[i], e[i], v);
   }
   return silu_f(v);
 }
 
-// A workgroup per head.  A thread owns one value channel of N consecutive rows of the
-// state, in registers from the first token to the last.  Both products with the
-// state are taken of the decayed one: S^T q = (g S)^T q + u (k . q).
-template <typename T, int N>
+constexpr int kScanThreads = 512, kScanCols = 32, kScanSlices = kScanThreads / kScanCols;
+
+// Grid (heads, slices of 32 value channels).  A thread owns one value channel of N
+// consecutive rows of the state, in registers from the first token to the last.  Both
+// products with the state are taken of the decayed one: S^T q = (g S)^T q + u (k . q).
+template <int N>
 __global__ void __launch_bounds__(kScanThreads)
 delta_scan_kernel(DeltaRows a) {
-  extern __shared__ __attribute__((aligned(16))) float lds[];
-  __shared__ float red[kScanWaves], dots[3];
+  __shared__ __attribute__((aligned(16))) float q[kScanSlices * N], k[kScanSlices * N], decay[kScanSlices * N];
+  __shared__ float v[kScanCols], part[2][kScanSlices][kScanCols], dots[3];
+  extern __shared__ __attribute__((aligned(16))) float lds[]; // inner decay, inner gate
   const DeltaShape &s = a.s;
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int h = blockIdx.x, group = s.heads / s.kv_heads, g = h / group;
-  const int dim = s.dim, vdim = s.vdim;
-  const int vcols = (vdim + 63) & ~63, slices = kScanThreads / vcols;
-  const int padded = slices * N; // rows of the state with those past the last, which stay zero
-  float *q = lds, *k = q + padded, *decay = k + padded, *v = decay + padded, *gate = v + vdim;
-  float *inner_d = gate + vdim, *inner_g = inner_d + ((s.decay_rank + 3) & ~3);
-  float *part = inner_g + ((s.gate_rank + 3) & ~3); // [2][slices][vcols]
-  const int c = tid % vcols, slice = tid / vcols;
-  const bool owner = slice < slices && c < vdim;
-  float *S = a.state + (int64_t)h * dim * vdim + min(c, vdim - 1);
-  const int d0 = min(slice, slices - 1) * N;
+  const int h = blockIdx.x, v0 = blockIdx.y * kScanCols;
+  const int dim = s.dim, vdim = s.vdim, vcols = min(kScanCols, vdim - v0);
+  float *inner_d = lds, *inner_g = lds + ((s.decay_rank + 3) & ~3);
+  const int c = tid % kScanCols, slice = tid / kScanCols, d0 = slice * N;
+  const bool owner = c < vcols;
+  float *S = a.state + (int64_t)h * dim * vdim + v0 + min(c, vcols - 1);
   float st[N];
 #pragma unroll
   for (int i = 0; i < N; ++i)
-    st[i] = owner && d0 + i < dim ? S[(int64_t)(d0 + i) * vdim] : 0.f;
-  for (int i = dim + tid; i < padded; i += kScanThreads)
+    st[i] = S[(int64_t)min(d0 + i, dim - 1) * vdim];
+  // this thread's share of the low-rank projections' outer rows, if they are short: from
+  // the same trip to memory
+  constexpr int kPreRows = 3, kPreRuns = 2, kRowStep = kScanThreads / 8;
+  const bool pre = dim + vcols <= kPreRows * kRowStep && s.decay_rank % 8 == 0 && s.gate_rank % 8 == 0 &&
+                   max(s.decay_rank, s.gate_rank) <= kPreRuns * 64;
+  auto low_row = [&](int i) { // row i: the decay of channel i, then the gates of the slice
+    return i < dim ? s.decay_w + ((int64_t)h * dim + i) * s.decay_rank
+                   : s.gate_w + ((int64_t)h * vdim + v0 + i - dim) * s.gate_rank;
+  };
+  uint4 low[kPreRows][kPreRuns];
+  float bias[kPreRows];
+  if (pre) {
+#pragma unroll
+    for (int m = 0; m < kPreRows; ++m) {
+      const int i = min((tid >> 3) + m * kRowStep, dim + vcols - 1);
+      const uint16_t *w = low_row(i);
+      const int n = i < dim ? s.decay_rank : s.gate_rank;
+#pragma unroll
+      for (int j = 0; j < kPreRuns; ++j) // past the end: times zero
+        low[m][j] = *reinterpret_cast<const uint4 *>(w + min((tid & 7) * 8 + j * 64, n - 8));
+      bias[m] = s.decay_bias[(int64_t)h * dim + min(i, dim - 1)];
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < N; ++i)
+    st[i] = owner && d0 + i < dim ? st[i] : 0.f;
+  for (int i = dim + tid; i < kScanSlices * N; i += kScanThreads)
     q[i] = k[i] = decay[i] = 0.f;
+  const int group = s.heads / s.kv_heads, g = h / group;
   const int p0 = a.pos ? *a.pos : a.start;
-  const float speed = s.decay_speed[h];
+  const float speed = s.decay_speed[h], root = sqrtf((float)dim);
   for (int r = 0; r < a.rows; ++r) {
     const float *row = a.proj + (int64_t)r * a.ld;
     const int p = p0 + r;
-    for (int i = tid; i < 2 * dim + vdim; i += kScanThreads) {
+    for (int i = tid; i < 2 * dim + vcols; i += kScanThreads) {
       const int col = i < dim ? s.q_at + g * dim + i
                       : i < 2 * dim ? s.k_at + g * dim + i - dim
-                                    : s.v_at + h * vdim + i - 2 * dim;
+                                    : s.v_at + h * vdim + v0 + i - 2 * dim;
       const float x = short_conv(s, row, a.ld, r, a.ring, p, col);
       (i < dim ? q[i] : i < 2 * dim ? k[i - dim] : v[i - 2 * dim]) = x;
       // no workgroup reads this slot: it is the one of position p - taps
-      if (a.rows == 1 && (i >= 2 * dim || h == g * group))
+      if (a.rows == 1 && (i >= 2 * dim || (v0 == 0 && h == g * group)))
         a.ring[(int64_t)(p % s.taps) * s.channels + col] = row[col];
     }
     for (int i = tid; i < s.decay_rank; i += kScanThreads)
       inner_d[i] = row[s.decay_at + i];
     for (int i = tid; i < s.gate_rank; i += kScanThreads)
       inner_g[i] = row[s.gate_at + i];
+    const float beta = sigmoid_f(row[s.beta_at + h]);
     __syncthreads();
-    for (int i = tid >> 3; i < dim + vdim; i += kScanThreads / 8) {
-      if (i < dim) {
-        const int64_t at = (int64_t)h * dim + i;
-        const float z = row_dot8(s.decay_w + at * s.decay_rank, inner_d, s.decay_rank);
-        if ((tid & 7) == 0)
-          decay[i] = expf(speed * softplus_f(z + s.decay_bias[at]));
-      } else {
-        const float z = row_dot8(s.gate_w + ((int64_t)h * vdim + i - dim) * s.gate_rank, inner_g, s.gate_rank);
-        if ((tid & 7) == 0)
-          gate[i - dim] = sigmoid_f(z);
+    auto finish_low = [&](int i, float z, float bias_i) {
+      if (tid & 7)
+        return;
+      if (i < dim)
+        decay[i] = fast_exp(speed * softplus_f(z + bias_i));
+      else
+        a.gate[(int64_t)r * s.heads * vdim + (int64_t)h * vdim + v0 + i - dim] = z;
+    };
+    if (pre) {
+#pragma unroll
+      for (int m = 0; m < kPreRows; ++m) {
+        const int i = (tid >> 3) + m * kRowStep;
+        if (i >= dim + vcols)
+          break;
+        const int n = i < dim ? s.decay_rank : s.gate_rank;
+        const float *x = i < dim ? inner_d : inner_g;
+        float z = 0.f;
+#pragma unroll
+        for (int j = 0; j < kPreRuns; ++j) {
+          const int k0 = (tid & 7) * 8 + j * 64;
+          if (k0 < n)
+            z = dot_run8(low[m][j], x + k0, z);
+        }
+        finish_low(i, sum8(z), bias[m]);
       }
+    } else {
+      for (int i = tid >> 3; i < dim + vcols; i += kRowStep)
+        finish_low(i, row_dot8(low_row(i), i < dim ? inner_d : inner_g, i < dim ? s.decay_rank : s.gate_rank),
+                   s.decay_bias[(int64_t)h * dim + min(i, dim - 1)]);
     }
     if (wave < 3) {
       const float *x = wave == 1 ? k : q, *y = wave == 0 ? q : k;
@@ -133,7 +195,7 @@ delta_scan_kernel(DeltaRows a) {
         dots[wave] = t;
     }
     __syncthreads();
-    const float rq = 1.0f / sqrtf(dots[0] + kUnitEps) / sqrtf((float)dim), rk = 1.0f / sqrtf(dots[1] + kUnitEps);
+    const float rq = 1.0f / sqrtf(dots[0] + kUnitEps) / root, rk = 1.0f / sqrtf(dots[1] + kUnitEps);
     float sk = 0.f, sq = 0.f;
 #pragma unroll
     for (int i = 0; i < N; i += 4) {
@@ -147,19 +209,16 @@ delta_scan_kernel(DeltaRows a) {
         sq = fmaf(st[i + j], qq[j], sq);
       }
     }
-    if (slice < slices) {
-      part[slice * vcols + c] = sk;
-      part[(slices + slice) * vcols + c] = sq;
-    }
+    part[0][slice][c] = sk;
+    part[1][slice][c] = sq;
     __syncthreads();
     sk = sq = 0.f;
-    for (int i = 0; i < slices; ++i) {
-      sk += part[i * vcols + c];
-      sq += part[(slices + i) * vcols + c];
+#pragma unroll
+    for (int i = 0; i < kScanSlices; ++i) {
+      sk += part[0][i][c];
+      sq += part[1][i][c];
     }
-    const float beta = sigmoid_f(row[s.beta_at + h]);
-    const float u = owner ? beta * (v[c] - sk * rk) : 0.f;
-    const float ku = rk * u;
+    const float ku = owner ? rk * beta * (v[c] - sk * rk) : 0.f;
 #pragma unroll
     for (int i = 0; i < N; i += 4) {
       const f32x4 kk = *reinterpret_cast<const f32x4 *>(k + d0 + i);
@@ -167,20 +226,10 @@ delta_scan_kernel(DeltaRows a) {
       for (int j = 0; j < 4; ++j)
         st[i + j] = fmaf(kk[j], ku, st[i + j]);
     }
-    const float o = rq * fmaf(ku, dots[2], sq);
-    const float ss = wave_sum(slice == 0 && owner ? o * o : 0.f);
-    if (lane == 0)
-      red[wave] = ss;
-    __syncthreads();
-    if (slice == 0 && owner) {
-      float t = 0.f;
-      for (int w = 0; w < vcols / 64; ++w)
-        t += red[w];
-      const float f = 1.0f / sqrtf(t / (float)vdim + s.eps);
-      store_act<T>(static_cast<T *>(a.out) + (int64_t)r * a.out_ld + (int64_t)h * vdim + c,
-                   o * f * s.norm_w[c] * gate[c]);
-    }
-    __syncthreads(); // the next row takes the places of this one
+    if (slice == 0 && owner)
+      a.o[(int64_t)r * s.heads * vdim + (int64_t)h * vdim + v0 + c] = rq * fmaf(ku, dots[2], sq);
+    if (r + 1 < a.rows)
+      __syncthreads(); // the next row takes the places of this one
   }
 #pragma unroll
   for (int i = 0; i < N; ++i)
@@ -210,7 +259,7 @@ int keep_rows(const DeltaRows &a, hipStream_t stream) {
 
 bool delta_ok(const DeltaRows &a) {
   const DeltaShape &s = a.s;
-  return a.proj && a.ring && a.state && a.out && a.rows > 0 && (!a.pos || a.rows == 1) && s.heads > 0 &&
+  return a.proj && a.ring && a.state && a.rows > 0 && (!a.pos || a.rows == 1) && s.heads > 0 &&
          s.kv_heads > 0 && s.heads % s.kv_heads == 0 && s.dim > 0 && s.vdim > 0 && s.taps > 0 &&
          s.decay_rank > 0 && s.gate_rank > 0 && s.channels > 0 && s.conv_w && s.decay_w && s.gate_w &&
          s.decay_bias && s.decay_speed && s.norm_w;
@@ -222,6 +271,7 @@ bool delta_ok(const DeltaRows &a) {
 constexpr int kC = kDeltaChunk, kBlock = 16, kBlocks = kC / kBlock;
 constexpr int kChunkThreads = 512;
 constexpr float kLog2e = 1.44269504088896341f;
+constexpr float kLeast = -200.f; // of a decay's log2: 2^-200 is no f32 number, the same as none left
 __device__ __forceinline__ float exp2_f(float x) { return __builtin_amdgcn_exp2f(x); }
 
 // Where the parts of a chunk and head lie in the workspace, in floats.
@@ -253,14 +303,97 @@ struct DeltaPrepArgs {
   float *dots; // [rows][kv_heads]: q . k
 };
 
+constexpr int kPrepRows = 8;
+
+// A column of kPrepRows rows through a convolution of TAPS taps: all inputs are asked
+// for at once, and each is loaded once.
+template <int TAPS>
+__device__ __forceinline__ void conv_rows(const DeltaPrepArgs &a, int r0, int c, float (&out)[kPrepRows]) {
+  const DeltaShape &s = a.s;
+  float x[kPrepRows + TAPS - 1], w[TAPS];
+#pragma unroll
+  for (int i = 0; i < kPrepRows + TAPS - 1; ++i)
+    x[i] = a.proj[(int64_t)min(r0 + i - (TAPS - 1), a.rows - 1) * a.ld + c];
+#pragma unroll
+  for (int t = 0; t < TAPS; ++t)
+    w[t] = s.conv_w[(int64_t)t * s.channels + c];
+#pragma unroll
+  for (int r = 0; r < kPrepRows; ++r) {
+    float v = 0.f;
+#pragma unroll
+    for (int t = 0; t < TAPS; ++t)
+      v = fmaf(w[t], x[r + t], v);
+    out[r] = silu_f(v);
+  }
+}
+
+// A wavefront per kPrepRows rows and head (not the first rows, whose convolution reaches
+// into the ring), like delta_prep_kernel; heads of at most 128 values.
+template <int TAPS> __global__ void __launch_bounds__(256) delta_prep_rows_kernel(DeltaPrepArgs a) {
+  const DeltaShape &s = a.s;
+  const int lane = threadIdx.x & 63;
+  const int u = blockIdx.y * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r0 = (blockIdx.x + 1) * kPrepRows;
+  if (u >= s.kv_heads + s.heads)
+    return;
+  float *out = a.conv + (int64_t)r0 * s.channels;
+  const int rows = min(kPrepRows, a.rows - r0);
+  if (u >= s.kv_heads) {
+    const int at = s.v_at + (u - s.kv_heads) * s.vdim;
+    for (int i = lane; i < s.vdim; i += 64) {
+      float v[kPrepRows];
+      conv_rows<TAPS>(a, r0, at + i, v);
+#pragma unroll
+      for (int r = 0; r < kPrepRows; ++r)
+        if (r < rows)
+          out[(int64_t)r * s.channels + at + i] = v[r];
+    }
+    return;
+  }
+  const int qa = s.q_at + u * s.dim, ka = s.k_at + u * s.dim;
+  float q[2][kPrepRows], k[2][kPrepRows];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    const int i = lane + j * 64;
+    if (i < s.dim) {
+      conv_rows<TAPS>(a, r0, qa + i, q[j]);
+      conv_rows<TAPS>(a, r0, ka + i, k[j]);
+    } else {
+#pragma unroll
+      for (int r = 0; r < kPrepRows; ++r)
+        q[j][r] = k[j][r] = 0.f;
+    }
+  }
+  const float root = sqrtf((float)s.dim);
+#pragma unroll
+  for (int r = 0; r < kPrepRows; ++r) {
+    const float qq = wave_sum(fmaf(q[0][r], q[0][r], q[1][r] * q[1][r]));
+    const float kk = wave_sum(fmaf(k[0][r], k[0][r], k[1][r] * k[1][r]));
+    const float qk = wave_sum(fmaf(q[0][r], k[0][r], q[1][r] * k[1][r]));
+    const float rq = 1.0f / sqrtf(qq + kUnitEps) / root, rk = 1.0f / sqrtf(kk + kUnitEps);
+    if (r >= rows)
+      continue;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int i = lane + j * 64;
+      if (i < s.dim) {
+        out[(int64_t)r * s.channels + qa + i] = q[j][r] * rq;
+        out[(int64_t)r * s.channels + ka + i] = k[j][r] * rk;
+      }
+    }
+    if (lane == 0)
+      a.dots[(int64_t)(r0 + r) * s.kv_heads + u] = qk * rq * rk;
+  }
+}
+
 // A wavefront per row and head: convolution and silu of a query and key head, made unit
 // vectors, or of a value head.
-__global__ void __launch_bounds__(256) delta_prep_kernel(DeltaPrepArgs a) {
+__global__ void __launch_bounds__(256) delta_prep_kernel(DeltaPrepArgs a, int rows) {
   const DeltaShape &s = a.s;
   const int lane = threadIdx.x & 63;
   const int64_t id = (int64_t)blockIdx.x * 4 + __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int units = s.kv_heads + s.heads;
-  if (id >= (int64_t)a.rows * units)
+  if (id >= (int64_t)rows * units)
     return;
   const int r = (int)(id / units), u = (int)(id - (int64_t)r * units), p = a.start + r;
   const float *row = a.proj + (int64_t)r * a.ld;
@@ -307,6 +440,7 @@ struct DeltaChunkArgs {
   const float *conv, *dots, *decay; // decay: [rows][ld_decay], before bias and softplus
   const float *proj;
   int ld, ld_decay, rows;
+  bool quads; // rows can be read four floats at a time
   float *parts;
   ChunkParts at;
 };
@@ -331,14 +465,47 @@ __global__ void __launch_bounds__(kChunkThreads) delta_chunk_kernel(DeltaChunkAr
   {
     const float speed = s.decay_speed[h] * kLog2e;
     const float *conv = a.conv + (int64_t)r0 * s.channels;
-    for (int i = tid; i < kC * dp; i += kChunkThreads) {
+    const float *bias = s.decay_bias + h * dim, *raw = a.decay + (int64_t)r0 * a.ld_decay + h * dim;
+    if (a.quads) { // four channels a time, several rows in flight
+      const int cols = dp / 4, per = kChunkThreads / cols, d = tid % cols * 4;
+      const int dl = d < dim ? d : 0;
+      const f32x4 bb = *reinterpret_cast<const f32x4 *>(bias + dl);
+      constexpr int kFlight = 4;
+      for (int t0 = tid / cols; t0 < kC && tid < per * cols; t0 += per * kFlight) {
+        f32x4 k[kFlight], q[kFlight], z[kFlight];
+#pragma unroll
+        for (int i = 0; i < kFlight; ++i) {
+          const int64_t r = min(t0 + i * per, rows - 1);
+          k[i] = *reinterpret_cast<const f32x4 *>(conv + r * s.channels + s.k_at + g * dim + dl);
+          q[i] = *reinterpret_cast<const f32x4 *>(conv + r * s.channels + s.q_at + g * dim + dl);
+          z[i] = *reinterpret_cast<const f32x4 *>(raw + r * a.ld_decay + dl);
+        }
+#pragma unroll
+        for (int i = 0; i < kFlight; ++i) {
+          const int t = t0 + i * per;
+          if (t >= kC)
+            continue;
+          const bool some = t < rows && d < dim; // a row past the last: no write, no decay
+          f32x4 l;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            l[j] = some ? fmaxf(speed * softplus_f(z[i][j] + bb[j]), kLeast) : 0.f;
+            k[i][j] = some ? k[i][j] : 0.f;
+            q[i][j] = some ? q[i][j] : 0.f;
+          }
+          *reinterpret_cast<f32x4 *>(ks + t * row_at + d) = k[i];
+          *reinterpret_cast<f32x4 *>(qs + t * row_at + d) = q[i];
+          *reinterpret_cast<f32x4 *>(gs + t * row_at + d) = l;
+        }
+      }
+    }
+    for (int i = tid; !a.quads && i < kC * dp; i += kChunkThreads) {
       const int r = i / dp, d = i - r * dp;
       float k = 0.f, q = 0.f, l = 0.f; // a row past the last: no write, no decay
       if (r < rows && d < dim) {
         k = conv[(int64_t)r * s.channels + s.k_at + g * dim + d];
         q = conv[(int64_t)r * s.channels + s.q_at + g * dim + d];
-        l = speed * softplus_f(a.decay[(int64_t)(r0 + r) * a.ld_decay + h * dim + d] + s.decay_bias[h * dim + d]);
-        l = fmaxf(l, -200.f); // 2^-200 is no f32 number: the same as none left
+        l = fmaxf(speed * softplus_f(raw[(int64_t)r * a.ld_decay + d] + bias[d]), kLeast);
       }
       ks[r * row_at + d] = k;
       qs[r * row_at + d] = q;
@@ -477,16 +644,16 @@ __global__ void __launch_bounds__(kChunkThreads) delta_chunk_kernel(DeltaChunkAr
     }
 #pragma unroll
     for (int t = 1; t < kC; ++t) {
-      float sum = x[t];
+      float sum[4] = {x[t], 0.f, 0.f, 0.f}; // four sums: none waits for the one before
 #pragma unroll
       for (int y = 0; y < t; y += 4) {
         const f32x4 m = *reinterpret_cast<const f32x4 *>(as + t * kARow + y);
 #pragma unroll
         for (int j = 0; j < 4; ++j)
           if (y + j < t)
-            sum = fmaf(-m[j], x[y + j], sum);
+            sum[j] = fmaf(-m[j], x[y + j], sum[j]);
       }
-      x[t] = sum;
+      x[t] = (sum[0] + sum[1]) + (sum[2] + sum[3]);
     }
     if (i < dp) {
 #pragma unroll
@@ -668,37 +835,41 @@ Workspace workspace(const DeltaShape &s, int rows) {
 
 int launch_delta_scan(const DeltaRows &a, hipStream_t stream) {
   const DeltaShape &s = a.s;
-  BH_REQUIRE(delta_ok(a), "delta_scan: bad argument");
-  const int vcols = (int)round_up(s.vdim, 64);
-  BH_REQUIRE(vcols <= kScanThreads, "delta_scan: value heads of %d", s.vdim);
-  const int slices = kScanThreads / vcols, per = (int)ceil_div(s.dim, slices);
-  const int rows_per = per <= 8 ? 8 : per <= 16 ? 16 : per <= 32 ? 32 : 64;
-  const size_t lds = sizeof(float) * (3 * (size_t)slices * rows_per + 2 * (size_t)s.vdim + round_up(s.decay_rank, 4) +
-                                      round_up(s.gate_rank, 4) + 2 * (size_t)slices * vcols);
-  constexpr size_t kLimit = 64 * 1024;
-  BH_REQUIRE(per <= 64 && lds <= kLimit, "delta_scan: a state of %d x %d", s.dim, s.vdim);
-#define BH_SCAN(T, N)                                                                              \
-  hipLaunchKernelGGL((delta_scan_kernel<T, N>), dim3((unsigned)s.heads), dim3(kScanThreads), lds,  \
-                     stream, a)
-#define BH_SCANS(T)                                                                                \
-  do {                                                                                             \
-    if (rows_per == 8)                                                                             \
-      BH_SCAN(T, 8);                                                                               \
-    else if (rows_per == 16)                                                                       \
-      BH_SCAN(T, 16);                                                                              \
-    else if (rows_per == 32)                                                                       \
-      BH_SCAN(T, 32);                                                                              \
-    else                                                                                           \
-      BH_SCAN(T, 64);                                                                              \
-  } while (0)
-  if (a.act_f32)
-    BH_SCANS(float);
+  BH_REQUIRE(delta_ok(a) && a.o && a.gate, "delta_scan: bad argument");
+  const int per = (int)ceil_div(s.dim, kScanSlices);
+  const size_t lds = sizeof(float) * (size_t)(round_up(s.decay_rank, 4) + round_up(s.gate_rank, 4));
+  BH_REQUIRE(per <= 64 && lds <= 40 * 1024, "delta_scan: key heads of %d, ranks of %d and %d", s.dim, s.decay_rank,
+             s.gate_rank);
+  const dim3 grid((unsigned)s.heads, (unsigned)ceil_div(s.vdim, kScanCols));
+#define BH_SCAN(N) hipLaunchKernelGGL(delta_scan_kernel<N>, grid, dim3(kScanThreads), lds, stream, a)
+  if (per <= 4)
+    BH_SCAN(4);
+  else if (per <= 8)
+    BH_SCAN(8);
+  else if (per <= 16)
+    BH_SCAN(16);
+  else if (per <= 32)
+    BH_SCAN(32);
   else
-    BH_SCANS(bf16_bits);
-#undef BH_SCANS
+    BH_SCAN(64);
 #undef BH_SCAN
   BH_CHECK_HIP(hipGetLastError());
   return a.rows > 1 ? keep_rows(a, stream) : BUDDY_HIP_OK;
+}
+
+int launch_delta_gate(const DeltaShape &s, const float *o, const float *gate, int ld_gate, int rows, void *out,
+                      int out_ld, bool act_f32, hipStream_t stream) {
+  BH_REQUIRE(o && gate && out && rows > 0 && s.heads > 0 && s.vdim > 0 && s.norm_w, "delta_gate: bad argument");
+  DeltaGateArgs e{s.heads, s.vdim, rows, ld_gate, out_ld, s.eps};
+  const dim3 grid((unsigned)ceil_div((int64_t)rows * s.heads, 4));
+  if (act_f32)
+    hipLaunchKernelGGL(delta_gate_kernel<float>, grid, dim3(256), 0, stream, o, gate, s.norm_w,
+                       static_cast<float *>(out), e);
+  else
+    hipLaunchKernelGGL(delta_gate_kernel<bf16_bits>, grid, dim3(256), 0, stream, o, gate, s.norm_w,
+                       static_cast<bf16_bits *>(out), e);
+  BH_CHECK_HIP(hipGetLastError());
+  return BUDDY_HIP_OK;
 }
 
 size_t delta_workspace(const DeltaShape &s, int rows) {
@@ -709,7 +880,7 @@ size_t delta_workspace(const DeltaShape &s, int rows) {
 
 int launch_delta_chunks(const DeltaRows &a, float *ws, hipStream_t stream) {
   const DeltaShape &s = a.s;
-  BH_REQUIRE(delta_ok(a) && !a.pos && ws && ((uintptr_t)ws & 15) == 0 && delta_workspace(s, a.rows) > 0 &&
+  BH_REQUIRE(delta_ok(a) && a.out && !a.pos && ws && ((uintptr_t)ws & 15) == 0 && delta_workspace(s, a.rows) > 0 &&
                  s.decay.tiles && s.gate.tiles && s.decay.K == s.decay_rank && s.gate.K == s.gate_rank &&
                  s.decay.N >= s.heads * s.dim && s.gate.N >= s.heads * s.vdim,
              "delta_chunks: bad argument");
@@ -729,14 +900,28 @@ int launch_delta_chunks(const DeltaRows &a, float *ws, hipStream_t stream) {
       return rc;
   }
   DeltaPrepArgs p{s, a.proj, a.ring, a.ld, a.rows, a.start, ws + w.conv, ws + w.dots};
-  hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)ceil_div((int64_t)a.rows * (s.kv_heads + s.heads), 4)),
-                     dim3(256), 0, stream, p);
+  const int units = s.kv_heads + s.heads;
+  const bool blocks = s.dim <= 128 && s.taps >= 2 && s.taps <= 4 && a.rows > kPrepRows;
+  const int singly = blocks ? kPrepRows : a.rows; // the first rows, or all of them
+  hipLaunchKernelGGL(delta_prep_kernel, dim3((unsigned)ceil_div((int64_t)singly * units, 4)), dim3(256), 0, stream, p,
+                     singly);
+  if (blocks) {
+    const dim3 grid((unsigned)ceil_div(a.rows - kPrepRows, kPrepRows), (unsigned)ceil_div(units, 4));
+    if (s.taps == 2)
+      hipLaunchKernelGGL(delta_prep_rows_kernel<2>, grid, dim3(256), 0, stream, p);
+    else if (s.taps == 3)
+      hipLaunchKernelGGL(delta_prep_rows_kernel<3>, grid, dim3(256), 0, stream, p);
+    else
+      hipLaunchKernelGGL(delta_prep_rows_kernel<4>, grid, dim3(256), 0, stream, p);
+  }
   BH_CHECK_HIP(hipGetLastError());
   if ((rc = keep_rows(a, stream)))
     return rc;
   const int chunks = (int)ceil_div(a.rows, kC);
-  DeltaChunkArgs c{s, ws + w.conv, ws + w.dots, ws + w.decay, a.proj, a.ld, s.decay.N, a.rows, ws + w.parts,
-                   chunk_parts(s)};
+  DeltaChunkArgs c{s, ws + w.conv, ws + w.dots, ws + w.decay, a.proj, a.ld, s.decay.N, a.rows, false,
+                   ws + w.parts, chunk_parts(s)};
+  c.quads = s.dim % 4 == 0 && s.q_at % 4 == 0 && s.k_at % 4 == 0 && s.channels % 4 == 0 &&
+            ((uintptr_t)s.decay_bias & 15) == 0;
   static DynLdsOnce once;
   BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)delta_chunk_kernel, (int)kChunkLdsLimit));
   hipLaunchKernelGGL(delta_chunk_kernel, dim3((unsigned)chunks, (unsigned)s.heads), dim3(kChunkThreads),
@@ -754,16 +939,7 @@ int launch_delta_chunks(const DeltaRows &a, float *ws, hipStream_t stream) {
   else
     hipLaunchKernelGGL(delta_carry_kernel<8>, grid, dim3(256), 0, stream, k);
   BH_CHECK_HIP(hipGetLastError());
-  DeltaGateArgs e{s.heads, s.vdim, a.rows, s.gate.N, a.out_ld, s.eps};
-  const dim3 rows_grid((unsigned)ceil_div((int64_t)a.rows * s.heads, 4));
-  if (a.act_f32)
-    hipLaunchKernelGGL(delta_gate_kernel<float>, rows_grid, dim3(256), 0, stream, ws + w.out, ws + w.gate, s.norm_w,
-                       static_cast<float *>(a.out), e);
-  else
-    hipLaunchKernelGGL(delta_gate_kernel<bf16_bits>, rows_grid, dim3(256), 0, stream, ws + w.out, ws + w.gate,
-                       s.norm_w, static_cast<bf16_bits *>(a.out), e);
-  BH_CHECK_HIP(hipGetLastError());
-  return BUDDY_HIP_OK;
+  return launch_delta_gate(s, ws + w.out, ws + w.gate, s.gate.N, a.rows, a.out, a.out_ld, a.act_f32, stream);
 }
 
 } // namespace bh

@@ -34,6 +34,10 @@ template <typename T> __device__ __forceinline__ Frag<float> widened(const Frag<
   else
     return f;
 }
+__device__ __forceinline__ void store_quad(float *p, f32x4 v) { *reinterpret_cast<f32x4 *>(p) = v; }
+__device__ __forceinline__ void store_quad(bf16_bits *p, f32x4 v) {
+  *reinterpret_cast<uint2 *>(p) = uint2{pack_bf(v[0], v[1]), pack_bf(v[2], v[3])};
+}
 __device__ __forceinline__ void set_elem(Frag<float> &f, int j, float v) {
   if (j < 4)
     f.lo[j] = v;
@@ -329,11 +333,14 @@ struct HeadRowsArgs {
   int map_heads, kv_maps, kv_heads, dim, vdim, vdim16, half;
   int ld, q_at, k_at, v_at, rows, start;
   int cache_rows, ring_mask;
+  int quads; // whole heads are rotated, and moved four pairs at a time
   float scale, rot_gain;
 };
 
+constexpr int kValueSlice = 32; // channels of a value head that are turned round at once
+
 // The first `rows` workgroups: a token's queries and keys.  The others: 64 positions of
-// a value head, turned round in LDS.
+// a slice of a value head, turned round in LDS.
 template <typename T>
 __global__ void __launch_bounds__(256)
 head_rows_kernel(const float *__restrict__ proj, T *__restrict__ keys, T *__restrict__ values_t,
@@ -352,6 +359,31 @@ head_rows_kernel(const float *__restrict__ proj, T *__restrict__ keys, T *__rest
     __syncthreads();
     T *qo = queries + (int64_t)blockIdx.x * a.map_heads * dim32;
     const int slot = p & a.ring_mask;
+    if (a.quads) {
+      const int per = a.half / 4;
+      for (int i = tid; i < (a.map_heads + a.kv_maps) * per; i += 256) {
+        const int h = i / per, f = (i - h * per) * 4, g = h - a.map_heads;
+        const float *src = row + (g < 0 ? a.q_at + h * a.dim : a.k_at + g * a.dim) + f;
+        T *dst = (g < 0 ? qo + (int64_t)h * dim32 : keys + ((int64_t)g * a.cache_rows + slot) * dim32) + f;
+        const f32x4 u = *reinterpret_cast<const f32x4 *>(src), v = *reinterpret_cast<const f32x4 *>(src + a.half);
+        const float m = g < 0 ? a.scale : 1.0f;
+        f32x4 x, y;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const float c = lds[f + j] * m, s = lds[a.half + f + j] * m;
+          x[j] = u[j] * c - v[j] * s;
+          y[j] = v[j] * c + u[j] * s;
+        }
+        store_quad(dst, x);
+        store_quad(dst + a.half, y);
+      }
+      const int pad = dim32 - a.dim;
+      for (int i = tid; i < (a.map_heads + a.kv_maps) * pad; i += 256) {
+        const int h = i / pad, d = a.dim + i - h * pad, g = h - a.map_heads;
+        store_act<T>((g < 0 ? qo + (int64_t)h * dim32 : keys + ((int64_t)g * a.cache_rows + slot) * dim32) + d, 0.f);
+      }
+      return;
+    }
     for (int h = tid >> 6; h < a.map_heads + a.kv_maps; h += 4) {
       const int g = h - a.map_heads;
       const float *src = row + (g < 0 ? a.q_at + h * a.dim : a.k_at + g * a.dim);
@@ -362,21 +394,25 @@ head_rows_kernel(const float *__restrict__ proj, T *__restrict__ keys, T *__rest
     }
     return;
   }
-  const int b = blockIdx.x - a.rows, g = b % a.kv_heads;
+  int b = blockIdx.x - a.rows;
+  const int slices = (a.vdim16 + kValueSlice - 1) / kValueSlice, c0 = b % slices * kValueSlice;
+  b /= slices;
+  const int g = b % a.kv_heads;
   const int t0 = (a.start & ~(kTile - 1)) + b / a.kv_heads * kTile; // aligned positions
   const int p0 = max(t0, a.start), p1 = min(t0 + kTile, a.start + a.rows);
-  const int vrow = a.vdim16 + 1;
-  for (int i = tid; i < kTile * a.vdim16; i += 256) {
-    const int r = i / a.vdim16, c = i - r * a.vdim16, p = t0 + r;
-    if (p >= p0 && p < p1)
-      lds[r * vrow + c] = c < a.vdim ? proj[(int64_t)(p - a.start) * a.ld + a.v_at + g * a.vdim + c] : 0.f;
+  constexpr int vrow = kValueSlice + 1;
+#pragma unroll
+  for (int i0 = 0; i0 < kTile * kValueSlice; i0 += 256) {
+    const int i = i0 + tid, r = i / kValueSlice, x = i % kValueSlice, c = c0 + x, p = t0 + r;
+    lds[r * vrow + x] = p >= p0 && p < p1 && c < a.vdim
+                            ? proj[(int64_t)(p - a.start) * a.ld + a.v_at + g * a.vdim + c] : 0.f;
   }
   __syncthreads();
   const int r = tid & 63, p = t0 + r;
   if (p < p0 || p >= p1)
     return;
-  for (int c = tid >> 6; c < a.vdim16; c += 4)
-    store_act<T>(values_t + ((int64_t)g * a.vdim16 + c) * a.cache_rows + (p & a.ring_mask), lds[r * vrow + c]);
+  for (int x = tid >> 6; x < kValueSlice && c0 + x < a.vdim16; x += 4)
+    store_act<T>(values_t + ((int64_t)g * a.vdim16 + c0 + x) * a.cache_rows + (p & a.ring_mask), lds[r * vrow + x]);
 }
 
 struct HeadAttnArgs {
@@ -651,13 +687,13 @@ int launch_attention_any(const HeadRows &a, OUT *out, const HeadAttnArgs &p, hip
 template <typename T> int launch_rows(const HeadRows &a, hipStream_t stream) {
   const HeadShape &s = a.s;
   HeadRowsArgs r{s.map_heads(), s.kv_heads * s.maps, s.kv_heads, s.dim, s.vdim, s.vdim16(), s.rot_dims / 2,
-                 a.ld, a.q_at, a.k_at, a.v_at, a.rows, a.start, s.rows, s.ring_mask, s.scale, s.rot_gain};
+                 a.ld, a.q_at, a.k_at, a.v_at, a.rows, a.start, s.rows, s.ring_mask, 0, s.scale, s.rot_gain};
+  r.quads = s.rot_dims == s.dim && s.dim % 8 == 0 && a.ld % 4 == 0 && a.q_at % 4 == 0 && a.k_at % 4 == 0 &&
+            (((uintptr_t)a.proj | (uintptr_t)a.queries | (uintptr_t)a.keys) & 15) == 0;
   const int value_tiles = (a.start + a.rows - 1) / kTile - a.start / kTile + 1;
-  const size_t lds = sizeof(float) * std::max((size_t)s.rot_dims, (size_t)kTile * (s.vdim16() + 1));
-  static DynLdsOnce once;
-  BH_CHECK_HIP(ensure_dyn_lds(once, (const void *)head_rows_kernel<T>, (int)kLdsLimit));
-  hipLaunchKernelGGL(head_rows_kernel<T>, dim3((unsigned)(a.rows + value_tiles * s.kv_heads)), dim3(256), lds,
-                     stream, a.proj, static_cast<T *>(a.keys), static_cast<T *>(a.values_t),
+  const int value_groups = value_tiles * s.kv_heads * (int)ceil_div(s.vdim16(), kValueSlice);
+  const size_t lds = sizeof(float) * std::max((size_t)s.rot_dims, (size_t)kTile * (kValueSlice + 1));
+  hipLaunchKernelGGL(head_rows_kernel<T>, dim3((unsigned)(a.rows + value_groups)), dim3(256), lds, stream, a.proj, static_cast<T *>(a.keys), static_cast<T *>(a.values_t),
                      static_cast<T *>(a.queries), s.turns, s.dim32(), r);
   BH_CHECK_HIP(hipGetLastError());
   HeadAttnArgs p{s.map_heads(), s.heads / s.kv_heads, s.maps, s.vdim, s.vdim16() / 16, s.dim32(), window_of(s),

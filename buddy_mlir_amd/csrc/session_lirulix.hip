@@ -141,8 +141,8 @@ struct LirulixSession : FolderSession {
   int longest = 1; // visible keys, at most
 
   // one token
-  float *x[2] = {nullptr, nullptr}, *y = nullptr, *proj = nullptr, *mix = nullptr, *act = nullptr,
-        *hrow = nullptr, *part_acc = nullptr, *part_ml = nullptr;
+  float *x[2] = {nullptr, nullptr}, *y = nullptr, *proj = nullptr, *mix = nullptr, *mix_gate = nullptr,
+        *act = nullptr, *hrow = nullptr, *part_acc = nullptr, *part_ml = nullptr;
 
   // a block of a prompt
   float *pf_x = nullptr, *pf_y = nullptr, *pf_proj = nullptr, *pf_maps = nullptr, *pf_delta = nullptr,
@@ -318,8 +318,9 @@ struct LirulixSession : FolderSession {
     hrow = device_zeros<float>((size_t)W);
     y = device_zeros<float>((size_t)width16());
     proj = device_zeros<float>((size_t)max_proj);
-    mix = device_zeros<float>((size_t)mix_max);
-    act = device_zeros<float>((size_t)ff_max);
+    mix = device_zeros<float>((size_t)round_up(mix_max, 64));
+    mix_gate = device_zeros<float>((size_t)round_up(mix_max, 64));
+    act = device_zeros<float>((size_t)round_up(ff_max, 64));
     if (parts) {
       part_acc = device_zeros<float>((size_t)parts);
       part_ml = device_zeros<float>((size_t)parts_ml);
@@ -372,10 +373,18 @@ struct LirulixSession : FolderSession {
       }
       return launch_row_gemv(g, stream);
     };
-    auto plain_gemv = [&](const Bf16Matrix &M, const float *src) {
+    auto plain_gemv = [&](const Bf16Matrix &M, const float *src, const DeltaShape *delta = nullptr) {
       RowGemv g;
+      if (delta) { // the mixer's norm and gate stand ahead of the product
+        g.input = kRowHeadGated;
+        g.weight = delta->norm_w;
+        g.gate = mix_gate;
+        g.head_dim = delta->vdim;
+        g.eps = delta->eps;
+      }
       g.W = M;
       g.src = src;
+      g.src_padded = true;
       g.out = y;
       pending = y;
       return launch_row_gemv(g, stream);
@@ -393,7 +402,8 @@ struct LirulixSession : FolderSession {
         d.pos = state + 1;
         d.ring = r.ring;
         d.state = r.state;
-        d.out = mix;
+        d.o = mix;
+        d.gate = mix_gate;
         rc = launch_delta_scan(d, stream);
       } else {
         HeadStep s;
@@ -411,7 +421,7 @@ struct LirulixSession : FolderSession {
         s.out = mix;
         rc = launch_head_step(s, span, stream);
       }
-      if (rc || (rc = plain_gemv(L.o, mix)))
+      if (rc || (rc = plain_gemv(L.o, mix, c.kind == kDelta ? &L.delta : nullptr)))
         return rc;
       if (c.ff && ((rc = norm_gemv(L.gate_up, L.norm2, nullptr, act, true)) || (rc = plain_gemv(L.down, act))))
         return rc;
@@ -449,7 +459,7 @@ struct LirulixSession : FolderSession {
         if (L.head.maps > 1 || L.head.gated)
           maps = std::max(maps, (size_t)L.head.map_heads() * L.head.vdim);
       } else {
-        delta = std::max(delta, delta_workspace(L.delta, rows));
+        delta = std::max({delta, delta_workspace(L.delta, rows), 2 * n * L.delta.heads * L.delta.vdim});
       }
       ff = std::max(ff, (size_t)round_up(cfg.layers[i].ff, 16));
     }
@@ -480,8 +490,14 @@ struct LirulixSession : FolderSession {
       d.out = pf_mix;
       d.out_ld = ld_mix;
       d.act_f32 = opt.f32;
-      return n < kScanRows || !delta_workspace(L.delta, n) ? launch_delta_scan(d, stream)
-                                                           : launch_delta_chunks(d, pf_delta, stream);
+      if (n >= kScanRows && delta_workspace(L.delta, n))
+        return launch_delta_chunks(d, pf_delta, stream);
+      const int width = L.delta.heads * L.delta.vdim;
+      d.o = pf_delta;
+      d.gate = pf_delta + (size_t)n * width;
+      const int rc = launch_delta_scan(d, stream);
+      return rc ? rc
+                : launch_delta_gate(L.delta, d.o, d.gate, width, n, pf_mix, ld_mix, opt.f32, stream);
     }
     HeadRows a;
     a.s = L.head;
