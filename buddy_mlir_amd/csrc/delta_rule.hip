@@ -453,13 +453,14 @@ __global__ void __launch_bounds__(kChunkThreads) delta_chunk_kernel(DeltaChunkAr
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int c = blockIdx.x, h = blockIdx.y, g = h / (s.heads / s.kv_heads);
   const int dim = s.dim, dp = a.at.dp, row_at = dp + 4;
-  constexpr int kARow = kC + 4;
+  constexpr int kARow = kC + 4, kIRow = kBlock + 4;
   float *ks = lds;                  // [64][row_at]
   float *qs = ks + kC * row_at;     // [64][row_at]
   float *gs = qs + kC * row_at;     // [64][row_at]: log2 decay, summed from the block's first token
   float *as = gs + kC * row_at;     // [64][kARow]: beta_t a_ts
   float *tot = as + kC * kARow;     // [kBlocks][dp]: a block's sum
   float *beta = tot + kBlocks * dp; // [64]
+  float *inv = beta + kC;           // [64][kIRow]: inverses of the blocks' own triangles
   const int r0 = c * kC, rows = min(kC, a.rows - r0);
   float *out = a.parts + ((int64_t)c * s.heads + h) * a.at.size;
   {
@@ -598,72 +599,110 @@ __global__ void __launch_bounds__(kChunkThreads) delta_chunk_kernel(DeltaChunkAr
     }
   }
   __syncthreads();
-  auto before = [&](int b, int d) { // decay of the blocks ahead of block b
-    float v = 0.f;
-    for (int i = 0; i < b; ++i)
-      v += tot[i * dp + d];
-    return v;
-  };
-  if (wave >= 4) {
-    for (int i = tid - 256; i < kC * dp; i += 256) {
-      const int t = i / dp, d = i - t * dp;
-      out[a.at.q + i] = qs[t * row_at + d] * exp2_f(before(t / kBlock, d) + gs[t * row_at + d]);
-    }
-    for (int i = tid - 256; i < kC * dp; i += 256) {
-      const int d = i / kC, t = i - d * kC, b = t / kBlock;
-      float left = tot[b * dp + d] - gs[t * row_at + d];
-      for (int j = b + 1; j < kBlocks; ++j)
-        left += tot[j * dp + d];
-      out[a.at.kt + i] = ks[t * row_at + d] * exp2_f(left);
-    }
-    for (int d = tid - 256; d < dp; d += 256)
-      out[a.at.last + d] = exp2_f(before(kBlocks, d));
-    return;
-  }
-  // the triangular system, a thread per right-hand side
-  const int v16 = a.at.v16;
-  for (int i = tid; i < dp + v16; i += 256) {
-    float x[kC];
-    if (i < dp) {
+  // the inverse of a block's own triangle, a lane per column, on one wavefront; the
+  // others write what the carry takes as it is
+  if (wave == 0) {
+    const int b = lane >> 4;
+    const float *m = as + b * kBlock * (kARow + 1); // the block's triangle
+    float x[kBlock];
 #pragma unroll
-      for (int b = 0; b < kBlocks; ++b) {
-        const float ahead = before(b, i);
-#pragma unroll
-        for (int t = b * kBlock; t < (b + 1) * kBlock; ++t)
-          x[t] = beta[t] * ks[t * row_at + i] * exp2_f(ahead + gs[t * row_at + i]);
-      }
-    } else {
-      const int v = i - dp;
-      const float *src = a.conv + (int64_t)r0 * s.channels + s.v_at + h * s.vdim + min(v, s.vdim - 1);
-#pragma unroll
-      for (int t = 0; t < kC; ++t)
-        x[t] = src[(int64_t)min(t, rows - 1) * s.channels];
-#pragma unroll
-      for (int t = 0; t < kC; ++t)
-        x[t] = v < s.vdim ? x[t] * beta[t] : 0.f;
-    }
-#pragma unroll
-    for (int t = 1; t < kC; ++t) {
-      float sum[4] = {x[t], 0.f, 0.f, 0.f}; // four sums: none waits for the one before
+    for (int t = 0; t < kBlock; ++t) {
+      float sum[4] = {t == col ? 1.f : 0.f, 0.f, 0.f, 0.f}; // none waits for the one before
 #pragma unroll
       for (int y = 0; y < t; y += 4) {
-        const f32x4 m = *reinterpret_cast<const f32x4 *>(as + t * kARow + y);
+        const f32x4 v = *reinterpret_cast<const f32x4 *>(m + t * kARow + y);
 #pragma unroll
         for (int j = 0; j < 4; ++j)
           if (y + j < t)
-            sum[j] = fmaf(-m[j], x[y + j], sum[j]);
+            sum[j] = fmaf(-v[j], x[y + j], sum[j]);
       }
       x[t] = (sum[0] + sum[1]) + (sum[2] + sum[3]);
+      inv[(b * kBlock + t) * kIRow + col] = x[t];
     }
+  } else {
+    const int id = tid - 64, n = kChunkThreads - 64, cols = dp / 4;
+    for (int i = id; i < kC * cols; i += n) {
+      const int t = i / cols, d = (i - t * cols) * 4;
+      f32x4 l = *reinterpret_cast<const f32x4 *>(gs + t * row_at + d);
+      for (int b = 0; b < t / kBlock; ++b)
+        l += *reinterpret_cast<const f32x4 *>(tot + b * dp + d);
+      f32x4 q = *reinterpret_cast<const f32x4 *>(qs + t * row_at + d);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        q[j] *= exp2_f(l[j]);
+      *reinterpret_cast<f32x4 *>(out + a.at.q + t * dp + d) = q;
+    }
+    for (int i = id; i < kC * cols; i += n) {
+      const int t = i % kC, d = i / kC * 4, b = t / kBlock;
+      f32x4 l = *reinterpret_cast<const f32x4 *>(tot + b * dp + d) - *reinterpret_cast<const f32x4 *>(gs + t * row_at + d);
+      for (int j = b + 1; j < kBlocks; ++j)
+        l += *reinterpret_cast<const f32x4 *>(tot + j * dp + d);
+      const f32x4 k = *reinterpret_cast<const f32x4 *>(ks + t * row_at + d);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        out[a.at.kt + (d + j) * kC + t] = k[j] * exp2_f(l[j]);
+    }
+    for (int d = id; d < dp; d += n)
+      out[a.at.last + d] = exp2_f((tot[d] + tot[dp + d]) + (tot[2 * dp + d] + tot[3 * dp + d]));
+  }
+  __syncthreads();
+  // The triangular system, 16 right-hand sides at a time: block by block, what earlier
+  // blocks wrote is taken off and the block's inverse applied.  A lane's four rows of a
+  // result are its share of the next product's operand as they lie.
+  for (int ct = wave; ct < (dp + a.at.v16) / 16; ct += kChunkThreads / 64) {
+    f32x4 x[kBlocks];
+    const int i = ct * 16 + col, v = i - dp;
     if (i < dp) {
+      float ahead = 0.f;
 #pragma unroll
-      for (int t = 0; t < kC; ++t)
-        out[a.at.w + t * dp + i] = x[t];
+      for (int b = 0; b < kBlocks; ++b) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int t = b * kBlock + quad * 4 + r;
+          x[b][r] = beta[t] * ks[t * row_at + i] * exp2_f(ahead + gs[t * row_at + i]);
+        }
+        ahead += tot[b * dp + i];
+      }
     } else {
-      float *u = out + a.at.ut + (i - dp) * kC;
+      const float *src = a.conv + (int64_t)r0 * s.channels + s.v_at + h * s.vdim + min(v, s.vdim - 1);
 #pragma unroll
-      for (int t = 0; t < kC; t += 4)
-        *reinterpret_cast<f32x4 *>(u + t) = f32x4{x[t], x[t + 1], x[t + 2], x[t + 3]};
+      for (int b = 0; b < kBlocks; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          x[b][r] = src[(int64_t)min(b * kBlock + quad * 4 + r, rows - 1) * s.channels];
+#pragma unroll
+      for (int b = 0; b < kBlocks; ++b)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          x[b][r] = v < s.vdim ? x[b][r] * beta[b * kBlock + quad * 4 + r] : 0.f;
+    }
+#pragma unroll
+    for (int b = 0; b < kBlocks; ++b) {
+      f32x4 rhs = x[b];
+#pragma unroll
+      for (int e = 0; e < b; ++e) {
+        const f32x4 m = *reinterpret_cast<const f32x4 *>(as + (b * kBlock + col) * kARow + e * kBlock + quad * 4);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          rhs = mfma_f32(-m[j], x[e][j], rhs);
+      }
+      const f32x4 m = *reinterpret_cast<const f32x4 *>(inv + (b * kBlock + col) * kIRow + quad * 4);
+      f32x4 y{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        y = mfma_f32(m[j], rhs[j], y);
+      x[b] = y;
+    }
+#pragma unroll
+    for (int b = 0; b < kBlocks; ++b) {
+      const int t = b * kBlock + quad * 4;
+      if (i < dp) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          out[a.at.w + (t + r) * dp + i] = x[b][r];
+      } else {
+        *reinterpret_cast<f32x4 *>(out + a.at.ut + v * kC + t) = x[b];
+      }
     }
   }
 }
@@ -807,7 +846,7 @@ delta_gate_kernel(const float *__restrict__ o, const float *__restrict__ gate, c
 
 constexpr size_t kChunkLdsLimit = 156 * 1024;
 size_t chunk_lds(const DeltaShape &s) {
-  return sizeof(float) * ((size_t)3 * kC * (s.dim32() + 4) + (size_t)kC * (kC + 4) + kBlocks * s.dim32() + kC);
+  return sizeof(float) * ((size_t)3 * kC * (s.dim32() + 4) + (size_t)kC * (kC + 4) + kBlocks * s.dim32() + kC + kC * (kBlock + 4));
 }
 struct Workspace {
   size_t conv, dots, decay, gate, out, parts, size; // offsets in floats
