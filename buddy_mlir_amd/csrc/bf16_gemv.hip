@@ -584,7 +584,8 @@ moe_down_kernel(const uint4 *__restrict__ down, const float *__restrict__ act,
   // lane j: the j-th chosen expert and its softmax weight
   const int cj = a.top > 0 ? chosen[min(lane, a.top - 1)] : 0;
   const float zj = lane < a.top ? a.chosen_logit[lane] : -INFINITY;
-  const float ej = lane < a.top ? expf(zj - wave_max(zj)) : 0.f;
+  const float most = wave_max(zj); // with all lanes, not under the condition below
+  const float ej = lane < a.top ? expf(zj - most) : 0.f;
   const float wj = ej / wave_sum(ej);
 
   const int routed = a.top * a.ktiles, total = routed + a.shared_ktiles;

@@ -252,7 +252,8 @@ __global__ void __launch_bounds__(256) route_pick_kernel(RouteRows a) {
       }
     }
   }
-  const float e = lane < a.top ? expf(mine - wave_max(mine)) : 0.f;
+  const float most = wave_max(mine); // with all lanes, not under the condition below
+  const float e = lane < a.top ? expf(mine - most) : 0.f;
   const float w = e / wave_sum(e);
   if (lane < a.top) {
     a.chosen[row * a.top + lane] = mine_idx;
