@@ -64,6 +64,20 @@ template <> __device__ __forceinline__ void store4<bf16_bits>(bf16_bits *p, f32x
   *reinterpret_cast<uint2 *>(p) = uint2{pack_bf(v[0], v[1]), pack_bf(v[2], v[3])};
 }
 
+// Workgroups go to the eight dies in turn, each with an L2 of its own.  A die takes a run
+// of tiles, in panels of kPanel column blocks by all row blocks: the workgroups that it
+// runs at the same time share rows and channels.
+constexpr int kDies = 8, kPanel = 4;
+__device__ __forceinline__ void place_tile(int &bx, int &by) {
+  const int gx = gridDim.x, gy = gridDim.y, total = gx * gy, id = blockIdx.y * gx + blockIdx.x;
+  const int die = id % kDies, q = total / kDies, r = total % kDies;
+  const int t = die * q + min(die, r) + id / kDies;
+  const int panel = t / (kPanel * gy), rest = t - panel * kPanel * gy;
+  const int width = min(kPanel, gx - panel * kPanel);
+  by = rest / width;
+  bx = panel * kPanel + rest - by * width;
+}
+
 template <typename T, int RT, int GT, int OUT, bool GROUPED>
 __global__ void __launch_bounds__(kGemmThreads)
 rows_gemm_kernel(const uint4 *__restrict__ W, int ktiles, int steps, GemmDev a) {
@@ -77,7 +91,10 @@ rows_gemm_kernel(const uint4 *__restrict__ W, int ktiles, int steps, GemmDev a) 
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
 
-  int row0 = blockIdx.y * kRows, rows = a.rows;
+  int bx = blockIdx.x, by = blockIdx.y;
+  if constexpr (!GROUPED)
+    place_tile(bx, by);
+  int row0 = by * kRows, rows = a.rows;
   const int *list = nullptr;
   if constexpr (GROUPED) {
     // blockIdx.y counts the row blocks of all experts: find this one's expert
@@ -130,7 +147,7 @@ rows_gemm_kernel(const uint4 *__restrict__ W, int ktiles, int steps, GemmDev a) 
     src[i] = static_cast<const T *>(a.A) + (int64_t)pr * a.lda;
   }
 
-  const int ch0 = (blockIdx.x * 4 + wave) * kGroups; // first channel group of this wavefront
+  const int ch0 = (bx * 4 + wave) * kGroups; // first channel group of this wavefront
   const uint4 *wp[GT];
 #pragma unroll
   for (int g = 0; g < GT; ++g) {
